@@ -28,7 +28,10 @@ elements of a token are divided by their one root mean square, weights ``q_norm`
 size, and likewise the keys); values that are the keys (``values_are_keys``: there is no ``v``
 projection, a key head's value is that head's key as projected, bias included, before any norm); a
 query temperature (``q_temp`` = (coef, every): the normed queries at position ``p`` are multiplied by
-``1 + coef * ln(floor((p + 1) / every) + 1)``, float32).
+``1 + coef * ln(floor((p + 1) / every) + 1)``, float32); turned values (``value_turn``, a base: the value
+of position ``j`` is rotated by ``j`` over all its elements, first half against second half with
+frequencies ``base^(-2m/value_dim)``, and cached so; each head's output at position ``i`` is rotated back
+by ``i``, so that what a query takes from a key depends on their distance alone).
 """
 
 from __future__ import annotations
@@ -40,6 +43,7 @@ import torch
 from ..registry import part_class, register_part
 from .base import Mixer
 from .plan import CacheSpec, PartSpec, TensorDecl
+from .rope import half_frequencies
 
 
 @register_part("mixer", "gqa_attention")
@@ -65,6 +69,7 @@ class GroupedQueryAttention(Mixer):
         qk_norm_scope: str = "head",
         values_are_keys: bool = False,
         q_temp: tuple[float, int] | None = None,
+        value_turn: float | None = None,
         tensors=None,
     ):
         super().__init__(tensors)
@@ -107,6 +112,14 @@ class GroupedQueryAttention(Mixer):
                                       "over the whole projection")
         if self.values_are_keys and self.value_dim != self.head_dim:
             raise ValueError("values that are the keys have the keys' size")
+        self.value_turn = self.turn_freq_cpu = self.turn_freq = self.turn_key = None
+        if value_turn is not None:
+            if self.joint_norm or output_gate or self.value_dim % 2:
+                raise ValueError("turned values have an even size, and go without a q/k norm over the whole projection "
+                                 "and without an output gate")
+            self.value_turn = float(value_turn)
+            self.turn_freq_cpu = half_frequencies(self.value_dim, self.value_turn)
+            self.turn_key = ("rope_half", self.value_dim, self.value_turn)
         self.position = None
         if position is not None:
             self.position = part_class("position", position.kind)(**position.args, tensors=position.tensors)
@@ -150,6 +163,8 @@ class GroupedQueryAttention(Mixer):
             + ([self._name("g")] if self.output_gate else [])
         self.qkv = fetch.fused(names, dim=0)
         self.o = fetch.matrix(self._name("o"))
+        if self.turn_freq_cpu is not None:
+            self.turn_freq = fetch.constant(self.turn_freq_cpu)
         if self.has_bias:  # one vector over the product's columns; a gate's columns get zeros
             pieces = [fetch.vector_f32(self._name(n)) for n in ("q_bias", "k_bias", "v_bias")[: 2 if self.values_are_keys else 3]]
             if self.output_gate:
@@ -197,7 +212,7 @@ class GroupedQueryAttention(Mixer):
             self.position.rotate_in_place(ctx, qkv, nq + nkv, self.bias)
         elif self.bias is not None:
             ops.bias_rotate_pairs(qkv, self.bias, ctx.positions, None, 0, d)
-        fused = self.position is None or in_place or self.position.fused_form == "neox_full"
+        fused = self.position is None or in_place or self.position.fused_form in ("neox_full", "half")
         inv_freq = None if self.position is None or in_place or not fused else self.position.inv_freq
         # what only some designs have travels by name, and only where it is set
         more = {}
@@ -211,11 +226,16 @@ class GroupedQueryAttention(Mixer):
             more["keep_first"] = self.keep_first
         if self.sink:
             more["sink"] = True
+        if self.turn_freq is not None:
+            if not fused:
+                raise NotImplementedError("turned values beside an encoding without a fused form")
+            more["value_turn"] = (self.turn_freq, self.turn_key)
         gate_width = nq * dv if self.output_gate else 0
         if gate_width:
             # the gate's columns stay where the product put them: the attention reads them there
             more["gate"] = qkv[:, qkv.shape[1] - gate_width:]
-        if fused and ops.fuses_decode_attention(ctx, qkv, nq, nkv, d, cache, **more):
+        if fused and ops.fuses_decode_attention(ctx, qkv, nq, nkv, d, cache,
+                                                **({"rot_pairs": inv_freq.numel()} if inv_freq is not None else {}), **more):
             # a step of single tokens: all of it inside the attention kernel
             attn = ops.decode_attention(qkv, cache, ctx, nq, nkv, d, self.scale, self.window,
                                         self.q_norm, self.k_norm, eps, inv_freq,
@@ -223,7 +243,7 @@ class GroupedQueryAttention(Mixer):
             return ops.linear_for_residual(attn, self.o)
         if fused:
             # norm, rotation and the cache write in one pass over qkv
-            shape = {k: more[k] for k in ("value_dim",) if k in more}
+            shape = {k: more[k] for k in ("value_dim", "value_turn") if k in more}
             if gate_width:
                 shape["extra"] = gate_width
             q = ops.qk_norm_rope_store(

@@ -145,9 +145,10 @@ class Norm(Part):
 class PositionEncoding(Part):
     role = "position"
     # An encoding that the fused q/k kernel can apply itself says which of the kernel's forms
-    # it is; the attention mixer then never calls ``rotate``. The one form there is:
+    # it is; the attention mixer then never calls ``rotate``. The forms there are:
     # ``"neox_full"``, the rotation of all ``head_dim`` elements, first half against second
-    # half, by the angles ``position * self.inv_freq[j]`` (float32 [head_dim / 2] on the device).
+    # half, by the angles ``position * self.inv_freq[j]`` (float32 [head_dim / 2] on the device);
+    # ``"half"``, the same over the first ``2 len(inv_freq)`` elements, the others passing unchanged.
     # None (the default) means the mixer norms, calls ``rotate`` and stores, as three steps.
     fused_form: str | None = None
     # Encodings with equal keys rotate by equal angles: the layers of a step then share one table
@@ -178,11 +179,14 @@ class StreamUpdate:
 class NormedUpdate:
     """A sub-layer output that joins the residual stream through a norm of its own:
     ``x <- x + y / rms(y) * weight`` (``rms`` with ``eps`` inside the root). Like a plain ``delta``
-    it is applied by the norm that comes next, which also normalises the sum."""
+    it is applied by the norm that comes next, which also normalises the sum, or by the sub-layer's
+    block that reads the stream as it is. ``groups``: ``y`` is divided into that many equal parts, each
+    over its own ``rms``."""
 
     y: torch.Tensor       # [T, H], or float32 planes [P, T, H] whose sum it is
     weight: torch.Tensor  # float32 [H]
     eps: float
+    groups: int = 1
 
 
 @dataclass

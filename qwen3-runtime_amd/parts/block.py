@@ -1,6 +1,7 @@
 """Arrangements of a layer's parts: the pre-norm residual block, over one residual stream or
-over several (hyper-connections), the block with a norm on both sides of each sub-layer, and
-the block whose mixer and feed-forward read one norm and join the stream in one scaled sum.
+over several (hyper-connections), the block with a norm on both sides of each sub-layer, the
+block with a norm behind each sub-layer only, and the block whose mixer and feed-forward read one
+norm and join the stream in one scaled sum.
 
 ``x += mixer(norm_in(x)); x += feed_forward(norm_post(x))``: the form the
 reference's oracle writes (tests/cpu/reference_qwen3.py:79-110) and its model
@@ -69,6 +70,46 @@ class SandwichNormBlock(Block):
             return residual, pending
         x = self.norm_post.forward(ctx, residual, pending)
         return residual, NormedUpdate(self.feed_forward.forward(ctx, x), self.after_ff.weight, self.after_ff.eps)
+
+
+@register_part("block", "output_norm")
+class OutputNormBlock(Block):
+    """A norm behind each sub-layer only: ``x += norm_after(mixer(x))``, then
+    ``x += norm_after_ff(feed_forward(x))``. The sub-layers read the stream itself, in the activations'
+    type; the norm travels with a sub-layer's output as a ``NormedUpdate``, which is applied in the
+    pass that reads the stream for the next sub-layer (or by the model's last norm)."""
+
+    norm_names = ("after_mixer", "after_ff")
+
+    def __init__(self, mixer, feed_forward, norms, tensors=None):
+        super().__init__(tensors)
+        self.mixer = mixer
+        self.feed_forward = feed_forward
+        self.after_mixer, self.after_ff = norms["after_mixer"], norms.get("after_ff")
+        if (feed_forward is None) != (self.after_ff is None):
+            raise ValueError("a feed-forward and the norm behind it come together")
+
+    def children(self):
+        return tuple(p for p in (self.mixer, self.after_mixer, self.feed_forward, self.after_ff) if p is not None)
+
+    @staticmethod
+    def _read(ctx, residual, delta):
+        """Apply what is pending to the stream and return the stream as the sub-layers read it."""
+        if delta is None:
+            return ctx.ops.group_norm_update(residual, None, None, None, 1, ctx.dtype)
+        return ctx.ops.group_norm_update(residual, delta.y, (delta.weight, delta.eps), None, delta.groups, ctx.dtype)
+
+    @staticmethod
+    def _pending(y, norm):
+        return NormedUpdate(y, norm.weight, norm.eps, norm.groups)
+
+    def forward(self, ctx, residual, delta, cache):
+        x = self._read(ctx, residual, delta)
+        pending = self._pending(self.mixer.forward(ctx, x, cache), self.after_mixer)
+        if self.feed_forward is None:
+            return residual, pending
+        x = self._read(ctx, residual, pending)
+        return residual, self._pending(self.feed_forward.forward(ctx, x), self.after_ff)
 
 
 @register_part("block", "hyper_connections")

@@ -5,7 +5,7 @@
 no bias and no scaling of logits (reference: qwen3_runtime/models/qwen3.py:265-266).
 The embedding starts the float32 residual stream; logits come out in float32.
 Either takes a constant ``scale`` (1 by default): the embedding's rows times it, in float32, and
-the float32 logits times it.
+the float32 logits times it. The head's ``softcap``: the logits become ``cap * tanh(logits / cap)``, float32.
 """
 
 from __future__ import annotations
@@ -49,8 +49,9 @@ class LinearHead(Part):
 
     role = "head"
 
-    def __init__(self, vocab_size: int, hidden_size: int, scale: float = 1.0, tensors=None):
+    def __init__(self, vocab_size: int, hidden_size: int, scale: float = 1.0, softcap: float | None = None, tensors=None):
         super().__init__(tensors)
+        self.softcap = None if softcap is None else float(softcap)
         self.vocab_size = int(vocab_size)
         self.hidden_size = int(hidden_size)
         self.scale = float(scale)
@@ -64,7 +65,9 @@ class LinearHead(Part):
 
     def forward(self, ctx, x):
         logits = ctx.ops.linear(x, self.weight, out_f32=True)
-        return logits if self.scale == 1.0 else ctx.ops.scale(logits, self.scale)
+        if self.scale != 1.0:
+            logits = ctx.ops.scale(logits, self.scale)
+        return logits if self.softcap is None else ctx.ops.softcap(logits, self.softcap)
 
     def step_cost(self, spans, rows, elem_bytes):
         # the whole matrix, multiplied with the wanted rows only

@@ -21,6 +21,9 @@ tensor ``correction`` [experts] is added to the scores for the choice alone; the
 chosen experts' scores without it. ``renormalise``: the chosen scores are divided by their sum
 (plus 1e-20). ``weight_scale``: the weights are multiplied by it at the end.
 ``activation="relu2"``: experts without a gate, ``down_e( relu(up_e(x))^2 )``, tensors ``up`` and ``down``.
+``weight_on="input"`` (gated experts): a weight scales its expert's input instead of its output, and the
+outputs are summed as they are: ``sum_j expert_j(w_j x)``. Both of an expert's first products are linear,
+so the weight multiplies them in float32 in front of the activation.
 """
 
 from __future__ import annotations
@@ -40,7 +43,7 @@ class RoutedSwiGLU(FeedForward):
                  router_bias: bool = True, scoring: str = "softmax_top", groups: int = 1, keep: int | None = None,
                  activation: str = "swiglu", limit: float = 0.0, shared_size: int | None = None,
                  shared_limit: float | None = None, group_score: str = "top2", correction: bool = False,
-                 renormalise: bool = False, weight_scale: float = 1.0, tensors=None):
+                 renormalise: bool = False, weight_scale: float = 1.0, weight_on: str = "output", tensors=None):
         super().__init__(tensors)
         self.hidden_size = int(hidden_size)
         self.intermediate_size = int(intermediate_size)
@@ -59,6 +62,9 @@ class RoutedSwiGLU(FeedForward):
         self.has_correction, self.renormalise, self.weight_scale = bool(correction), bool(renormalise), float(weight_scale)
         if (self.has_correction or self.renormalise) and scoring == "softmax_top":
             raise ValueError("a correction of the choice and renormalised weights go with scores over all experts")
+        if weight_on not in ("output", "input") or (weight_on == "input" and not self.gated):
+            raise ValueError(f"weights on the experts' {weight_on!r}: on their output, or on the input of gated experts")
+        self.weight_on = weight_on
         if not self.gated and shared_size:
             raise NotImplementedError("a shared expert beside experts without a gate")
         self.groups = int(groups)
@@ -126,7 +132,8 @@ class RoutedSwiGLU(FeedForward):
 
     def forward(self, ctx, x):
         ops = ctx.ops
-        plain = self.scoring == "softmax_top" and self.groups == 1 and self.activation == "swiglu"
+        plain = (self.scoring == "softmax_top" and self.groups == 1 and self.activation == "swiglu" and not self.shared_size
+                 and self.weight_on == "output")
         if plain:
             index, weight = ops.route_top(x, self.router, self.router_bias, self.top)
             return ops.moe_swiglu(x, self.gate_up, self.down, index, weight)
@@ -136,6 +143,8 @@ class RoutedSwiGLU(FeedForward):
         index, weight = ops.route_top(x, self.router, self.router_bias, self.top, scoring=self.scoring,
                                       groups=self.groups, keep=self.keep, **how)
         more = {"activation": self.activation, "limit": self.limit}
+        if self.weight_on == "input":
+            more["weight_on_input"] = True
         if not self.shared_size:
             return ops.moe_swiglu(x, self.gate_up, self.down, index, weight, **more)
         act = ops.gated_linear(x, self.shared_gate_up, activation=self.activation, limit=self.shared_limit)

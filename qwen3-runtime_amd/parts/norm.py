@@ -16,6 +16,10 @@ sub-layer's output times a weight per stream), and what is normalised is the sum
 streams weighted by ``read``; a ``ScaledUpdate`` (the outputs of sub-layers that ran side by side,
 each times a vector) joins one stream as ``x + sum_i s_i * y_i``; a norm built with ``streams=S`` and called without ``read`` takes
 the plain sum (the model's last norm).
+
+``groups``: the RMS norm in parts: the vector is divided into that many equal parts of neighbours, each
+over its own root mean square, and the whole multiplied by the weight; also the norm on a pending
+output (``NormedUpdate.groups``) that this norm adds first.
 """
 
 from __future__ import annotations
@@ -31,8 +35,13 @@ from .plan import TensorDecl
 class RMSNorm(Norm):
     has_bias = False
 
-    def __init__(self, size: int, eps: float, streams: int = 1, delta_scale: float = 1.0, tensors=None):
+    def __init__(self, size: int, eps: float, streams: int = 1, delta_scale: float = 1.0, groups: int = 1, tensors=None):
         super().__init__(tensors)
+        self.groups = int(groups)
+        if self.groups < 1 or int(size) % self.groups:
+            raise ValueError(f"a norm of {size} elements in {groups} equal parts")
+        if self.groups > 1 and (streams > 1 or self.has_bias or delta_scale != 1.0):
+            raise ValueError("a norm in groups goes with the RMS norm over one stream and the plain sum")
         self.size = int(size)
         self.eps = float(eps)
         self.streams = int(streams)
@@ -61,6 +70,13 @@ class RMSNorm(Norm):
         With ``rows`` (int32 indices) only those rows are normalised and
         returned, packed; ``residual`` is then left as it is.
         """
+        if self.groups > 1 or (isinstance(delta, NormedUpdate) and delta.groups > 1):
+            after = None
+            if isinstance(delta, NormedUpdate):
+                if delta.groups != self.groups:
+                    raise NotImplementedError(f"an update normed in {delta.groups} groups meets a norm in {self.groups}")
+                after, delta = (delta.weight, delta.eps), delta.y
+            return ctx.ops.group_norm_update(residual, delta, after, (self.weight, self.eps), self.groups, ctx.dtype, rows)
         if residual.dim() == 3:  # several streams
             return ctx.ops.mix_norm(residual, delta, self.read_all if read is None else read, self.weight,
                                     self.bias, self.eps, ctx.dtype, rows)

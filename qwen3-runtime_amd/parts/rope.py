@@ -6,6 +6,8 @@ into its first and second half ``x1 | x2`` and rotated pairwise:
 (reference: qwen3_runtime/layers/rope.py:7-21). Angles, sine and cosine are
 float32. The same angles serve every head; values are not rotated.
 
+``rope_half``: the same pairing over the first ``dims`` elements of a head only.
+
 ``rope_pairs``: only the first ``dims`` elements of a head turn, element ``2i`` paired with
 ``2i + 1`` (the interleaved layout): ``(u, v) -> (u cos a - v sin a, v cos a + u sin a)`` with
 ``a = pos * f_i``, ``f_i = base^(-2i/dims)``; the rest of the head passes unchanged. The
@@ -51,6 +53,34 @@ class RotaryNeox(PositionEncoding):
     def rotate(self, ctx, q, k):
         """Unfused form: rotate already-normed q ``[T, nq, D]`` and k ``[T, nkv, D]``."""
         return ctx.ops.rope_neox(q, k, ctx.positions, self.inv_freq)
+
+
+@register_part("position", "rope_half")
+class RotaryHalf(PositionEncoding):
+    """The first ``dims`` elements of a head turn, element ``i`` against ``i + dims / 2``; the rest passes."""
+
+    fused_form = "half"
+
+    def __init__(self, head_dim: int, dims: int, base: float, tensors=None):
+        super().__init__(tensors)
+        if dims % 2 or not 2 <= dims <= head_dim or head_dim % 2:
+            raise ValueError(f"{dims} rotated elements in heads of {head_dim}: both even, the first no larger")
+        self.head_dim, self.dims, self.base = int(head_dim), int(dims), float(base)
+        self.inv_freq_cpu = half_frequencies(self.dims, self.base)
+        self.inv_freq = None
+        self.angles_key = ("rope_half", self.dims, self.base)
+
+    def load(self, fetch):
+        self.inv_freq = fetch.constant(self.inv_freq_cpu)
+
+    def rotate(self, ctx, q, k):
+        raise NotImplementedError("this encoding runs inside the kernel that norms and stores")
+
+
+def half_frequencies(dims: int, base: float) -> torch.Tensor:
+    """``base^(-2i/dims)``, ``i < dims / 2``: computed in float64 and rounded once."""
+    i = torch.arange(dims // 2, dtype=torch.float64)
+    return (base ** (-2.0 * i / dims)).to(torch.float32)
 
 
 @register_part("position", "rope_pairs")

@@ -57,13 +57,14 @@ def head_rmsnorm(x, weight, eps, compute=torch.float32):
     return x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * weight.to(compute)
 
 
-def rope_rotate(x, positions, inv_freq, compute=torch.float32):
-    """x [T, heads, D] (compute dtype); angles = float32(pos) * inv_freq in float32."""
-    d = x.shape[-1]
-    ang = (positions.to(torch.float32)[:, None] * inv_freq.to(torch.float32)[None, :]).to(compute)
+def rope_rotate(x, positions, inv_freq, compute=torch.float32, sign=1.0):
+    """x [T, heads, D] (compute dtype); angles = float32(pos) * inv_freq in float32. The first
+    2 len(inv_freq) elements turn, first half against second half; the others pass."""
+    n = inv_freq.numel()
+    ang = (sign * positions.to(torch.float32)[:, None] * inv_freq.to(torch.float32)[None, :]).to(compute)
     cos, sin = ang.cos()[:, None, :], ang.sin()[:, None, :]
-    x1, x2 = x[..., : d // 2], x[..., d // 2:]
-    return torch.cat((x1 * cos - x2 * sin, x2 * cos + x1 * sin), dim=-1)
+    x1, x2 = x[..., :n], x[..., n: 2 * n]
+    return torch.cat((x1 * cos - x2 * sin, x2 * cos + x1 * sin, x[..., 2 * n:]), dim=-1)
 
 
 def qk_norm_split(qkv, nq, nkv, d, q_w, k_w, eps, compute=torch.float32):
@@ -86,7 +87,8 @@ def kv_store(k, v, k_cache, v_cache, slots, page_size):
 
 def qk_norm_rope_store(qkv, nq, nkv, d, q_w, k_w, eps, inv_freq, positions,
                        k_cache=None, v_cache=None, slots=None, page_size=None, compute=torch.float32,
-                       value_dim=None):
+                       value_dim=None, value_turn=None):
+    """``value_turn`` (frequencies, a name): the values turn by their positions before they are cached."""
     t = qkv.shape[0]
     dv = d if value_dim is None else value_dim
     q = qkv[:, : nq * d].reshape(t, nq, d)
@@ -97,6 +99,8 @@ def qk_norm_rope_store(qkv, nq, nkv, d, q_w, k_w, eps, inv_freq, positions,
     if inv_freq is not None:
         q = rope_rotate(q, positions, inv_freq, compute)
         k = rope_rotate(k, positions, inv_freq, compute)
+    if value_turn is not None:
+        v = rope_rotate(v.to(compute), positions, value_turn[0], compute)
     if k_cache is not None:
         kv_store(k, v, k_cache, v_cache, slots, page_size)
     return q.to(qkv.dtype).reshape(t, nq * d)
@@ -116,8 +120,9 @@ def gather_kv(k_cache, v_cache, table_row, lo, hi, page_size):
 
 def paged_attention(q, k_cache, v_cache, cu_q, kv_lens, block_table, page_size, nq, nkv, d,
                     scale, window=None, compute=torch.float32, round_probs=False, chunk=None, softcap=None,
-                    value_dim=None, gate=None, keep_first=0, sink=False):
-    """q [T, nq*D] -> [T, nq*Dv]. ``keep_first``: beside a window the sequence's first tokens stay
+                    value_dim=None, gate=None, keep_first=0, sink=False, value_turn=None):
+    """q [T, nq*D] -> [T, nq*Dv]. ``value_turn`` (frequencies, a name): each head's output is turned back by
+    the query's position. ``keep_first``: beside a window the sequence's first tokens stay
     visible; ``sink``: one more term of score 0 in the softmax's denominator.
     Query row i of a sequence sits at position
     kv_len - q_len + i and sees keys j <= its position (and > position - window, or, with
@@ -171,7 +176,10 @@ def paged_attention(q, k_cache, v_cache, cu_q, kv_lens, block_table, page_size, 
             probs = torch.softmax(scores, dim=-1)
         if round_probs:
             probs = probs.to(q.dtype).to(compute)
-        ctx = torch.einsum("hqk,khd->qhd", probs, v).reshape(q_len, nq * dv)
+        ctx = torch.einsum("hqk,khd->qhd", probs, v)
+        if value_turn is not None:
+            ctx = rope_rotate(ctx, qpos[:, 0], value_turn[0], compute, sign=-1.0)
+        ctx = ctx.reshape(q_len, nq * dv)
         if gate is not None:
             ctx = ctx * torch.sigmoid(gate[a:b].to(compute))
         out[a:b] = ctx.to(q.dtype)
@@ -253,8 +261,10 @@ def gated(g, u, activation="swiglu", limit=0.0):
     return g * torch.sigmoid(g) * u
 
 
-def moe_swiglu(x, gate_up, down, index, weight, compute=torch.float32, activation="swiglu", limit=0.0):
-    """x [T, H]; gate_up [E, 2I, H]; down [E, H, I]; index/weight [T, top] -> [T, H] (float32)."""
+def moe_swiglu(x, gate_up, down, index, weight, compute=torch.float32, activation="swiglu", limit=0.0,
+               weight_on_input=False):
+    """x [T, H]; gate_up [E, 2I, H]; down [E, H, I]; index/weight [T, top] -> [T, H] (float32).
+    ``weight_on_input``: the weights scale the experts' first products instead of their outputs."""
     t, h = x.shape
     inter = gate_up.shape[1] // 2
     out = torch.zeros((t, h), dtype=torch.float32, device=x.device)
@@ -263,11 +273,14 @@ def moe_swiglu(x, gate_up, down, index, weight, compute=torch.float32, activatio
         for e in index[:, j].unique().tolist():
             sel = (index[:, j] == e).nonzero()[:, 0]
             gu = (xc[sel] @ gate_up[e].to(compute).T).to(x.dtype).to(compute)
+            if weight_on_input:
+                gu = gu * weight[sel, j, None]
             if activation == "relu2":  # no gate: the tensor holds the up rows alone
                 act = torch.relu(gu).pow(2).to(x.dtype).to(compute)
             else:
                 act = gated(gu[:, :inter], gu[:, inter:], activation, limit).to(x.dtype).to(compute)
-            out[sel] += weight[sel, j, None] * (act @ down[e].to(compute).T).to(torch.float32)
+            y = (act @ down[e].to(compute).T).to(torch.float32)
+            out[sel] += y if weight_on_input else weight[sel, j, None] * y
     return out
 
 
@@ -306,8 +319,10 @@ def bias_rotate_pairs(x, bias, positions, freq, rot_heads, head_dim):
     return x
 
 
-def delta_conv(y, channels, taps, tail, cu_q, slots, segments, unit_eps):
-    """Causal convolution + silu + unit vectors per head, span by span; ``tail`` updated in place."""
+def delta_conv(y, channels, taps, tail, cu_q, slots, segments, unit_eps, first=0, bias=None):
+    """Causal convolution (+ ``bias``) + silu + unit vectors per head, span by span, over the columns
+    ``first .. first + channels``; ``tail`` updated in place."""
+    y = y[:, first:]
     k = taps.shape[1]
     out = torch.empty((y.shape[0], channels), dtype=torch.float32, device=y.device)
     for s in range(len(cu_q) - 1):
@@ -315,7 +330,7 @@ def delta_conv(y, channels, taps, tail, cu_q, slots, segments, unit_eps):
         slot = int(slots[s])
         x = y[a:b, :channels].to(torch.float32)
         full = torch.cat([tail[slot, :, : k - 1].T, x], dim=0) if k > 1 else x
-        acc = torch.zeros_like(x)
+        acc = torch.zeros_like(x) if bias is None else bias[None, :].expand_as(x).clone()
         for j in range(k):
             acc = acc + full[j: j + (b - a)] * taps[:, j]
         out[a:b] = acc * torch.sigmoid(acc)
@@ -449,6 +464,56 @@ def retention_rule(qkv, decay, state, cu_q, slots, heads, dim, vdim):
     return out
 
 
+def state_space(xbc, step, dt_bias, a_log, skip, state, cu_q, slots, heads, groups, n, vdim):
+    """S <- exp(-exp(a_log) softplus(step + dt_bias)) S + (softplus(..) x) B^T; y = S C + skip x, per sequence and
+    head from the slot's state [slots, heads, vdim, n]. ``xbc`` float32 [T, heads vdim | groups n | groups n]."""
+    t = xbc.shape[0]
+    x = xbc[:, : heads * vdim].view(t, heads, vdim)
+    b = xbc[:, heads * vdim: heads * vdim + groups * n].reshape(t, groups, n).repeat_interleave(heads // groups, dim=1)
+    c = xbc[:, heads * vdim + groups * n:].reshape(t, groups, n).repeat_interleave(heads // groups, dim=1)
+    dt = torch.nn.functional.softplus(step.to(torch.float32) + dt_bias, threshold=1e9)
+    decay = torch.exp(-torch.exp(a_log)[None, :] * dt)
+    out = torch.empty((t, heads, vdim), dtype=torch.float32, device=xbc.device)
+    for s in range(len(cu_q) - 1):
+        slot = int(slots[s])
+        st = state[slot].clone()  # [heads, vdim, n]
+        for i in range(int(cu_q[s]), int(cu_q[s + 1])):
+            st = st * decay[i][:, None, None] + (dt[i][:, None] * x[i])[:, :, None] * b[i][:, None, :]
+            out[i] = torch.einsum("hvd,hd->hv", st, c[i]) + skip[:, None] * x[i]
+        state[slot] = st
+    return out
+
+
+def group_normed(x, weight, eps, groups):
+    parts = x.reshape(*x.shape[:-1], groups, x.shape[-1] // groups)
+    y = parts * torch.rsqrt(parts.pow(2).mean(-1, keepdim=True) + eps)
+    return y.reshape(x.shape) * weight
+
+
+def gated_group_norm(o, gate, weight, eps, groups, out_dtype):
+    """The read-out [T, heads, vdim] times silu(gate), RMS-normed in ``groups`` equal parts."""
+    z = gate.to(torch.float32)
+    return group_normed(o.reshape(o.shape[0], -1) * z * torch.sigmoid(z), weight, eps, groups).to(out_dtype)
+
+
+def group_norm_update(residual, y, after, norm, groups, out_dtype, rows=None):
+    """``residual += y`` in place, ``y`` first normed in groups if ``after`` = (weight, eps) is given; the rows of
+    the sum normed in groups by ``norm`` = (weight, eps), or (None) as they are. With ``rows`` only those, and
+    ``residual`` is left alone."""
+    x = residual if rows is None else residual[rows.long()]
+    if y is not None:
+        y = planes_sum(y)
+        y = y if rows is None else y[rows.long()]
+        if after is not None:
+            y = group_normed(y, after[0], after[1], groups)
+        if rows is None:
+            residual += y
+            x = residual
+        else:
+            x = x + y
+    return (x if norm is None else group_normed(x, norm[0], norm[1], groups)).to(out_dtype, copy=True)
+
+
 def unary_act(x, kind):
     if kind != "relu2":
         raise ValueError(kind)
@@ -503,6 +568,18 @@ class TorchOps:
 
     def scale(self, x, factor):
         return x.mul_(factor)
+
+    def softcap(self, x, limit):
+        return x.div_(limit).tanh_().mul_(limit)
+
+    def group_norm_update(self, residual, y, after, norm, groups, out_dtype, rows=None):
+        return group_norm_update(residual, y, after, norm, groups, out_dtype, rows)
+
+    def gated_group_norm(self, o, gate, weight, eps, groups, out_dtype):
+        return gated_group_norm(o, gate, weight, eps, groups, out_dtype)
+
+    def state_space(self, ctx, xbc, step, dt_bias, a_log, skip, state, heads, groups, n, vdim):
+        return state_space(xbc, step, dt_bias, a_log, skip, state, ctx.cu_q, ctx.state_slots, heads, groups, n, vdim)
 
     def new_rows(self, t, width, dtype, device):
         return torch.empty((t, width), dtype=dtype, device=device)
@@ -566,8 +643,8 @@ class TorchOps:
     def bias_rotate_pairs(self, x, bias, positions, freq, rot_heads, head_dim):
         return bias_rotate_pairs(x, bias, positions, freq, rot_heads, head_dim)
 
-    def delta_conv(self, ctx, y, channels, taps, tail, segments, unit_eps):
-        return delta_conv(y, channels, taps, tail, ctx.cu_q, ctx.state_slots, segments, unit_eps)
+    def delta_conv(self, ctx, y, channels, taps, tail, segments, unit_eps, first=0, bias=None):
+        return delta_conv(y, channels, taps, tail, ctx.cu_q, ctx.state_slots, segments, unit_eps, first, bias)
 
     def delta_rule(self, ctx, qkv, beta, a_logits, a_log, dt_bias, state, heads, kv_heads, dim, vdim, per_channel):
         return delta_rule(qkv, beta, a_logits, a_log, dt_bias, state, ctx.cu_q, ctx.state_slots, heads, kv_heads,
@@ -583,13 +660,13 @@ class TorchOps:
         return linear(x, w, False, self.compute)
 
     def qk_norm_rope_store(self, qkv, nq, nkv, d, q_w, k_w, eps, inv_freq, positions, cache, ctx=None,
-                           angles_key=None, value_dim=None, extra=0):
+                           angles_key=None, value_dim=None, extra=0, value_turn=None):
         if cache is None:
             return qk_norm_rope_store(qkv, nq, nkv, d, q_w, k_w, eps, inv_freq, positions,
                                       compute=self.compute, value_dim=value_dim)
         return qk_norm_rope_store(qkv, nq, nkv, d, q_w, k_w, eps, inv_freq, positions,
                                   cache.k, cache.v, cache.group.slots, cache.group.page_size, self.compute,
-                                  value_dim=value_dim)
+                                  value_dim=value_dim, value_turn=value_turn)
 
     def mix_norm(self, streams, update, read, weight, bias, eps, out_dtype, rows=None):
         return mix_norm(streams, update, read, weight, bias, eps, out_dtype, rows, self.compute)
@@ -599,8 +676,8 @@ class TorchOps:
         return route_top(x, router, router_bias, top, scoring, groups, keep, group_score, correction, renormalise,
                          weight_scale)
 
-    def moe_swiglu(self, x, gate_up, down, index, weight, activation="swiglu", limit=0.0):
-        return moe_swiglu(x, gate_up, down, index, weight, self.compute, activation, limit)
+    def moe_swiglu(self, x, gate_up, down, index, weight, activation="swiglu", limit=0.0, weight_on_input=False):
+        return moe_swiglu(x, gate_up, down, index, weight, self.compute, activation, limit, weight_on_input)
 
     def fuses_decode_attention(self, ctx, qkv, nq, nkv, d, cache, **more):
         return False  # no one-kernel form of a decode step's attention here: the steps above, in order
@@ -616,10 +693,11 @@ class TorchOps:
         kv_store(k, v, cache.k, cache.v, cache.group.slots, cache.group.page_size)
 
     def paged_attention(self, q, cache, ctx, nq, nkv, d, scale, window, chunk=None, softcap=None, value_dim=None,
-                        gate=None, keep_first=0, sink=False):
+                        gate=None, keep_first=0, sink=False, value_turn=None):
         return paged_attention(q, cache.k, cache.v, ctx.cu_q, ctx.kv_lens, cache.group.block_table,
                                cache.group.page_size, nq, nkv, d, scale, window, self.compute, chunk=chunk,
-                               softcap=softcap, value_dim=value_dim, gate=gate, keep_first=keep_first, sink=sink)
+                               softcap=softcap, value_dim=value_dim, gate=gate, keep_first=keep_first, sink=sink,
+                               value_turn=value_turn)
 
     def swiglu(self, gate_up):
         return swiglu(gate_up, self.compute)
