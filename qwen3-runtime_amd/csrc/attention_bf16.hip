@@ -80,7 +80,7 @@ struct AttnTileArgs {
   long qkv_stride;
   const float* q_weight;   // [D] or null: no norm
   const float* k_weight;
-  const float* rope;       // [T, D]: cosines of the D / 2 angles, then their sines; null: no rotation
+  const float* rope;       // [T, 2 rope_pairs]: cosines of the angles, then their sines; null: no rotation
   const int* slots;        // [T]: place of the token in the cache, page * page_size + offset
   float eps;
   // Decoding over sequences of very different lengths: instead of num_splits equal parts of every
@@ -107,6 +107,11 @@ struct AttnTileArgs {
   // 1: the softmax's denominator has one more term of score 0 and no value,
   // p_j = exp(s_j) / (1 + sum exp(s_j)): added where the sums are final (here, or in the merge).
   int sink;
+  int rope_pairs;          // with `rope`: pairs (j, j + rope_pairs) that turn, a multiple of 32 up to D / 2
+  // Turned values: [T, D], the cosines of a token's D / 2 angles, then their sines; null: values as they
+  // are. The cached values are turned by their own positions, element j against j + D / 2, and a row's
+  // output is turned back by its token's angles where it is written (here, or in the merge).
+  const float* turn;
 };
 
 // The first key position that the query at position p sees. It does not fall as p grows, so for a
@@ -141,6 +146,40 @@ __device__ __forceinline__ float gate_factor(const bf16_t* __restrict__ gate, lo
   return 1.0f / (1.0f + __expf(-x));
 }
 
+// A row's output turned back by its token's angles (`angles`: cosines, then sines), in the registers of
+// the prompt kernels: this lane holds elements 16 i + 4 quad + r of its row. With D a multiple of 32 an
+// element and its partner D / 2 away lie in one lane; else the partner lies in the lane two quads away
+// (all four lanes of a row come here together).
+__device__ __forceinline__ void turn_back(f32x4_t* o, const float* __restrict__ angles, int quad) {
+  if constexpr (DB % 2 == 0) {
+#pragma unroll
+    for (int i = 0; i < DB / 2; ++i) {
+      const f32x4_t c = *(const f32x4_t*)(angles + 16 * i + 4 * quad), s = *(const f32x4_t*)(angles + D / 2 + 16 * i + 4 * quad);
+      const f32x4_t u = o[i], v = o[i + DB / 2];
+      o[i] = u * c + v * s;
+      o[i + DB / 2] = v * c - u * s;
+    }
+  } else {
+    constexpr int H = (DB - 1) / 2;
+    const bool upper = quad >= 2;
+    f32x4_t across[DB];
+#pragma unroll
+    for (int i = 0; i < DB; ++i)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) across[i][r] = __shfl_xor(o[i][r], 32, 64);
+#pragma unroll
+    for (int i = 0; i < DB; ++i) {
+      f32x4_t p;
+      if (i < H) p = upper ? across[i + H + 1] : across[i + H];
+      else if (i == H) p = upper ? across[0] : across[DB - 1];
+      else p = upper ? across[i - H] : across[i - H - 1];
+      const bool low = i < H || (i == H && !upper);
+      const int j = 16 * i + 4 * quad - (low ? 0 : D / 2);
+      const f32x4_t c = *(const f32x4_t*)(angles + j), s = *(const f32x4_t*)(angles + D / 2 + j);
+      o[i] = low ? o[i] * c + p * s : o[i] * c - p * s;
+    }
+  }
+}
 
 // One tile of 16 rows meets one block of 32 keys: sc holds the raw scores (this lane: its row,
 // keys base + 8 quad + e), vv the block's values as MFMA operands. Online softmax in base 2;
@@ -514,6 +553,7 @@ __global__ __launch_bounds__(256, (RT <= 2 && D <= 256) ? 2 : 1) void attention_
     lt += __shfl_xor(lt, 32, 64);
     if (!row_valid[t]) continue;
     if (a.sink && a.num_splits == 1) add_sink(m[t], lt, o[t]);
+    if (a.turn && a.num_splits == 1) turn_back(o[t], a.turn + row_index[t] / a.nq * D, quad);
     const float inv = lt > 0.f ? 1.0f / lt : 0.f;
     if (a.num_splits == 1) {
       bf16_t* op = a.out + row_index[t] * D;
@@ -904,6 +944,7 @@ __global__ __launch_bounds__(256 * G, G == 1 ? 2 : 1) void attention_bf16_prefil
     lt += __shfl_xor(lt, 32, 64);
     if (!row_valid[t] || !wave_has_rows || grp != 0) continue;
     if (a.sink && a.num_splits == 1) add_sink(m[t], lt, o[t]);
+    if (a.turn && a.num_splits == 1) turn_back(o[t], a.turn + row_index[t] / a.nq * D, quad);
     const float inv = lt > 0.f ? 1.0f / lt : 0.f;
     if (a.num_splits == 1) {
       bf16_t* op = a.out + row_index[t] * D;
@@ -929,13 +970,16 @@ __global__ __launch_bounds__(256 * G, G == 1 ? 2 : 1) void attention_bf16_prefil
 
 // Few splits: every load is asked for before the first is used (clamped indices, so none stands
 // under a branch), one trip to memory instead of two; the sums are those of the kernel's loop.
-// A thread takes elements threadIdx.x and threadIdx.x + blockDim.x of the row.
+// A thread takes elements threadIdx.x and threadIdx.x + blockDim.x of the row; with turned values the two
+// of a pair, threadIdx.x and threadIdx.x + D / 2.
 template <int MAX>
 __device__ __forceinline__ void merge_few(const float* __restrict__ part_o, const float* __restrict__ lse,
                                           bf16_t* __restrict__ out, int num_splits, size_t row,
-                                          const bf16_t* __restrict__ gate, long gate_stride, int nq, int sink) {
+                                          const bf16_t* __restrict__ gate, long gate_stride, int nq, int sink,
+                                          const float* __restrict__ turn) {
   float ls[MAX], pv[2][MAX];
-  const int d0 = min((int)threadIdx.x, D - 1), d1 = min((int)(threadIdx.x + blockDim.x), D - 1);
+  const int second = turn ? D / 2 : (int)blockDim.x;
+  const int d0 = min((int)threadIdx.x, D - 1), d1 = min((int)threadIdx.x + second, D - 1);
   const float g0 = gate_factor(gate, gate_stride, nq, row, d0), g1 = gate_factor(gate, gate_stride, nq, row, d1);
 #pragma unroll
   for (int s = 0; s < MAX; ++s) {
@@ -962,6 +1006,16 @@ __device__ __forceinline__ void merge_few(const float* __restrict__ part_o, cons
       }
     }
   }
+  if (turn) {
+    if ((int)threadIdx.x < D / 2) {
+      const float* angles = turn + row / nq * D + threadIdx.x;
+      const float c = angles[0], s = angles[D / 2], inv = wsum > 0.f ? 1.0f / wsum : 0.f;
+      const float u = acc[0] * inv, v = acc[1] * inv;
+      out[row * D + threadIdx.x] = (bf16_t)((u * c + v * s) * g0);
+      out[row * D + threadIdx.x + D / 2] = (bf16_t)((v * c - u * s) * g1);
+    }
+    return;
+  }
   if ((int)threadIdx.x < D) out[row * D + threadIdx.x] = (bf16_t)(wsum > 0.f ? acc[0] / wsum * g0 : 0.f);
   if ((int)(threadIdx.x + blockDim.x) < D)
     out[row * D + threadIdx.x + blockDim.x] = (bf16_t)(wsum > 0.f ? acc[1] / wsum * g1 : 0.f);
@@ -971,21 +1025,22 @@ __device__ __forceinline__ void merge_few(const float* __restrict__ part_o, cons
 // (a thread takes two elements of the row: 32, 64 or, for heads wider than 128, 256 threads a row)
 __global__ void attention_merge_kernel(const float* __restrict__ part_o, const float* __restrict__ part_lse,
                                        bf16_t* __restrict__ out, int num_splits, const int* __restrict__ tokens,
-                                       int nq, const bf16_t* __restrict__ gate, long gate_stride, int sink) {
+                                       int nq, const bf16_t* __restrict__ gate, long gate_stride, int sink,
+                                       const float* __restrict__ turn) {
   // rows are (token, query head); with a token list the grid walks the listed tokens' rows only
   const size_t row = tokens ? (size_t)tokens[blockIdx.x / nq] * nq + blockIdx.x % nq : blockIdx.x;
   const float* lse = part_lse + row * num_splits;
   if (num_splits <= 64 && D <= 2 * (int)blockDim.x) {
-    if (num_splits <= 8) merge_few<8>(part_o, lse, out, num_splits, row, gate, gate_stride, nq, sink);
-    else if (num_splits <= 16) merge_few<16>(part_o, lse, out, num_splits, row, gate, gate_stride, nq, sink);
-    else if (num_splits <= 32) merge_few<32>(part_o, lse, out, num_splits, row, gate, gate_stride, nq, sink);
-    else merge_few<64>(part_o, lse, out, num_splits, row, gate, gate_stride, nq, sink);
+    if (num_splits <= 8) merge_few<8>(part_o, lse, out, num_splits, row, gate, gate_stride, nq, sink, turn);
+    else if (num_splits <= 16) merge_few<16>(part_o, lse, out, num_splits, row, gate, gate_stride, nq, sink, turn);
+    else if (num_splits <= 32) merge_few<32>(part_o, lse, out, num_splits, row, gate, gate_stride, nq, sink, turn);
+    else merge_few<64>(part_o, lse, out, num_splits, row, gate, gate_stride, nq, sink, turn);
     return;
   }
   float mx = -INFINITY;
   for (int s = 0; s < num_splits; ++s) mx = fmaxf(mx, lse[s]);
   if (sink) mx = fmaxf(mx, 0.f);
-  for (int d = threadIdx.x; d < D; d += blockDim.x) {
+  auto element = [&](int d) -> float {
     float acc = 0.f, wsum = sink ? exp2f(-mx) : 0.f;
     if (mx != -INFINITY) {
       const float* po = part_o + row * num_splits * D + d;
@@ -996,8 +1051,19 @@ __global__ void attention_merge_kernel(const float* __restrict__ part_o, const f
         if (w > 0.f) acc += w * po[(size_t)s * D];
       }
     }
-    out[row * D + d] = (bf16_t)(wsum > 0.f ? acc / wsum * gate_factor(gate, gate_stride, nq, row, d) : 0.f);
+    return wsum > 0.f ? acc / wsum : 0.f;
+  };
+  if (turn) {
+    for (int d = threadIdx.x; d < D / 2; d += blockDim.x) {
+      const float* angles = turn + row / nq * D + d;
+      const float c = angles[0], s = angles[D / 2], u = element(d), v = element(d + D / 2);
+      out[row * D + d] = (bf16_t)((u * c + v * s) * gate_factor(gate, gate_stride, nq, row, d));
+      out[row * D + d + D / 2] = (bf16_t)((v * c - u * s) * gate_factor(gate, gate_stride, nq, row, d + D / 2));
+    }
+    return;
   }
+  for (int d = threadIdx.x; d < D; d += blockDim.x)
+    out[row * D + d] = (bf16_t)(element(d) * gate_factor(gate, gate_stride, nq, row, d));
 }
 
 // ------------------------------------------------------------------ decoding
@@ -1091,15 +1157,15 @@ __device__ __forceinline__ void block_compute(KvBlock& blk, const bf16x8_t* qreg
 }
 
 // One head of a token's product (x, D elements, D a multiple of 64) as an MFMA operand: RMSNorm
-// over the head in float32 (weight after the normalisation), NeoX rotation pairing element j
-// with j + D / 2 by the angles of `rope`, rounded to bfloat16 last, as the kernel that writes
+// over the head in float32 (weight after the normalisation), rotation pairing element j < pairs
+// with j + pairs by the angles of `rope` (a multiple of 32 of them), rounded to bfloat16 last, as the kernel that writes
 // queries and keys to memory does. A lane holds elements 32 i + 8 quad .. + 7 of k-step i, so a
-// pair lies in one lane (k-steps i and i + KFULL / 2) and the head's sum of squares in the four
+// pair lies in one lane (k-steps i and i + pairs / 32) and the head's sum of squares in the four
 // lanes of a row.
 __device__ __forceinline__ void head_as_operand(const bf16_t* __restrict__ x, const float* __restrict__ w,
-                                                const float* __restrict__ rope, float eps, int quad,
+                                                const float* __restrict__ rope, int pairs, float eps, int quad,
                                                 bf16x8_t* out) {
-  constexpr int KF = KFULL > 0 ? KFULL : 1, HALF_STEPS = KF / 2;
+  constexpr int KF = KFULL > 0 ? KFULL : 1;
   float v[KF][8];
   float ss = 0.f;
 #pragma unroll
@@ -1121,16 +1187,21 @@ __device__ __forceinline__ void head_as_operand(const bf16_t* __restrict__ x, co
       for (int e = 0; e < 8; ++e) v[i][e] = v[i][e] * inv * w[32 * i + 8 * quad + e];
   }
   if (rope) {
+    const int steps = pairs >> 5;  // the same for the whole launch
 #pragma unroll
-    for (int i = 0; i < HALF_STEPS; ++i)
+    for (int n = 1; n <= KF / 2; ++n) {
+      if (n != steps) continue;
 #pragma unroll
-      for (int e = 0; e < 8; ++e) {
-        const int j = 32 * i + 8 * quad + e;
-        const float cs = rope[j], sn = rope[D / 2 + j];
-        const float x1 = v[i][e], x2 = v[i + HALF_STEPS][e];
-        v[i][e] = x1 * cs - x2 * sn;
-        v[i + HALF_STEPS][e] = x2 * cs + x1 * sn;
-      }
+      for (int i = 0; i < n; ++i)
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          const int j = 32 * i + 8 * quad + e;
+          const float cs = rope[j], sn = rope[32 * n + j];
+          const float x1 = v[i][e], x2 = v[i + n][e];
+          v[i][e] = x1 * cs - x2 * sn;
+          v[i + n][e] = x2 * cs + x1 * sn;
+        }
+    }
   }
 #pragma unroll
   for (int i = 0; i < KF; ++i)
@@ -1207,15 +1278,24 @@ __global__ __launch_bounds__(64 * DW, D <= 128 ? 2 : 1) void attention_bf16_deco
   // the others left)
   auto own_token = [&]() {
     const bf16_t* raw = a.qkv + (size_t)q_begin * a.qkv_stride;
-    const float* rope = a.rope ? a.rope + (size_t)q_begin * D : nullptr;
-    head_as_operand(raw + (size_t)head * D, a.q_weight, rope, a.eps, quad, qreg);
+    const float* rope = a.rope ? a.rope + (size_t)q_begin * 2 * a.rope_pairs : nullptr;
+    const float* turn = a.turn ? a.turn + (size_t)q_begin * D : nullptr;
+    head_as_operand(raw + (size_t)head * D, a.q_weight, rope, a.rope_pairs, a.eps, quad, qreg);
     const bool at_end = split == last_split;
     const bool adds_own = at_end && wave == DW - 1, stores_own = at_end && wave == (2 * DW - 2) % DW;
     if (adds_own || stores_own) {  // uniform over the wave
       const bf16_t* kraw = raw + ((size_t)a.nq + kvh) * D;
       const bf16_t* vraw = raw + ((size_t)a.nq + a.nkv + kvh) * D;
       bf16x8_t kreg[KFULL > 0 ? KFULL : 1];
-      head_as_operand(kraw, a.k_weight, rope, a.eps, quad, kreg);
+      head_as_operand(kraw, a.k_weight, rope, a.rope_pairs, a.eps, quad, kreg);
+      // the token's own value, turned by its position where values are
+      auto own_value = [&](int d) -> bf16_t {
+        if (!turn) return vraw[d];
+        const bool low = d < D / 2;
+        const int j = low ? d : d - D / 2;
+        const float x = (float)vraw[d], y = (float)vraw[low ? d + D / 2 : j], c = turn[j], sn = turn[D / 2 + j];
+        return (bf16_t)(low ? x * c - y * sn : x * c + y * sn);
+      };
       if (stores_own) {
         const int slot = a.slots[q_begin];
         const int page = slot / a.page_size, off = slot - page * a.page_size;
@@ -1225,7 +1305,7 @@ __global__ __launch_bounds__(64 * DW, D <= 128 ? 2 : 1) void attention_bf16_deco
 #pragma unroll
           for (int i = 0; i < KFULL; ++i) *(bf16x8_t*)(kdst + 32 * i + 8 * quad) = kreg[i];
         }
-        for (int d = lane; d < D; d += 64) vdst[(size_t)d * a.page_size] = vraw[d];
+        for (int d = lane; d < D; d += 64) vdst[(size_t)d * a.page_size] = own_value(d);
       }
       if (adds_own) {
         // a block of keys that holds this one key, in the place of key first_pos: operand row 0
@@ -1241,7 +1321,7 @@ __global__ __launch_bounds__(64 * DW, D <= 128 ? 2 : 1) void attention_bf16_deco
         for (int i = 0; i < DB; ++i) {
 #pragma unroll
           for (int e = 0; e < 8; ++e) vv[i][e] = (bf16_t)0.0f;
-          if (quad == 0) vv[i][0] = vraw[16 * i + r16];
+          if (quad == 0) vv[i][0] = own_value(16 * i + r16);
         }
         tile_update(sc, vv, true, first_pos, quad, row_valid, qpos, a.window, a.chunk, 0, 0, a.scale_log2, m, l, o);
       }
@@ -1313,15 +1393,15 @@ __global__ __launch_bounds__(64 * DW, D <= 128 ? 2 : 1) void attention_bf16_deco
   __syncthreads();
 
   const size_t tile_row0 = (size_t)q_begin * a.nq;  // rows of this sequence start here, in units of heads
-  for (int idx = threadIdx.x; idx < 16 * D; idx += 64 * DW) {
-    const int row = idx / D, d = idx - row * D;
-    if (row >= n_rows) continue;
-    float mm = -INFINITY;
+  const bool sink_here = a.sink && a.num_splits == 1;
+  // element d of row `row`: the waves' parts joined, and the row's reference and sum
+  auto joined = [&](int row, int d, float& mm, float& den) -> float {
+    mm = -INFINITY;
 #pragma unroll
     for (int w = 0; w < DW; ++w) mm = fmaxf(mm, lds_m[w * 16 + row]);
-    const bool sink_here = a.sink && a.num_splits == 1;
     if (sink_here) mm = fmaxf(mm, 0.f);
-    float num = 0.f, den = sink_here ? exp2f(-mm) : 0.f;
+    float num = 0.f;
+    den = sink_here ? exp2f(-mm) : 0.f;
     if (mm != -INFINITY) {
 #pragma unroll
       for (int w = 0; w < DW; ++w) {
@@ -1330,9 +1410,29 @@ __global__ __launch_bounds__(64 * DW, D <= 128 ? 2 : 1) void attention_bf16_deco
         den += f * lds_l[w * 16 + row];
       }
     }
+    return den > 0.f ? num / den : 0.f;
+  };
+  if (a.turn && a.num_splits == 1) {  // the two elements of a pair at a time, turned back
+    for (int idx = threadIdx.x; idx < n_rows * (D / 2); idx += 64 * DW) {
+      const int row = idx / (D / 2), d = idx - row * (D / 2);
+      float mm, den;
+      const float u = joined(row, d, mm, den), v = joined(row, d + D / 2, mm, den);
+      const int rt = row / g, rh = row - rt * g;
+      const size_t row_index = tile_row0 + (size_t)rt * a.nq + kvh * g + rh;
+      const float* angles = a.turn + (size_t)(q_begin + rt) * D + d;
+      const float c = angles[0], sn = angles[D / 2];
+      a.out[row_index * D + d] = (bf16_t)((u * c + v * sn) * gate_factor(a.gate, a.gate_stride, a.nq, row_index, d));
+      a.out[row_index * D + d + D / 2] = (bf16_t)((v * c - u * sn) * gate_factor(a.gate, a.gate_stride, a.nq, row_index, d + D / 2));
+    }
+    return;  // one split: there are no parts to mark empty
+  }
+  for (int idx = threadIdx.x; idx < 16 * D; idx += 64 * DW) {
+    const int row = idx / D, d = idx - row * D;
+    if (row >= n_rows) continue;
+    float mm, den;
+    const float val = joined(row, d, mm, den);
     const int rt = row / g, rh = row - rt * g;
     const size_t row_index = tile_row0 + (size_t)rt * a.nq + kvh * g + rh;
-    const float val = den > 0.f ? num / den : 0.f;
     if (a.num_splits == 1) {
       a.out[row_index * D + d] = (bf16_t)(val * gate_factor(a.gate, a.gate_stride, a.nq, row_index, d));
     } else {
@@ -1410,6 +1510,8 @@ extern "C" int qrt_attention_bf16_decode(const AttnTileArgs* args, int num_rows_
                     (uintptr_t)a.qkv % 16 == 0,
                 "attention (decode, own token from the product): %d query heads per key head, stride %ld",
                 a.nq / a.nkv, a.qkv_stride);
+      QRT_CHECK(!a.rope || (a.rope_pairs >= 32 && a.rope_pairs % 32 == 0 && a.rope_pairs <= D / 2),
+                "attention (decode, own token from the product): %d pairs turn (multiples of 32 up to %d)", a.rope_pairs, D / 2);
       if (smem > 64 * 1024) {
         static bool allowed_fused = false;
         if (!allowed_fused) {
@@ -1433,7 +1535,7 @@ extern "C" int qrt_attention_bf16_decode(const AttnTileArgs* args, int num_rows_
     const int merge_rows = a.merge_tokens ? a.num_merge_tokens * a.nq : num_rows_total;
     if (merge_rows > 0)
       attention_merge_kernel<<<dim3(merge_rows), dim3(D > 128 ? 256 : (D >= 64 ? 64 : 32)), 0, stream>>>(
-          a.part_o, a.part_lse, a.out, a.num_splits, a.merge_tokens, a.nq, a.gate, a.gate_stride, a.sink);
+          a.part_o, a.part_lse, a.out, a.num_splits, a.merge_tokens, a.nq, a.gate, a.gate_stride, a.sink, a.turn);
     QRT_LAUNCH_CHECK("attention_merge");
   }
   return 0;
@@ -1493,7 +1595,7 @@ extern "C" int qrt_attention_bf16(const AttnTileArgs* args, int num_rows_total, 
     const int merge_rows = a.merge_tokens ? a.num_merge_tokens * a.nq : num_rows_total;
     if (merge_rows > 0)
       attention_merge_kernel<<<dim3(merge_rows), dim3(D > 128 ? 256 : (D >= 64 ? 64 : 32)), 0, stream>>>(
-          a.part_o, a.part_lse, a.out, a.num_splits, a.merge_tokens, a.nq, a.gate, a.gate_stride, a.sink);
+          a.part_o, a.part_lse, a.out, a.num_splits, a.merge_tokens, a.nq, a.gate, a.gate_stride, a.sink, a.turn);
     QRT_LAUNCH_CHECK("attention_merge");
   }
   return 0;

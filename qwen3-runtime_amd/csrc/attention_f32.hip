@@ -33,6 +33,7 @@ struct AttnArgs {
   long gate_stride;
   int keep_first;  // with a window: keys j < keep_first are seen too
   int sink;        // 1: one more term exp(0) in the denominator
+  const float* turn;  // [T, Dv] or null: cosines of the token's Dv / 2 angles, then their sines; the output is turned back by them
 };
 
 #define MAX_D 1024
@@ -107,11 +108,26 @@ __global__ __launch_bounds__(64) void attention_f32_kernel(AttnArgs a) {
   T* o = (T*)a.out + ((size_t)t * a.nq + h) * Dv;
   const T* gate = a.gate ? (const T*)a.gate + (size_t)t * a.gate_stride + (size_t)h * Dv : nullptr;
   const float inv = l > 0.f ? 1.0f / l : 0.f;
+  const float* angles = a.turn ? a.turn + (size_t)t * Dv : nullptr;
+  if (angles) {  // partners meet in LDS, which the queries no longer need
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < MAX_D / 64; ++i)
+      if (lane + 64 * i < Dv) qs[lane + 64 * i] = acc[i];
+    __syncthreads();
+  }
 #pragma unroll
   for (int i = 0; i < MAX_D / 64; ++i) {
     const int d = lane + 64 * i;
     if (d < Dv) {
       float v = acc[i] * inv;
+      if (angles) {
+        const int half = Dv >> 1;
+        const bool low = d < half;
+        const int j = low ? d : d - half;
+        const float p = qs[low ? d + half : j] * inv, c = angles[j], s = angles[half + j];
+        v = low ? v * c + p * s : v * c - p * s;
+      }
       if (gate) v *= 1.0f / (1.0f + expf(-to_f32<T>(gate[d])));
       o[d] = from_f32<T>(v);
     }
@@ -129,6 +145,7 @@ extern "C" int qrt_attention_f32(const AttnArgs* args, int dtype, hipStream_t st
   QRT_CHECK(a.chunk >= 0 && !(a.chunk > 0 && a.window > 0), "attention: a window or a chunk size, not both");
   QRT_CHECK(a.softcap >= 0.f, "attention: negative score cap");
   QRT_CHECK(a.keep_first >= 0 && (a.keep_first == 0 || a.window > 0), "attention: first keys are kept beside a window");
+  QRT_CHECK(!a.turn || a.value_dim % 2 == 0, "attention: turned values of odd size %d", a.value_dim);
   QRT_CHECK(a.nq <= 65535, "attention: too many heads");
   if (a.num_tokens == 0) return 0;
   dim3 grid(a.num_tokens, a.nq), block(64);

@@ -139,21 +139,25 @@ extern "C" int qrt_accumulate(float* acc, const void* y, int y_code, int y_plane
   return 0;
 }
 
-// out[t, i] = act(gu[t, i], gu[t, I + i]) for the gated activations of common.h
+// out[t, i] = act(by * gu[t, i], by * gu[t, I + i]) for the gated activations of common.h; by = 1, or, with
+// `scale`, scale[order[t]] (order null: scale[t])
 template <typename T>
-__global__ void gated_act_kernel(const T* __restrict__ gu, T* __restrict__ out, int inter, int kind, float limit) {
+__global__ void gated_act_kernel(const T* __restrict__ gu, T* __restrict__ out, int inter, int kind, float limit,
+                                 const float* __restrict__ scale, const int* __restrict__ order) {
   const T* row = gu + (size_t)blockIdx.x * 2 * inter;
+  const float by = scale ? scale[order ? order[blockIdx.x] : blockIdx.x] : 1.0f;
   for (int i = threadIdx.x; i < inter; i += blockDim.x)
-    out[(size_t)blockIdx.x * inter + i] = from_f32<T>(gated_act(to_f32<T>(row[i]), to_f32<T>(row[inter + i]), kind, limit));
+    out[(size_t)blockIdx.x * inter + i] =
+        from_f32<T>(gated_act(to_f32<T>(row[i]) * by, to_f32<T>(row[inter + i]) * by, kind, limit));
 }
 
 extern "C" int qrt_gated_act(const void* gu, void* out, int dtype, int num_tokens, int inter, int kind, float limit,
-                             hipStream_t stream) {
+                             const float* scale, const int* order, hipStream_t stream) {
   QRT_CHECK(num_tokens >= 0 && inter > 0, "gated_act: bad sizes");
   QRT_CHECK(kind == QRT_ACT_SWIGLU || kind == QRT_ACT_CLAMPED, "gated_act: unknown activation %d", kind);
   if (num_tokens == 0) return 0;
-  if (dtype == QRT_F32) gated_act_kernel<float><<<dim3(num_tokens), 256, 0, stream>>>((const float*)gu, (float*)out, inter, kind, limit);
-  else if (dtype == QRT_BF16) gated_act_kernel<bf16_t><<<dim3(num_tokens), 256, 0, stream>>>((const bf16_t*)gu, (bf16_t*)out, inter, kind, limit);
+  if (dtype == QRT_F32) gated_act_kernel<float><<<dim3(num_tokens), 256, 0, stream>>>((const float*)gu, (float*)out, inter, kind, limit, scale, order);
+  else if (dtype == QRT_BF16) gated_act_kernel<bf16_t><<<dim3(num_tokens), 256, 0, stream>>>((const bf16_t*)gu, (bf16_t*)out, inter, kind, limit, scale, order);
   else return qrt_fail("gated_act: unknown dtype %d", dtype);
   QRT_LAUNCH_CHECK("gated_act");
   return 0;
@@ -348,6 +352,20 @@ extern "C" int qrt_scale(float* x, float factor, long n, hipStream_t stream) {
   if (n == 0) return 0;
   scale_kernel<<<dim3((unsigned)((n + 255) / 256)), 256, 0, stream>>>(x, factor, n);
   QRT_LAUNCH_CHECK("scale");
+  return 0;
+}
+
+// x = limit * tanh(x / limit), float32, in place (a cap on the logits)
+__global__ void softcap_kernel(float* __restrict__ x, float limit, long n) {
+  const long i = (long)blockIdx.x * 256 + threadIdx.x;
+  if (i < n) x[i] = limit * tanhf(x[i] / limit);
+}
+
+extern "C" int qrt_softcap(float* x, float limit, long n, hipStream_t stream) {
+  QRT_CHECK(n >= 0 && limit > 0.f, "softcap: bad size or limit");
+  if (n == 0) return 0;
+  softcap_kernel<<<dim3((unsigned)((n + 255) / 256)), 256, 0, stream>>>(x, limit, n);
+  QRT_LAUNCH_CHECK("softcap");
   return 0;
 }
 

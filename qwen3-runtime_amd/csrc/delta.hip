@@ -38,6 +38,7 @@ struct ConvArgs {
   // every span is one token (a decode step): the wave that reads a channel's tail also moves it on,
   // and no second kernel runs
   int fuse_tail;
+  const float* bias;        // [C] or null: added to the convolution, before silu
 };
 
 template <typename T>
@@ -63,7 +64,7 @@ __global__ __launch_bounds__(256) void conv_unit_kernel(ConvArgs a) {
     y[r] = 0.f;
     const int c = c0 + lane + 64 * r;
     if (lane + 64 * r < width) {
-      float acc = 0.f;
+      float acc = a.bias ? a.bias[c] : 0.f;
       for (int j = 0; j < K; ++j) {
         const int back = K - 1 - j;        // this tap reads the token `back` places earlier
         const float in = back <= i ? to_f32<T>(x[(size_t)(t - back) * a.x_stride + c])
@@ -106,13 +107,14 @@ __global__ __launch_bounds__(256) void conv_unit_tile_kernel(ConvArgs a) {
   const int c0 = a.seg_first[seg] + h * width;
   const int t0 = tile * CONV_TILE, nt = min(CONV_TILE, a.num_tokens - t0);
   const T* x = (const T*)a.x;
-  float w[2][K], xw[2][CONV_TILE + K - 1], y[2][CONV_TILE];
+  float w[2][K], xw[2][CONV_TILE + K - 1], y[2][CONV_TILE], bias[2];
 #pragma unroll
   for (int r = 0; r < 2; ++r) {
     const bool on = lane + 64 * r < width;
     const int c = c0 + (on ? lane + 64 * r : 0);
 #pragma unroll
     for (int j = 0; j < K; ++j) w[r][j] = a.taps[(size_t)c * K + j];
+    bias[r] = a.bias ? a.bias[c] : 0.f;
 #pragma unroll
     for (int j = 0; j < CONV_TILE + K - 1; ++j) {
       const int row = t0 - (K - 1) + j;
@@ -131,7 +133,7 @@ __global__ __launch_bounds__(256) void conv_unit_tile_kernel(ConvArgs a) {
     const float* tail = a.tail + (size_t)a.state_slots[s] * a.channels * (K - 1);
 #pragma unroll
     for (int r = 0; r < 2; ++r) {
-      float acc = 0.f;
+      float acc = bias[r];
 #pragma unroll
       for (int j = 0; j < K; ++j) {
         float in = xw[r][tt + j];

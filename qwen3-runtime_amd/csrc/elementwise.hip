@@ -217,9 +217,11 @@ extern "C" int qrt_add_rmsnorm(float* residual, const void* delta, int delta_dty
 
 // ------------------------------------------------------------------ SwiGLU
 // out[t, i] = silu(gu[t, i]) * gu[t, I + i],  silu(x) = x / (1 + exp(-x)), in float32.
-// VEC elements per thread and access: 8 for bfloat16 rows whose halves start on 16 bytes.
+// VEC elements per thread and access: 8 for bfloat16 rows whose halves start on 16 bytes. With `scale`
+// both halves of row t are first multiplied by scale[order[t]] (order null: scale[t]).
 template <typename T, int VEC>
-__global__ __launch_bounds__(256) void swiglu_kernel(const T* __restrict__ gu, T* __restrict__ out, int inter) {
+__global__ __launch_bounds__(256) void swiglu_kernel(const T* __restrict__ gu, T* __restrict__ out, int inter,
+                                                     const float* __restrict__ scale, const int* __restrict__ order) {
   typedef T vec_t __attribute__((ext_vector_type(VEC)));
   // a block per token: no division to find the row, and two loads of each half in flight per thread
   // (120 MB read and written for 2,048 tokens of the 4B shape in 23.6 us, 5.1 TB/s, as the
@@ -228,6 +230,7 @@ __global__ __launch_bounds__(256) void swiglu_kernel(const T* __restrict__ gu, T
   const T* u_row = g_row + inter;
   T* o_row = out + (size_t)blockIdx.x * inter;
   constexpr int U = 2;
+  const float by = scale ? scale[order ? order[blockIdx.x] : blockIdx.x] : 1.0f;
   for (int i0 = threadIdx.x * VEC; i0 < inter; i0 += U * 256 * VEC) {
     vec_t g[U], u[U];
 #pragma unroll
@@ -245,8 +248,8 @@ __global__ __launch_bounds__(256) void swiglu_kernel(const T* __restrict__ gu, T
         vec_t o;
 #pragma unroll
         for (int e = 0; e < VEC; ++e) {
-          const float gf = to_f32<T>(g[k][e]);
-          o[e] = from_f32<T>(gf / (1.0f + expf(-gf)) * to_f32<T>(u[k][e]));
+          const float gf = to_f32<T>(g[k][e]) * by;
+          o[e] = from_f32<T>(gf / (1.0f + expf(-gf)) * (to_f32<T>(u[k][e]) * by));
         }
         *(vec_t*)(o_row + i) = o;
       }
@@ -255,21 +258,22 @@ __global__ __launch_bounds__(256) void swiglu_kernel(const T* __restrict__ gu, T
 }
 
 template <typename T, int VEC>
-static void swiglu_launch(const void* gate_up, void* out, int num_tokens, int inter, hipStream_t stream) {
-  swiglu_kernel<T, VEC><<<dim3((unsigned)num_tokens), 256, 0, stream>>>((const T*)gate_up, (T*)out, inter);
+static void swiglu_launch(const void* gate_up, void* out, int num_tokens, int inter, const float* scale, const int* order,
+                          hipStream_t stream) {
+  swiglu_kernel<T, VEC><<<dim3((unsigned)num_tokens), 256, 0, stream>>>((const T*)gate_up, (T*)out, inter, scale, order);
 }
 
-extern "C" int qrt_swiglu(const void* gate_up, void* out, int dtype, int num_tokens, int inter,
-                          hipStream_t stream) {
+extern "C" int qrt_swiglu(const void* gate_up, void* out, int dtype, int num_tokens, int inter, const float* scale,
+                          const int* order, hipStream_t stream) {
   QRT_CHECK(num_tokens >= 0 && inter > 0, "swiglu: bad sizes T=%d I=%d", num_tokens, inter);
   if ((size_t)num_tokens * inter == 0) return 0;
   const bool aligned = ((uintptr_t)gate_up % 16 == 0) && ((uintptr_t)out % 16 == 0);
   if (dtype == QRT_F32) {
-    if (aligned && inter % 4 == 0) swiglu_launch<float, 4>(gate_up, out, num_tokens, inter, stream);
-    else swiglu_launch<float, 1>(gate_up, out, num_tokens, inter, stream);
+    if (aligned && inter % 4 == 0) swiglu_launch<float, 4>(gate_up, out, num_tokens, inter, scale, order, stream);
+    else swiglu_launch<float, 1>(gate_up, out, num_tokens, inter, scale, order, stream);
   } else if (dtype == QRT_BF16) {
-    if (aligned && inter % 8 == 0) swiglu_launch<bf16_t, 8>(gate_up, out, num_tokens, inter, stream);
-    else swiglu_launch<bf16_t, 1>(gate_up, out, num_tokens, inter, stream);
+    if (aligned && inter % 8 == 0) swiglu_launch<bf16_t, 8>(gate_up, out, num_tokens, inter, scale, order, stream);
+    else swiglu_launch<bf16_t, 1>(gate_up, out, num_tokens, inter, scale, order, stream);
   } else {
     return qrt_fail("swiglu: unknown dtype %d", dtype);
   }
@@ -280,8 +284,10 @@ extern "C" int qrt_swiglu(const void* gate_up, void* out, int dtype, int num_tok
 // ------------------------------- per-head norm + rotary + cache write
 // One wave per (token, head) over the nq query heads, nkv key heads and nkv
 // value heads of a token. Query and key heads: optional RMSNorm over the head
-// (weight [D]), optional NeoX rotation with angle = float(pos) * inv_freq[j]
-// pairing element j with j + D/2. Value heads are copied. Keys and values go to
+// (weight [D]), optional rotation of the first 2 rot_pairs elements with angle =
+// float(pos) * inv_freq[j], pairing element j with j + rot_pairs (NeoX: all D elements);
+// the rest passes. Value heads are copied, or, with v_rope, turned over all their
+// elements, first half against second half. Keys and values go to
 // the paged cache (keys [page, head, offset, D], values [page, head, D, offset])
 // and/or to dense outputs; queries go to q_out.
 struct QkArgs {
@@ -300,12 +306,28 @@ struct QkArgs {
   void* v_cache;
   int num_tokens, nq, nkv, nv, head_dim, page_size;
   float eps;
-  // [T, head_dim] or null: the cosines of the tokens' head_dim / 2 angles, then their sines, as
+  // [T, 2 rot_pairs] or null: the cosines of the tokens' angles, then their sines, as
   // rope_table makes them. The kernel for many tokens looks them up instead of computing them in
   // every layer (inv_freq and positions are still given: the kernel for few tokens computes).
   const float* rope;
   int value_dim;  // elements of a value head; 0: head_dim
+  int rot_pairs;  // pairs that turn; 0: head_dim / 2
+  const float* v_rope;  // [T, value_dim] or null: cosines of the value's value_dim / 2 angles, then their sines
 };
+
+// Where the two elements of pair p of a head lie (p < D / 2): the pairs that turn come first, then the
+// elements that pass, halved the same way. A run of 8 pairs that starts on a multiple of 8 is two runs of
+// neighbours as long as rot_pairs is a multiple of 8.
+__device__ __forceinline__ int pair_lo(int p, int rp) { return p < rp ? p : p + rp; }
+__device__ __forceinline__ int pair_hi(int p, int rp, int half) { return p < rp ? p + rp : p + half; }
+
+// element i of a value head turned by its token's angles (table row: cosines, then sines)
+template <typename T>
+__device__ __forceinline__ void turned_pair(const T* src, const float* angles, int i, int half, T* lo, T* hi) {
+  const float u = to_f32<T>(src[i]), v = to_f32<T>(src[i + half]), c = angles[i], s = angles[half + i];
+  *lo = from_f32<T>(u * c - v * s);
+  *hi = from_f32<T>(v * c + u * s);
+}
 
 template <typename T>
 __global__ void qk_norm_rope_store_kernel(QkArgs a) {
@@ -315,12 +337,29 @@ __global__ void qk_norm_rope_store_kernel(QkArgs a) {
   if (item >= (long)a.num_tokens * heads) return;
   const int t = (int)(item / heads);
   const int h = (int)(item - (long)t * heads);
-  const int D = a.head_dim, half = D >> 1;
+  const int D = a.head_dim, half = D >> 1, rp = a.rot_pairs;
 
-  if (h >= a.nq + a.nkv) {  // value head: copy
+  if (h >= a.nq + a.nkv) {  // value head: copy, or turn
     const int hv = h - a.nq - a.nkv;
     const int Dv = a.value_dim;
     const T* src = (const T*)a.v_in + (size_t)t * a.v_stride + (size_t)hv * Dv;
+    if (a.v_rope) {
+      const float* angles = a.v_rope + (size_t)t * Dv;
+      T* dense = a.v_out ? (T*)a.v_out + ((size_t)t * a.nv + hv) * Dv : nullptr;
+      T* paged = nullptr;
+      if (a.slots) {
+        const int slot = a.slots[t];
+        const int page = slot / a.page_size, off = slot - page * a.page_size;
+        paged = (T*)a.v_cache + ((size_t)page * a.nv + hv) * Dv * a.page_size + off;
+      }
+      for (int i = lane; i < (Dv >> 1); i += 64) {
+        T lo, hi;
+        turned_pair<T>(src, angles, i, Dv >> 1, &lo, &hi);
+        if (dense) { dense[i] = lo; dense[i + (Dv >> 1)] = hi; }
+        if (paged) { paged[(size_t)i * a.page_size] = lo; paged[(size_t)(i + (Dv >> 1)) * a.page_size] = hi; }
+      }
+      return;
+    }
     if (a.v_out) {
       T* dst = (T*)a.v_out + ((size_t)t * a.nv + hv) * Dv;
       for (int i = lane; i < Dv; i += 64) dst[i] = src[i];
@@ -340,7 +379,7 @@ __global__ void qk_norm_rope_store_kernel(QkArgs a) {
                       : (const T*)a.k_in + (size_t)t * a.k_stride + (size_t)hh * D;
   const float* w = is_q ? a.q_weight : a.k_weight;
 
-  // each lane owns the pairs (p, p + D/2) for p = lane, lane + 64, ... (D <= 512).
+  // each lane owns the pairs p = lane, lane + 64, ... (D <= 512; see pair_lo and pair_hi).
   // Everything the lane will need is loaded before the first use (norm weights, position,
   // frequencies, slot), so that the kernel costs one round of memory latency, not four.
   float x1[4], x2[4], w1[4], w2[4], fr[4];
@@ -354,13 +393,13 @@ __global__ void qk_norm_rope_store_kernel(QkArgs a) {
     w1[i] = w2[i] = 1.f;
     fr[i] = 0.f;
     if (p < half) {
-      x1[i] = to_f32<T>(src[p]);
-      x2[i] = to_f32<T>(src[p + half]);
+      x1[i] = to_f32<T>(src[pair_lo(p, rp)]);
+      x2[i] = to_f32<T>(src[pair_hi(p, rp, half)]);
       if (w) {
-        w1[i] = w[p];
-        w2[i] = w[p + half];
+        w1[i] = w[pair_lo(p, rp)];
+        w2[i] = w[pair_hi(p, rp, half)];
       }
-      if (a.inv_freq) fr[i] = a.inv_freq[p];
+      if (a.inv_freq && p < rp) fr[i] = a.inv_freq[p];
     }
   }
 #pragma unroll
@@ -378,7 +417,7 @@ __global__ void qk_norm_rope_store_kernel(QkArgs a) {
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
       const int p = lane + 64 * i;
-      if (p < half) {
+      if (p < rp) {
         const float ang = pos * fr[i];
         float sn, c;
         sincos_angle(ang, &sn, &c);
@@ -402,15 +441,16 @@ __global__ void qk_norm_rope_store_kernel(QkArgs a) {
     const int p = lane + 64 * i;
     if (p < half) {
       const T y1 = from_f32<T>(x1[i]), y2 = from_f32<T>(x2[i]);
-      if (dense) { dense[p] = y1; dense[p + half] = y2; }
-      if (paged) { paged[p] = y1; paged[p + half] = y2; }
+      const int lo = pair_lo(p, rp), hi = pair_hi(p, rp, half);
+      if (dense) { dense[lo] = y1; dense[hi] = y2; }
+      if (paged) { paged[lo] = y1; paged[hi] = y2; }
     }
   }
 }
 
 // The same work for head sizes 16, 32, ..., 512 (powers of two) with every access 8 elements
-// wide. Norm and rotation: a lane owns 8 neighbouring elements of the first half of a head and
-// their partners in the second half, head_dim / 16 lanes share a head, a wave covers
+// wide. Norm and rotation: a lane owns 8 neighbouring pairs of a head (with all elements turning: 8
+// neighbours of the first half and their partners in the second), head_dim / 16 lanes share a head, a wave covers
 // 64 / (head_dim / 16) heads per pass and computes the sines and cosines of its token once for
 // all passes it makes. Values: a wave takes 8 tokens of one head, turns them round in LDS and
 // writes, for each head element, the 8 tokens as one piece of the transposed page; that needs
@@ -423,7 +463,7 @@ __global__ __launch_bounds__(256) void qk_norm_rope_store_wide_kernel(QkArgs a, 
                                                                       int passes_per_wave) {
   extern __shared__ __align__(32) unsigned char smem_raw[];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
-  const int D = a.head_dim, half = D >> 1;
+  const int D = a.head_dim, half = D >> 1, rp = a.rot_pairs;
 
   if ((int)blockIdx.x < rope_blocks) {
     const int hp = 64 / lph, nh = a.nq + a.nkv;
@@ -433,15 +473,17 @@ __global__ __launch_bounds__(256) void qk_norm_rope_store_wide_kernel(QkArgs a, 
     if (item >= (long)a.num_tokens * groups) return;
     const int t = (int)(item / groups), grp = (int)(item - (long)t * groups);
     const int c = lane & (lph - 1), hl = lane / lph;
+    const bool turns = a.inv_freq && 8 * c < rp;
+    const int lo = pair_lo(8 * c, rp), hi = pair_hi(8 * c, rp, half);
     float sn[8], cs[8];
-    if (a.rope) {
-      const float* angles = a.rope + (size_t)t * D + 8 * c;
+    if (a.rope && turns) {
+      const float* angles = a.rope + (size_t)t * 2 * rp + 8 * c;
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
         cs[e] = angles[e];
-        sn[e] = angles[half + e];
+        sn[e] = angles[rp + e];
       }
-    } else if (a.inv_freq) {
+    } else if (turns) {
       const float pos = (float)a.positions[t];
 #pragma unroll
       for (int e = 0; e < 8; ++e) sincos_angle(pos * a.inv_freq[8 * c + e], &sn[e], &cs[e]);
@@ -457,7 +499,7 @@ __global__ __launch_bounds__(256) void qk_norm_rope_store_wide_kernel(QkArgs a, 
       const T* src = is_q ? (const T*)a.q_in + (size_t)t * a.q_stride + (size_t)hh * D
                           : (const T*)a.k_in + (size_t)t * a.k_stride + (size_t)hh * D;
       const float* w = is_q ? a.q_weight : a.k_weight;
-      const Vec8<T> r1 = *(const Vec8<T>*)(src + 8 * c), r2 = *(const Vec8<T>*)(src + half + 8 * c);
+      const Vec8<T> r1 = *(const Vec8<T>*)(src + lo), r2 = *(const Vec8<T>*)(src + hi);
       float x1[8], x2[8];
       float ss = 0.f;
 #pragma unroll
@@ -471,15 +513,15 @@ __global__ __launch_bounds__(256) void qk_norm_rope_store_wide_kernel(QkArgs a, 
         const float inv = rsqrtf(ss / (float)D + a.eps);
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
-          x1[e] = x1[e] * inv * w[8 * c + e];
-          x2[e] = x2[e] * inv * w[half + 8 * c + e];
+          x1[e] = x1[e] * inv * w[lo + e];
+          x2[e] = x2[e] * inv * w[hi + e];
         }
       }
       Vec8<T> y1, y2;
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
         float u1 = x1[e], u2 = x2[e];
-        if (a.inv_freq) {
+        if (turns) {
           u1 = x1[e] * cs[e] - x2[e] * sn[e];
           u2 = x2[e] * cs[e] + x1[e] * sn[e];
         }
@@ -490,13 +532,13 @@ __global__ __launch_bounds__(256) void qk_norm_rope_store_wide_kernel(QkArgs a, 
       if (is_q && a.q_out) dense = (T*)a.q_out + ((size_t)t * a.nq + hh) * D;
       if (!is_q && a.k_out) dense = (T*)a.k_out + ((size_t)t * a.nkv + hh) * D;
       if (dense) {
-        *(Vec8<T>*)(dense + 8 * c) = y1;
-        *(Vec8<T>*)(dense + half + 8 * c) = y2;
+        *(Vec8<T>*)(dense + lo) = y1;
+        *(Vec8<T>*)(dense + hi) = y2;
       }
       if (!is_q && a.slots) {
         T* paged = (T*)a.k_cache + (((size_t)page * a.nkv + hh) * a.page_size + off) * D;
-        *(Vec8<T>*)(paged + 8 * c) = y1;
-        *(Vec8<T>*)(paged + half + 8 * c) = y2;
+        *(Vec8<T>*)(paged + lo) = y1;
+        *(Vec8<T>*)(paged + hi) = y2;
       }
     }
     return;
@@ -511,6 +553,31 @@ __global__ __launch_bounds__(256) void qk_norm_rope_store_wide_kernel(QkArgs a, 
   const int row = D + 8;  // padded: the 8 tokens of an element lie in different banks
   T* tile = (T*)smem_raw + (size_t)wave * 8 * row;
   const int chunks = D >> 3;
+  if (a.v_rope) {  // 8 neighbouring pairs at a time, turned on their way into LDS
+    const int hc = D >> 4;
+    for (int idx = lane; idx < 8 * hc; idx += 64) {
+      const int j = idx / hc, c = idx - j * hc;
+      if (j < nvalid) {
+        const T* src = (const T*)a.v_in + (size_t)(t0 + j) * a.v_stride + (size_t)hv * D + 8 * c;
+        const float* angles = a.v_rope + (size_t)(t0 + j) * D + 8 * c;
+        const Vec8<T> u = *(const Vec8<T>*)src, v = *(const Vec8<T>*)(src + half);
+        Vec8<T> y1, y2;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          const float x1 = to_f32<T>(u.v[e]), x2 = to_f32<T>(v.v[e]), cs = angles[e], sn = angles[half + e];
+          y1.v[e] = from_f32<T>(x1 * cs - x2 * sn);
+          y2.v[e] = from_f32<T>(x2 * cs + x1 * sn);
+        }
+        *(Vec8<T>*)(tile + j * row + 8 * c) = y1;
+        *(Vec8<T>*)(tile + j * row + half + 8 * c) = y2;
+        if (a.v_out) {
+          T* dense = (T*)a.v_out + ((size_t)(t0 + j) * a.nv + hv) * D + 8 * c;
+          *(Vec8<T>*)dense = y1;
+          *(Vec8<T>*)(dense + half) = y2;
+        }
+      }
+    }
+  } else
   for (int idx = lane; idx < 8 * chunks; idx += 64) {
     const int j = idx / chunks, c = idx - j * chunks;
     if (j < nvalid) {
@@ -555,6 +622,9 @@ extern "C" int qrt_qk_norm_rope_store(const QkArgs* args, int dtype, long num_ca
   QRT_CHECK(!a.inv_freq || a.positions, "qk_norm_rope_store: rotation without positions");
   if (a.value_dim == 0) a.value_dim = a.head_dim;
   QRT_CHECK(a.value_dim > 0, "qk_norm_rope_store: bad value size %d", a.value_dim);
+  if (a.rot_pairs == 0) a.rot_pairs = a.head_dim / 2;
+  QRT_CHECK(a.rot_pairs > 0 && a.rot_pairs <= a.head_dim / 2, "qk_norm_rope_store: %d pairs turn in heads of %d", a.rot_pairs, a.head_dim);
+  QRT_CHECK(!a.v_rope || a.value_dim % 2 == 0, "qk_norm_rope_store: turned values of odd size %d", a.value_dim);
   if (a.slots) {
     QRT_CHECK(a.k_cache && a.v_cache && a.page_size > 0 && num_cache_pages > 0,
               "qk_norm_rope_store: cache write without cache");
@@ -568,7 +638,7 @@ extern "C" int qrt_qk_norm_rope_store(const QkArgs* args, int dtype, long num_ca
   const int D = a.head_dim;
   // few tokens (decoding): the time is the launch and one round of memory latency, and the
   // one-head-per-wave kernel has the shorter chain
-  const bool wide = a.num_tokens >= 32 && D >= 16 && a.value_dim == D && (D & (D - 1)) == 0 && a.q_stride % 8 == 0 && a.k_stride % 8 == 0 &&
+  const bool wide = a.num_tokens >= 32 && D >= 16 && a.value_dim == D && (D & (D - 1)) == 0 && a.rot_pairs % 8 == 0 && a.q_stride % 8 == 0 && a.k_stride % 8 == 0 &&
                     a.v_stride % 8 == 0 && lined_up(a.q_in) && lined_up(a.k_in) && lined_up(a.v_in) &&
                     lined_up(a.q_out) && lined_up(a.k_out) && lined_up(a.v_out) && lined_up(a.k_cache) &&
                     lined_up(a.v_cache);

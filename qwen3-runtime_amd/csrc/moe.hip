@@ -37,6 +37,9 @@ __device__ __forceinline__ float lane_dot(const T* __restrict__ w, const float* 
   return acc;
 }
 
+// Weights on the experts' input (`in_weight`, per pair): expert(w x). The first products are linear, so
+// the weight multiplies their float32 sums in front of the activation, and the outputs are summed as
+// they are (the output weights are then null).
 // An expert's activation: the gated ones of common.h, or, for experts without a gate, the square
 // of relu of the one product (`u` unused).
 #define QRT_ACT_RELU2 2
@@ -194,7 +197,8 @@ extern "C" int qrt_route_top(const void* x, int x_dtype, const float* router, co
 template <typename T>
 __global__ __launch_bounds__(256) void moe_gate_up_kernel(const T* __restrict__ x, const T* __restrict__ gate_up,
                                                           const int* __restrict__ index, T* __restrict__ act,
-                                                          int hidden, int inter, int top, int act_kind, float limit) {
+                                                          int hidden, int inter, int top, int act_kind, float limit,
+                                                          const float* __restrict__ in_weight) {
   extern __shared__ float xs[];  // [hidden]
   const int p = blockIdx.x, t = p / top;
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
@@ -205,13 +209,14 @@ __global__ __launch_bounds__(256) void moe_gate_up_kernel(const T* __restrict__ 
   const bool gated = act_kind != QRT_ACT_RELU2;  // without a gate an expert's rows are the up rows alone
   const T* w = gate_up + (size_t)e * (gated ? 2 : 1) * inter * hidden;
   const int i0 = (blockIdx.y * 4 + wave) * ROWS_PER_WAVE;
+  const float by = in_weight ? in_weight[p] : 1.0f;
 #pragma unroll
   for (int r = 0; r < ROWS_PER_WAVE; ++r) {
     const int i = i0 + r;
     if (i >= inter) break;
     const float g = wave_sum(lane_dot<T>(w + (size_t)i * hidden, xs, hidden, lane, wide));
     const float u = gated ? wave_sum(lane_dot<T>(w + (size_t)(inter + i) * hidden, xs, hidden, lane, wide)) : 0.f;
-    if (lane == 0) act[(size_t)p * inter + i] = from_f32<T>(expert_act(g, u, act_kind, limit));
+    if (lane == 0) act[(size_t)p * inter + i] = from_f32<T>(expert_act(g * by, u * by, act_kind, limit));
   }
 }
 
@@ -234,7 +239,7 @@ __global__ __launch_bounds__(256) void moe_down_kernel(const T* __restrict__ act
     for (int j = 0; j < top; ++j) {
       const int e = index[(size_t)t * top + j];
       const float d = wave_sum(lane_dot<T>(down + ((size_t)e * hidden + n) * inter, as + (size_t)j * inter, inter, lane, wide));
-      sum = fmaf(weight[(size_t)t * top + j], d, sum);
+      sum = fmaf(weight ? weight[(size_t)t * top + j] : 1.0f, d, sum);
     }
     if (lane == 0) out[(size_t)t * hidden + n] = sum;
   }
@@ -242,7 +247,10 @@ __global__ __launch_bounds__(256) void moe_down_kernel(const T* __restrict__ act
 
 extern "C" int qrt_moe_pairs(const void* x, const void* gate_up, const void* down, const int* index,
                              const float* weight, void* act, float* out, int dtype, int num_tokens, int hidden,
-                             int inter, int experts, int top, int act_kind, float limit, hipStream_t stream) {
+                             int inter, int experts, int top, int act_kind, float limit, int weight_on_input,
+                             hipStream_t stream) {
+  const float* in_weight = weight_on_input ? weight : nullptr;
+  if (weight_on_input) weight = nullptr;
   QRT_CHECK(num_tokens >= 0 && hidden > 0 && inter > 0 && experts > 0 && top > 0, "moe: bad sizes");
   QRT_CHECK(act_kind == QRT_ACT_SWIGLU || act_kind == QRT_ACT_CLAMPED || act_kind == QRT_ACT_RELU2, "moe: unknown activation %d", act_kind);
   QRT_CHECK((size_t)hidden * 4 <= 64 * 1024 && (size_t)top * inter * 4 <= 64 * 1024,
@@ -253,10 +261,10 @@ extern "C" int qrt_moe_pairs(const void* x, const void* gate_up, const void* dow
   dim3 g1(num_tokens * top, (inter + per_block - 1) / per_block), g2(num_tokens, (hidden + per_block - 1) / per_block);
   QRT_CHECK(g1.y <= 65535 && g2.y <= 65535, "moe: rows too wide for one launch");
   if (dtype == QRT_F32) {
-    moe_gate_up_kernel<float><<<g1, 256, hidden * 4, stream>>>((const float*)x, (const float*)gate_up, index, (float*)act, hidden, inter, top, act_kind, limit);
+    moe_gate_up_kernel<float><<<g1, 256, hidden * 4, stream>>>((const float*)x, (const float*)gate_up, index, (float*)act, hidden, inter, top, act_kind, limit, in_weight);
     moe_down_kernel<float><<<g2, 256, top * inter * 4, stream>>>((const float*)act, (const float*)down, index, weight, out, hidden, inter, top);
   } else {
-    moe_gate_up_kernel<bf16_t><<<g1, 256, hidden * 4, stream>>>((const bf16_t*)x, (const bf16_t*)gate_up, index, (bf16_t*)act, hidden, inter, top, act_kind, limit);
+    moe_gate_up_kernel<bf16_t><<<g1, 256, hidden * 4, stream>>>((const bf16_t*)x, (const bf16_t*)gate_up, index, (bf16_t*)act, hidden, inter, top, act_kind, limit, in_weight);
     moe_down_kernel<bf16_t><<<g2, 256, top * inter * 4, stream>>>((const bf16_t*)act, (const bf16_t*)down, index, weight, out, hidden, inter, top);
   }
   QRT_LAUNCH_CHECK("moe_pairs");
@@ -326,7 +334,7 @@ __global__ void moe_combine_kernel(const T* __restrict__ y, const int* __restric
     float sum = 0.f;
     for (int j = 0; j < top; ++j) {
       const size_t p = (size_t)t * top + j;
-      sum = fmaf(weight[p], to_f32<T>(y[moe_row(place[p], index[p], offsets, padded) * hidden + c]), sum);
+      sum = fmaf(weight ? weight[p] : 1.0f, to_f32<T>(y[moe_row(place[p], index[p], offsets, padded) * hidden + c]), sum);
     }
     out[(size_t)t * hidden + c] = sum;
   }
@@ -377,7 +385,8 @@ template <typename T, int R, int MODE>
 __global__ __launch_bounds__(256) void moe_rows_by_expert_kernel(const T* __restrict__ in, const T* __restrict__ w,
                                                                  const int* __restrict__ order,
                                                                  const int* __restrict__ offsets, T* __restrict__ out,
-                                                                 int K, int N, int top, int act_kind, float limit) {
+                                                                 int K, int N, int top, int act_kind, float limit,
+                                                                 const float* __restrict__ in_weight) {
   constexpr int VEC = 16 / sizeof(T);
   constexpr bool GATED = MODE == 1;
   constexpr bool FIRST = MODE != 0;  // the experts' first product: input by token, output by pair
@@ -425,10 +434,11 @@ __global__ __launch_bounds__(256) void moe_rows_by_expert_kernel(const T* __rest
 #pragma unroll
     for (int r = 0; r < NR; ++r) acc[r] = wave_sum(acc[r]);
     if (lane == 0) {
+      const float by = FIRST && in_weight ? in_weight[p] : 1.0f;
 #pragma unroll
       for (int r = 0; r < R; ++r) {
         if (n0 + r >= N) break;
-        if (FIRST) out[(size_t)p * N + n0 + r] = from_f32<T>(expert_act(acc[r], GATED ? acc[NR - R + r] : 0.f, act_kind, limit));
+        if (FIRST) out[(size_t)p * N + n0 + r] = from_f32<T>(expert_act(acc[r] * by, GATED ? acc[NR - R + r] * by : 0.f, act_kind, limit));
         else out[(size_t)(first + i) * N + n0 + r] = from_f32<T>(acc[r]);
       }
     }
@@ -437,32 +447,34 @@ __global__ __launch_bounds__(256) void moe_rows_by_expert_kernel(const T* __rest
 
 template <typename T, int R, int MODE>
 static void moe_rows_launch(const void* in, const void* w, const int* order, const int* offsets, void* out, int K, int N,
-                            int experts, int top, int act_kind, float limit, hipStream_t stream) {
+                            int experts, int top, int act_kind, float limit, const float* in_weight, hipStream_t stream) {
   dim3 grid(experts, (N + R - 1) / R);
   const size_t smem = (size_t)(MODE == 1 ? 2 * R : R) * K * sizeof(T);
-  moe_rows_by_expert_kernel<T, R, MODE><<<grid, 256, smem, stream>>>((const T*)in, (const T*)w, order, offsets, (T*)out, K, N, top, act_kind, limit);
+  moe_rows_by_expert_kernel<T, R, MODE><<<grid, 256, smem, stream>>>((const T*)in, (const T*)w, order, offsets, (T*)out, K, N, top, act_kind, limit, in_weight);
 }
 
 template <typename T, int MODE>
 static int moe_rows_pick(const void* in, const void* w, const int* order, const int* offsets, void* out, int K, int N,
-                         int experts, int top, int act_kind, float limit, hipStream_t stream) {
+                         int experts, int top, int act_kind, float limit, const float* in_weight, hipStream_t stream) {
   // as many rows a block as 48 KB of LDS hold, eight at most
   const size_t row_bytes = (size_t)(MODE == 1 ? 2 : 1) * K * sizeof(T);
   const int fit = (int)(48 * 1024 / row_bytes);
-  if (fit >= 8) moe_rows_launch<T, 8, MODE>(in, w, order, offsets, out, K, N, experts, top, act_kind, limit, stream);
-  else if (fit >= 4) moe_rows_launch<T, 4, MODE>(in, w, order, offsets, out, K, N, experts, top, act_kind, limit, stream);
-  else if (fit >= 2) moe_rows_launch<T, 2, MODE>(in, w, order, offsets, out, K, N, experts, top, act_kind, limit, stream);
-  else if (fit >= 1) moe_rows_launch<T, 1, MODE>(in, w, order, offsets, out, K, N, experts, top, act_kind, limit, stream);
+  if (fit >= 8) moe_rows_launch<T, 8, MODE>(in, w, order, offsets, out, K, N, experts, top, act_kind, limit, in_weight, stream);
+  else if (fit >= 4) moe_rows_launch<T, 4, MODE>(in, w, order, offsets, out, K, N, experts, top, act_kind, limit, in_weight, stream);
+  else if (fit >= 2) moe_rows_launch<T, 2, MODE>(in, w, order, offsets, out, K, N, experts, top, act_kind, limit, in_weight, stream);
+  else if (fit >= 1) moe_rows_launch<T, 1, MODE>(in, w, order, offsets, out, K, N, experts, top, act_kind, limit, in_weight, stream);
   else return qrt_fail("moe: rows of %d elements do not fit the block's memory", K);
   return 0;
 }
 
+// in_weight [pairs] or null: weights on the experts' input
 // x [T, H] -> act [pairs, I] (by pair) -> y [pairs, H] (by place); order and offsets from qrt_moe_group
 extern "C" int qrt_moe_by_expert(const void* x, const void* gate_up, const void* down, const int* order,
                                  const int* offsets, void* act, void* y, int dtype, int hidden, int inter, int experts,
-                                 int top, int act_kind, float limit, hipStream_t stream) {
+                                 int top, int act_kind, float limit, const float* in_weight, hipStream_t stream) {
   QRT_CHECK(hidden > 0 && inter > 0 && experts >= 1 && experts <= MAX_EXPERTS && top > 0, "moe: bad sizes");
   QRT_CHECK(act_kind == QRT_ACT_SWIGLU || act_kind == QRT_ACT_CLAMPED || act_kind == QRT_ACT_RELU2, "moe: unknown activation %d", act_kind);
+  QRT_CHECK(!in_weight || act_kind != QRT_ACT_RELU2, "moe: weights on the input go with gated experts");
   QRT_CHECK(dtype == QRT_F32 || dtype == QRT_BF16, "moe: unknown dtype %d", dtype);
   const int vec = dtype == QRT_F32 ? 4 : 8;
   QRT_CHECK(hidden % vec == 0 && inter % vec == 0, "moe: widths %d and %d are no multiples of %d", hidden, inter, vec);
@@ -470,14 +482,14 @@ extern "C" int qrt_moe_by_expert(const void* x, const void* gate_up, const void*
   int rc;
   if (dtype == QRT_F32) {
     rc = act_kind == QRT_ACT_RELU2
-             ? moe_rows_pick<float, 2>(x, gate_up, order, offsets, act, hidden, inter, experts, top, act_kind, limit, stream)
-             : moe_rows_pick<float, 1>(x, gate_up, order, offsets, act, hidden, inter, experts, top, act_kind, limit, stream);
-    if (rc == 0) rc = moe_rows_pick<float, 0>(act, down, order, offsets, y, inter, hidden, experts, top, act_kind, limit, stream);
+             ? moe_rows_pick<float, 2>(x, gate_up, order, offsets, act, hidden, inter, experts, top, act_kind, limit, in_weight, stream)
+             : moe_rows_pick<float, 1>(x, gate_up, order, offsets, act, hidden, inter, experts, top, act_kind, limit, in_weight, stream);
+    if (rc == 0) rc = moe_rows_pick<float, 0>(act, down, order, offsets, y, inter, hidden, experts, top, act_kind, limit, nullptr, stream);
   } else {
     rc = act_kind == QRT_ACT_RELU2
-             ? moe_rows_pick<bf16_t, 2>(x, gate_up, order, offsets, act, hidden, inter, experts, top, act_kind, limit, stream)
-             : moe_rows_pick<bf16_t, 1>(x, gate_up, order, offsets, act, hidden, inter, experts, top, act_kind, limit, stream);
-    if (rc == 0) rc = moe_rows_pick<bf16_t, 0>(act, down, order, offsets, y, inter, hidden, experts, top, act_kind, limit, stream);
+             ? moe_rows_pick<bf16_t, 2>(x, gate_up, order, offsets, act, hidden, inter, experts, top, act_kind, limit, in_weight, stream)
+             : moe_rows_pick<bf16_t, 1>(x, gate_up, order, offsets, act, hidden, inter, experts, top, act_kind, limit, in_weight, stream);
+    if (rc == 0) rc = moe_rows_pick<bf16_t, 0>(act, down, order, offsets, y, inter, hidden, experts, top, act_kind, limit, nullptr, stream);
   }
   if (rc != 0) return rc;
   QRT_LAUNCH_CHECK("moe_by_expert");

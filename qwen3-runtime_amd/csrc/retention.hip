@@ -1,6 +1,11 @@
-// Retention: the recurrence of linear attention with a constant decay per head, float32.
+// Recurrences of linear attention with one decay per head, float32.
 //
-//   S <- decay_h S + k v^T;   o = S^T q          (S [dim, vdim] per sequence and head)
+//   S <- d S + k v^T;   o = S^T q                (S [dim, vdim] per sequence and head)
+//
+// Retention: d is a constant of the head. State-space form (STEP): a step size per token and head,
+// D = softplus(logit + bias), makes both the decay d = exp(-exp(a_log) D) and the written value v = D x,
+// the read-out has a skip, o = S^T q + skip x, and neighbouring heads share keys and queries (head h has
+// those of h / share).
 //
 // over each sequence's tokens of the step, from the state in the sequence's slot, which is left
 // there for the next step: [slots, heads, vdim, dim], a value channel's column of S contiguous.
@@ -23,6 +28,9 @@ struct RetentionArgs {
   float* out;             // [T, heads, vdim]
   const int* cu_q; const int* state_slots;
   int heads, dim, vdim;
+  int share;              // heads that have one key and query in common (1: each its own)
+  const void* step; long step_stride; int step_code;   // [T, heads] step logits, float32 or bfloat16; null: retention
+  const float* step_bias; const float* a_log; const float* skip;  // [heads]
 };
 
 #define RT_COLS 16   // columns of the state per block
@@ -43,7 +51,7 @@ __device__ __forceinline__ float row16_sum(float x) {
 // G groups of four rows a lane: heads of up to 64 G key elements (padded with zero rows). RT_TILE
 // tokens a tile: 16 (8 for the widest heads: what fits 64 KB), or 4 for steps of single tokens,
 // whose blocks then are all resident at once with a quarter of the LDS and of the loads.
-template <int G, int RT_TILE>
+template <int G, int RT_TILE, bool STEP>
 __global__ __launch_bounds__(256) void retention_kernel(RetentionArgs a) {
   constexpr int DP = 64 * G;                          // rows staged
   constexpr int NQK = 2 * RT_TILE * DP / 256;         // q and k elements a thread fetches per tile
@@ -51,6 +59,7 @@ __global__ __launch_bounds__(256) void retention_kernel(RetentionArgs a) {
   __shared__ __attribute__((aligned(16))) float ks[RT_TILE * DP];
   __shared__ float vs[RT_TILE * RT_COLS];
   __shared__ float os[RT_TILE * RT_COLS];
+  __shared__ float ds[RT_TILE], steps[RT_TILE];  // a token's decay and step size (STEP)
   const int seq = blockIdx.x, head = blockIdx.y, col0 = blockIdx.z * RT_COLS;
   const int t0 = a.cu_q[seq], t1 = a.cu_q[seq + 1];
   if (t1 <= t0) return;
@@ -58,7 +67,9 @@ __global__ __launch_bounds__(256) void retention_kernel(RetentionArgs a) {
   const int sub = threadIdx.x & 15, colg = threadIdx.x >> 4;  // lane within its column, column of the block
   const int col = col0 + colg;
   const bool col_ok = col < vdim;
-  const float decay = a.decay[head];
+  const float decay = STEP ? 0.f : a.decay[head];
+  const float rate = STEP ? expf(a.a_log[head]) : 0.f, bias = STEP ? a.step_bias[head] : 0.f, skip = STEP ? a.skip[head] : 0.f;
+  const int qk_head = head / a.share;
   float* st = a.state + (((size_t)a.state_slots[seq] * a.heads + head) * vdim + min(col, vdim - 1)) * dim;
   const bool vec = (dim & 3) == 0;  // a lane's four rows are 16 aligned bytes of the column
   float s[G][4];
@@ -74,7 +85,7 @@ __global__ __launch_bounds__(256) void retention_kernel(RetentionArgs a) {
     }
   }
   // what this thread fetches of a tile: elements threadIdx.x + 256 i of q | k ([which][token][row]), one of v
-  float pre[NQK], pre_v;
+  float pre[NQK], pre_v, pre_step = 0.f;
   auto fetch = [&](int base) {
     const int n = min(RT_TILE, t1 - base);
 #pragma unroll
@@ -82,10 +93,14 @@ __global__ __launch_bounds__(256) void retention_kernel(RetentionArgs a) {
       const int e = threadIdx.x + 256 * i;
       const int which = e / (RT_TILE * DP), tok = (e / DP) % RT_TILE, d = e % DP;
       const bool ok = tok < n && d < dim;
-      const float* row = a.qkv + (size_t)(base + min(tok, n - 1)) * a.channels + (which ? a.k_first : a.q_first) + head * dim;
+      const float* row = a.qkv + (size_t)(base + min(tok, n - 1)) * a.channels + (which ? a.k_first : a.q_first) + qk_head * dim;
       pre[i] = ok ? row[d] : 0.f;
     }
     const int tok = min((int)threadIdx.x / RT_COLS, RT_TILE - 1), c = threadIdx.x % RT_COLS;
+    if (STEP && (int)threadIdx.x < n) {
+      const size_t at = (size_t)(base + threadIdx.x) * a.step_stride + head;
+      pre_step = a.step_code == QRT_F32 ? ((const float*)a.step)[at] : (float)((const bf16_t*)a.step)[at];
+    }
     pre_v = (tok < n && col0 + c < vdim) ? a.qkv[(size_t)(base + tok) * a.channels + a.v_first + head * vdim + col0 + c] : 0.f;
   };
   fetch(t0);
@@ -99,41 +114,36 @@ __global__ __launch_bounds__(256) void retention_kernel(RetentionArgs a) {
       else ks[e - RT_TILE * DP] = pre[i];
     }
     if (threadIdx.x < RT_TILE * RT_COLS) vs[threadIdx.x] = pre_v;
+    if (STEP && threadIdx.x < RT_TILE) {
+      const float z = pre_step + bias;
+      const float sp = z > 20.f ? z : log1pf(expf(z));
+      steps[threadIdx.x] = sp;
+      ds[threadIdx.x] = expf(-rate * sp);
+    }
     __syncthreads();
     if (base + RT_TILE < t1) fetch(base + RT_TILE);  // on its way during the walk
+    auto token = [&](int i) {
+      const float x = vs[i * RT_COLS + colg];
+      const float d = STEP ? ds[i] : decay, v = STEP ? x * steps[i] : x;
+      float acc = 0.f;
+#pragma unroll
+      for (int g = 0; g < G; ++g) {
+        const float4 kd = *(const float4*)(ks + i * DP + 4 * (sub + 16 * g));
+        const float4 qd = *(const float4*)(qs + i * DP + 4 * (sub + 16 * g));
+        s[g][0] = fmaf(d, s[g][0], kd.x * v); acc = fmaf(s[g][0], qd.x, acc);
+        s[g][1] = fmaf(d, s[g][1], kd.y * v); acc = fmaf(s[g][1], qd.y, acc);
+        s[g][2] = fmaf(d, s[g][2], kd.z * v); acc = fmaf(s[g][2], qd.z, acc);
+        s[g][3] = fmaf(d, s[g][3], kd.w * v); acc = fmaf(s[g][3], qd.w, acc);
+      }
+      acc = row16_sum(acc);
+      if (STEP) acc = fmaf(skip, x, acc);
+      if (sub == 0) os[i * RT_COLS + colg] = acc;
+    };
     if (n == RT_TILE) {
 #pragma unroll 4
-      for (int i = 0; i < RT_TILE; ++i) {
-        const float v = vs[i * RT_COLS + colg];
-        float acc = 0.f;
-#pragma unroll
-        for (int g = 0; g < G; ++g) {
-          const float4 kd = *(const float4*)(ks + i * DP + 4 * (sub + 16 * g));
-          const float4 qd = *(const float4*)(qs + i * DP + 4 * (sub + 16 * g));
-          s[g][0] = fmaf(decay, s[g][0], kd.x * v); acc = fmaf(s[g][0], qd.x, acc);
-          s[g][1] = fmaf(decay, s[g][1], kd.y * v); acc = fmaf(s[g][1], qd.y, acc);
-          s[g][2] = fmaf(decay, s[g][2], kd.z * v); acc = fmaf(s[g][2], qd.z, acc);
-          s[g][3] = fmaf(decay, s[g][3], kd.w * v); acc = fmaf(s[g][3], qd.w, acc);
-        }
-        acc = row16_sum(acc);
-        if (sub == 0) os[i * RT_COLS + colg] = acc;
-      }
+      for (int i = 0; i < RT_TILE; ++i) token(i);
     } else {
-      for (int i = 0; i < n; ++i) {
-        const float v = vs[i * RT_COLS + colg];
-        float acc = 0.f;
-#pragma unroll
-        for (int g = 0; g < G; ++g) {
-          const float4 kd = *(const float4*)(ks + i * DP + 4 * (sub + 16 * g));
-          const float4 qd = *(const float4*)(qs + i * DP + 4 * (sub + 16 * g));
-          s[g][0] = fmaf(decay, s[g][0], kd.x * v); acc = fmaf(s[g][0], qd.x, acc);
-          s[g][1] = fmaf(decay, s[g][1], kd.y * v); acc = fmaf(s[g][1], qd.y, acc);
-          s[g][2] = fmaf(decay, s[g][2], kd.z * v); acc = fmaf(s[g][2], qd.z, acc);
-          s[g][3] = fmaf(decay, s[g][3], kd.w * v); acc = fmaf(s[g][3], qd.w, acc);
-        }
-        acc = row16_sum(acc);
-        if (sub == 0) os[i * RT_COLS + colg] = acc;
-      }
+      for (int i = 0; i < n; ++i) token(i);
     }
     __syncthreads();
     {  // the tile's read-outs: thread (token, column)
@@ -160,19 +170,29 @@ extern "C" int qrt_retention(const RetentionArgs* args, int num_tokens, int num_
   RetentionArgs a = *args;
   QRT_CHECK(num_tokens >= 0 && num_seqs >= 0 && num_slots > 0, "retention: bad counts");
   QRT_CHECK(a.heads > 0 && a.heads <= 65535 && a.dim > 0 && a.dim <= 512 && a.vdim > 0, "retention: %d heads of %d x %d", a.heads, a.dim, a.vdim);
-  QRT_CHECK(a.channels >= 2 * a.heads * a.dim + a.heads * a.vdim, "retention: %d channels hold no q, k and v", a.channels);
+  if (a.share == 0) a.share = 1;
+  QRT_CHECK(a.share > 0 && a.heads % a.share == 0, "retention: %d heads, %d of which share a key", a.heads, a.share);
+  QRT_CHECK(a.channels >= 2 * (a.heads / a.share) * a.dim + a.heads * a.vdim, "retention: %d channels hold no q, k and v", a.channels);
+  QRT_CHECK(a.step ? a.step_bias && a.a_log && a.skip && a.step_stride >= a.heads : a.decay != nullptr,
+            "retention: neither constant decays nor step logits with their bias, rate and skip");
   if (num_tokens == 0 || num_seqs == 0) return 0;
   const dim3 grid(num_seqs, a.heads, (a.vdim + RT_COLS - 1) / RT_COLS);
   const int groups = (a.dim + 63) / 64;
+#define GO(G, TILE)                                                                 \
+  do {                                                                              \
+    if (a.step) retention_kernel<G, TILE, true><<<grid, 256, 0, stream>>>(a);       \
+    else retention_kernel<G, TILE, false><<<grid, 256, 0, stream>>>(a);             \
+  } while (0)
   if (num_tokens <= 2 * num_seqs) {  // decoded tokens, mostly
-    if (groups <= 1) retention_kernel<1, 4><<<grid, 256, 0, stream>>>(a);
-    else if (groups <= 2) retention_kernel<2, 4><<<grid, 256, 0, stream>>>(a);
-    else if (groups <= 4) retention_kernel<4, 4><<<grid, 256, 0, stream>>>(a);
-    else retention_kernel<8, 4><<<grid, 256, 0, stream>>>(a);
-  } else if (groups <= 1) retention_kernel<1, 16><<<grid, 256, 0, stream>>>(a);
-  else if (groups <= 2) retention_kernel<2, 16><<<grid, 256, 0, stream>>>(a);
-  else if (groups <= 4) retention_kernel<4, 16><<<grid, 256, 0, stream>>>(a);
-  else retention_kernel<8, 8><<<grid, 256, 0, stream>>>(a);
+    if (groups <= 1) GO(1, 4);
+    else if (groups <= 2) GO(2, 4);
+    else if (groups <= 4) GO(4, 4);
+    else GO(8, 4);
+  } else if (groups <= 1) GO(1, 16);
+  else if (groups <= 2) GO(2, 16);
+  else if (groups <= 4) GO(4, 16);
+  else GO(8, 8);
+#undef GO
   QRT_LAUNCH_CHECK("retention");
   return 0;
 }

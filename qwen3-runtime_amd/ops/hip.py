@@ -44,7 +44,7 @@ class _QkArgs(Structure):
         ("k_cache", c_void_p), ("v_cache", c_void_p),
         ("num_tokens", c_int), ("nq", c_int), ("nkv", c_int), ("nv", c_int),
         ("head_dim", c_int), ("page_size", c_int), ("eps", c_float), ("rope", c_void_p),
-        ("value_dim", c_int),
+        ("value_dim", c_int), ("rot_pairs", c_int), ("v_rope", c_void_p),
     ]
 
 
@@ -55,7 +55,7 @@ class _AttnArgs(Structure):
         ("table_width", c_int), ("num_tokens", c_int), ("nq", c_int), ("nkv", c_int),
         ("head_dim", c_int), ("page_size", c_int), ("window", c_int), ("scale", c_float),
         ("chunk", c_int), ("softcap", c_float), ("value_dim", c_int), ("gate", c_void_p), ("gate_stride", c_long),
-        ("keep_first", c_int), ("sink", c_int),
+        ("keep_first", c_int), ("sink", c_int), ("turn", c_void_p),
     ]
 
 
@@ -82,6 +82,7 @@ class _AttnTileArgs(Structure):
         ("max_items", c_int), ("items", c_void_p),
         ("chunk", c_int), ("cap_in", c_float), ("cap_out", c_float),
         ("gate", c_void_p), ("gate_stride", c_long), ("keep_first", c_int), ("sink", c_int),
+        ("rope_pairs", c_int), ("turn", c_void_p),
     ]
 
 
@@ -91,7 +92,7 @@ class _ConvArgs(Structure):
         ("cu_q", c_void_p), ("seq_of_token", c_void_p), ("state_slots", c_void_p), ("out", c_void_p),
         ("num_tokens", c_int), ("channels", c_int), ("num_taps", c_int), ("nseg", c_int),
         ("seg_first", c_int * 4), ("seg_heads", c_int * 4), ("seg_width", c_int * 4), ("seg_mode", c_int * 4),
-        ("total_heads", c_int), ("unit_eps", c_float), ("fuse_tail", c_int),
+        ("total_heads", c_int), ("unit_eps", c_float), ("fuse_tail", c_int), ("bias", c_void_p),
     ]
 
 
@@ -118,7 +119,9 @@ class _RetentionArgs(Structure):
     _fields_ = [
         ("qkv", c_void_p), ("channels", c_int), ("q_first", c_int), ("k_first", c_int), ("v_first", c_int),
         ("decay", c_void_p), ("state", c_void_p), ("out", c_void_p), ("cu_q", c_void_p), ("state_slots", c_void_p),
-        ("heads", c_int), ("dim", c_int), ("vdim", c_int),
+        ("heads", c_int), ("dim", c_int), ("vdim", c_int), ("share", c_int),
+        ("step", c_void_p), ("step_stride", c_long), ("step_code", c_int),
+        ("step_bias", c_void_p), ("a_log", c_void_p), ("skip", c_void_p),
     ]
 
 
@@ -281,6 +284,12 @@ class HipOps:
         self._check(self.lib, self.lib.qrt_scale(_ptr(x), c_float(factor), c_long(x.numel()), _stream()))
         return x
 
+    def softcap(self, x, limit):
+        """``x = limit * tanh(x / limit)`` in place, float32."""
+        _need(x, "x", torch.float32)
+        self._check(self.lib, self.lib.qrt_softcap(_ptr(x), c_float(limit), c_long(x.numel()), _stream()))
+        return x
+
     def unary_act(self, x, kind):
         """An activation without a gate, element by element: ``relu2`` is ``max(x, 0)^2``."""
         _need(x, "x")
@@ -358,6 +367,49 @@ class HipOps:
         self._check(self.lib, self.lib.qrt_scaled_add_rmsnorm(
             _ptr(residual), ptrs, codes, counts, scales, c_int(n), c_long(t * h), _ptr(weight), c_float(eps), _ptr(rows),
             _ptr(out), _CODE[out_dtype], c_int(n_out), c_int(h), _stream()))
+        return out
+
+    # ---- norms in groups of the row ---------------------------------------------------
+    def group_norm_update(self, residual, y, after, norm, groups, out_dtype, rows=None):
+        """``residual += y`` in place (``y`` a matrix or float32 planes, or None: nothing is pending), ``y``
+        first RMS-normed in ``groups`` equal parts of the row if ``after`` = (weight, eps) is given; returns
+        the rows of the sum in ``out_dtype``, normed likewise by ``norm`` = (weight, eps), or (None) as they
+        are. With ``rows`` only those, and ``residual`` is left alone."""
+        t, h = residual.shape
+        _need(residual, "residual", torch.float32)
+        if groups < 1 or h % groups:
+            raise OpsError(f"a norm of {h} elements in {groups} equal parts")
+        py, cy, ny = (None, F32, 1) if y is None else _planes(y, t, h, "sub-layer output")
+        wa, ea = (None, 0.0) if after is None else after
+        wn, en = (None, 0.0) if norm is None else norm
+        for name, w in (("weight of the norm behind the sub-layer", wa), ("norm weight", wn)):
+            if w is not None:
+                _need(w, name, torch.float32, (h,))
+        n_out = t
+        if rows is not None:
+            _need(rows, "rows", torch.int32)
+            n_out = rows.numel()
+        out = torch.empty((n_out, h), dtype=out_dtype, device=residual.device)
+        self._check(self.lib, self.lib.qrt_group_norm_update(
+            _ptr(residual), py, c_int(cy), c_int(ny), c_long(t * h), _ptr(wa), c_float(ea), _ptr(wn), c_float(en), _ptr(rows),
+            _ptr(out), _CODE[out_dtype], c_int(n_out), c_int(h), c_int(groups), _stream()))
+        return out
+
+    def gated_group_norm(self, o, gate, weight, eps, groups, out_dtype):
+        """``v = o * silu(gate)`` over all heads of a token, then the RMS norm of ``v`` in ``groups`` equal parts
+        times ``weight``; ``gate`` may be columns of a wider matrix. [T, heads * vdim]."""
+        t, heads, vdim = o.shape
+        width = heads * vdim
+        _need(o, "read-out", torch.float32)
+        _need(weight, "read-out norm weight", torch.float32, (width,))
+        if not gate.is_cuda or tuple(gate.shape) != (t, width) or gate.stride(1) != 1 or gate.dtype not in _CODE:
+            raise OpsError(f"gate {tuple(gate.shape)} {gate.dtype} does not fit {t} tokens of {width} channels")
+        if groups < 1 or width % groups:
+            raise OpsError(f"a norm of {width} elements in {groups} equal parts")
+        out = torch.empty((t, width), dtype=out_dtype, device=o.device)
+        self._check(self.lib, self.lib.qrt_gated_group_norm(
+            _ptr(o), c_void_p(gate.data_ptr()), c_long(gate.stride(0)), _CODE[gate.dtype], _ptr(weight), c_float(eps), _ptr(out),
+            _CODE[out_dtype], c_int(t), c_int(width), c_int(groups), _stream()))
         return out
 
     # ---- attention through a latent, retention ------------------------------------------
@@ -485,6 +537,33 @@ class HipOps:
         self._check(self.lib, self.lib.qrt_retention(byref(a), c_int(t), c_int(ctx.num_seqs), c_int(state.shape[0]), _stream()))
         return out
 
+    def state_space(self, ctx, xbc, step, step_bias, a_log, skip, state, heads, groups, n, vdim):
+        """Per sequence and head from the slot's state (float32 [slots, heads, vdim, n], updated in place):
+        ``D = softplus(step + step_bias); S <- exp(-exp(a_log) D) S + (D x) B^T; y = S C + skip x``. ``xbc``
+        float32 [T, heads * vdim | groups * n | groups * n] (x, B, C; head h uses group h // (heads /
+        groups)); ``step`` [T, heads] may be columns of a wider matrix. Returns y, float32 [T, heads, vdim]."""
+        t = ctx.num_tokens
+        c = heads * vdim + 2 * groups * n
+        _need(xbc, "x | B | C", torch.float32, (t, c))
+        _need(state, "state", torch.float32, (state.shape[0], heads, vdim, n))
+        if not step.is_cuda or tuple(step.shape) != (t, heads) or step.stride(1) != 1 or step.dtype not in _CODE:
+            raise OpsError(f"step logits: {tuple(step.shape)} {step.dtype} with strides {step.stride()} for {t} tokens of {heads}")
+        if heads % groups:
+            raise OpsError(f"{heads} heads in {groups} groups")
+        a = _RetentionArgs()
+        a.qkv, a.channels = xbc.data_ptr(), c
+        a.v_first, a.k_first, a.q_first = 0, heads * vdim, heads * vdim + groups * n
+        a.step, a.step_stride, a.step_code = step.data_ptr(), step.stride(0), _CODE[step.dtype]
+        for name, w in (("step_bias", step_bias), ("a_log", a_log), ("skip", skip)):
+            setattr(a, name, _need(w, name, torch.float32, (heads,)).data_ptr())
+        out = torch.empty((t, heads, vdim), dtype=torch.float32, device=xbc.device)
+        a.state, a.out = state.data_ptr(), out.data_ptr()
+        a.cu_q = _need(ctx.cu_q, "cu_q", torch.int32, (ctx.num_seqs + 1,)).data_ptr()
+        a.state_slots = _need(ctx.state_slots, "state_slots", torch.int32, (ctx.num_seqs,)).data_ptr()
+        a.heads, a.dim, a.vdim, a.share = heads, n, vdim, heads // groups
+        self._check(self.lib, self.lib.qrt_retention(byref(a), c_int(t), c_int(ctx.num_seqs), c_int(state.shape[0]), _stream()))
+        return out
+
     # ---- steps between sub-layers that are neither a product nor a plain norm -----------
     def norm_mean(self, ya, wa, yb, wb, eps):
         """``(rmsnorm(ya) * wa + rmsnorm(yb) * wb) / 2`` over the rows, float32 [T, H]; either input a
@@ -518,17 +597,25 @@ class HipOps:
         self._check(self.lib, self.lib.qrt_accumulate(_ptr(acc), py, c_int(cy), c_int(ny), c_long(t * h), _stream()))
         return acc
 
-    def gated_act(self, gate_up, activation="swiglu", limit=0.0):
-        """The gated activation of [T, 2I] (gate columns first): ``swiglu``, or ``clamped``."""
+    def gated_act(self, gate_up, activation="swiglu", limit=0.0, scale=None, order=None):
+        """The gated activation of [T, 2I] (gate columns first): ``swiglu``, or ``clamped``. With ``scale``
+        (float32 [T]) both halves of row t are first multiplied by ``scale[order[t]]`` (``order`` None: ``scale[t]``)."""
+        if scale is not None:
+            _need(scale, "row scales", torch.float32)
+            if order is not None:
+                _need(order, "order", torch.int32, (gate_up.shape[0],))
+            if scale.numel() != gate_up.shape[0]:
+                raise OpsError(f"{scale.numel()} row scales for {gate_up.shape[0]} rows")
         if activation == "swiglu":
-            return self.swiglu(gate_up)
+            return self.swiglu(gate_up, scale, order)
         _need(gate_up, "gate_up")
         t, two_i = gate_up.shape
         if two_i % 2:
             raise OpsError(f"gate_up has odd width {two_i}")
         out = torch.empty((t, two_i // 2), dtype=gate_up.dtype, device=gate_up.device)
         self._check(self.lib, self.lib.qrt_gated_act(_ptr(gate_up), _ptr(out), _CODE[gate_up.dtype], c_int(t),
-                                                     c_int(two_i // 2), c_int(ACTIVATIONS[activation]), c_float(limit), _stream()))
+                                                     c_int(two_i // 2), c_int(ACTIVATIONS[activation]), c_float(limit),
+                                                     _ptr(scale), _ptr(order), _stream()))
         return out
 
     def bias_rotate_pairs(self, x, bias, positions, freq, rot_heads, head_dim):
@@ -550,9 +637,9 @@ class HipOps:
         return x
 
     # ---- gated delta rule ---------------------------------------------------------------
-    def delta_conv(self, ctx, y, channels, taps, tail, segments, unit_eps):
-        """The first ``channels`` columns of ``y`` [T, W] through their causal convolutions
-        (``taps`` float32 [C, K]) and silu, then per head as ``segments`` say, each (heads, width,
+    def delta_conv(self, ctx, y, channels, taps, tail, segments, unit_eps, first=0, bias=None):
+        """``channels`` columns of ``y`` [T, W], from column ``first`` on, through their causal convolutions
+        (``taps`` float32 [C, K]; ``bias`` float32 [C] or None is added) and silu, then per head as ``segments`` say, each (heads, width,
         mode): 0 as it is, 1 scaled to a unit vector, 2 that times width^(-1/2). float32 [T, C].
         ``tail`` [slots, C, K-1] float32 holds each request's last inputs and is brought up to date."""
         t, w = y.shape
@@ -561,21 +648,23 @@ class HipOps:
         _need(taps, "taps", torch.float32, (channels, k))
         slots = tail.shape[0]
         _need(tail, "convolution tail", torch.float32, (slots, channels, max(k - 1, 1)))
-        if t != ctx.num_tokens or channels > w or not 1 <= len(segments) <= 4:
+        if t != ctx.num_tokens or first < 0 or first + channels > w or not 1 <= len(segments) <= 4:
             raise OpsError(f"delta_conv: {t} rows for {ctx.num_tokens} tokens, {channels} channels in {w} columns")
         a = _ConvArgs()
-        a.x, a.x_stride, a.taps, a.tail = y.data_ptr(), y.stride(0), taps.data_ptr(), tail.data_ptr()
+        a.x, a.x_stride, a.taps, a.tail = y.data_ptr() + first * y.element_size(), y.stride(0), taps.data_ptr(), tail.data_ptr()
+        if bias is not None:
+            a.bias = _need(bias, "convolution bias", torch.float32, (channels,)).data_ptr()
         a.cu_q = _need(ctx.cu_q, "cu_q", torch.int32, (ctx.num_seqs + 1,)).data_ptr()
         a.seq_of_token = _need(ctx.seq_of_token, "seq_of_token", torch.int32, (t,)).data_ptr()
         a.state_slots = _need(ctx.state_slots, "state_slots", torch.int32, (ctx.num_seqs,)).data_ptr()
         out = torch.empty((t, channels), dtype=torch.float32, device=y.device)
         a.out, a.num_tokens, a.channels, a.num_taps, a.nseg, a.unit_eps = out.data_ptr(), t, channels, k, len(segments), unit_eps
-        first = 0
+        at = 0
         for i, (heads, width, mode) in enumerate(segments):
-            a.seg_first[i], a.seg_heads[i], a.seg_width[i], a.seg_mode[i] = first, heads, width, mode
-            first += heads * width
-        if first != channels:
-            raise OpsError(f"delta_conv: segments cover {first} of {channels} channels")
+            a.seg_first[i], a.seg_heads[i], a.seg_width[i], a.seg_mode[i] = at, heads, width, mode
+            at += heads * width
+        if at != channels:
+            raise OpsError(f"delta_conv: segments cover {at} of {channels} channels")
         self._check(self.lib, self.lib.qrt_delta_conv(byref(a), _CODE[y.dtype], c_int(ctx.num_seqs), c_int(slots),
                                                       c_int(ctx.max_q_len), _stream()))
         return out
@@ -691,10 +780,14 @@ class HipOps:
                                                      c_int(bool(renormalise)), c_float(weight_scale), _stream()))
         return index, weight
 
-    def moe_swiglu(self, x, gate_up, down, index, weight, activation="swiglu", limit=0.0, out=None):
+    def moe_swiglu(self, x, gate_up, down, index, weight, activation="swiglu", limit=0.0, out=None, weight_on_input=False):
         """``sum_j weight[t, j] * down[e] (silu(gate[e] x) * (up[e] x))`` with ``e = index[t, j]``;
         ``gate_up`` [E, 2I, H] (gate rows first), ``down`` [E, H, I]. float32 [T, H]. ``activation="relu2"``:
-        experts without a gate, ``down[e] relu(up[e] x)^2``, and ``gate_up`` is the up rows alone, [E, I, H]."""
+        experts without a gate, ``down[e] relu(up[e] x)^2``, and ``gate_up`` is the up rows alone, [E, I, H].
+        ``weight_on_input`` (gated experts): a weight scales its expert's input, ``sum_j expert_j(weight[t, j] x)``:
+        it multiplies the first products in float32 in front of the activation, and nothing after it."""
+        if weight_on_input and activation == "relu2":
+            raise OpsError("weights on the experts' input go with gated experts")
         t, h = x.shape
         n, rows_e, _ = gate_up.shape
         inter = rows_e if activation == "relu2" else rows_e // 2
@@ -713,7 +806,7 @@ class HipOps:
         pairs = t * top
         if (pairs >= self.moe_grouped_min_pairs and pairs >= self.moe_grouped_pairs_per_expert * n
                 and not torch.cuda.is_current_stream_capturing()):
-            return self._moe_grouped(x, gate_up, down, index, weight, out, activation, limit)
+            return self._moe_grouped(x, gate_up, down, index, weight, out, activation, limit, weight_on_input)
         kind = (c_int(ACTIVATIONS[activation]), c_float(limit))
         act = torch.empty((t * top, inter), dtype=x.dtype, device=x.device)
         vec = 16 // x.element_size()
@@ -727,14 +820,16 @@ class HipOps:
                                                          c_int(pairs), c_int(n), _stream()))
             self._check(self.lib, self.lib.qrt_moe_by_expert(_ptr(x), _ptr(gate_up), _ptr(down), _ptr(order), _ptr(offsets),
                                                              _ptr(act), _ptr(y), _CODE[x.dtype], c_int(h), c_int(inter),
-                                                             c_int(n), c_int(top), *kind, _stream()))
+                                                             c_int(n), c_int(top), *kind, _ptr(weight) if weight_on_input else None,
+                                                            _stream()))
             self._check(self.lib, self.lib.qrt_moe_combine(_ptr(y), _ptr(place), _ptr(index), _ptr(offsets), c_int(0),
-                                                           _ptr(weight), _ptr(out), _CODE[x.dtype], c_int(t), c_int(h),
-                                                           c_int(top), _stream()))
+                                                           None if weight_on_input else _ptr(weight), _ptr(out),
+                                                           _CODE[x.dtype], c_int(t), c_int(h), c_int(top), _stream()))
             return out
         self._check(self.lib, self.lib.qrt_moe_pairs(_ptr(x), _ptr(gate_up), _ptr(down), _ptr(index), _ptr(weight),
                                                      _ptr(act), _ptr(out), _CODE[x.dtype], c_int(t), c_int(h),
-                                                     c_int(inter), c_int(n), c_int(top), *kind, _stream()))
+                                                     c_int(inter), c_int(n), c_int(top), *kind, c_int(bool(weight_on_input)),
+                                                     _stream()))
         return out
 
     # Steps of many tokens run the experts one by one, each on the rows of its own tokens, with
@@ -748,7 +843,7 @@ class HipOps:
     # walks the expert's tokens; below it, once per pair (fewer launches, and pairs rarely meet).
     moe_by_expert_pairs_per_expert = 1
 
-    def _moe_grouped(self, x, gate_up, down, index, weight, out, activation="swiglu", limit=0.0):
+    def _moe_grouped(self, x, gate_up, down, index, weight, out, activation="swiglu", limit=0.0, weight_on_input=False):
         t, h = x.shape
         n, top = gate_up.shape[0], index.shape[1]
         pairs = t * top
@@ -770,6 +865,8 @@ class HipOps:
                                                       _stream()))
         y = torch.empty((pairs, h), dtype=x.dtype, device=dev)
         busy = [(e, bounds[e], bounds[e + 1]) for e in range(n) if bounds[e + 1] > bounds[e]]
+        # weights on the input: each row's own, found through the order of the rows, in front of the activation
+        scaled = {"scale": weight.view(-1), "order": order} if weight_on_input else {}
         if x.dtype == torch.bfloat16:
             # what bounds this form is the host's time per launch, so an expert costs two of them:
             # its products go straight into its rows of one buffer each (the library's for more
@@ -780,7 +877,8 @@ class HipOps:
                     torch.mm(xs[a:b], gate_up[e].t(), out=both[a:b])
                 else:
                     both[a:b] = self.linear(xs[a:b], gate_up[e])
-            act = self.unary_act(both, activation) if activation == "relu2" else self.gated_act(both, activation, limit)
+            act = self.unary_act(both, activation) if activation == "relu2" else \
+                self.gated_act(both, activation, limit, **scaled)
             for e, a, b in busy:
                 if b - a > self.own_max_rows:
                     torch.mm(act[a:b], down[e].t(), out=y[a:b])
@@ -790,12 +888,15 @@ class HipOps:
             for e, a, b in busy:
                 if activation == "relu2":
                     act = self.unary_act(self.linear(xs[a:b], gate_up[e]), activation)
+                elif weight_on_input:
+                    act = self.gated_act(self.linear(xs[a:b], gate_up[e]), activation, limit,
+                                         weight.view(-1)[order[a:b].long()].contiguous())
                 else:
                     act = self.gated_linear(xs[a:b], gate_up[e], activation, limit)
                 y[a:b] = self.linear(act, down[e])
         self._check(self.lib, self.lib.qrt_moe_combine(_ptr(y), _ptr(place), _ptr(index), _ptr(offsets), c_int(padded),
-                                                       _ptr(weight), _ptr(out), _CODE[x.dtype], c_int(t), c_int(h),
-                                                       c_int(top), _stream()))
+                                                       None if weight_on_input else _ptr(weight), _ptr(out),
+                                                       _CODE[x.dtype], c_int(t), c_int(h), c_int(top), _stream()))
         return out
 
     def sigmoid_gate(self, out, gate):
@@ -808,14 +909,14 @@ class HipOps:
                                                         _CODE[out.dtype], c_int(t), c_int(w), _stream()))
         return out
 
-    def swiglu(self, gate_up):
+    def swiglu(self, gate_up, scale=None, order=None):
         _need(gate_up, "gate_up")
         t, two_i = gate_up.shape
         if two_i % 2:
             raise OpsError(f"gate_up has odd width {two_i}")
         out = torch.empty((t, two_i // 2), dtype=gate_up.dtype, device=gate_up.device)
         self._check(self.lib, self.lib.qrt_swiglu(_ptr(gate_up), _ptr(out), _CODE[gate_up.dtype],
-                                                  c_int(t), c_int(two_i // 2), _stream()))
+                                                  c_int(t), c_int(two_i // 2), _ptr(scale), _ptr(order), _stream()))
         return out
 
     # ---- matrix products -------------------------------------------------------
@@ -996,9 +1097,11 @@ class HipOps:
     rope_table_from_tokens = 256
 
     def qk_norm_rope_store(self, qkv, nq, nkv, d, q_w, k_w, eps, inv_freq, positions, cache, ctx=None,
-                           angles_key=None, value_dim=None, extra=0):
-        """Per-head RMSNorm of queries and keys, NeoX rotation, and the write of keys and values into
-        the cache, in one pass over ``qkv``; returns the queries. With the step's context given,
+                           angles_key=None, value_dim=None, extra=0, value_turn=None):
+        """Per-head RMSNorm of queries and keys, rotation of their first ``2 len(inv_freq)`` elements (first
+        half of those against second half), and the write of keys and values into
+        the cache, in one pass over ``qkv``; returns the queries. ``value_turn`` (frequencies, a name for them
+        as ``angles_key``): the values turn too, over all their elements, before they are stored. With the step's context given,
         the angles of a long step come from ``rope_table`` (``angles_key`` as there). Values may
         have ``value_dim`` elements a head; ``extra`` columns behind them are left alone."""
         t, width = qkv.shape
@@ -1008,7 +1111,10 @@ class HipOps:
             if w is not None:
                 _need(w, name, torch.float32, (d,))
         if inv_freq is not None:
-            _need(inv_freq, "inv_freq", torch.float32, (d // 2,))
+            pairs = inv_freq.numel()
+            _need(inv_freq, "inv_freq", torch.float32, (pairs,))
+            if not 1 <= pairs <= d // 2:
+                raise OpsError(f"{pairs} pairs turn in heads of {d}")
             _need(positions, "positions", torch.int32, (t,))
         q = torch.empty((t, nq * d), dtype=qkv.dtype, device=qkv.device)
         es = qkv.element_size()
@@ -1024,6 +1130,12 @@ class HipOps:
         a.q_out = q.data_ptr()
         a.num_tokens, a.nq, a.nkv, a.nv, a.head_dim, a.eps = t, nq, nkv, nkv, d, eps
         a.value_dim = dv
+        if inv_freq is not None:
+            a.rot_pairs = pairs
+        if value_turn is not None and cache is not None:
+            if ctx is None or value_turn[0].numel() * 2 != dv:
+                raise OpsError(f"turned values of {dv} take the step's context and {dv // 2} frequencies")
+            a.v_rope = self.rope_table(ctx, *value_turn).data_ptr()
         pages = 0
         if cache is not None:
             pages = self._check_cache(cache, nkv, d, qkv.dtype, dv)
@@ -1144,11 +1256,12 @@ class HipOps:
         return table
 
     def fuses_decode_attention(self, ctx, qkv, nq, nkv, d, cache, value_dim=None, chunk=None, softcap=None,
-                               gate=None, keep_first=0, sink=False) -> bool:
+                               gate=None, keep_first=0, sink=False, rot_pairs=None, value_turn=None) -> bool:
         """Whether ``decode_attention`` serves this step: one token per sequence, bfloat16, a head
-        size that keeps a rotation pair in one lane (a multiple of 64, up to 256), at most 16
+        size that keeps a rotation pair in one lane (a multiple of 64, up to 256; ``rot_pairs``, the pairs
+        of a head that turn, a multiple of 32), at most 16
         query heads per key head, and a layer that writes its own cache."""
-        if value_dim not in (None, d):
+        if value_dim not in (None, d) or (rot_pairs is not None and rot_pairs % 32):
             return False
         return (self.fuse_decode and qkv.dtype == torch.bfloat16 and ctx.max_q_len == 1
                 and ctx.num_tokens == ctx.num_seqs and d % 64 == 0 and d <= 256 and nq // nkv <= 16
@@ -1156,7 +1269,8 @@ class HipOps:
                 and cache.k.dtype == torch.bfloat16)
 
     def decode_attention(self, qkv, cache, ctx, nq, nkv, d, scale, window, q_w, k_w, eps, inv_freq,
-                         angles_key=None, chunk=None, softcap=None, gate=None, value_dim=None, keep_first=0, sink=False):
+                         angles_key=None, chunk=None, softcap=None, gate=None, value_dim=None, keep_first=0, sink=False,
+                         value_turn=None):
         """``paged_attention(qk_norm_rope_store(qkv, ...))`` for a step of single tokens, in one
         kernel: each block forms its queries from ``qkv`` (RMSNorm per head, NeoX rotation by the
         step's angle table), attends over the cached keys before the token, adds the token's own
@@ -1179,15 +1293,27 @@ class HipOps:
         if not scale > 0:
             raise OpsError(f"the bfloat16 attention kernels take a positive score scale, not {scale}")
         own = {"qkv": qkv, "q_weight": q_w, "k_weight": k_w, "eps": eps,
-               "rope": None if inv_freq is None else self.rope_table(ctx, inv_freq, angles_key)}
+               "rope": None if inv_freq is None else self.rope_table(ctx, inv_freq, angles_key),
+               "rope_pairs": 0 if inv_freq is None else inv_freq.numel()}
         out = torch.empty((t, nq * d), dtype=qkv.dtype, device=qkv.device)
         self._launch_attention(None, out, cache, ctx, nq, nkv, d, scale, window or 0, None, True, own,
-                               chunk=chunk or 0, softcap=softcap or 0.0, gate=gate, keep_first=keep_first, sink=sink)
+                               chunk=chunk or 0, softcap=softcap or 0.0, gate=gate, keep_first=keep_first, sink=sink,
+                               turn=self._turn_table(ctx, value_turn, d))
         return out
 
+    def _turn_table(self, ctx, value_turn, dv):
+        """The step's angles of turned values of ``dv`` elements (None: values are not turned)."""
+        if value_turn is None:
+            return None
+        if value_turn[0].numel() * 2 != dv:
+            raise OpsError(f"{value_turn[0].numel()} frequencies for turned values of {dv}")
+        return self.rope_table(ctx, *value_turn)
+
     def paged_attention(self, q, cache, ctx, nq, nkv, d, scale, window, chunk=None, softcap=None, value_dim=None,
-                        gate=None, keep_first=0, sink=False):
-        """Attention of every query over its sequence's cache. Beyond the plain form: a mask of
+                        gate=None, keep_first=0, sink=False, value_turn=None):
+        """Attention of every query over its sequence's cache. ``value_turn`` (frequencies, a name for
+        them): the cached values are turned by their positions, and each head's output is turned back by
+        the query's. Beyond the plain form: a mask of
         chunks instead of a window (``chunk``), a tanh cap on the scaled scores (``softcap``),
         values of ``value_dim`` elements, and a ``gate`` [T, nq * value_dim] (columns of a wider
         matrix will do) whose sigmoid multiplies the output."""
@@ -1209,7 +1335,7 @@ class HipOps:
             raise OpsError("first keys are kept in sight beside a window")
         if dv == d and q.dtype == torch.bfloat16 and d % 16 == 0 and d <= 512 and ps % 8 == 0:
             self._attention_mfma(q, out, cache, ctx, nq, nkv, d, scale, window or 0, chunk or 0, softcap or 0.0, gate,
-                                 keep_first=int(keep_first), sink=bool(sink))
+                                 keep_first=int(keep_first), sink=bool(sink), turn=self._turn_table(ctx, value_turn, dv))
         else:
             a = _AttnArgs()
             a.q, a.out, a.k_cache, a.v_cache = q.data_ptr(), out.data_ptr(), cache.k.data_ptr(), cache.v.data_ptr()
@@ -1222,6 +1348,7 @@ class HipOps:
             if gate is not None:
                 a.gate, a.gate_stride = gate.data_ptr(), gate.stride(0)
             a.keep_first, a.sink = int(keep_first), int(bool(sink))
+            a.turn = _addr(self._turn_table(ctx, value_turn, dv))
             self._check(self.lib, self.lib.qrt_attention_f32(byref(a), _CODE[q.dtype], _stream()))
         return out
 
@@ -1351,7 +1478,7 @@ class HipOps:
     split_launch_min_kv = 1024
 
     def _attention_mfma(self, q, out, cache, ctx, nq, nkv, d, scale, window, chunk=0, softcap=0.0, gate=None,
-                        keep_first=0, sink=False):
+                        keep_first=0, sink=False, turn=None):
         """Which kernel for which sequences. Steps of decoded tokens only: the decode kernel.
         Other steps: the prompt kernels; but sequences of at most 16 rows with a long context
         (decoded tokens beside a prompt portion) would each walk all their keys in one block
@@ -1361,7 +1488,7 @@ class HipOps:
             raise OpsError(f"the bfloat16 attention kernels take a positive score scale, not {scale}")
         g = nq // nkv
         seqs = range(ctx.num_seqs)
-        more = {"keep_first": keep_first, "sink": sink}
+        more = {"keep_first": keep_first, "sink": sink, "turn": turn}
         if ctx.max_q_len * g <= 16 and d <= 256:
             return self._launch_attention(q, out, cache, ctx, nq, nkv, d, scale, window, None, True, chunk=chunk, softcap=softcap, gate=gate, **more)
         small = [s for s in seqs if ctx.q_lens_host[s] * g <= 16]
@@ -1375,7 +1502,7 @@ class HipOps:
         self._launch_attention(q, out, cache, ctx, nq, nkv, d, scale, window, None, False, chunk=chunk, softcap=softcap, gate=gate, **more)
 
     def _launch_attention(self, q, out, cache, ctx, nq, nkv, d, scale, window, subset, decode, own=None,
-                          chunk=0, softcap=0.0, gate=None, keep_first=0, sink=False):
+                          chunk=0, softcap=0.0, gate=None, keep_first=0, sink=False, turn=None):
         """One launch over the sequences in ``subset`` (None: all of the step's). ``own``: the
         decode kernel takes the tokens' queries, own keys and own values from the q/k/v product
         (``decode_attention``); ``q`` is then None. ``chunk``: a mask of chunks in place of a
@@ -1428,6 +1555,7 @@ class HipOps:
         a.chunk = chunk
         # beside a window the sequence's first keys stay in sight; a sink: one more term in the softmax's sum
         a.keep_first, a.sink = int(keep_first), int(bool(sink))
+        a.turn = _addr(turn)  # float32 [T, d]: angles by which the outputs are turned back
         if softcap:
             a.cap_in, a.cap_out = scale / softcap, softcap / scale
         if gate is not None:
@@ -1456,6 +1584,7 @@ class HipOps:
         else:  # the token's own query, key and value come from the product that made them
             a.qkv, a.qkv_stride = own["qkv"].data_ptr(), own["qkv"].shape[1]
             a.q_weight, a.k_weight, a.rope = _addr(own["q_weight"]), _addr(own["k_weight"]), _addr(own["rope"])
+            a.rope_pairs = own["rope_pairs"]
             a.slots, a.eps = cache.group.slots.data_ptr(), own["eps"]
         a.cu_q = _need(ctx.cu_q, "cu_q", torch.int32, (ctx.num_seqs + 1,)).data_ptr()
         a.kv_lens = _need(ctx.kv_lens, "kv_lens", torch.int32, (ctx.num_seqs,)).data_ptr()
