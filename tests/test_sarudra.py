@@ -450,7 +450,7 @@ def test_weights_scale_the_experts_input(backend, width, ff, experts, top, share
     if activation == "swiglu":
         elsewhere = torch.stack([sum(weight[i, j] * P.gated(x[i].double(), w64, f"e{int(index[i, j])}.") for j in range(top)) for i in range(t)])
         here = want - (P.gated(x.double(), w64, "shared.") if shared else 0.0)
-        assert ((elsewhere - here).abs().amax(1) / row_bound(want, dtype)).max() > 5
+        assert ((elsewhere - here).abs().amax(1) / row_bound(want, "float32")).max() > 50
 
 
 @pytest.mark.parametrize("backend", BACKENDS)
