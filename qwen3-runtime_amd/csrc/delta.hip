@@ -30,7 +30,7 @@ struct ConvArgs {
   const float* taps;        // [C, K], the last column multiplies the current token
   const float* tail;        // [slots, C, K-1]
   const int* cu_q; const int* seq_of_token; const int* state_slots;
-  float* out;               // [T, C] float32
+  void* out;                // [T, C], float32 or bfloat16 (out_code)
   int num_tokens, channels, num_taps, nseg;
   int seg_first[4], seg_heads[4], seg_width[4], seg_mode[4];
   int total_heads;
@@ -39,7 +39,13 @@ struct ConvArgs {
   // and no second kernel runs
   int fuse_tail;
   const float* bias;        // [C] or null: added to the convolution, before silu
+  int out_code;
 };
+
+__device__ __forceinline__ void conv_store(const ConvArgs& a, size_t i, float v) {
+  if (a.out_code == QRT_BF16) ((bf16_t*)a.out)[i] = (bf16_t)v;
+  else ((float*)a.out)[i] = v;
+}
 
 template <typename T>
 __global__ __launch_bounds__(256) void conv_unit_kernel(ConvArgs a) {
@@ -84,7 +90,7 @@ __global__ __launch_bounds__(256) void conv_unit_kernel(ConvArgs a) {
   }
 #pragma unroll
   for (int r = 0; r < 8; ++r)
-    if (lane + 64 * r < width) a.out[(size_t)t * a.channels + c0 + lane + 64 * r] = y[r] * mul;
+    if (lane + 64 * r < width) conv_store(a, (size_t)t * a.channels + c0 + lane + 64 * r, y[r] * mul);
 }
 
 // The same for steps of many tokens, K <= 4 taps and heads of at most 128 channels: a wave takes
@@ -158,7 +164,7 @@ __global__ __launch_bounds__(256) void conv_unit_tile_kernel(ConvArgs a) {
 #pragma unroll
       for (int r = 0; r < 2; ++r)
         if (lane + 64 * r < width)
-          a.out[(size_t)(t0 + tt) * a.channels + c0 + lane + 64 * r] = mode ? y[r][tt] * ss[tt] : y[r][tt];
+          conv_store(a, (size_t)(t0 + tt) * a.channels + c0 + lane + 64 * r, mode ? y[r][tt] * ss[tt] : y[r][tt]);
     }
   }
 }
@@ -203,6 +209,7 @@ __global__ void conv_tail_kernel(const T* __restrict__ x, long x_stride, float* 
 extern "C" int qrt_delta_conv(const ConvArgs* args, int dtype, int num_seqs, int num_slots, int max_span,
                               hipStream_t stream) {
   ConvArgs a = *args;
+  QRT_CHECK(a.out_code == QRT_F32 || a.out_code == QRT_BF16, "delta_conv: unknown output type %d", a.out_code);
   a.fuse_tail = max_span == 1 && a.num_tokens == num_seqs;
   QRT_CHECK(a.num_tokens >= 0 && a.channels > 0 && a.nseg >= 1 && a.nseg <= 4, "delta_conv: bad sizes");
   QRT_CHECK(a.num_taps >= 1 && a.num_taps <= DELTA_MAX_TAPS, "delta_conv: %d taps (1 to %d)", a.num_taps, DELTA_MAX_TAPS);

@@ -7,7 +7,8 @@
 //
 // A block per row. `wpg` waves share a group and `slots` groups are worked on at once, by neighbouring
 // waves, so that a group's sum of squares is a wave's sum (wpg = 1) or one exchange over a few floats
-// of LDS. A lane takes VEC neighbouring elements at a time and keeps KEEP such pieces in registers, all
+// of LDS. A lane takes VEC neighbouring elements at a time and keeps KEEP such pieces in registers (one in
+// steps of few rows, which spread a group over as many waves as it has pieces for), all
 // of them and the weights asked for before the first use; what a wider group has beyond them is read
 // a second time. The order of the additions is fixed by the row's shape and the launch alone.
 #include "common.h"
@@ -22,11 +23,21 @@ struct GroupSource {  // a matrix (float32 or bfloat16), or float32 planes whose
   const void* p; int code; int planes; long plane_stride;
 };
 
-template <int VEC>
+// PL: the number of planes where it is known when compiling (1: a matrix of either type), -1: any.
+template <int VEC, int PL>
 __device__ __forceinline__ typename VecOf<VEC>::f source_at(const GroupSource& y, size_t i) {
   typedef typename VecOf<VEC>::f fvec;
   typedef typename VecOf<VEC>::b bvec;
   fvec v;
+  if (PL > 1) {
+    fvec part[PL > 1 ? PL : 1];
+#pragma unroll
+    for (int k = 0; k < PL; ++k) part[k] = *(const fvec*)((const float*)y.p + (size_t)k * y.plane_stride + i);
+    v = part[0];
+#pragma unroll
+    for (int k = 1; k < PL; ++k) v += part[k];
+    return v;
+  }
   if (y.code == QRT_BF16) {
     const bvec b = *(const bvec*)((const bf16_t*)y.p + i);
 #pragma unroll
@@ -35,7 +46,7 @@ __device__ __forceinline__ typename VecOf<VEC>::f source_at(const GroupSource& y
   }
   const float* p = (const float*)y.p;
   v = *(const fvec*)(p + i);
-  if (y.planes == 1) return v;
+  if (PL == 1 || y.planes == 1) return v;
   // up to eight planes asked for together (one that is not there: the first again, dropped), added in order
   fvec part[7];
 #pragma unroll
@@ -78,12 +89,10 @@ __device__ __forceinline__ void store_vec(TO* p, const typename VecOf<VEC>::f& v
   *(ovec*)p = o;
 }
 
-#define GN_KEEP 4
-
 // r = rows ? rows[b] : b
 // x = residual[r] + (w_after ? y[r] / rms(y[r]) * w_after : y[r])   (y.p null: residual[r]); written back
 // without `rows`;  out[b] = weight ? x / rms(x) * weight : x
-template <typename TO, int VEC>
+template <typename TO, int VEC, int KEEP, int PL>
 __global__ __launch_bounds__(1024) void group_norm_update_kernel(float* __restrict__ residual, GroupSource y,
                                                                  const float* __restrict__ w_after, float eps_after,
                                                                  const float* __restrict__ weight, float eps,
@@ -99,12 +108,12 @@ __global__ __launch_bounds__(1024) void group_norm_update_kernel(float* __restri
   const fvec zero = {};
   for (int g = slot; g < groups; g += slots) {
     const int base = g * size;
-    fvec vx[GN_KEEP], vy[GN_KEEP], wa[GN_KEEP], wn[GN_KEEP];
+    fvec vx[KEEP], vy[KEEP], wa[KEEP], wn[KEEP];
 #pragma unroll
-    for (int j = 0; j < GN_KEEP; ++j) {
+    for (int j = 0; j < KEEP; ++j) {
       const int i = base + min(first + j * stride, size - VEC);  // beyond the group: some element of it, dropped below
       vx[j] = *(const fvec*)(residual + row + i);
-      vy[j] = y.p ? source_at<VEC>(y, row + i) : zero;
+      vy[j] = y.p ? source_at<VEC, PL>(y, row + i) : zero;
       wa[j] = w_after ? *(const fvec*)(w_after + i) : zero;
       wn[j] = weight ? *(const fvec*)(weight + i) : zero;
     }
@@ -112,9 +121,9 @@ __global__ __launch_bounds__(1024) void group_norm_update_kernel(float* __restri
     if (w_after) {
       float s = 0.f;
 #pragma unroll
-      for (int j = 0; j < GN_KEEP; ++j)
+      for (int j = 0; j < KEEP; ++j)
         if (first + j * stride < size) s += squares<VEC>(vy[j]);
-      for (int i = first + GN_KEEP * stride; i < size; i += stride) s += squares<VEC>(source_at<VEC>(y, row + base + i));
+      for (int i = first + KEEP * stride; i < size; i += stride) s += squares<VEC>(source_at<VEC, PL>(y, row + base + i));
       iy = 1.0f / sqrtf(group_sum(s, red, slot, wpg) / (float)size + eps_after);
     }
     auto joined = [&](const fvec& x, const fvec& d, const fvec& w) -> fvec {
@@ -124,7 +133,7 @@ __global__ __launch_bounds__(1024) void group_norm_update_kernel(float* __restri
     const bool write_back = y.p && !rows;
     float s = 0.f;
 #pragma unroll
-    for (int j = 0; j < GN_KEEP; ++j) {
+    for (int j = 0; j < KEEP; ++j) {
       vx[j] = joined(vx[j], vy[j], wa[j]);
       if (first + j * stride < size) {
         s += squares<VEC>(vx[j]);
@@ -132,8 +141,8 @@ __global__ __launch_bounds__(1024) void group_norm_update_kernel(float* __restri
         if (!weight) store_vec<VEC, TO>(out + orow + base + first + j * stride, vx[j]);
       }
     }
-    for (int i = base + first + GN_KEEP * stride; i < base + size; i += stride) {
-      const fvec x = joined(*(const fvec*)(residual + row + i), y.p ? source_at<VEC>(y, row + i) : zero,
+    for (int i = base + first + KEEP * stride; i < base + size; i += stride) {
+      const fvec x = joined(*(const fvec*)(residual + row + i), y.p ? source_at<VEC, PL>(y, row + i) : zero,
                             w_after ? *(const fvec*)(w_after + i) : zero);
       s += squares<VEC>(x);
       if (write_back) *(fvec*)(residual + row + i) = x;
@@ -142,12 +151,12 @@ __global__ __launch_bounds__(1024) void group_norm_update_kernel(float* __restri
     if (!weight) continue;
     const float ix = 1.0f / sqrtf(group_sum(s, red, slot, wpg) / (float)size + eps);
 #pragma unroll
-    for (int j = 0; j < GN_KEEP; ++j)
+    for (int j = 0; j < KEEP; ++j)
       if (first + j * stride < size) store_vec<VEC, TO>(out + orow + base + first + j * stride, vx[j] * ix * wn[j]);
-    for (int i = base + first + GN_KEEP * stride; i < base + size; i += stride) {
+    for (int i = base + first + KEEP * stride; i < base + size; i += stride) {
       fvec x = *(const fvec*)(residual + row + i);  // the sum already, where it was written back
       if (!write_back)
-        x = joined(x, y.p ? source_at<VEC>(y, row + i) : zero, w_after ? *(const fvec*)(w_after + i) : zero);
+        x = joined(x, y.p ? source_at<VEC, PL>(y, row + i) : zero, w_after ? *(const fvec*)(w_after + i) : zero);
       store_vec<VEC, TO>(out + orow + i, x * ix * *(const fvec*)(weight + i));
     }
   }
@@ -155,7 +164,7 @@ __global__ __launch_bounds__(1024) void group_norm_update_kernel(float* __restri
 
 // o [T, width] float32, gate rows `gate_stride` elements apart:
 // v = o * silu(gate);  out = v / rms(v, per group) * weight
-template <typename TG, typename TO, int VEC>
+template <typename TG, typename TO, int VEC, int KEEP>
 __global__ __launch_bounds__(1024) void gated_group_norm_kernel(const float* __restrict__ o, const TG* __restrict__ gate,
                                                                 long gate_stride, const float* __restrict__ weight, float eps,
                                                                 TO* __restrict__ out, int width, int groups, int wpg, int slots) {
@@ -179,10 +188,10 @@ __global__ __launch_bounds__(1024) void gated_group_norm_kernel(const float* __r
   };
   for (int g = slot; g < groups; g += slots) {
     const int base = g * size;
-    fvec v[GN_KEEP], w[GN_KEEP];
-    gvec z[GN_KEEP];
+    fvec v[KEEP], w[KEEP];
+    gvec z[KEEP];
 #pragma unroll
-    for (int j = 0; j < GN_KEEP; ++j) {
+    for (int j = 0; j < KEEP; ++j) {
       const int i = base + min(first + j * stride, size - VEC);
       v[j] = *(const fvec*)(orow + i);
       z[j] = *(const gvec*)(grow + i);
@@ -190,17 +199,17 @@ __global__ __launch_bounds__(1024) void gated_group_norm_kernel(const float* __r
     }
     float s = 0.f;
 #pragma unroll
-    for (int j = 0; j < GN_KEEP; ++j) {
+    for (int j = 0; j < KEEP; ++j) {
       v[j] = gated(v[j], z[j]);
       if (first + j * stride < size) s += squares<VEC>(v[j]);
     }
-    for (int i = base + first + GN_KEEP * stride; i < base + size; i += stride)
+    for (int i = base + first + KEEP * stride; i < base + size; i += stride)
       s += squares<VEC>(gated(*(const fvec*)(orow + i), *(const gvec*)(grow + i)));
     const float inv = 1.0f / sqrtf(group_sum(s, red, slot, wpg) / (float)size + eps);
 #pragma unroll
-    for (int j = 0; j < GN_KEEP; ++j)
+    for (int j = 0; j < KEEP; ++j)
       if (first + j * stride < size) store_vec<VEC, TO>(dst + base + first + j * stride, v[j] * inv * w[j]);
-    for (int i = base + first + GN_KEEP * stride; i < base + size; i += stride)
+    for (int i = base + first + KEEP * stride; i < base + size; i += stride)
       store_vec<VEC, TO>(dst + i, gated(*(const fvec*)(orow + i), *(const gvec*)(grow + i)) * inv * *(const fvec*)(weight + i));
   }
 }
@@ -216,11 +225,14 @@ static void group_launch_shape(int rows, int size, int groups, int vec, int* wpg
   const int most = 16 / groups;
   const int per_wave = 64 * vec;
   const int pieces = (size + per_wave - 1) / per_wave;   // waves for one piece a lane
-  const int enough = (pieces + GN_KEEP - 1) / GN_KEEP;   // waves that keep the group in registers
+  const int enough = (pieces + 3) / 4;                   // waves that keep the group in registers, four pieces a lane
   const int want = rows <= 256 ? pieces : enough;
   *wpg = want < 1 ? 1 : (want > most ? most : want);
   *slots = groups;
 }
+
+// pieces a lane keeps: one where that is all there is
+static int group_keep(int size, int wpg, int vec) { return size <= wpg * 64 * vec ? 1 : 4; }
 
 static bool lined_up(const void* p, size_t bytes) { return (uintptr_t)p % bytes == 0; }
 
@@ -239,10 +251,26 @@ extern "C" int qrt_group_norm_update(float* residual, const void* y, int y_code,
   int wpg, slots;
   group_launch_shape(num_out, size, groups, vec4 ? 4 : 1, &wpg, &slots);
   const dim3 grid(num_out), block(64 * wpg * slots);
-#define GO(TO, VEC) group_norm_update_kernel<TO, VEC><<<grid, block, 0, stream>>>(residual, src, w_after, eps_after, weight, eps, \
-                                                                                  rows, (TO*)out, hidden, groups, wpg, slots)
-  if (out_dtype == QRT_F32) { if (vec4) GO(float, 4); else GO(float, 1); }
-  else { if (vec4) GO(bf16_t, 4); else GO(bf16_t, 1); }
+  const int keep = group_keep(size, wpg, vec4 ? 4 : 1), pl = y ? y_planes : 1;
+#define GO(TO, VEC, KEEP, PL) group_norm_update_kernel<TO, VEC, KEEP, PL><<<grid, block, 0, stream>>>( \
+    residual, src, w_after, eps_after, weight, eps, rows, (TO*)out, hidden, groups, wpg, slots)
+#define PICK(TO)                              \
+  do {                                        \
+    if (!vec4) GO(TO, 1, 4, -1);              \
+    else if (keep == 4 && pl == 1) GO(TO, 4, 4, 1); \
+    else if (keep == 4) GO(TO, 4, 4, -1);     \
+    else if (pl == 1) GO(TO, 4, 1, 1);        \
+    else if (pl == 2) GO(TO, 4, 1, 2);        \
+    else if (pl == 3) GO(TO, 4, 1, 3);        \
+    else if (pl == 4) GO(TO, 4, 1, 4);        \
+    else if (pl == 5) GO(TO, 4, 1, 5);        \
+    else if (pl == 8) GO(TO, 4, 1, 8);        \
+    else if (pl == 9) GO(TO, 4, 1, 9);        \
+    else GO(TO, 4, 1, -1);                    \
+  } while (0)
+  if (out_dtype == QRT_F32) PICK(float);
+  else PICK(bf16_t);
+#undef PICK
 #undef GO
   QRT_LAUNCH_CHECK("group_norm_update");
   return 0;
@@ -263,9 +291,10 @@ extern "C" int qrt_gated_group_norm(const float* o, const void* gate, long gate_
   int wpg, slots;
   group_launch_shape(num_tokens, size, groups, vec4 ? 4 : 1, &wpg, &slots);
   const dim3 grid(num_tokens), block(64 * wpg * slots);
-#define GO(TG, TO, VEC) gated_group_norm_kernel<TG, TO, VEC><<<grid, block, 0, stream>>>(o, (const TG*)gate, gate_stride, weight, eps, \
-                                                                                        (TO*)out, width, groups, wpg, slots)
-#define PICK(TG, TO) do { if (vec4) GO(TG, TO, 4); else GO(TG, TO, 1); } while (0)
+  const int keep = group_keep(size, wpg, vec4 ? 4 : 1);
+#define GO(TG, TO, VEC, KEEP) gated_group_norm_kernel<TG, TO, VEC, KEEP><<<grid, block, 0, stream>>>( \
+    o, (const TG*)gate, gate_stride, weight, eps, (TO*)out, width, groups, wpg, slots)
+#define PICK(TG, TO) do { if (!vec4) GO(TG, TO, 1, 4); else if (keep == 4) GO(TG, TO, 4, 4); else GO(TG, TO, 4, 1); } while (0)
   if (gate_dtype == QRT_F32 && out_dtype == QRT_F32) PICK(float, float);
   else if (gate_dtype == QRT_BF16) PICK(bf16_t, bf16_t);
   else PICK(float, bf16_t);

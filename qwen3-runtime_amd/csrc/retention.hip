@@ -22,7 +22,8 @@
 #include <math.h>
 
 struct RetentionArgs {
-  const float* qkv; int channels, q_first, k_first, v_first;
+  const void* qkv;        // [T, channels] float32, or (STEP) bfloat16
+  int channels, q_first, k_first, v_first;
   const float* decay;     // [heads]
   float* state;           // [slots, heads, vdim, dim]
   float* out;             // [T, heads, vdim]
@@ -31,6 +32,8 @@ struct RetentionArgs {
   int share;              // heads that have one key and query in common (1: each its own)
   const void* step; long step_stride; int step_code;   // [T, heads] step logits, float32 or bfloat16; null: retention
   const float* step_bias; const float* a_log; const float* skip;  // [heads]
+  int qkv_code;
+  const int* seq_ids;     // the sequences of this launch; null: all of the step's
 };
 
 #define RT_COLS 16   // columns of the state per block
@@ -51,7 +54,7 @@ __device__ __forceinline__ float row16_sum(float x) {
 // G groups of four rows a lane: heads of up to 64 G key elements (padded with zero rows). RT_TILE
 // tokens a tile: 16 (8 for the widest heads: what fits 64 KB), or 4 for steps of single tokens,
 // whose blocks then are all resident at once with a quarter of the LDS and of the loads.
-template <int G, int RT_TILE, bool STEP>
+template <int G, int RT_TILE, bool STEP, typename TI>
 __global__ __launch_bounds__(256) void retention_kernel(RetentionArgs a) {
   constexpr int DP = 64 * G;                          // rows staged
   constexpr int NQK = 2 * RT_TILE * DP / 256;         // q and k elements a thread fetches per tile
@@ -60,10 +63,11 @@ __global__ __launch_bounds__(256) void retention_kernel(RetentionArgs a) {
   __shared__ float vs[RT_TILE * RT_COLS];
   __shared__ float os[RT_TILE * RT_COLS];
   __shared__ float ds[RT_TILE], steps[RT_TILE];  // a token's decay and step size (STEP)
-  const int seq = blockIdx.x, head = blockIdx.y, col0 = blockIdx.z * RT_COLS;
+  const int seq = a.seq_ids ? a.seq_ids[blockIdx.x] : blockIdx.x, head = blockIdx.y, col0 = blockIdx.z * RT_COLS;
   const int t0 = a.cu_q[seq], t1 = a.cu_q[seq + 1];
   if (t1 <= t0) return;
   const int dim = a.dim, vdim = a.vdim;
+  const TI* qkv = (const TI*)a.qkv;
   const int sub = threadIdx.x & 15, colg = threadIdx.x >> 4;  // lane within its column, column of the block
   const int col = col0 + colg;
   const bool col_ok = col < vdim;
@@ -93,15 +97,15 @@ __global__ __launch_bounds__(256) void retention_kernel(RetentionArgs a) {
       const int e = threadIdx.x + 256 * i;
       const int which = e / (RT_TILE * DP), tok = (e / DP) % RT_TILE, d = e % DP;
       const bool ok = tok < n && d < dim;
-      const float* row = a.qkv + (size_t)(base + min(tok, n - 1)) * a.channels + (which ? a.k_first : a.q_first) + qk_head * dim;
-      pre[i] = ok ? row[d] : 0.f;
+      const TI* row = qkv + (size_t)(base + min(tok, n - 1)) * a.channels + (which ? a.k_first : a.q_first) + qk_head * dim;
+      pre[i] = ok ? to_f32<TI>(row[d]) : 0.f;
     }
     const int tok = min((int)threadIdx.x / RT_COLS, RT_TILE - 1), c = threadIdx.x % RT_COLS;
     if (STEP && (int)threadIdx.x < n) {
       const size_t at = (size_t)(base + threadIdx.x) * a.step_stride + head;
       pre_step = a.step_code == QRT_F32 ? ((const float*)a.step)[at] : (float)((const bf16_t*)a.step)[at];
     }
-    pre_v = (tok < n && col0 + c < vdim) ? a.qkv[(size_t)(base + tok) * a.channels + a.v_first + head * vdim + col0 + c] : 0.f;
+    pre_v = (tok < n && col0 + c < vdim) ? to_f32<TI>(qkv[(size_t)(base + tok) * a.channels + a.v_first + head * vdim + col0 + c]) : 0.f;
   };
   fetch(t0);
   for (int base = t0; base < t1; base += RT_TILE) {
@@ -171,6 +175,7 @@ extern "C" int qrt_retention(const RetentionArgs* args, int num_tokens, int num_
   QRT_CHECK(num_tokens >= 0 && num_seqs >= 0 && num_slots > 0, "retention: bad counts");
   QRT_CHECK(a.heads > 0 && a.heads <= 65535 && a.dim > 0 && a.dim <= 512 && a.vdim > 0, "retention: %d heads of %d x %d", a.heads, a.dim, a.vdim);
   if (a.share == 0) a.share = 1;
+  QRT_CHECK(a.qkv_code == QRT_F32 || (a.qkv_code == QRT_BF16 && a.step), "retention: unknown input type %d", a.qkv_code);
   QRT_CHECK(a.share > 0 && a.heads % a.share == 0, "retention: %d heads, %d of which share a key", a.heads, a.share);
   QRT_CHECK(a.channels >= 2 * (a.heads / a.share) * a.dim + a.heads * a.vdim, "retention: %d channels hold no q, k and v", a.channels);
   QRT_CHECK(a.step ? a.step_bias && a.a_log && a.skip && a.step_stride >= a.heads : a.decay != nullptr,
@@ -180,8 +185,9 @@ extern "C" int qrt_retention(const RetentionArgs* args, int num_tokens, int num_
   const int groups = (a.dim + 63) / 64;
 #define GO(G, TILE)                                                                 \
   do {                                                                              \
-    if (a.step) retention_kernel<G, TILE, true><<<grid, 256, 0, stream>>>(a);       \
-    else retention_kernel<G, TILE, false><<<grid, 256, 0, stream>>>(a);             \
+    if (a.step && a.qkv_code == QRT_BF16) retention_kernel<G, TILE, true, bf16_t><<<grid, 256, 0, stream>>>(a); \
+    else if (a.step) retention_kernel<G, TILE, true, float><<<grid, 256, 0, stream>>>(a); \
+    else retention_kernel<G, TILE, false, float><<<grid, 256, 0, stream>>>(a);      \
   } while (0)
   if (num_tokens <= 2 * num_seqs) {  // decoded tokens, mostly
     if (groups <= 1) GO(1, 4);

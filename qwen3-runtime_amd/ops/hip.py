@@ -93,6 +93,7 @@ class _ConvArgs(Structure):
         ("num_tokens", c_int), ("channels", c_int), ("num_taps", c_int), ("nseg", c_int),
         ("seg_first", c_int * 4), ("seg_heads", c_int * 4), ("seg_width", c_int * 4), ("seg_mode", c_int * 4),
         ("total_heads", c_int), ("unit_eps", c_float), ("fuse_tail", c_int), ("bias", c_void_p),
+        ("out_code", c_int),
     ]
 
 
@@ -121,7 +122,16 @@ class _RetentionArgs(Structure):
         ("decay", c_void_p), ("state", c_void_p), ("out", c_void_p), ("cu_q", c_void_p), ("state_slots", c_void_p),
         ("heads", c_int), ("dim", c_int), ("vdim", c_int), ("share", c_int),
         ("step", c_void_p), ("step_stride", c_long), ("step_code", c_int),
-        ("step_bias", c_void_p), ("a_log", c_void_p), ("skip", c_void_p),
+        ("step_bias", c_void_p), ("a_log", c_void_p), ("skip", c_void_p), ("qkv_code", c_int), ("seq_ids", c_void_p),
+    ]
+
+
+class _SpaceArgs(Structure):
+    _fields_ = [
+        ("xbc", c_void_p), ("channels", c_int), ("step", c_void_p), ("step_stride", c_long), ("step_code", c_int),
+        ("step_bias", c_void_p), ("a_log", c_void_p), ("skip", c_void_p), ("state", c_void_p), ("out", c_void_p),
+        ("cu_q", c_void_p), ("state_slots", c_void_p), ("seq_ids", c_void_p),
+        ("heads", c_int), ("groups", c_int), ("n", c_int), ("p", c_int),
     ]
 
 
@@ -540,29 +550,63 @@ class HipOps:
     def state_space(self, ctx, xbc, step, step_bias, a_log, skip, state, heads, groups, n, vdim):
         """Per sequence and head from the slot's state (float32 [slots, heads, vdim, n], updated in place):
         ``D = softplus(step + step_bias); S <- exp(-exp(a_log) D) S + (D x) B^T; y = S C + skip x``. ``xbc``
-        float32 [T, heads * vdim | groups * n | groups * n] (x, B, C; head h uses group h // (heads /
-        groups)); ``step`` [T, heads] may be columns of a wider matrix. Returns y, float32 [T, heads, vdim]."""
+        [T, heads * vdim | groups * n | groups * n] (x, B, C; head h uses group h // (heads / groups)),
+        float32 or bfloat16; ``step`` [T, heads] may be columns of a wider matrix. Returns y, float32 [T, heads,
+        vdim]. Float32 inputs, short spans and odd sizes go token by token; long spans of bfloat16
+        inputs chunk by chunk, in a launch of their own beside the short ones of the same step."""
         t = ctx.num_tokens
         c = heads * vdim + 2 * groups * n
-        _need(xbc, "x | B | C", torch.float32, (t, c))
+        _need(xbc, "x | B | C", shape=(t, c))
         _need(state, "state", torch.float32, (state.shape[0], heads, vdim, n))
         if not step.is_cuda or tuple(step.shape) != (t, heads) or step.stride(1) != 1 or step.dtype not in _CODE:
             raise OpsError(f"step logits: {tuple(step.shape)} {step.dtype} with strides {step.stride()} for {t} tokens of {heads}")
         if heads % groups:
             raise OpsError(f"{heads} heads in {groups} groups")
-        a = _RetentionArgs()
-        a.qkv, a.channels = xbc.data_ptr(), c
-        a.v_first, a.k_first, a.q_first = 0, heads * vdim, heads * vdim + groups * n
-        a.step, a.step_stride, a.step_code = step.data_ptr(), step.stride(0), _CODE[step.dtype]
-        for name, w in (("step_bias", step_bias), ("a_log", a_log), ("skip", skip)):
-            setattr(a, name, _need(w, name, torch.float32, (heads,)).data_ptr())
+        consts = {name: _need(w, name, torch.float32, (heads,)).data_ptr()
+                  for name, w in (("step_bias", step_bias), ("a_log", a_log), ("skip", skip))}
+        cu_q = _need(ctx.cu_q, "cu_q", torch.int32, (ctx.num_seqs + 1,)).data_ptr()
+        slots = _need(ctx.state_slots, "state_slots", torch.int32, (ctx.num_seqs,)).data_ptr()
         out = torch.empty((t, heads, vdim), dtype=torch.float32, device=xbc.device)
-        a.state, a.out = state.data_ptr(), out.data_ptr()
-        a.cu_q = _need(ctx.cu_q, "cu_q", torch.int32, (ctx.num_seqs + 1,)).data_ptr()
-        a.state_slots = _need(ctx.state_slots, "state_slots", torch.int32, (ctx.num_seqs,)).data_ptr()
-        a.heads, a.dim, a.vdim, a.share = heads, n, vdim, heads // groups
-        self._check(self.lib, self.lib.qrt_retention(byref(a), c_int(t), c_int(ctx.num_seqs), c_int(state.shape[0]), _stream()))
+        chunked, short, num_chunked, short_tokens = self._space_split(ctx, xbc, n, vdim)
+        if num_chunked:
+            b = _SpaceArgs()
+            b.xbc, b.channels, b.step, b.step_stride, b.step_code = xbc.data_ptr(), c, step.data_ptr(), step.stride(0), _CODE[step.dtype]
+            b.state, b.out, b.cu_q, b.state_slots, b.seq_ids = state.data_ptr(), out.data_ptr(), cu_q, slots, _addr(chunked)
+            b.heads, b.groups, b.n, b.p = heads, groups, n, vdim
+            for name, ptr in consts.items():
+                setattr(b, name, ptr)
+            self._check(self.lib, self.lib.qrt_state_space_chunks(byref(b), c_int(num_chunked), _stream()))
+        if num_chunked < ctx.num_seqs:
+            a = _RetentionArgs()
+            a.qkv, a.qkv_code, a.channels = xbc.data_ptr(), _CODE[xbc.dtype], c
+            a.v_first, a.k_first, a.q_first = 0, heads * vdim, heads * vdim + groups * n
+            a.step, a.step_stride, a.step_code = step.data_ptr(), step.stride(0), _CODE[step.dtype]
+            for name, ptr in consts.items():
+                setattr(a, name, ptr)
+            a.state, a.out, a.cu_q, a.state_slots, a.seq_ids = state.data_ptr(), out.data_ptr(), cu_q, slots, _addr(short)
+            a.heads, a.dim, a.vdim, a.share = heads, n, vdim, heads // groups
+            self._check(self.lib, self.lib.qrt_retention(byref(a), c_int(short_tokens), c_int(ctx.num_seqs - num_chunked),
+                                                         c_int(state.shape[0]), _stream()))
         return out
+
+    # spans of at least this many tokens run chunk by chunk
+    space_chunk_min_tokens = 16
+
+    def _space_split(self, ctx, xbc, n, vdim):
+        """(ids of the sequences that run chunk by chunk or None for all, ids of the others or None for
+        all, how many of the first, tokens of the others): the same for every layer of the step."""
+        if xbc.dtype != torch.bfloat16 or n > 256 or n % 8 or vdim % 8 or ctx.max_q_len < self.space_chunk_min_tokens:
+            return None, None, 0, ctx.num_tokens
+        plan = ctx.scratch.get("space_split")
+        if plan is None:
+            is_long = [q >= self.space_chunk_min_tokens for q in ctx.q_lens_host]
+            if all(is_long):
+                plan = (None, None, ctx.num_seqs, 0)
+            else:
+                ids = lambda keep: torch.tensor([s for s, x in enumerate(is_long) if x == keep], dtype=torch.int32, device=xbc.device)  # noqa: E731
+                plan = (ids(True), ids(False), sum(is_long), sum(q for q, x in zip(ctx.q_lens_host, is_long) if not x))
+            ctx.scratch["space_split"] = plan
+        return plan
 
     # ---- steps between sub-layers that are neither a product nor a plain norm -----------
     def norm_mean(self, ya, wa, yb, wb, eps):
@@ -637,10 +681,10 @@ class HipOps:
         return x
 
     # ---- gated delta rule ---------------------------------------------------------------
-    def delta_conv(self, ctx, y, channels, taps, tail, segments, unit_eps, first=0, bias=None):
+    def delta_conv(self, ctx, y, channels, taps, tail, segments, unit_eps, first=0, bias=None, out_dtype=torch.float32):
         """``channels`` columns of ``y`` [T, W], from column ``first`` on, through their causal convolutions
         (``taps`` float32 [C, K]; ``bias`` float32 [C] or None is added) and silu, then per head as ``segments`` say, each (heads, width,
-        mode): 0 as it is, 1 scaled to a unit vector, 2 that times width^(-1/2). float32 [T, C].
+        mode): 0 as it is, 1 scaled to a unit vector, 2 that times width^(-1/2). [T, C] in ``out_dtype``.
         ``tail`` [slots, C, K-1] float32 holds each request's last inputs and is brought up to date."""
         t, w = y.shape
         _need(y, "projections")
@@ -657,7 +701,8 @@ class HipOps:
         a.cu_q = _need(ctx.cu_q, "cu_q", torch.int32, (ctx.num_seqs + 1,)).data_ptr()
         a.seq_of_token = _need(ctx.seq_of_token, "seq_of_token", torch.int32, (t,)).data_ptr()
         a.state_slots = _need(ctx.state_slots, "state_slots", torch.int32, (ctx.num_seqs,)).data_ptr()
-        out = torch.empty((t, channels), dtype=torch.float32, device=y.device)
+        out = torch.empty((t, channels), dtype=out_dtype, device=y.device)
+        a.out_code = _CODE[out_dtype]
         a.out, a.num_tokens, a.channels, a.num_taps, a.nseg, a.unit_eps = out.data_ptr(), t, channels, k, len(segments), unit_eps
         at = 0
         for i, (heads, width, mode) in enumerate(segments):

@@ -12,7 +12,8 @@ token, with ``step = softplus(dt + dt_bias)``::
 The heads' ``y`` are concatenated, multiplied by ``silu(z)``, RMS-normed in ``norm_groups`` equal parts
 (eps inside the root, one weight vector over all channels) and projected out. ``S`` starts at zero and
 is float32; it and the convolution's last ``taps - 1`` inputs are the request's state, kept in its slot
-from step to step. Step sizes, decays, recurrence and norm are float32 in every mode.
+from step to step. Step sizes, decays, recurrence and norm are float32 in every mode; the convolution's
+output is in the activations' type.
 """
 
 from __future__ import annotations
@@ -85,9 +86,10 @@ class StateSpace(Mixer):
         state, tail = cache
         inner = self.inner
         y = ops.linear(x, self.proj)  # z | x | B | C | dt, read where they lie
-        whole, rest = divmod(self.channels, 64)
-        segments = tuple(s for s in ((whole, 64, 0), (1, rest, 0)) if s[0] * s[1])
-        xbc = ops.delta_conv(ctx, y, self.channels, self.conv, tail.state, segments, 0.0, first=inner, bias=self.conv_bias)
+        whole, rest = divmod(self.channels, 128)  # what a wave of the convolution takes at a time
+        segments = tuple(s for s in ((whole, 128, 0), (1, rest, 0)) if s[0] * s[1])
+        xbc = ops.delta_conv(ctx, y, self.channels, self.conv, tail.state, segments, 0.0, first=inner, bias=self.conv_bias,
+                             out_dtype=ctx.dtype)
         step = y[:, inner + self.channels:]
         out = ops.state_space(ctx, xbc, step, self.dt_bias, self.a_log, self.skip, state.state, self.heads, self.groups,
                               self.state_dim, self.vdim)

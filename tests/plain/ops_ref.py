@@ -319,7 +319,7 @@ def bias_rotate_pairs(x, bias, positions, freq, rot_heads, head_dim):
     return x
 
 
-def delta_conv(y, channels, taps, tail, cu_q, slots, segments, unit_eps, first=0, bias=None):
+def delta_conv(y, channels, taps, tail, cu_q, slots, segments, unit_eps, first=0, bias=None, out_dtype=torch.float32):
     """Causal convolution (+ ``bias``) + silu + unit vectors per head, span by span, over the columns
     ``first .. first + channels``; ``tail`` updated in place."""
     y = y[:, first:]
@@ -345,7 +345,7 @@ def delta_conv(y, channels, taps, tail, cu_q, slots, segments, unit_eps, first=0
                 seg = seg * width ** -0.5
             out[:, first: first + heads * width] = seg.reshape(-1, heads * width)
         first += heads * width
-    return out
+    return out.to(out_dtype)
 
 
 def delta_rule(qkv, beta, a_logits, a_log, dt_bias, state, cu_q, slots, heads, kv_heads, dim, vdim, per_channel):
@@ -468,6 +468,7 @@ def state_space(xbc, step, dt_bias, a_log, skip, state, cu_q, slots, heads, grou
     """S <- exp(-exp(a_log) softplus(step + dt_bias)) S + (softplus(..) x) B^T; y = S C + skip x, per sequence and
     head from the slot's state [slots, heads, vdim, n]. ``xbc`` float32 [T, heads vdim | groups n | groups n]."""
     t = xbc.shape[0]
+    xbc = xbc.to(torch.float32)
     x = xbc[:, : heads * vdim].view(t, heads, vdim)
     b = xbc[:, heads * vdim: heads * vdim + groups * n].reshape(t, groups, n).repeat_interleave(heads // groups, dim=1)
     c = xbc[:, heads * vdim + groups * n:].reshape(t, groups, n).repeat_interleave(heads // groups, dim=1)
@@ -643,8 +644,8 @@ class TorchOps:
     def bias_rotate_pairs(self, x, bias, positions, freq, rot_heads, head_dim):
         return bias_rotate_pairs(x, bias, positions, freq, rot_heads, head_dim)
 
-    def delta_conv(self, ctx, y, channels, taps, tail, segments, unit_eps, first=0, bias=None):
-        return delta_conv(y, channels, taps, tail, ctx.cu_q, ctx.state_slots, segments, unit_eps, first, bias)
+    def delta_conv(self, ctx, y, channels, taps, tail, segments, unit_eps, first=0, bias=None, out_dtype=torch.float32):
+        return delta_conv(y, channels, taps, tail, ctx.cu_q, ctx.state_slots, segments, unit_eps, first, bias, out_dtype)
 
     def delta_rule(self, ctx, qkv, beta, a_logits, a_log, dt_bias, state, heads, kv_heads, dim, vdim, per_channel):
         return delta_rule(qkv, beta, a_logits, a_log, dt_bias, state, ctx.cu_q, ctx.state_slots, heads, kv_heads,

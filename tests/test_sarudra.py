@@ -128,7 +128,7 @@ def spans(device, lens, slots):
     for n in lens:
         cu.append(cu[-1] + n)
     return SimpleNamespace(num_tokens=cu[-1], num_seqs=len(lens), cu_q=i32(cu), state_slots=i32(slots), max_q_len=max(lens),
-                           seq_of_token=i32([s for s, n in enumerate(lens) for _ in range(n)]), q_lens_host=list(lens))
+                           seq_of_token=i32([s for s, n in enumerate(lens) for _ in range(n)]), q_lens_host=list(lens), scratch={})
 
 
 def recurrence_inputs(t, heads, groups, n, p, seed):
@@ -153,17 +153,19 @@ STATE_SIZES = [(6, 2, 16, 24), (4, 4, 32, 16), (3, 1, 40, 7), (2, 1, 128, 64), (
 def test_state_space_recurrence_against_the_rule_written_out(backend, heads, groups, n, p):
     """The recurrence alone: a whole span, portions down to one token with the state in its slot, a second
     sequence beside the first. Every head's step bias and rate differ, so heads mixed up would show, and
-    so would heads that read another group's vectors. Step logits reach from -10 to 25."""
+    so would heads that read another group's vectors. Step logits reach from -10 to 25. With bfloat16 inputs
+    long spans go chunk by chunk; the short spans of the same step go token by token beside them."""
     device, dtype = backend
     ops, dt = make_ops(device), DT[dtype]
     t = 40 if device == "cpu" else 330
     x, b, c, step, bias = recurrence_inputs(t, heads, groups, n, p, seed=heads + n)
+    x, b, c = (v.to(dt).float() for v in (x, b, c))
     step[3], step[9] = -10.0, 25.0
     step = step.to(dt)
     a_log, skip = rnd(heads, seed=20) - 2.0, 1 + rnd(heads, seed=21)
     want = plain_recurrence(x, b, c, step.float(), bias, a_log, skip)
-    rows = torch.cat([v.reshape(t, -1) for v in (x, b, c)], 1).to(device)
-    other = torch.cat([v.reshape(t, -1) for v in recurrence_inputs(t, heads, groups, n, p, seed=99)[:3]], 1).to(device)
+    rows = torch.cat([v.reshape(t, -1) for v in (x, b, c)], 1).to(dt).to(device)
+    other = torch.cat([v.reshape(t, -1) for v in recurrence_inputs(t, heads, groups, n, p, seed=99)[:3]], 1).to(dt).to(device)
     wide = torch.cat([rnd(t, 3).to(dt), step], 1).to(device)
     consts = tuple(v.to(device) for v in (bias, a_log, skip))
     for sizes in ((t,), (37, 2, 1, 1, 16, 5), (130, 3, 64), (64, 65))[: 2 if device == "cpu" else 4]:
@@ -171,10 +173,11 @@ def test_state_space_recurrence_against_the_rule_written_out(backend, heads, gro
         state[3] = state[1] = 0.0
         got = []
         for at, k in in_steps(t, sizes):
-            ctx = spans(device, [k, k], [1, 3])
-            both = torch.cat([other[at: at + k], rows[at: at + k]]).contiguous()
-            steps = torch.cat([wide[at: at + k], wide[at: at + k]])[:, 3:]
-            got.append(ops.state_space(ctx, both, steps, *consts, state, heads, groups, n, p).cpu()[k:])
+            m = 1 + at % min(k, 4) if len(sizes) > 2 else k   # beside a span of another length
+            ctx = spans(device, [m, k], [1, 3])
+            both = torch.cat([other[at: at + m], rows[at: at + k]]).contiguous()
+            steps = torch.cat([wide[at: at + m], wide[at: at + k]])[:, 3:]
+            got.append(ops.state_space(ctx, both, steps, *consts, state, heads, groups, n, p).cpu()[m:])
         scale = float(want.abs().max())
         torch.testing.assert_close(torch.cat(got).double(), want, atol=2e-5 * scale, rtol=1e-4)
         assert torch.isnan(state[0]).all() and torch.isnan(state[2]).all()  # other slots are left alone
@@ -187,20 +190,21 @@ def test_a_write_from_far_back_is_read_and_a_slot_taken_again_is_empty(backend, 
     across many portions, is read whole, less the decay since; a second head forgets fast and has nothing
     left. Zeroed as when a slot is taken again, the state gives the skip alone."""
     device, dtype = backend
-    ops = make_ops(device)
+    ops, dt = make_ops(device), DT[dtype]
     t, heads = 420, 2
     unit = lambda v: v / v.norm(dim=-1, keepdim=True)  # noqa: E731
     x, b = rnd(t, heads, p, seed=2), unit(rnd(t, 1, n, seed=3))
     direction = unit(rnd(n, seed=77))
     b = b - (b @ direction)[..., None] * direction
     b[5, 0], x[5] = direction, 9.0
+    b, x, direction = (v.to(dt).float() for v in (b, x, direction))
     c = torch.zeros(t, 1, n)
     c[-1, 0] = direction
     step, bias = torch.zeros(t, heads), torch.tensor([0.3, -0.2])
     a_log, skip = torch.tensor([-12.0, 0.0]), torch.tensor([0.5, 2.0])
     want = plain_recurrence(x, b, c, step, bias, a_log, skip)
-    assert (want[-1, 0] - 0.5 * x[-1, 0]).abs().min() > 5.0 and (want[-1, 1] - 2.0 * x[-1, 1]).abs().max() < 1e-4
-    rows = torch.cat([v.reshape(t, -1) for v in (x, b, c)], 1).to(device)
+    assert (want[-1, 0] - 0.5 * x[-1, 0]).abs().min() > 5.0 and (want[-1, 1] - 2.0 * x[-1, 1]).abs().max() < (1e-4 if dtype == "float32" else 0.1)
+    rows = torch.cat([v.reshape(t, -1) for v in (x, b, c)], 1).to(dt).to(device)
     consts = tuple(v.to(device) for v in (bias, a_log, skip))
     state = torch.zeros(2, heads, p, n, device=device)
     got = [ops.state_space(spans(device, [k], [1]), rows[at: at + k].contiguous(), step[:k].to(device), *consts, state, heads, 1, n, p).cpu()
