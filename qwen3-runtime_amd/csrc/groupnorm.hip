@@ -231,8 +231,11 @@ static void group_launch_shape(int rows, int size, int groups, int vec, int* wpg
   *slots = groups;
 }
 
-// pieces a lane keeps: one where that is all there is
-static int group_keep(int size, int wpg, int vec) { return size <= wpg * 64 * vec ? 1 : 4; }
+// pieces a lane keeps: one or two where that is all there is
+static int group_keep(int size, int wpg, int vec) {
+  const int wave_pieces = wpg * 64 * vec;
+  return size <= wave_pieces ? 1 : size <= 2 * wave_pieces ? 2 : 4;
+}
 
 static bool lined_up(const void* p, size_t bytes) { return (uintptr_t)p % bytes == 0; }
 
@@ -259,6 +262,9 @@ extern "C" int qrt_group_norm_update(float* residual, const void* y, int y_code,
     if (!vec4) GO(TO, 1, 4, -1);              \
     else if (keep == 4 && pl == 1) GO(TO, 4, 4, 1); \
     else if (keep == 4) GO(TO, 4, 4, -1);     \
+    else if (keep == 2 && pl == 1) GO(TO, 4, 2, 1); \
+    else if (keep == 2 && pl == 2) GO(TO, 4, 2, 2); \
+    else if (keep == 2) GO(TO, 4, 2, -1);     \
     else if (pl == 1) GO(TO, 4, 1, 1);        \
     else if (pl == 2) GO(TO, 4, 1, 2);        \
     else if (pl == 3) GO(TO, 4, 1, 3);        \
@@ -294,7 +300,7 @@ extern "C" int qrt_gated_group_norm(const float* o, const void* gate, long gate_
   const int keep = group_keep(size, wpg, vec4 ? 4 : 1);
 #define GO(TG, TO, VEC, KEEP) gated_group_norm_kernel<TG, TO, VEC, KEEP><<<grid, block, 0, stream>>>( \
     o, (const TG*)gate, gate_stride, weight, eps, (TO*)out, width, groups, wpg, slots)
-#define PICK(TG, TO) do { if (!vec4) GO(TG, TO, 1, 4); else if (keep == 4) GO(TG, TO, 4, 4); else GO(TG, TO, 4, 1); } while (0)
+#define PICK(TG, TO) do { if (!vec4) GO(TG, TO, 1, 4); else if (keep == 4) GO(TG, TO, 4, 4); else if (keep == 2) GO(TG, TO, 4, 2); else GO(TG, TO, 4, 1); } while (0)
   if (gate_dtype == QRT_F32 && out_dtype == QRT_F32) PICK(float, float);
   else if (gate_dtype == QRT_BF16) PICK(bf16_t, bf16_t);
   else PICK(float, bf16_t);

@@ -3,14 +3,15 @@
 //   D_t = softplus(step_t + bias), a_t = exp(-exp(a_log) D_t)
 //   S <- a_t S + D_t x_t B_t^T;   y_t = S C_t + skip x_t            (S [P, N] per sequence and head)
 //
-// With l_t = sum of log a over the chunk up to and including t, a chunk of 64 tokens is three products:
+// With l_t = sum of log a (base 2 in the code) over the chunk up to and including t, a chunk of 64 tokens is three products:
 //
 //   y_t  = sum_{s <= t} [ exp(l_t - l_s) D_s (C_t . B_s) + skip (s = t) ] x_s  +  exp(l_t) S_0 C_t
 //   S_64 = exp(l_63) S_0 + sum_s exp(l_63 - l_s) D_s x_s B_s^T
 //
 // x, B and C come in bfloat16 (the short convolution's output) and are exact as operands. What is
-// float32 (the bracket, the state as an operand, the weighted x of the state's update) enters as three
-// bfloat16 terms whose sum is the float32 value to 24 bits; sums are float32, and so are step sizes,
+// float32 enters as a sum of bfloat16 terms: the weighted x of the state's update as three, which hold
+// all 24 bits, so that the state is kept to float32; the bracket and the state as they are read out as two
+// (17 bits; a read-out is gated, normed and rounded to 8). Sums are float32, and so are step sizes,
 // logarithms of decays and exponentials. The exponents are differences l_t - l_s <= 0, so nothing
 // overflows however fast a head forgets. The recurrence written out token by token is in retention.hip;
 // the two differ by the rounding of float32 sums.
@@ -20,7 +21,8 @@
 // the accumulator tiles of the update (tile i: rows n = 16 i + 4 quad + r, column p = lane & 15), which
 // read in pairs are also the operand of the product with C (two runs of four neighbouring n a lane; C
 // is read from LDS in the same order). B is staged by rows for C . B and transposed for the update, x
-// transposed; a thread turns 8 x 8 pieces round in registers on the way into LDS. The next chunk's
+// transposed; for the transposed ones a thread turns 8 x 8 pieces round in registers on the way into LDS
+// (neighbouring threads take neighbouring tokens, so that they write neighbouring pieces of a row). The next chunk's
 // global loads are in flight while a chunk is computed. The bracket is computed once for the block,
 // 16 rows a wave, in the layout its product wants (the keys of two 16-row tiles permuted so that a lane
 // ends up with eight neighbouring s for its t), and shared through LDS.
@@ -40,25 +42,47 @@ struct SpaceArgs {
 };
 
 constexpr int CHUNK = 64;
-constexpr int TERMS = 3;
+constexpr int READ_TERMS = 2, WRITE_TERMS = 3;  // bfloat16 terms of a float32 value in a read-out, in the state's update
 constexpr int TROW = CHUNK + 16;   // elements of a transposed row in LDS: 32 bytes modulo 64
 
+// v as a sum of COUNT bfloat16 terms, the last one rounded, those before cut off (8 bits each: what is
+// left is exact, and three terms hold a float32's 24 bits). Two values' halves leave in one register.
+template <int COUNT>
 __device__ __forceinline__ void split_terms(const float* v, bf16x8_t* out) {
+  float r[8];
 #pragma unroll
-  for (int e = 0; e < 8; ++e) {
-    float r = v[e];
+  for (int e = 0; e < 8; ++e) r[e] = v[e];
 #pragma unroll
-    for (int k = 0; k < TERMS; ++k) {
-      const bf16_t t = (bf16_t)r;
-      out[k][e] = t;
-      r -= (float)t;
-    }
+  for (int k = 0; k < COUNT - 1; ++k) {
+    u32x4_t bits;
+#pragma unroll
+    for (int e = 0; e < 4; ++e)  // the upper halves of two neighbours
+      bits[e] = __builtin_amdgcn_perm(__float_as_uint(r[2 * e + 1]), __float_as_uint(r[2 * e]), 0x07060302u);
+    out[k] = __builtin_bit_cast(bf16x8_t, bits);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) r[e] -= __uint_as_float(__float_as_uint(r[e]) & 0xffff0000u);
   }
+#pragma unroll
+  for (int e = 0; e < 8; ++e) out[COUNT - 1][e] = (bf16_t)r[e];
+}
+
+// sum over the lanes up to and including this one (DPP: shifts within rows of 16, then the rows before)
+__device__ __forceinline__ float wave_running_sum(float x) {
+#define STEP_(ctrl, rows)                                                                                         \
+  x += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, x), ctrl, rows, 0xF, false))
+  STEP_(0x111, 0xF);  // row_shr 1, 2, 4, 8: a lane without a source adds 0
+  STEP_(0x112, 0xF);
+  STEP_(0x114, 0xF);
+  STEP_(0x118, 0xF);
+  STEP_(0x142, 0xA);  // row_bcast 15 into rows 1 and 3
+  STEP_(0x143, 0xC);  // row_bcast 31 into rows 2 and 3
+#undef STEP_
+  return x;
 }
 
 // KS steps of 32 state elements (N padded with zeros)
 template <int KS>
-__global__ __launch_bounds__(256) void state_space_chunk_kernel(SpaceArgs a) {
+__global__ __launch_bounds__(256, 1) void state_space_chunk_kernel(SpaceArgs a) {
   constexpr int NP = 32 * KS, BROW = NP + 16;
   constexpr int B_TASKS = 32 * KS, TASKS = B_TASKS + 64;     // 8 x 8 pieces of B and of x
   constexpr int R = (TASKS + 255) / 256;
@@ -67,9 +91,11 @@ __global__ __launch_bounds__(256) void state_space_chunk_kernel(SpaceArgs a) {
   bf16_t* crow = brow + CHUNK * BROW;      // [64][BROW]
   bf16_t* bt = crow + CHUNK * BROW;        // [NP][TROW]
   bf16_t* xt = bt + NP * TROW;             // [64][TROW]
-  bf16_t* pm = xt + CHUNK * TROW;          // [6][TERMS][64 lanes][8]
-  float* dts = (float*)(pm + 6 * TERMS * 512);  // [64] step sizes
-  float* acs = dts + CHUNK;                // [64] logarithms of the decay since the chunk's start
+  bf16_t* pm = xt + CHUNK * TROW;          // [6][READ_TERMS][64 lanes][8]
+  float* dts = (float*)(pm + 6 * READ_TERMS * 512);  // [64] step sizes
+  float* acs = dts + CHUNK;                // [64] base-2 logarithms of the decay since the chunk's start, the token's own included
+  float* since = acs + CHUNK;              // [64] 2^acs: what is left of the state before the chunk
+  float* left = since + CHUNK;             // [64] step size times what is left of the token's write at the chunk's end
 
   const int tid = threadIdx.x, lane = tid & 63, wave = uniform_wave_number();
   const int r16 = lane & 15, quad = lane >> 4;
@@ -79,7 +105,7 @@ __global__ __launch_bounds__(256) void state_space_chunk_kernel(SpaceArgs a) {
   if (t1 <= t0) return;
   const int N = a.n, P = a.p, group = head / (a.heads / a.groups);
   const int x_col = head * P + p0, b_col = a.heads * P + group * N, c_col = b_col + a.groups * N;
-  const float rate = expf(a.a_log[head]), bias = a.step_bias[head], skip = a.skip[head];
+  const float rate = expf(a.a_log[head]) * 1.4426950408889634f, bias = a.step_bias[head], skip = a.skip[head];
   const bool has_tile = p0 + 16 * wave < P;   // the same for the whole wave
   const int my_p = p0 + 16 * wave + r16;
   const bool p_ok = my_p < P;
@@ -92,34 +118,61 @@ __global__ __launch_bounds__(256) void state_space_chunk_kernel(SpaceArgs a) {
     S[i] = (p_ok && nn < N) ? *(const f32x4_t*)(st + nn) : (f32x4_t){0.f, 0.f, 0.f, 0.f};
   }
 
-  bf16x8_t pre[R][8], pre_c[KS];
+  bf16x8_t pre[R][8], pre_b[KS], pre_c[KS];
   float pre_step = 0.f;
+  const bool padded = N < NP || p0 + 64 > P;   // some pieces lie outside the state: zeros (the same for the block)
   // piece `task`: of B (tokens 8 sg .., channels 8 cg ..) or of x
   auto where = [&](int task, int& sg, int& cg, bool& is_b, bool& ok) {
     is_b = task < B_TASKS;
-    const int idx = is_b ? task : task - B_TASKS, per = is_b ? 4 * KS : 8;
-    sg = idx / per;
-    cg = idx - sg * per;
-    ok = is_b ? 8 * cg < N : p0 + 8 * cg < P;
+    const int idx = is_b ? task : task - B_TASKS;
+    sg = idx & 7;
+    cg = idx >> 3;
+    ok = !padded || (is_b ? 8 * cg < N : p0 + 8 * cg < P);
   };
+  // where a thread reads: element offsets from a chunk's first token, in a chunk of 64 whole tokens
+  int at_piece[R], at_row[KS];
+#pragma unroll
+  for (int r = 0; r < R; ++r) {
+    int sg, cg;
+    bool is_b, ok;
+    where(tid + 256 * r, sg, cg, is_b, ok);
+    at_piece[r] = 8 * sg * a.channels + (is_b ? b_col : x_col) + (ok ? 8 * cg : 0);
+  }
+#pragma unroll
+  for (int k = 0; k < KS; ++k) {
+    const int piece = tid + 256 * k, row = piece / (4 * KS), cg = piece - row * (4 * KS);
+    at_row[k] = row * a.channels + (8 * cg < N ? 8 * cg : 0);
+  }
   auto fetch = [&](int c0) {
+    const bf16_t* base = a.xbc + (size_t)c0 * a.channels;
+    if (c0 + CHUNK <= t1) {
 #pragma unroll
-    for (int r = 0; r < R; ++r) {
-      const int task = tid + 256 * r;
-      if (task < TASKS) {
-        int sg, cg;
-        bool is_b, ok;
-        where(task, sg, cg, is_b, ok);
-        const int col = (is_b ? b_col : x_col) + (ok ? 8 * cg : 0);
+      for (int r = 0; r < R; ++r)
+        if (tid + 256 * r < TASKS) {
 #pragma unroll
-        for (int j = 0; j < 8; ++j)  // tokens after the span's last: the last one again, weighed by zero below
-          pre[r][j] = *(const bf16x8_t*)(a.xbc + (size_t)min(c0 + 8 * sg + j, t1 - 1) * a.channels + col);
+          for (int j = 0; j < 8; ++j) pre[r][j] = *(const bf16x8_t*)(base + at_piece[r] + j * a.channels);
+        }
+#pragma unroll
+      for (int k = 0; k < KS; ++k) {
+        pre_b[k] = *(const bf16x8_t*)(base + at_row[k] + b_col);
+        pre_c[k] = *(const bf16x8_t*)(base + at_row[k] + c_col);
       }
-    }
+    } else {  // tokens after the span's last: the last one again, weighed by zero below
+      const int last = t1 - 1 - c0;
 #pragma unroll
-    for (int k = 0; k < KS; ++k) {
-      const int piece = tid + 256 * k, row = piece / (4 * KS), cg = piece - row * (4 * KS);
-      pre_c[k] = *(const bf16x8_t*)(a.xbc + (size_t)min(c0 + row, t1 - 1) * a.channels + c_col + (8 * cg < N ? 8 * cg : 0));
+      for (int r = 0; r < R; ++r)
+        if (tid + 256 * r < TASKS) {
+          const int sg = (tid + 256 * r < B_TASKS ? tid + 256 * r : tid + 256 * r - B_TASKS) & 7;
+#pragma unroll
+          for (int j = 0; j < 8; ++j)
+            pre[r][j] = *(const bf16x8_t*)(base + at_piece[r] + (min(8 * sg + j, last) - 8 * sg) * a.channels);
+        }
+#pragma unroll
+      for (int k = 0; k < KS; ++k) {
+        const int row = (tid + 256 * k) / (4 * KS), back = (min(row, last) - row) * a.channels;
+        pre_b[k] = *(const bf16x8_t*)(base + at_row[k] + back + b_col);
+        pre_c[k] = *(const bf16x8_t*)(base + at_row[k] + back + c_col);
+      }
     }
     if (tid < CHUNK) {
       const size_t at = (size_t)min(c0 + tid, t1 - 1) * a.step_stride + head;
@@ -136,10 +189,8 @@ __global__ __launch_bounds__(256) void state_space_chunk_kernel(SpaceArgs a) {
         bool is_b, ok;
         where(task, sg, cg, is_b, ok);
 #pragma unroll
-        for (int j = 0; j < 8; ++j) {
-          if (!ok) pre[r][j] = zero8;
-          if (is_b) *(bf16x8_t*)(brow + (8 * sg + j) * BROW + 8 * cg) = pre[r][j];
-        }
+        for (int j = 0; j < 8; ++j)
+          if (padded && !ok) pre[r][j] = zero8;
         bf16_t* dst = is_b ? bt : xt;
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
@@ -153,19 +204,21 @@ __global__ __launch_bounds__(256) void state_space_chunk_kernel(SpaceArgs a) {
 #pragma unroll
     for (int k = 0; k < KS; ++k) {
       const int piece = tid + 256 * k, row = piece / (4 * KS), cg = piece - row * (4 * KS);
-      *(bf16x8_t*)(crow + row * BROW + 8 * cg) = 8 * cg < N ? pre_c[k] : zero8;
+      if (padded && 8 * cg >= N) pre_b[k] = pre_c[k] = zero8;
+      // row 32 kb + 16 s2 + 4 q + r of `brow` is token 32 kb + 8 q + 4 s2 + r: the 16 lanes of an operand
+      // read 16 neighbouring rows
+      const int brow_at = (row & 32) + ((row & 4) << 2) + ((row & 24) >> 1) + (row & 3);
+      *(bf16x8_t*)(brow + brow_at * BROW + 8 * cg) = pre_b[k];
+      *(bf16x8_t*)(crow + row * BROW + 8 * cg) = pre_c[k];
     }
     if (wave == 0) {
       const float z = pre_step + bias;
       const float d = c0 + lane < t1 ? (z > 20.f ? z : log1pf(expf(z))) : 0.f;
-      float v = -rate * d;
-#pragma unroll
-      for (int o = 1; o < 64; o <<= 1) {
-        const float u = __shfl_up(v, o, 64);
-        if (lane >= o) v += u;
-      }
+      const float v = wave_running_sum(-rate * d);
       dts[lane] = d;
       acs[lane] = v;
+      since[lane] = __builtin_amdgcn_exp2f(v);
+      left[lane] = d * __builtin_amdgcn_exp2f(__int_as_float(__builtin_amdgcn_readlane(__float_as_int(v), 63)) - v);
     }
   };
 
@@ -179,87 +232,120 @@ __global__ __launch_bounds__(256) void state_space_chunk_kernel(SpaceArgs a) {
       const int t = 16 * wave + r16;
       const float lt = acs[t];
       for (int kb = 0; kb <= (wave >> 1); ++kb) {
-        f32x4_t sc[2];
+        // everything the rows need from LDS is asked for before the first product
+        bf16x8_t kk[2][KS], cc[KS];
+        f32x4_t ls[2], dd[2];
+#pragma unroll
+        for (int j = 0; j < KS; ++j) {
+          cc[j] = *(const bf16x8_t*)(crow + t * BROW + 32 * j + 8 * quad);
+#pragma unroll
+          for (int s2 = 0; s2 < 2; ++s2)
+            kk[s2][j] = *(const bf16x8_t*)(brow + (32 * kb + 16 * s2 + r16) * BROW + 32 * j + 8 * quad);
+        }
 #pragma unroll
         for (int s2 = 0; s2 < 2; ++s2) {
-          sc[s2] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
-          const int key = 32 * kb + 8 * (r16 >> 2) + 4 * s2 + (r16 & 3);
-#pragma unroll
-          for (int j = 0; j < KS; ++j)
-            sc[s2] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const bf16x8_t*)(brow + key * BROW + 32 * j + 8 * quad),
-                                                             *(const bf16x8_t*)(crow + t * BROW + 32 * j + 8 * quad), sc[s2], 0, 0, 0);
+          ls[s2] = *(const f32x4_t*)(acs + 32 * kb + 8 * quad + 4 * s2);
+          dd[s2] = *(const f32x4_t*)(dts + 32 * kb + 8 * quad + 4 * s2);
         }
+        f32x4_t sc[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+#pragma unroll
+        for (int j = 0; j < KS; ++j)
+#pragma unroll
+          for (int s2 = 0; s2 < 2; ++s2) sc[s2] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kk[s2][j], cc[j], sc[s2], 0, 0, 0);
         float m[8];
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
           const int s = 32 * kb + 8 * quad + e;
-          const float w = s <= t ? expf(lt - acs[s]) * dts[s] : 0.f;
-          m[e] = sc[e >> 2][e & 3] * w + (s == t ? skip : 0.f);
+          // keys after the row's token: the exponent is held at 0 (so that nothing overflows) and the weight is 0
+          const float w = __builtin_amdgcn_exp2f(fminf(lt - ls[e >> 2][e & 3], 0.f)) * dd[e >> 2][e & 3];
+          m[e] = sc[e >> 2][e & 3] * (s <= t ? w : 0.f) + (s == t ? skip : 0.f);
         }
-        bf16x8_t terms[TERMS];
-        split_terms(m, terms);
+        bf16x8_t terms[READ_TERMS];
+        split_terms<READ_TERMS>(m, terms);
         const int combo = wave < 2 ? wave : 2 * wave - 2 + kb;
 #pragma unroll
-        for (int k = 0; k < TERMS; ++k) *(bf16x8_t*)(pm + ((combo * TERMS + k) * 64 + lane) * 8) = terms[k];
+        for (int k = 0; k < READ_TERMS; ++k) *(bf16x8_t*)(pm + ((combo * READ_TERMS + k) * 64 + lane) * 8) = terms[k];
       }
     }
     __syncthreads();
     if (has_tile) {
-      bf16x8_t sterm[KS][TERMS], xa[2];
+      bf16x8_t sterm[KS][READ_TERMS], xa[2];
 #pragma unroll
       for (int j = 0; j < KS; ++j) {
         float v[8];
 #pragma unroll
         for (int e = 0; e < 8; ++e) v[e] = S[2 * j + (e >> 2)][e & 3];
-        split_terms(v, sterm[j]);
+        split_terms<READ_TERMS>(v, sterm[j]);
       }
 #pragma unroll
       for (int kb = 0; kb < 2; ++kb) xa[kb] = *(const bf16x8_t*)(xt + (16 * wave + r16) * TROW + 32 * kb + 8 * quad);
-#pragma unroll
-      for (int t4 = 0; t4 < 4; ++t4) {
-        f32x4_t own = {0.f, 0.f, 0.f, 0.f}, before[TERMS];
+      // the operands of a 16-row tile, asked for a tile ahead (where the registers allow it)
+      constexpr bool AHEAD = KS <= 4;
+      bf16x8_t pt[2][2 * READ_TERMS], ct[2][KS];
+      auto ask = [&](int t4) {
 #pragma unroll
         for (int kb = 0; kb <= (t4 >> 1); ++kb) {
           const int combo = t4 < 2 ? t4 : 2 * t4 - 2 + kb;
 #pragma unroll
-          for (int k = 0; k < TERMS; ++k)
-            own = __builtin_amdgcn_mfma_f32_16x16x32_bf16(xa[kb], *(const bf16x8_t*)(pm + ((combo * TERMS + k) * 64 + lane) * 8), own, 0, 0, 0);
+          for (int k = 0; k < READ_TERMS; ++k) pt[t4 & 1][kb * READ_TERMS + k] = *(const bf16x8_t*)(pm + ((combo * READ_TERMS + k) * 64 + lane) * 8);
         }
-#pragma unroll
-        for (int k = 0; k < TERMS; ++k) before[k] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int j = 0; j < KS; ++j) {
           const bf16_t* cp = crow + (16 * t4 + r16) * BROW + 32 * j + 4 * quad;
           const bf16x4_t lo = *(const bf16x4_t*)cp, hi = *(const bf16x4_t*)(cp + 16);
-          const bf16x8_t cb = __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7);
-#pragma unroll
-          for (int k = 0; k < TERMS; ++k) before[k] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sterm[j][k], cb, before[k], 0, 0, 0);
+          ct[t4 & 1][j] = __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7);
         }
+      };
+      f32x4_t lw[2][2];
+      float gone[4];
+#pragma unroll
+      for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+        for (int h = 0; h < 2; ++h) lw[kb][h] = *(const f32x4_t*)(left + 32 * kb + 8 * quad + 4 * h);
+#pragma unroll
+      for (int t4 = 0; t4 < 4; ++t4) gone[t4] = since[16 * t4 + r16];
+      const float whole = since[CHUNK - 1];
+      if (AHEAD) ask(0);
+#pragma unroll
+      for (int t4 = 0; t4 < 4; ++t4) {
+        if (!AHEAD) ask(t4);
+        else if (t4 < 3) ask(t4 + 1);
+        f32x4_t own = {0.f, 0.f, 0.f, 0.f}, before[READ_TERMS];
+#pragma unroll
+        for (int kb = 0; kb <= (t4 >> 1); ++kb)
+#pragma unroll
+          for (int k = 0; k < READ_TERMS; ++k) own = __builtin_amdgcn_mfma_f32_16x16x32_bf16(xa[kb], pt[t4 & 1][kb * READ_TERMS + k], own, 0, 0, 0);
+#pragma unroll
+        for (int k = 0; k < READ_TERMS; ++k) before[k] = (f32x4_t){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int j = 0; j < KS; ++j)
+#pragma unroll
+          for (int k = 0; k < READ_TERMS; ++k)
+            before[k] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(sterm[j][k], ct[t4 & 1][j], before[k], 0, 0, 0);
         const int tok = c0 + 16 * t4 + r16, p = p0 + 16 * wave + 4 * quad;
-        const float since = expf(acs[16 * t4 + r16]);
-        const f32x4_t y = own + since * (before[0] + (before[1] + before[2]));
+        const f32x4_t y = own + gone[t4] * (before[0] + before[1]);
         if (tok < t1 && p < P) *(f32x4_t*)(a.out + ((size_t)tok * a.heads + head) * P + p) = y;
       }
-      const float last = acs[CHUNK - 1], whole = expf(last);
+      bf16x8_t bn[2][2 * KS], xw[2][WRITE_TERMS];
 #pragma unroll
-      for (int i = 0; i < 2 * KS; ++i) S[i] *= whole;
+      for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+        for (int i = 0; i < 2 * KS; ++i) bn[kb][i] = *(const bf16x8_t*)(bt + (16 * i + r16) * TROW + 32 * kb + 8 * quad);
 #pragma unroll
       for (int kb = 0; kb < 2; ++kb) {
         float v[8];
 #pragma unroll
-        for (int e = 0; e < 8; ++e) {
-          const int s = 32 * kb + 8 * quad + e;
-          v[e] = (float)xa[kb][e] * (dts[s] * expf(last - acs[s]));
-        }
-        bf16x8_t xw[TERMS];
-        split_terms(v, xw);
-#pragma unroll
-        for (int i = 0; i < 2 * KS; ++i) {
-          const bf16x8_t bn = *(const bf16x8_t*)(bt + (16 * i + r16) * TROW + 32 * kb + 8 * quad);
-#pragma unroll
-          for (int k = 0; k < TERMS; ++k) S[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(bn, xw[k], S[i], 0, 0, 0);
-        }
+        for (int e = 0; e < 8; ++e) v[e] = (float)xa[kb][e] * lw[kb][e >> 2][e & 3];
+        split_terms<WRITE_TERMS>(v, xw[kb]);
       }
+#pragma unroll
+      for (int i = 0; i < 2 * KS; ++i) S[i] *= whole;
+#pragma unroll
+      for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+        for (int k = 0; k < WRITE_TERMS; ++k)
+#pragma unroll
+          for (int i = 0; i < 2 * KS; ++i) S[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(bn[kb][i], xw[kb][k], S[i], 0, 0, 0);
     }
     __syncthreads();  // the next chunk takes the same LDS
   }
@@ -275,7 +361,7 @@ __global__ __launch_bounds__(256) void state_space_chunk_kernel(SpaceArgs a) {
 template <int KS>
 static int space_launch(const SpaceArgs& a, int num_seqs, hipStream_t stream) {
   constexpr int NP = 32 * KS, BROW = NP + 16;
-  constexpr size_t smem = (size_t)(2 * CHUNK * BROW + NP * TROW + CHUNK * TROW + 6 * TERMS * 512) * sizeof(bf16_t) + 2 * CHUNK * sizeof(float);
+  constexpr size_t smem = (size_t)(2 * CHUNK * BROW + NP * TROW + CHUNK * TROW + 6 * READ_TERMS * 512) * sizeof(bf16_t) + 4 * CHUNK * sizeof(float);
   static_assert(smem <= 160 * 1024, "the chunk does not fit a compute unit's LDS");
   static bool allowed = smem <= 64 * 1024;  // once: not again inside every stream capture
   if (!allowed) {
