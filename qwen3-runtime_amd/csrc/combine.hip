@@ -1,8 +1,7 @@
 // Small float32 steps between sub-layers that are neither a product nor a plain norm:
 // the mean of several outputs each RMS-normed first (mixers side by side), the residual
 // stream joined with the embedding for a product that re-enters it (a looped span's entry),
-// a sum of two sub-layer outputs (routed and shared experts), and gated activations other than
-// SwiGLU. Inputs that are sub-layer outputs may be one matrix [T, H] (float32 or bfloat16) or
+// a sum of two sub-layer outputs (routed and shared experts). Inputs that are sub-layer outputs may be one matrix [T, H] (float32 or bfloat16) or
 // float32 planes [P, T, H] whose sum they are.
 #include "common.h"
 #include <math.h>
@@ -139,30 +138,6 @@ extern "C" int qrt_accumulate(float* acc, const void* y, int y_code, int y_plane
   return 0;
 }
 
-// out[t, i] = act(by * gu[t, i], by * gu[t, I + i]) for the gated activations of common.h; by = 1, or, with
-// `scale`, scale[order[t]] (order null: scale[t])
-template <typename T>
-__global__ void gated_act_kernel(const T* __restrict__ gu, T* __restrict__ out, int inter, int kind, float limit,
-                                 const float* __restrict__ scale, const int* __restrict__ order) {
-  const T* row = gu + (size_t)blockIdx.x * 2 * inter;
-  const float by = scale ? scale[order ? order[blockIdx.x] : blockIdx.x] : 1.0f;
-  for (int i = threadIdx.x; i < inter; i += blockDim.x)
-    out[(size_t)blockIdx.x * inter + i] =
-        from_f32<T>(gated_act(to_f32<T>(row[i]) * by, to_f32<T>(row[inter + i]) * by, kind, limit));
-}
-
-extern "C" int qrt_gated_act(const void* gu, void* out, int dtype, int num_tokens, int inter, int kind, float limit,
-                             const float* scale, const int* order, hipStream_t stream) {
-  QRT_CHECK(num_tokens >= 0 && inter > 0, "gated_act: bad sizes");
-  QRT_CHECK(kind == QRT_ACT_SWIGLU || kind == QRT_ACT_CLAMPED, "gated_act: unknown activation %d", kind);
-  if (num_tokens == 0) return 0;
-  if (dtype == QRT_F32) gated_act_kernel<float><<<dim3(num_tokens), 256, 0, stream>>>((const float*)gu, (float*)out, inter, kind, limit, scale, order);
-  else if (dtype == QRT_BF16) gated_act_kernel<bf16_t><<<dim3(num_tokens), 256, 0, stream>>>((const bf16_t*)gu, (bf16_t*)out, inter, kind, limit, scale, order);
-  else return qrt_fail("gated_act: unknown dtype %d", dtype);
-  QRT_LAUNCH_CHECK("gated_act");
-  return 0;
-}
-
 // ------------------------------------------------ a sub-layer output with a norm of its own
 // r = rows ? rows[b] : b
 // d = y[r] / rms(y[r]) * w_after;  x = residual[r] + d  (written back without `rows`);
@@ -242,7 +217,7 @@ extern "C" int qrt_norm_add_rmsnorm(float* residual, const void* y, int y_code, 
 }
 
 // ------------------------------------------------ a sum of scaled sub-layer outputs, then the norm
-// x = residual[r] + sum_i s_i * y_i[r]  (element by element; written back without `rows`);
+// x = residual[r] + sum_i s_i * y_i[r] (+ vector)  (element by element; written back without `rows`);
 // out[b] = x / rms(x) * w.  Everything float32. One block of 1,024 threads per row; a thread keeps
 // its elements in registers (rows up to 4,096 wide; the rest of a wider row is computed again),
 // all terms, vectors and weights asked for before the first is used. The terms are added in order.
@@ -251,11 +226,13 @@ struct ScaledTerms {
   Planes y[SA_TERMS];
   const float* scale[SA_TERMS];
   int count;
+  const float* vector;  // [H] or null: one more addend, the same for every row
 };
 
 template <int N>
 __device__ __forceinline__ float scaled_sum_at(const ScaledTerms& s, float x, size_t at, int i) {
-  float part[N], sc[N];
+  float part[N > 0 ? N : 1], sc[N > 0 ? N : 1];
+  const float v = s.vector ? s.vector[i] : 0.f;
 #pragma unroll
   for (int k = 0; k < N; ++k) {
     part[k] = planes_at(s.y[k], at);
@@ -263,7 +240,7 @@ __device__ __forceinline__ float scaled_sum_at(const ScaledTerms& s, float x, si
   }
 #pragma unroll
   for (int k = 0; k < N; ++k) x = fmaf(sc[k], part[k], x);
-  return x;
+  return x + v;
 }
 
 template <typename TO, int N>
@@ -311,13 +288,19 @@ __global__ __launch_bounds__(1024) void scaled_add_rmsnorm_kernel(float* __restr
 
 // y, y_code, y_planes, scale: `count` entries each; all planes [P, T, H] lie `plane_stride` elements apart
 extern "C" int qrt_scaled_add_rmsnorm(float* residual, const void* const* y, const int* y_code, const int* y_planes,
-                                      const float* const* scale, int count, long plane_stride, const float* weight,
-                                      float eps, const int* rows, void* out, int out_dtype, int num_out, int hidden,
+                                      const float* const* scale, int count, const float* vector, long plane_stride,
+                                      const float* weight, float eps, const int* rows, void* out, int out_dtype, int num_out, int hidden,
                                       hipStream_t stream) {
-  QRT_CHECK(num_out >= 0 && hidden > 0 && count >= 1 && count <= SA_TERMS, "scaled_add_rmsnorm: %d terms (1..%d)", count, SA_TERMS);
+  QRT_CHECK(num_out >= 0 && hidden > 0 && count >= (vector ? 0 : 1) && count <= SA_TERMS, "scaled_add_rmsnorm: %d terms (1..%d)", count, SA_TERMS);
   ScaledTerms s;
   s.count = count;
+  s.vector = vector;
   for (int k = 0; k < SA_TERMS; ++k) {
+    if (count == 0) {
+      s.y[k] = Planes{nullptr, QRT_F32, 1, 0};
+      s.scale[k] = nullptr;
+      continue;
+    }
     const int kk = k < count ? k : 0;
     QRT_CHECK(y[kk] && scale[kk] && y_planes[kk] >= 1, "scaled_add_rmsnorm: term %d is not there", kk);
     QRT_CHECK(y_code[kk] == QRT_F32 || (y_code[kk] == QRT_BF16 && y_planes[kk] == 1), "scaled_add_rmsnorm: planes are float32");
@@ -331,7 +314,8 @@ extern "C" int qrt_scaled_add_rmsnorm(float* residual, const void* const* y, con
     scaled_add_rmsnorm_kernel<float, N><<<num_out, 1024, 0, stream>>>(residual, s, weight, eps, rows, (float*)out, hidden);   \
   else                                                                                                                        \
     scaled_add_rmsnorm_kernel<bf16_t, N><<<num_out, 1024, 0, stream>>>(residual, s, weight, eps, rows, (bf16_t*)out, hidden)
-  if (count == 1) { SA_LAUNCH(1); }
+  if (count == 0) { SA_LAUNCH(0); }
+  else if (count == 1) { SA_LAUNCH(1); }
   else if (count == 2) { SA_LAUNCH(2); }
   else if (count == 3) { SA_LAUNCH(3); }
   else { SA_LAUNCH(4); }

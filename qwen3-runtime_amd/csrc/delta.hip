@@ -40,6 +40,7 @@ struct ConvArgs {
   int fuse_tail;
   const float* bias;        // [C] or null: added to the convolution, before silu
   int out_code;
+  int no_activation;        // 1: the convolution's sum as it is, no silu behind it
 };
 
 __device__ __forceinline__ void conv_store(const ConvArgs& a, size_t i, float v) {
@@ -78,7 +79,7 @@ __global__ __launch_bounds__(256) void conv_unit_kernel(ConvArgs a) {
         acc = fmaf(a.taps[(size_t)c * K + j], in, acc);
         if (a.fuse_tail && j >= 1) tail[(size_t)c * (K - 1) + (j - 1)] = in;  // i is 0: the inputs were tail[0..K-2], x
       }
-      y[r] = acc / (1.0f + expf(-acc));
+      y[r] = a.no_activation ? acc : acc / (1.0f + expf(-acc));
       ss += y[r] * y[r];
     }
   }
@@ -146,7 +147,7 @@ __global__ __launch_bounds__(256) void conv_unit_tile_kernel(ConvArgs a) {
         if (K - 1 - j > i) in = (lane + 64 * r < width) ? tail[(size_t)(c0 + lane + 64 * r) * (K - 1) + (i + j)] : 0.f;
         acc = fmaf(w[r][j], in, acc);
       }
-      y[r][tt] = acc / (1.0f + __expf(-acc));
+      y[r][tt] = a.no_activation ? acc : acc / (1.0f + __expf(-acc));
       ss[tt] += y[r][tt] * y[r][tt];
     }
   }

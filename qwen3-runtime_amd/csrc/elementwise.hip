@@ -31,6 +31,52 @@ extern "C" int qrt_embed(const int* ids, const void* table, int table_dtype, flo
   return 0;
 }
 
+// out[t, :] = float(table[ids[t], :]) + float(pairs[row, :]) with row = (previous token * mul_prev +
+// ids[t] * mul_cur) mod buckets, or row `buckets` at position 0. The token before a span's first one
+// stands in the request's slot (last [slots, 1]); the block of the span's first token, the only one that
+// reads it there, puts the span's last token in its place.
+template <typename TW, typename TP>
+__global__ void embed_pairs_kernel(const int* __restrict__ ids, const int* __restrict__ positions,
+                                   const int* __restrict__ seq_of_token, const int* __restrict__ cu_q,
+                                   const int* __restrict__ state_slots, const TW* __restrict__ table,
+                                   const TP* __restrict__ pairs, int* last, float* __restrict__ out,
+                                   int hidden, int buckets, long mul_prev, long mul_cur) {
+  const int t = blockIdx.x;
+  const int s = seq_of_token[t], first = cu_q[s];
+  const int cur = ids[t];
+  const int prev = t > first ? ids[t - 1] : last[state_slots[s]];
+  if (t == first) {  // the same for the whole block
+    __syncthreads();  // everyone has read the slot
+    if (threadIdx.x == 0) last[state_slots[s]] = ids[cu_q[s + 1] - 1];
+  }
+  long r = (prev * mul_prev + cur * mul_cur) % buckets;
+  if (r < 0) r += buckets;
+  if (positions[t] == 0) r = buckets;
+  const TW* row = table + (size_t)cur * hidden;
+  const TP* add = pairs + (size_t)r * hidden;
+  float* o = out + (size_t)t * hidden;
+  for (int i = threadIdx.x; i < hidden; i += blockDim.x) o[i] = to_f32<TW>(row[i]) + to_f32<TP>(add[i]);
+}
+
+extern "C" int qrt_embed_pairs(const int* ids, const int* positions, const int* seq_of_token, const int* cu_q,
+                               const int* state_slots, const void* table, int table_dtype, const void* pairs, int pairs_dtype,
+                               int* last, float* out, int num_tokens, int hidden, int buckets, long mul_prev, long mul_cur,
+                               hipStream_t stream) {
+  QRT_CHECK(num_tokens >= 0 && hidden > 0 && buckets > 0, "embed_pairs: bad sizes T=%d H=%d, %d rows", num_tokens, hidden, buckets);
+  if (num_tokens == 0) return 0;
+  const dim3 grid(num_tokens), block(256);
+#define GO(TW, TP) embed_pairs_kernel<TW, TP><<<grid, block, 0, stream>>>(ids, positions, seq_of_token, cu_q, state_slots, \
+                   (const TW*)table, (const TP*)pairs, last, out, hidden, buckets, mul_prev, mul_cur)
+  if (table_dtype == QRT_F32 && pairs_dtype == QRT_F32) GO(float, float);
+  else if (table_dtype == QRT_BF16 && pairs_dtype == QRT_BF16) GO(bf16_t, bf16_t);
+  else if (table_dtype == QRT_F32 && pairs_dtype == QRT_BF16) GO(float, bf16_t);
+  else if (table_dtype == QRT_BF16 && pairs_dtype == QRT_F32) GO(bf16_t, float);
+  else return qrt_fail("embed_pairs: unknown table dtypes %d %d", table_dtype, pairs_dtype);
+#undef GO
+  QRT_LAUNCH_CHECK("embed_pairs");
+  return 0;
+}
+
 // ------------------------------------------------ rotation table of a step
 // out[t, j] = cos(pos[t] * inv_freq[j]), out[t, half + j] = sin(...), j < half: the angles of a
 // step's tokens, float32. Every layer of a step rotates by the same angles, so a step that
@@ -215,13 +261,15 @@ extern "C" int qrt_add_rmsnorm(float* residual, const void* delta, int delta_dty
   return 0;
 }
 
-// ------------------------------------------------------------------ SwiGLU
-// out[t, i] = silu(gu[t, i]) * gu[t, I + i],  silu(x) = x / (1 + exp(-x)), in float32.
+// ------------------------------------------------------------------ gated activations
+// out[t, i] = act(gu[t, i], gu[t, I + i]) * row_scale[t] for the activations of common.h (SWIGLU:
+// silu(x) = x / (1 + exp(-x)) of the first times the second), in float32; row_scale null: 1.
 // VEC elements per thread and access: 8 for bfloat16 rows whose halves start on 16 bytes. With `scale`
 // both halves of row t are first multiplied by scale[order[t]] (order null: scale[t]).
-template <typename T, int VEC>
-__global__ __launch_bounds__(256) void swiglu_kernel(const T* __restrict__ gu, T* __restrict__ out, int inter,
-                                                     const float* __restrict__ scale, const int* __restrict__ order) {
+template <typename T, int VEC, int KIND>
+__global__ __launch_bounds__(256) void gated_act_kernel(const T* __restrict__ gu, T* __restrict__ out, int inter, float limit,
+                                                        const float* __restrict__ scale, const int* __restrict__ order,
+                                                        const float* __restrict__ row_scale) {
   typedef T vec_t __attribute__((ext_vector_type(VEC)));
   // a block per token: no division to find the row, and two loads of each half in flight per thread
   // (120 MB read and written for 2,048 tokens of the 4B shape in 23.6 us, 5.1 TB/s, as the
@@ -231,6 +279,7 @@ __global__ __launch_bounds__(256) void swiglu_kernel(const T* __restrict__ gu, T
   T* o_row = out + (size_t)blockIdx.x * inter;
   constexpr int U = 2;
   const float by = scale ? scale[order ? order[blockIdx.x] : blockIdx.x] : 1.0f;
+  const float times = row_scale ? row_scale[blockIdx.x] : 1.0f;
   for (int i0 = threadIdx.x * VEC; i0 < inter; i0 += U * 256 * VEC) {
     vec_t g[U], u[U];
 #pragma unroll
@@ -247,10 +296,8 @@ __global__ __launch_bounds__(256) void swiglu_kernel(const T* __restrict__ gu, T
       if (i < inter) {
         vec_t o;
 #pragma unroll
-        for (int e = 0; e < VEC; ++e) {
-          const float gf = to_f32<T>(g[k][e]) * by;
-          o[e] = from_f32<T>(gf / (1.0f + expf(-gf)) * (to_f32<T>(u[k][e]) * by));
-        }
+        for (int e = 0; e < VEC; ++e)
+          o[e] = from_f32<T>(gated_act(to_f32<T>(g[k][e]) * by, to_f32<T>(u[k][e]) * by, KIND, limit) * times);
         *(vec_t*)(o_row + i) = o;
       }
     }
@@ -258,26 +305,31 @@ __global__ __launch_bounds__(256) void swiglu_kernel(const T* __restrict__ gu, T
 }
 
 template <typename T, int VEC>
-static void swiglu_launch(const void* gate_up, void* out, int num_tokens, int inter, const float* scale, const int* order,
-                          hipStream_t stream) {
-  swiglu_kernel<T, VEC><<<dim3((unsigned)num_tokens), 256, 0, stream>>>((const T*)gate_up, (T*)out, inter, scale, order);
+static void gated_act_launch(const void* gate_up, void* out, int num_tokens, int inter, int kind, float limit, const float* scale,
+                             const int* order, const float* row_scale, hipStream_t stream) {
+  const dim3 grid((unsigned)num_tokens);
+  if (kind == QRT_ACT_SWIGLU)
+    gated_act_kernel<T, VEC, QRT_ACT_SWIGLU><<<grid, 256, 0, stream>>>((const T*)gate_up, (T*)out, inter, limit, scale, order, row_scale);
+  else
+    gated_act_kernel<T, VEC, QRT_ACT_CLAMPED><<<grid, 256, 0, stream>>>((const T*)gate_up, (T*)out, inter, limit, scale, order, row_scale);
 }
 
-extern "C" int qrt_swiglu(const void* gate_up, void* out, int dtype, int num_tokens, int inter, const float* scale,
-                          const int* order, hipStream_t stream) {
-  QRT_CHECK(num_tokens >= 0 && inter > 0, "swiglu: bad sizes T=%d I=%d", num_tokens, inter);
+extern "C" int qrt_gated_act(const void* gate_up, void* out, int dtype, int num_tokens, int inter, int kind, float limit,
+                             const float* scale, const int* order, const float* row_scale, hipStream_t stream) {
+  QRT_CHECK(num_tokens >= 0 && inter > 0, "gated_act: bad sizes T=%d I=%d", num_tokens, inter);
+  QRT_CHECK(kind == QRT_ACT_SWIGLU || kind == QRT_ACT_CLAMPED, "gated_act: unknown activation %d", kind);
   if ((size_t)num_tokens * inter == 0) return 0;
   const bool aligned = ((uintptr_t)gate_up % 16 == 0) && ((uintptr_t)out % 16 == 0);
   if (dtype == QRT_F32) {
-    if (aligned && inter % 4 == 0) swiglu_launch<float, 4>(gate_up, out, num_tokens, inter, scale, order, stream);
-    else swiglu_launch<float, 1>(gate_up, out, num_tokens, inter, scale, order, stream);
+    if (aligned && inter % 4 == 0) gated_act_launch<float, 4>(gate_up, out, num_tokens, inter, kind, limit, scale, order, row_scale, stream);
+    else gated_act_launch<float, 1>(gate_up, out, num_tokens, inter, kind, limit, scale, order, row_scale, stream);
   } else if (dtype == QRT_BF16) {
-    if (aligned && inter % 8 == 0) swiglu_launch<bf16_t, 8>(gate_up, out, num_tokens, inter, scale, order, stream);
-    else swiglu_launch<bf16_t, 1>(gate_up, out, num_tokens, inter, scale, order, stream);
+    if (aligned && inter % 8 == 0) gated_act_launch<bf16_t, 8>(gate_up, out, num_tokens, inter, kind, limit, scale, order, row_scale, stream);
+    else gated_act_launch<bf16_t, 1>(gate_up, out, num_tokens, inter, kind, limit, scale, order, row_scale, stream);
   } else {
-    return qrt_fail("swiglu: unknown dtype %d", dtype);
+    return qrt_fail("gated_act: unknown dtype %d", dtype);
   }
-  QRT_LAUNCH_CHECK("swiglu");
+  QRT_LAUNCH_CHECK("gated_act");
   return 0;
 }
 

@@ -27,6 +27,18 @@ __device__ __forceinline__ bf16x8_t load_k8(const bf16_t* __restrict__ row, int 
   return v;
 }
 
+// What the gated products do with a gate and an up value: an activation of common.h, times a factor per
+// row of the activations (null: 1).
+struct GatedEpilogue {
+  int kind;
+  float limit;
+  const float* row_scale;
+  __device__ __forceinline__ float apply(float g, float u, int m) const {
+    const float v = gated_act(g, u, kind, limit);
+    return row_scale ? v * row_scale[m] : v;
+  }
+};
+
 template <int MT, int NT, bool ALIGNED, typename TO>
 __global__ __launch_bounds__(256) void gemm_bf16_kernel(const bf16_t* __restrict__ A, const bf16_t* __restrict__ W,
                                                          TO* __restrict__ C, int M, int N, int K) {
@@ -108,7 +120,7 @@ __global__ __launch_bounds__(256) void gemm_bf16_kernel(const bf16_t* __restrict
 template <int MB, int NW, int NT, int U, bool GATED, typename TO>
 __global__ __launch_bounds__(64 * NW) void gemm_bf16_skinny_kernel(const bf16_t* __restrict__ A,
                                                                     const bf16_t* __restrict__ W,
-                                                                    TO* __restrict__ C, int M, int N, int K) {
+                                                                    TO* __restrict__ C, int M, int N, int K, GatedEpilogue ep) {
   constexpr int WT = GATED ? 2 * NT : NT;  // weight tiles per block
   extern __shared__ float red[];            // [NW][WT][MB][4][64]
   const int lane = threadIdx.x & 63, wave = uniform_wave_number();
@@ -192,7 +204,7 @@ __global__ __launch_bounds__(64 * NW) void gemm_bf16_skinny_kernel(const bf16_t*
         if (nn + r < N) {
           // the gate and the up value are rounded to bfloat16 first, as the unfused kernels see them
           const float g = (float)(bf16_t)sum[r];
-          const float out = GATED ? g / (1.0f + expf(-g)) * (float)(bf16_t)sum2[r] : sum[r];
+          const float out = GATED ? ep.apply(g, (float)(bf16_t)sum2[r], m) : sum[r];
           C[(size_t)m * N + nn + r] = from_f32<TO>(out);
         }
       }
@@ -201,14 +213,14 @@ __global__ __launch_bounds__(64 * NW) void gemm_bf16_skinny_kernel(const bf16_t*
 }
 
 template <int MB, int NW, int NT, int U, bool GATED>
-static int launch_skinny(const bf16_t* a, const bf16_t* w, void* c, int out_dtype, int M, int N, int K,
+static int launch_skinny(const bf16_t* a, const bf16_t* w, void* c, int out_dtype, int M, int N, int K, const GatedEpilogue& ep,
                          hipStream_t stream) {
   dim3 grid((N + 16 * NT - 1) / (16 * NT)), block(64 * NW);
   const size_t smem = (size_t)NW * (GATED ? 2 : 1) * NT * MB * 4 * 64 * sizeof(float);
   if (out_dtype == QRT_BF16)
-    gemm_bf16_skinny_kernel<MB, NW, NT, U, GATED, bf16_t><<<grid, block, smem, stream>>>(a, w, (bf16_t*)c, M, N, K);
+    gemm_bf16_skinny_kernel<MB, NW, NT, U, GATED, bf16_t><<<grid, block, smem, stream>>>(a, w, (bf16_t*)c, M, N, K, ep);
   else if (out_dtype == QRT_F32)
-    gemm_bf16_skinny_kernel<MB, NW, NT, U, GATED, float><<<grid, block, smem, stream>>>(a, w, (float*)c, M, N, K);
+    gemm_bf16_skinny_kernel<MB, NW, NT, U, GATED, float><<<grid, block, smem, stream>>>(a, w, (float*)c, M, N, K, ep);
   else
     return qrt_fail("gemm_bf16: unknown output dtype %d", out_dtype);
   QRT_LAUNCH_CHECK("gemm_bf16_skinny");
@@ -216,11 +228,11 @@ static int launch_skinny(const bf16_t* a, const bf16_t* w, void* c, int out_dtyp
 }
 
 template <bool GATED>
-static int skinny(const bf16_t* a, const bf16_t* w, void* c, int out_dtype, int M, int N, int K, hipStream_t st) {
+static int skinny(const bf16_t* a, const bf16_t* w, void* c, int out_dtype, int M, int N, int K, const GatedEpilogue& ep, hipStream_t st) {
   const int tiles = (N + 15) / 16;
-  if (tiles >= 2048) return launch_skinny<1, 8, 2, 8, GATED>(a, w, c, out_dtype, M, N, K, st);
-  if (tiles >= 512 || K < 4096) return launch_skinny<1, 8, 1, 8, GATED>(a, w, c, out_dtype, M, N, K, st);
-  return launch_skinny<1, 16, 1, 8, GATED>(a, w, c, out_dtype, M, N, K, st);
+  if (tiles >= 2048) return launch_skinny<1, 8, 2, 8, GATED>(a, w, c, out_dtype, M, N, K, ep, st);
+  if (tiles >= 512 || K < 4096) return launch_skinny<1, 8, 1, 8, GATED>(a, w, c, out_dtype, M, N, K, ep, st);
+  return launch_skinny<1, 16, 1, 8, GATED>(a, w, c, out_dtype, M, N, K, ep, st);
 }
 
 // ---------------------------------------------------------------- few rows, whole cache lines
@@ -257,7 +269,7 @@ typedef void __attribute__((address_space(3)))* lds_ptr_t;
 template <int NW, int NT, int U, bool GATED, typename TO>
 __global__ __launch_bounds__(64 * NW) void gemm_bf16_rows_kernel(const bf16_t* __restrict__ A,
                                                                   const bf16_t* __restrict__ W,
-                                                                  TO* __restrict__ C, int M, int N, int K) {
+                                                                  TO* __restrict__ C, int M, int N, int K, GatedEpilogue ep) {
   constexpr int WT = GATED ? 2 * NT : NT, UNITS = WT + 1, LOADS = 2 * UNITS, SLOT = UNITS * 2048;
   constexpr int ONCE = 2;  // the cache policy of a non-temporal load
   static_assert((U - 1) * LOADS < 64, "the loads' counter holds 63");
@@ -355,7 +367,7 @@ __global__ __launch_bounds__(64 * NW) void gemm_bf16_rows_kernel(const bf16_t* _
       for (int r = 0; r < 4; ++r) {
         if (nn + r < N) {
           const float g = (float)(bf16_t)sum[r];  // rounded to bfloat16 first, as the unfused kernels see them
-          const float out = GATED ? g / (1.0f + expf(-g)) * (float)(bf16_t)sum2[r] : sum[r];
+          const float out = GATED ? ep.apply(g, (float)(bf16_t)sum2[r], m) : sum[r];
           C[(size_t)m * N + nn + r] = from_f32<TO>(out);
         }
       }
@@ -364,7 +376,7 @@ __global__ __launch_bounds__(64 * NW) void gemm_bf16_rows_kernel(const bf16_t* _
 }
 
 template <int NW, int NT, int U, bool GATED>
-static int launch_rows(const bf16_t* a, const bf16_t* w, void* c, int out_dtype, int M, int N, int K,
+static int launch_rows(const bf16_t* a, const bf16_t* w, void* c, int out_dtype, int M, int N, int K, const GatedEpilogue& ep,
                        hipStream_t stream, int k_parts) {
   constexpr int WT = GATED ? 2 * NT : NT;
   dim3 grid((N + 16 * NT - 1) / (16 * NT), k_parts), block(64 * NW);
@@ -379,7 +391,7 @@ static int launch_rows(const bf16_t* a, const bf16_t* w, void* c, int out_dtype,
         return qrt_fail("gemm_bf16: cannot get %zu bytes of LDS", smem);                                \
       allowed = true;                                                                                   \
     }                                                                                                   \
-    kernel<<<grid, block, smem, stream>>>(a, w, (TO*)c, M, N, K);                                       \
+    kernel<<<grid, block, smem, stream>>>(a, w, (TO*)c, M, N, K, ep);                                   \
   } while (0)
   if (out_dtype == QRT_BF16) GO(bf16_t);
   else if (out_dtype == QRT_F32) GO(float);
@@ -397,22 +409,22 @@ static int launch_rows(const bf16_t* a, const bf16_t* w, void* c, int out_dtype,
 // two tiles then start in the same memory channels: 14.0 us against 11.2 for the 8B q/k/v product)
 // and for a few hundred tiles of long rows. K cut into planes: two tiles a block from K = 9,728 on.
 template <bool GATED>
-static int few_rows(const bf16_t* a, const bf16_t* w, void* c, int out_dtype, int M, int N, int K, hipStream_t st,
+static int few_rows(const bf16_t* a, const bf16_t* w, void* c, int out_dtype, int M, int N, int K, const GatedEpilogue& ep, hipStream_t st,
                     int k_parts) {
   const int tiles = (N + 15) / 16;
-  if (GATED) return launch_rows<4, 1, 3, GATED>(a, w, c, out_dtype, M, N, K, st, 1);
+  if (GATED) return launch_rows<4, 1, 3, GATED>(a, w, c, out_dtype, M, N, K, ep, st, 1);
   if (k_parts > 1) {
-    if (K >= 9728) return launch_rows<4, 2, 2, GATED>(a, w, c, out_dtype, M, N, K, st, k_parts);
-    return launch_rows<4, 1, 2, GATED>(a, w, c, out_dtype, M, N, K, st, k_parts);
+    if (K >= 9728) return launch_rows<4, 2, 2, GATED>(a, w, c, out_dtype, M, N, K, ep, st, k_parts);
+    return launch_rows<4, 1, 2, GATED>(a, w, c, out_dtype, M, N, K, ep, st, k_parts);
   }
   if (K % 2048 == 0) {
-    if (tiles >= 2048) return launch_rows<4, 1, 3, GATED>(a, w, c, out_dtype, M, N, K, st, 1);
-    return launch_rows<4, 1, 2, GATED>(a, w, c, out_dtype, M, N, K, st, 1);
+    if (tiles >= 2048) return launch_rows<4, 1, 3, GATED>(a, w, c, out_dtype, M, N, K, ep, st, 1);
+    return launch_rows<4, 1, 2, GATED>(a, w, c, out_dtype, M, N, K, ep, st, 1);
   }
-  if (tiles >= 2048) return launch_rows<4, 2, 3, GATED>(a, w, c, out_dtype, M, N, K, st, 1);
-  if (tiles >= 384 && K <= 4096) return launch_rows<4, 2, 2, GATED>(a, w, c, out_dtype, M, N, K, st, 1);
-  if (tiles >= 384) return launch_rows<4, 1, 4, GATED>(a, w, c, out_dtype, M, N, K, st, 1);
-  return launch_rows<4, 1, 2, GATED>(a, w, c, out_dtype, M, N, K, st, 1);
+  if (tiles >= 2048) return launch_rows<4, 2, 3, GATED>(a, w, c, out_dtype, M, N, K, ep, st, 1);
+  if (tiles >= 384 && K <= 4096) return launch_rows<4, 2, 2, GATED>(a, w, c, out_dtype, M, N, K, ep, st, 1);
+  if (tiles >= 384) return launch_rows<4, 1, 4, GATED>(a, w, c, out_dtype, M, N, K, ep, st, 1);
+  return launch_rows<4, 1, 2, GATED>(a, w, c, out_dtype, M, N, K, ep, st, 1);
 }
 
 __device__ __forceinline__ void store4(float* p, const float (&o)[4]) {
@@ -457,7 +469,7 @@ __device__ bf16x8_t qrt_zero_tile[64];
 template <int MB, int KW, int NWV, int NT, int KC, bool GATED, typename TO>
 __global__ __launch_bounds__(64 * KW * NWV) void gemm_bf16_mid_rows_kernel(const bf16_t* __restrict__ A,
                                                                             const bf16_t* __restrict__ W,
-                                                                            TO* __restrict__ C, int M, int N, int K) {
+                                                                            TO* __restrict__ C, int M, int N, int K, GatedEpilogue ep) {
   constexpr int WT = GATED ? 2 * NT : NT;  // weight tiles per wave
   constexpr int PAIRS = KC / 2;            // pairs of k-steps per chunk
   constexpr int ACT = KC * MB / NWV;       // loads of activations a wave issues per chunk
@@ -637,7 +649,7 @@ __global__ __launch_bounds__(64 * KW * NWV) void gemm_bf16_mid_rows_kernel(const
       for (int r = 0; r < 4; ++r) {
         if (GATED) {  // gate and up value rounded to bfloat16 first, as the unfused kernels see them
           const float g = (float)(bf16_t)acc[t][b][r];
-          o[r] = g / (1.0f + expf(-g)) * (float)(bf16_t)acc[NT + t][b][r];
+          o[r] = ep.apply(g, (float)(bf16_t)acc[NT + t][b][r], m);
         } else {
           o[r] = acc[t][b][r];
         }
@@ -648,7 +660,7 @@ __global__ __launch_bounds__(64 * KW * NWV) void gemm_bf16_mid_rows_kernel(const
 }
 
 template <int MB, int KW, int NWV, int NT, int KC, bool GATED>
-static int launch_mid_rows(const bf16_t* a, const bf16_t* w, void* c, int out_dtype, int M, int N, int K,
+static int launch_mid_rows(const bf16_t* a, const bf16_t* w, void* c, int out_dtype, int M, int N, int K, const GatedEpilogue& ep,
                            hipStream_t stream, int k_parts) {
   constexpr int WT = GATED ? 2 * NT : NT;
   const int per_block = NWV * NT, tiles = N / 16;
@@ -670,7 +682,7 @@ static int launch_mid_rows(const bf16_t* a, const bf16_t* w, void* c, int out_dt
         return qrt_fail("gemm_bf16: cannot get %zu bytes of LDS", smem);                                \
       allowed = true;                                                                                   \
     }                                                                                                   \
-    kernel<<<grid, block, smem, stream>>>(a, w, (TO*)c, M, N, K);                                       \
+    kernel<<<grid, block, smem, stream>>>(a, w, (TO*)c, M, N, K, ep);                                   \
   } while (0)
   if (out_dtype == QRT_BF16) GO(bf16_t);
   else if (out_dtype == QRT_F32) GO(float);
@@ -694,21 +706,21 @@ static int launch_mid_rows(const bf16_t* a, const bf16_t* w, void* c, int out_dt
 // block would have to fetch more activations than weights, and the vendor library is faster.
 // Very many tiles (the vocabulary head): eight tiles on the staged activations.
 template <int MB>
-static int mid_rows(const bf16_t* a, const bf16_t* w, void* c, int out_dtype, int M, int N, int K, int gated,
+static int mid_rows(const bf16_t* a, const bf16_t* w, void* c, int out_dtype, int M, int N, int K, const GatedEpilogue& ep, int gated,
                     hipStream_t st, int k_parts) {
-  if (gated) return launch_mid_rows<MB, 1, 3, 1, 6, true>(a, w, c, out_dtype, M, N, K, st, 1);
+  if (gated) return launch_mid_rows<MB, 1, 3, 1, 6, true>(a, w, c, out_dtype, M, N, K, ep, st, 1);
   if (k_parts > 1) {
     if constexpr (MB % 2 == 0) {
-      if (MB > 4 || K % 2048 == 0) return launch_mid_rows<MB, 1, 8, 1, 4, false>(a, w, c, out_dtype, M, N, K, st, k_parts);
+      if (MB > 4 || K % 2048 == 0) return launch_mid_rows<MB, 1, 8, 1, 4, false>(a, w, c, out_dtype, M, N, K, ep, st, k_parts);
     } else {
-      if (K % 2048 == 0) return launch_mid_rows<MB, 1, 4, 1, 4, false>(a, w, c, out_dtype, M, N, K, st, k_parts);
+      if (K % 2048 == 0) return launch_mid_rows<MB, 1, 4, 1, 4, false>(a, w, c, out_dtype, M, N, K, ep, st, k_parts);
     }
-    if constexpr (MB <= 4) return launch_mid_rows<MB, 1, 4, 2, 8, false>(a, w, c, out_dtype, M, N, K, st, k_parts);
+    if constexpr (MB <= 4) return launch_mid_rows<MB, 1, 4, 2, 8, false>(a, w, c, out_dtype, M, N, K, ep, st, k_parts);
   }
   if constexpr (MB <= 4) {
-    if (N >= 32768) return launch_mid_rows<MB, 1, 4, 2, 8, false>(a, w, c, out_dtype, M, N, K, st, 1);
-    if (K % 2048 == 0) return launch_mid_rows<MB, 3, 2, 1, 4, false>(a, w, c, out_dtype, M, N, K, st, 1);
-    return launch_mid_rows<MB, 2, 2, 1, 8, false>(a, w, c, out_dtype, M, N, K, st, 1);
+    if (N >= 32768) return launch_mid_rows<MB, 1, 4, 2, 8, false>(a, w, c, out_dtype, M, N, K, ep, st, 1);
+    if (K % 2048 == 0) return launch_mid_rows<MB, 3, 2, 1, 4, false>(a, w, c, out_dtype, M, N, K, ep, st, 1);
+    return launch_mid_rows<MB, 2, 2, 1, 8, false>(a, w, c, out_dtype, M, N, K, ep, st, 1);
   }
   return qrt_fail("gemm_bf16: above 64 rows only the gated form and products cut along K have a kernel of their own (M=%d)", M);
 }
@@ -735,8 +747,8 @@ static int launch(const bf16_t* a, const bf16_t* w, void* c, int out_dtype, int 
 // k_parts > 1 (not gated, float32 out; K % 64 == 0, and shared or M <= 16): K is cut into that
 // many parts, each handled by blocks of its own, and C is [k_parts, M, N]: planes to be added by
 // the caller.
-extern "C" int qrt_gemm_bf16(const void* a, const void* w, void* c, int out_dtype, int M, int N, int K, int gated,
-                             int shared, int k_parts, hipStream_t stream) {
+static int gemm(const void* a, const void* w, void* c, int out_dtype, int M, int N, int K, int gated, int shared, int k_parts,
+                const GatedEpilogue& ep, hipStream_t stream) {
   QRT_CHECK(M >= 0 && N > 0 && K > 0, "gemm_bf16: bad sizes M=%d N=%d K=%d", M, N, K);
   QRT_CHECK(gated == 0 || gated == 1, "gemm_bf16: unknown mode %d", gated);
   QRT_CHECK(shared == 0 || shared == 1, "gemm_bf16: unknown kernel choice %d", shared);
@@ -750,22 +762,34 @@ extern "C" int qrt_gemm_bf16(const void* a, const void* w, void* c, int out_dtyp
     QRT_CHECK(M <= 128 && N % 16 == 0 && N <= (1 << 20) && K % 64 == 0 && K >= 128 && aligned,
               "gemm_bf16: the LDS-sharing kernel needs M <= 128, N %% 16 == 0, N <= 2^20, K %% 64 == 0, K >= 128 "
               "(M=%d N=%d K=%d)", M, N, K);
-    if (M <= 16) return mid_rows<1>(A, W, c, out_dtype, M, N, K, gated, stream, k_parts);
-    if (M <= 32) return mid_rows<2>(A, W, c, out_dtype, M, N, K, gated, stream, k_parts);
-    if (M <= 48) return mid_rows<3>(A, W, c, out_dtype, M, N, K, gated, stream, k_parts);
-    if (M <= 64) return mid_rows<4>(A, W, c, out_dtype, M, N, K, gated, stream, k_parts);
-    if (M <= 96) return mid_rows<6>(A, W, c, out_dtype, M, N, K, gated, stream, k_parts);
-    return mid_rows<8>(A, W, c, out_dtype, M, N, K, gated, stream, k_parts);
+    if (M <= 16) return mid_rows<1>(A, W, c, out_dtype, M, N, K, ep, gated, stream, k_parts);
+    if (M <= 32) return mid_rows<2>(A, W, c, out_dtype, M, N, K, ep, gated, stream, k_parts);
+    if (M <= 48) return mid_rows<3>(A, W, c, out_dtype, M, N, K, ep, gated, stream, k_parts);
+    if (M <= 64) return mid_rows<4>(A, W, c, out_dtype, M, N, K, ep, gated, stream, k_parts);
+    if (M <= 96) return mid_rows<6>(A, W, c, out_dtype, M, N, K, ep, gated, stream, k_parts);
+    return mid_rows<8>(A, W, c, out_dtype, M, N, K, ep, gated, stream, k_parts);
   }
   if (M <= 16 && aligned && K % 64 == 0)  // through LDS by direct loads: whole cache lines
-    return gated ? few_rows<true>(A, W, c, out_dtype, M, N, K, stream, 1)
-                 : few_rows<false>(A, W, c, out_dtype, M, N, K, stream, k_parts);
+    return gated ? few_rows<true>(A, W, c, out_dtype, M, N, K, ep, stream, 1)
+                 : few_rows<false>(A, W, c, out_dtype, M, N, K, ep, stream, k_parts);
   QRT_CHECK(k_parts == 1, "gemm_bf16: K parts need M <= 16 or the LDS-sharing kernel, and K %% 64 == 0 (M=%d K=%d)", M, K);
-  if (M <= 16 && aligned) return gated ? skinny<true>(A, W, c, out_dtype, M, N, K, stream)
-                                       : skinny<false>(A, W, c, out_dtype, M, N, K, stream);
+  if (M <= 16 && aligned) return gated ? skinny<true>(A, W, c, out_dtype, M, N, K, ep, stream)
+                                       : skinny<false>(A, W, c, out_dtype, M, N, K, ep, stream);
   QRT_CHECK(gated == 0, "gemm_bf16: the gated form needs K a multiple of 32 and M <= 16, or the LDS-sharing kernel "
             "(M=%d K=%d)", M, K);
   if (M <= 16) return launch<1, 2>(A, W, c, out_dtype, M, N, K, stream);
   if (M <= 32) return launch<2, 2>(A, W, c, out_dtype, M, N, K, stream);
   return launch<4, 4>(A, W, c, out_dtype, M, N, K, stream);
+}
+
+extern "C" int qrt_gemm_bf16(const void* a, const void* w, void* c, int out_dtype, int M, int N, int K, int gated,
+                             int shared, int k_parts, hipStream_t stream) {
+  return gemm(a, w, c, out_dtype, M, N, K, gated, shared, k_parts, GatedEpilogue{QRT_ACT_SWIGLU, 0.f, nullptr}, stream);
+}
+
+// The gated product with any activation of common.h, row m of the result times row_scale[m] (null: 1).
+extern "C" int qrt_gated_gemm_bf16(const void* a, const void* w, void* c, int out_dtype, int M, int N, int K, int shared,
+                                   int act_kind, float limit, const float* row_scale, hipStream_t stream) {
+  QRT_CHECK(act_kind == QRT_ACT_SWIGLU || act_kind == QRT_ACT_CLAMPED, "gated_gemm_bf16: unknown activation %d", act_kind);
+  return gemm(a, w, c, out_dtype, M, N, K, 1, shared, 1, GatedEpilogue{act_kind, limit, row_scale}, stream);
 }

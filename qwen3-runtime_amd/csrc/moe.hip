@@ -62,13 +62,14 @@ __global__ __launch_bounds__(1024) void route_top_kernel(const T* __restrict__ x
                                                          float* __restrict__ weight, int hidden, int experts, int top,
                                                          int sigmoid_scores, int groups, int keep, int group_max,
                                                          const float* __restrict__ correction, int renormalise,
-                                                         float weight_scale) {
+                                                         float weight_scale, float* __restrict__ gate) {
   __shared__ float logit[MAX_EXPERTS];
   __shared__ float score[MAX_EXPERTS];
   const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const T* xr = x + (size_t)t * hidden;
   const bool wide = hidden % 4 == 0;
-  for (int e = wave; e < experts; e += 16) {
+  // with `gate` the router has one more row, no expert: the sigmoid of its product is the token's gate
+  for (int e = wave; e < experts + (gate ? 1 : 0); e += 16) {
     const float* wr = router + (size_t)e * hidden;
     float acc = 0.f;
     if (wide) {
@@ -84,7 +85,10 @@ __global__ __launch_bounds__(1024) void route_top_kernel(const T* __restrict__ x
       for (int c = lane; c < hidden; c += 64) acc = fmaf(to_f32<T>(xr[c]), wr[c], acc);
     }
     const float z = wave_sum(acc);
-    if (lane == 0) logit[e] = z + (bias ? bias[e] : 0.f);
+    if (lane == 0) {
+      if (e < experts) logit[e] = z + (bias ? bias[e] : 0.f);
+      else gate[t] = 1.0f / (1.0f + expf(-z));
+    }
   }
   __syncthreads();
   if (wave != 0) return;
@@ -172,7 +176,7 @@ __global__ __launch_bounds__(1024) void route_top_kernel(const T* __restrict__ x
 extern "C" int qrt_route_top(const void* x, int x_dtype, const float* router, const float* bias, int* index,
                              float* weight, int num_tokens, int hidden, int experts, int top, int sigmoid_scores,
                              int groups, int keep, int group_max, const float* correction, int renormalise,
-                             float weight_scale, hipStream_t stream) {
+                             float weight_scale, float* gate, hipStream_t stream) {
   QRT_CHECK(groups >= 1 && groups <= 64 && experts % groups == 0 && keep >= 1 && keep <= groups &&
             (long)keep * (experts / groups) >= top,
             "route_top: %d groups of which %d stay do not fit %d experts of which %d are chosen", groups, keep, experts, top);
@@ -184,9 +188,9 @@ extern "C" int qrt_route_top(const void* x, int x_dtype, const float* router, co
   if (num_tokens == 0) return 0;
   dim3 grid(num_tokens), block(1024);
   if (x_dtype == QRT_F32)
-    route_top_kernel<float><<<grid, block, 0, stream>>>((const float*)x, router, bias, index, weight, hidden, experts, top, sigmoid_scores, groups, keep, group_max, correction, renormalise, weight_scale);
+    route_top_kernel<float><<<grid, block, 0, stream>>>((const float*)x, router, bias, index, weight, hidden, experts, top, sigmoid_scores, groups, keep, group_max, correction, renormalise, weight_scale, gate);
   else if (x_dtype == QRT_BF16)
-    route_top_kernel<bf16_t><<<grid, block, 0, stream>>>((const bf16_t*)x, router, bias, index, weight, hidden, experts, top, sigmoid_scores, groups, keep, group_max, correction, renormalise, weight_scale);
+    route_top_kernel<bf16_t><<<grid, block, 0, stream>>>((const bf16_t*)x, router, bias, index, weight, hidden, experts, top, sigmoid_scores, groups, keep, group_max, correction, renormalise, weight_scale, gate);
   else return qrt_fail("route_top: unknown dtype %d", x_dtype);
   QRT_LAUNCH_CHECK("route_top");
   return 0;

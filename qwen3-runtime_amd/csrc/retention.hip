@@ -6,6 +6,9 @@
 // D = softplus(logit + bias), makes both the decay d = exp(-exp(a_log) D) and the written value v = D x,
 // the read-out has a skip, o = S^T q + skip x, and neighbouring heads share keys and queries (head h has
 // those of h / share).
+// Matrix memory (GATES): what a token keeps of the state and what its write weighs come per token and
+// head as logarithms, and the state has one more column, whose value is always 1: the sum of the weighted
+// keys, whose read-out goes to a place of its own.
 //
 // over each sequence's tokens of the step, from the state in the sequence's slot, which is left
 // there for the next step: [slots, heads, vdim, dim], a value channel's column of S contiguous.
@@ -34,7 +37,11 @@ struct RetentionArgs {
   const float* step_bias; const float* a_log; const float* skip;  // [heads]
   int qkv_code;
   const int* seq_ids;     // the sequences of this launch; null: all of the step's
+  const float* gates;     // [T, 3, heads] (GATES): log keep, log write (a third row is not read here)
+  float* last_out;        // [T, heads] (GATES): the read-out of the state's last column
 };
+
+constexpr int RT_CONSTANT = 0, RT_STEP = 1, RT_GATES = 2;  // where decays and writes come from
 
 #define RT_COLS 16   // columns of the state per block
 
@@ -54,27 +61,29 @@ __device__ __forceinline__ float row16_sum(float x) {
 // G groups of four rows a lane: heads of up to 64 G key elements (padded with zero rows). RT_TILE
 // tokens a tile: 16 (8 for the widest heads: what fits 64 KB), or 4 for steps of single tokens,
 // whose blocks then are all resident at once with a quarter of the LDS and of the loads.
-template <int G, int RT_TILE, bool STEP, typename TI>
+template <int G, int RT_TILE, int MODE, typename TI>
 __global__ __launch_bounds__(256) void retention_kernel(RetentionArgs a) {
+  constexpr bool STEP = MODE == RT_STEP, GATES = MODE == RT_GATES, PER_TOKEN = STEP || GATES;
   constexpr int DP = 64 * G;                          // rows staged
   constexpr int NQK = 2 * RT_TILE * DP / 256;         // q and k elements a thread fetches per tile
   __shared__ __attribute__((aligned(16))) float qs[RT_TILE * DP];
   __shared__ __attribute__((aligned(16))) float ks[RT_TILE * DP];
   __shared__ float vs[RT_TILE * RT_COLS];
   __shared__ float os[RT_TILE * RT_COLS];
-  __shared__ float ds[RT_TILE], steps[RT_TILE];  // a token's decay and step size (STEP)
+  __shared__ float ds[RT_TILE], steps[RT_TILE];  // a token's decay and what its value is multiplied by (PER_TOKEN)
   const int seq = a.seq_ids ? a.seq_ids[blockIdx.x] : blockIdx.x, head = blockIdx.y, col0 = blockIdx.z * RT_COLS;
   const int t0 = a.cu_q[seq], t1 = a.cu_q[seq + 1];
   if (t1 <= t0) return;
   const int dim = a.dim, vdim = a.vdim;
+  const int cols = GATES ? vdim + 1 : vdim;  // columns of the state
   const TI* qkv = (const TI*)a.qkv;
   const int sub = threadIdx.x & 15, colg = threadIdx.x >> 4;  // lane within its column, column of the block
   const int col = col0 + colg;
-  const bool col_ok = col < vdim;
-  const float decay = STEP ? 0.f : a.decay[head];
+  const bool col_ok = col < cols;
+  const float decay = PER_TOKEN ? 0.f : a.decay[head];
   const float rate = STEP ? expf(a.a_log[head]) : 0.f, bias = STEP ? a.step_bias[head] : 0.f, skip = STEP ? a.skip[head] : 0.f;
   const int qk_head = head / a.share;
-  float* st = a.state + (((size_t)a.state_slots[seq] * a.heads + head) * vdim + min(col, vdim - 1)) * dim;
+  float* st = a.state + (((size_t)a.state_slots[seq] * a.heads + head) * cols + min(col, cols - 1)) * dim;
   const bool vec = (dim & 3) == 0;  // a lane's four rows are 16 aligned bytes of the column
   float s[G][4];
 #pragma unroll
@@ -89,7 +98,7 @@ __global__ __launch_bounds__(256) void retention_kernel(RetentionArgs a) {
     }
   }
   // what this thread fetches of a tile: elements threadIdx.x + 256 i of q | k ([which][token][row]), one of v
-  float pre[NQK], pre_v, pre_step = 0.f;
+  float pre[NQK], pre_v, pre_step = 0.f, pre_write = 0.f;
   auto fetch = [&](int base) {
     const int n = min(RT_TILE, t1 - base);
 #pragma unroll
@@ -105,7 +114,12 @@ __global__ __launch_bounds__(256) void retention_kernel(RetentionArgs a) {
       const size_t at = (size_t)(base + threadIdx.x) * a.step_stride + head;
       pre_step = a.step_code == QRT_F32 ? ((const float*)a.step)[at] : (float)((const bf16_t*)a.step)[at];
     }
-    pre_v = (tok < n && col0 + c < vdim) ? to_f32<TI>(qkv[(size_t)(base + tok) * a.channels + a.v_first + head * vdim + col0 + c]) : 0.f;
+    if (GATES && (int)threadIdx.x < n) {
+      const float* row = a.gates + (size_t)(base + threadIdx.x) * 3 * a.heads + head;
+      pre_step = row[0];
+      pre_write = row[a.heads];
+    }
+    pre_v = GATES && col0 + c == vdim ? 1.f : (tok < n && col0 + c < vdim) ? to_f32<TI>(qkv[(size_t)(base + tok) * a.channels + a.v_first + head * vdim + col0 + c]) : 0.f;
   };
   fetch(t0);
   for (int base = t0; base < t1; base += RT_TILE) {
@@ -124,11 +138,15 @@ __global__ __launch_bounds__(256) void retention_kernel(RetentionArgs a) {
       steps[threadIdx.x] = sp;
       ds[threadIdx.x] = expf(-rate * sp);
     }
+    if (GATES && threadIdx.x < RT_TILE) {
+      ds[threadIdx.x] = expf(pre_step);
+      steps[threadIdx.x] = expf(pre_write);
+    }
     __syncthreads();
     if (base + RT_TILE < t1) fetch(base + RT_TILE);  // on its way during the walk
     auto token = [&](int i) {
       const float x = vs[i * RT_COLS + colg];
-      const float d = STEP ? ds[i] : decay, v = STEP ? x * steps[i] : x;
+      const float d = PER_TOKEN ? ds[i] : decay, v = PER_TOKEN ? x * steps[i] : x;
       float acc = 0.f;
 #pragma unroll
       for (int g = 0; g < G; ++g) {
@@ -153,6 +171,7 @@ __global__ __launch_bounds__(256) void retention_kernel(RetentionArgs a) {
     {  // the tile's read-outs: thread (token, column)
       const int tok = threadIdx.x / RT_COLS, c = threadIdx.x % RT_COLS;
       if (tok < n && tok < RT_TILE && col0 + c < vdim) a.out[((size_t)(base + tok) * a.heads + head) * vdim + col0 + c] = os[threadIdx.x];
+      if (GATES && tok < n && tok < RT_TILE && col0 + c == vdim) a.last_out[(size_t)(base + tok) * a.heads + head] = os[threadIdx.x];
     }
   }
   if (col_ok) {
@@ -175,19 +194,22 @@ extern "C" int qrt_retention(const RetentionArgs* args, int num_tokens, int num_
   QRT_CHECK(num_tokens >= 0 && num_seqs >= 0 && num_slots > 0, "retention: bad counts");
   QRT_CHECK(a.heads > 0 && a.heads <= 65535 && a.dim > 0 && a.dim <= 512 && a.vdim > 0, "retention: %d heads of %d x %d", a.heads, a.dim, a.vdim);
   if (a.share == 0) a.share = 1;
-  QRT_CHECK(a.qkv_code == QRT_F32 || (a.qkv_code == QRT_BF16 && a.step), "retention: unknown input type %d", a.qkv_code);
+  QRT_CHECK(a.qkv_code == QRT_F32 || (a.qkv_code == QRT_BF16 && (a.step || a.gates)), "retention: unknown input type %d", a.qkv_code);
   QRT_CHECK(a.share > 0 && a.heads % a.share == 0, "retention: %d heads, %d of which share a key", a.heads, a.share);
   QRT_CHECK(a.channels >= 2 * (a.heads / a.share) * a.dim + a.heads * a.vdim, "retention: %d channels hold no q, k and v", a.channels);
-  QRT_CHECK(a.step ? a.step_bias && a.a_log && a.skip && a.step_stride >= a.heads : a.decay != nullptr,
+  QRT_CHECK(!a.gates || (a.last_out && !a.step), "retention: gates without a place for the last column's read-out, or beside step logits");
+  QRT_CHECK(a.gates ? true : a.step ? a.step_bias && a.a_log && a.skip && a.step_stride >= a.heads : a.decay != nullptr,
             "retention: neither constant decays nor step logits with their bias, rate and skip");
   if (num_tokens == 0 || num_seqs == 0) return 0;
-  const dim3 grid(num_seqs, a.heads, (a.vdim + RT_COLS - 1) / RT_COLS);
+  const dim3 grid(num_seqs, a.heads, (a.vdim + (a.gates ? 1 : 0) + RT_COLS - 1) / RT_COLS);
   const int groups = (a.dim + 63) / 64;
 #define GO(G, TILE)                                                                 \
   do {                                                                              \
-    if (a.step && a.qkv_code == QRT_BF16) retention_kernel<G, TILE, true, bf16_t><<<grid, 256, 0, stream>>>(a); \
-    else if (a.step) retention_kernel<G, TILE, true, float><<<grid, 256, 0, stream>>>(a); \
-    else retention_kernel<G, TILE, false, float><<<grid, 256, 0, stream>>>(a);      \
+    if (a.gates && a.qkv_code == QRT_BF16) retention_kernel<G, TILE, RT_GATES, bf16_t><<<grid, 256, 0, stream>>>(a); \
+    else if (a.gates) retention_kernel<G, TILE, RT_GATES, float><<<grid, 256, 0, stream>>>(a); \
+    else if (a.step && a.qkv_code == QRT_BF16) retention_kernel<G, TILE, RT_STEP, bf16_t><<<grid, 256, 0, stream>>>(a); \
+    else if (a.step) retention_kernel<G, TILE, RT_STEP, float><<<grid, 256, 0, stream>>>(a); \
+    else retention_kernel<G, TILE, RT_CONSTANT, float><<<grid, 256, 0, stream>>>(a);      \
   } while (0)
   if (num_tokens <= 2 * num_seqs) {  // decoded tokens, mostly
     if (groups <= 1) GO(1, 4);

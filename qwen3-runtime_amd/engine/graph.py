@@ -218,7 +218,7 @@ class DecodeGraph:
                 # now, to choose the length of its pieces by
                 if self.unequal:
                     self.ctx.scratch["attn_lens"] = [runner.cache.length(e.request_id) + 1 for e in entries]
-                self.cache_views = runner.cache.step_views(runner.model.plan.order, self.ctx.groups)
+                self.cache_views, self.embedding_views = runner._cache_views(self.ctx.groups)
             dev = self.views_dev
             runner.last_row_slots = dev["row_slots"]
             self.runs += 1
@@ -226,7 +226,7 @@ class DecodeGraph:
                 if self.runs < 2:
                     # the first call at this size runs eagerly: it fills the attention work list
                     # and warms the allocator; the capture happens on the second call
-                    return runner.model.forward(self.ctx, dev["ids"], self.cache_views, dev["rows"])
+                    return runner.model.forward(self.ctx, dev["ids"], self.cache_views, dev["rows"], self.embedding_views)
                 graph = torch.cuda.CUDAGraph()
                 torch.cuda.synchronize(runner.device)
                 # all graphs of a runner take their buffers from one pool: only one of them runs
@@ -244,7 +244,7 @@ class DecodeGraph:
                 gc.disable()
                 try:
                     with torch.cuda.graph(graph, pool=runner._graph_pool):
-                        self.logits = runner.model.forward(self.ctx, dev["ids"], self.cache_views, dev["rows"])
+                        self.logits = runner.model.forward(self.ctx, dev["ids"], self.cache_views, dev["rows"], self.embedding_views)
                 finally:
                     if collecting:
                         gc.enable()

@@ -158,10 +158,15 @@ class ModelRunner:
 
     def _forward(self, packed: PackedStep, dev: dict[str, torch.Tensor]):
         ctx = self._context(packed, dev)
-        views = self.cache.step_views(self.model.plan.order, ctx.groups)
+        views, own = self._cache_views(ctx.groups)
         rows = dev["rows"] if packed.num_rows else None
         with torch.inference_mode():
-            return self.model.forward(ctx, dev["ids"], views, rows)
+            return self.model.forward(ctx, dev["ids"], views, rows, own)
+
+    def _cache_views(self, groups):
+        """What the steps of the model's order see of their caches, and what its embedding sees of its own."""
+        plan = self.model.plan
+        return self.cache.step_views(plan.order, groups), tuple(self.cache.view(c, groups) for c in plan.embedding_cache)
 
     # ---- graph path ----------------------------------------------------------
     def _step_graph(self, entries: Sequence[StepEntry]):

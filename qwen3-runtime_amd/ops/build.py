@@ -36,7 +36,7 @@ FLAGS = [
 FLAGS += os.environ.get("QWEN3_RUNTIME_AMD_HIPCC_FLAGS", "").split()
 CORE_SOURCES = ["runtime.hip", "elementwise.hip", "gemm_f32.hip", "gemm_bf16.hip", "attention_f32.hip", "sampling.hip",
                 "streams.hip", "moe.hip", "delta.hip", "combine.hip", "rotary.hip", "latent.hip", "retention.hip", "jointnorm.hip", "groupnorm.hip",
-                "statespace.hip"]
+                "statespace.hip", "memory.hip"]
 
 
 class BuildError(RuntimeError):

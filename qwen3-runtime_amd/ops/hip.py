@@ -93,7 +93,7 @@ class _ConvArgs(Structure):
         ("num_tokens", c_int), ("channels", c_int), ("num_taps", c_int), ("nseg", c_int),
         ("seg_first", c_int * 4), ("seg_heads", c_int * 4), ("seg_width", c_int * 4), ("seg_mode", c_int * 4),
         ("total_heads", c_int), ("unit_eps", c_float), ("fuse_tail", c_int), ("bias", c_void_p),
-        ("out_code", c_int),
+        ("out_code", c_int), ("no_activation", c_int),
     ]
 
 
@@ -123,6 +123,7 @@ class _RetentionArgs(Structure):
         ("heads", c_int), ("dim", c_int), ("vdim", c_int), ("share", c_int),
         ("step", c_void_p), ("step_stride", c_long), ("step_code", c_int),
         ("step_bias", c_void_p), ("a_log", c_void_p), ("skip", c_void_p), ("qkv_code", c_int), ("seq_ids", c_void_p),
+        ("gates", c_void_p), ("last_out", c_void_p),
     ]
 
 
@@ -288,6 +289,26 @@ class HipOps:
                                                  c_int(t), c_int(v), c_int(h), c_float(scale), _stream()))
         return out
 
+    def embed_pairs(self, ctx, ids, table, pairs, mul_prev, mul_cur, last):
+        """Rows of ``table`` plus rows of ``pairs`` [buckets + 1, H], which (previous token * mul_prev + token *
+        mul_cur) mod buckets picks, the last one for a sequence's first token; float32 [T, H]. ``last`` int32
+        [slots, 1] holds each request's last token and is brought up to date."""
+        t, (_, h) = ids.numel(), table.shape
+        _need(ids, "ids", torch.int32, (ctx.num_tokens,))
+        _need(table, "embedding table")
+        _need(pairs, "table of pairs", shape=(pairs.shape[0], h))
+        _need(last, "last tokens", torch.int32, (last.shape[0], 1))
+        _need(ctx.positions, "positions", torch.int32, (t,))
+        _need(ctx.seq_of_token, "seq_of_token", torch.int32, (t,))
+        _need(ctx.cu_q, "cu_q", torch.int32, (ctx.num_seqs + 1,))
+        _need(ctx.state_slots, "state_slots", torch.int32, (ctx.num_seqs,))
+        out = torch.empty((t, h), dtype=torch.float32, device=table.device)
+        self._check(self.lib, self.lib.qrt_embed_pairs(
+            _ptr(ids), _ptr(ctx.positions), _ptr(ctx.seq_of_token), _ptr(ctx.cu_q), _ptr(ctx.state_slots), _ptr(table),
+            _CODE[table.dtype], _ptr(pairs), _CODE[pairs.dtype], _ptr(last), _ptr(out), c_int(t), c_int(h),
+            c_int(pairs.shape[0] - 1), c_long(mul_prev), c_long(mul_cur), _stream()))
+        return out
+
     def scale(self, x, factor):
         """``x *= factor`` in place, float32."""
         _need(x, "x", torch.float32)
@@ -354,16 +375,18 @@ class HipOps:
             c_float(eps), _ptr(rows), _ptr(out), _CODE[out_dtype], c_int(n_out), c_int(h), _stream()))
         return out
 
-    def scaled_add_rmsnorm(self, residual, parts, weight, eps, out_dtype, rows=None):
-        """``residual += sum_i scale_i * y_i`` in place, element by element (``parts``: up to four
-        (y, scale), ``y`` a matrix or float32 planes, ``scale`` float32 [H]), then the rows' RMS norm;
+    def scaled_add_rmsnorm(self, residual, parts, weight, eps, out_dtype, rows=None, vector=None):
+        """``residual += sum_i scale_i * y_i (+ vector)`` in place, element by element (``parts``: up to four
+        (y, scale), ``y`` a matrix or float32 planes, ``scale`` float32 [H]; ``vector`` float32 [H]), then the rows' RMS norm;
         with ``rows`` only those, and ``residual`` is left alone."""
         t, h = residual.shape
         _need(residual, "residual", torch.float32)
         _need(weight, "norm weight", torch.float32, (h,))
         n = len(parts)
-        if not 1 <= n <= 4:
+        if not (0 if vector is not None else 1) <= n <= 4:
             raise OpsError(f"a sum of {n} scaled outputs (1 to 4)")
+        if vector is not None:
+            _need(vector, "vector", torch.float32, (h,))
         ptrs, codes, counts, scales = (c_void_p * n)(), (c_int * n)(), (c_int * n)(), (c_void_p * n)()
         for i, (y, scale) in enumerate(parts):
             py, codes[i], counts[i] = _planes(y, t, h, "sub-layer output")
@@ -375,7 +398,7 @@ class HipOps:
             n_out = rows.numel()
         out = torch.empty((n_out, h), dtype=out_dtype, device=residual.device)
         self._check(self.lib, self.lib.qrt_scaled_add_rmsnorm(
-            _ptr(residual), ptrs, codes, counts, scales, c_int(n), c_long(t * h), _ptr(weight), c_float(eps), _ptr(rows),
+            _ptr(residual), ptrs, codes, counts, scales, c_int(n), _ptr(vector), c_long(t * h), _ptr(weight), c_float(eps), _ptr(rows),
             _ptr(out), _CODE[out_dtype], c_int(n_out), c_int(h), _stream()))
         return out
 
@@ -589,6 +612,61 @@ class HipOps:
                                                          c_int(state.shape[0]), _stream()))
         return out
 
+    # ---- matrix memory -----------------------------------------------------------------
+    def memory_gates(self, ctx, logits, bias, cap, top, heads):
+        """From the logits [T, heads input | heads forget] (float32; + ``bias``, softly held to ``cap``) and the
+        running maxima ``top`` [slots, heads] (brought up to date): float32 [T, 3, heads], the logarithms of
+        what a token keeps of the memory and of what its write weighs, and its running maximum."""
+        t = ctx.num_tokens
+        _need(logits, "gate logits", torch.float32, (t, 2 * heads))
+        _need(bias, "gate biases", torch.float32, (2 * heads,))
+        _need(top, "running maxima", torch.float32, (top.shape[0], heads))
+        _need(ctx.cu_q, "cu_q", torch.int32, (ctx.num_seqs + 1,))
+        _need(ctx.state_slots, "state_slots", torch.int32, (ctx.num_seqs,))
+        out = torch.empty((t, 3, heads), dtype=torch.float32, device=logits.device)
+        self._check(self.lib, self.lib.qrt_memory_gates(_ptr(logits), _ptr(bias), c_float(cap), _ptr(top), _ptr(out), _ptr(ctx.cu_q),
+                                                        _ptr(ctx.state_slots), c_int(heads), c_int(t), c_int(ctx.num_seqs), _stream()))
+        return out
+
+    def matrix_memory(self, ctx, y, gates, state, heads, dim, vdim):
+        """``S <- keep S + write k [v | 1]^T; o = S^T q`` over each sequence's tokens from its slot's state (float32
+        [slots, heads, vdim + 1, dim], updated in place). ``y`` [T, W]: its first columns are q | k | v; ``gates``
+        as ``memory_gates`` leaves them. Returns (o float32 [T, heads, vdim], the last column's [T, heads])."""
+        t, w = y.shape
+        c = 2 * heads * dim + heads * vdim
+        _need(y, "q | k | v", shape=(ctx.num_tokens, w))
+        if c > w:
+            raise OpsError(f"matrix_memory: {c} channels in {w} columns")
+        _need(state, "state", torch.float32, (state.shape[0], heads, vdim + 1, dim))
+        _need(gates, "gates", torch.float32, (t, 3, heads))
+        out = torch.empty((t, heads, vdim), dtype=torch.float32, device=y.device)
+        last = torch.empty((t, heads), dtype=torch.float32, device=y.device)
+        a = _RetentionArgs()
+        a.qkv, a.qkv_code, a.channels, a.q_first, a.k_first, a.v_first = y.data_ptr(), _CODE[y.dtype], w, 0, heads * dim, 2 * heads * dim
+        a.gates, a.last_out, a.state, a.out = gates.data_ptr(), last.data_ptr(), state.data_ptr(), out.data_ptr()
+        a.cu_q = _need(ctx.cu_q, "cu_q", torch.int32, (ctx.num_seqs + 1,)).data_ptr()
+        a.state_slots = _need(ctx.state_slots, "state_slots", torch.int32, (ctx.num_seqs,)).data_ptr()
+        a.heads, a.dim, a.vdim = heads, dim, vdim
+        self._check(self.lib, self.lib.qrt_retention(byref(a), c_int(t), c_int(ctx.num_seqs), c_int(state.shape[0]), _stream()))
+        return out, last
+
+    def memory_out(self, read, norm_read, gates, weight, out_gate, eps, q_scale, out_dtype):
+        """Per head ``o = s read / (max(|s norm_read|, exp(-m)) + 1e-6)`` (s = ``q_scale``), divided by its root mean
+        square, times ``weight`` (of all heads) and sigmoid(``out_gate``), columns of a wider matrix; [T, heads * vdim]."""
+        t, heads, vdim = read.shape
+        _need(read, "read-out", torch.float32)
+        _need(norm_read, "normaliser's read-out", torch.float32, (t, heads))
+        _need(gates, "gates", torch.float32, (t, 3, heads))
+        _need(weight, "read-out norm weight", torch.float32, (heads * vdim,))
+        if not out_gate.is_cuda or tuple(out_gate.shape) != (t, heads * vdim) or out_gate.stride(1) != 1 or out_gate.dtype not in _CODE:
+            raise OpsError(f"gate {tuple(out_gate.shape)} {out_gate.dtype} does not fit {t} tokens of {heads} heads of {vdim}")
+        out = torch.empty((t, heads * vdim), dtype=out_dtype, device=read.device)
+        self._check(self.lib, self.lib.qrt_memory_out(
+            _ptr(read), _ptr(norm_read), _ptr(gates), _ptr(weight), c_void_p(out_gate.data_ptr()), c_long(out_gate.stride(0)),
+            _CODE[out_gate.dtype], _ptr(out), _CODE[out_dtype], c_int(t), c_int(heads), c_int(vdim), c_float(eps), c_float(q_scale),
+            _stream()))
+        return out
+
     # spans of at least this many tokens run chunk by chunk
     space_chunk_min_tokens = 16
 
@@ -641,17 +719,17 @@ class HipOps:
         self._check(self.lib, self.lib.qrt_accumulate(_ptr(acc), py, c_int(cy), c_int(ny), c_long(t * h), _stream()))
         return acc
 
-    def gated_act(self, gate_up, activation="swiglu", limit=0.0, scale=None, order=None):
-        """The gated activation of [T, 2I] (gate columns first): ``swiglu``, or ``clamped``. With ``scale``
-        (float32 [T]) both halves of row t are first multiplied by ``scale[order[t]]`` (``order`` None: ``scale[t]``)."""
+    def gated_act(self, gate_up, activation="swiglu", limit=0.0, scale=None, order=None, row_scale=None):
+        """The gated activation of [T, 2I] (gate columns first): ``swiglu``, or ``clamped``, row t of it times
+        ``row_scale[t]`` (float32). With ``scale`` (float32 [T]) both halves of row t are first multiplied by ``scale[order[t]]`` (``order`` None: ``scale[t]``)."""
         if scale is not None:
             _need(scale, "row scales", torch.float32)
             if order is not None:
                 _need(order, "order", torch.int32, (gate_up.shape[0],))
             if scale.numel() != gate_up.shape[0]:
                 raise OpsError(f"{scale.numel()} row scales for {gate_up.shape[0]} rows")
-        if activation == "swiglu":
-            return self.swiglu(gate_up, scale, order)
+        if row_scale is not None:
+            _need(row_scale, "row factors", torch.float32, (gate_up.shape[0],))
         _need(gate_up, "gate_up")
         t, two_i = gate_up.shape
         if two_i % 2:
@@ -659,7 +737,7 @@ class HipOps:
         out = torch.empty((t, two_i // 2), dtype=gate_up.dtype, device=gate_up.device)
         self._check(self.lib, self.lib.qrt_gated_act(_ptr(gate_up), _ptr(out), _CODE[gate_up.dtype], c_int(t),
                                                      c_int(two_i // 2), c_int(ACTIVATIONS[activation]), c_float(limit),
-                                                     _ptr(scale), _ptr(order), _stream()))
+                                                     _ptr(scale), _ptr(order), _ptr(row_scale), _stream()))
         return out
 
     def bias_rotate_pairs(self, x, bias, positions, freq, rot_heads, head_dim):
@@ -681,9 +759,10 @@ class HipOps:
         return x
 
     # ---- gated delta rule ---------------------------------------------------------------
-    def delta_conv(self, ctx, y, channels, taps, tail, segments, unit_eps, first=0, bias=None, out_dtype=torch.float32):
+    def delta_conv(self, ctx, y, channels, taps, tail, segments, unit_eps, first=0, bias=None, out_dtype=torch.float32,
+                   activation="silu"):
         """``channels`` columns of ``y`` [T, W], from column ``first`` on, through their causal convolutions
-        (``taps`` float32 [C, K]; ``bias`` float32 [C] or None is added) and silu, then per head as ``segments`` say, each (heads, width,
+        (``taps`` float32 [C, K]; ``bias`` float32 [C] or None is added) and silu (``activation`` None: without), then per head as ``segments`` say, each (heads, width,
         mode): 0 as it is, 1 scaled to a unit vector, 2 that times width^(-1/2). [T, C] in ``out_dtype``.
         ``tail`` [slots, C, K-1] float32 holds each request's last inputs and is brought up to date."""
         t, w = y.shape
@@ -703,6 +782,9 @@ class HipOps:
         a.state_slots = _need(ctx.state_slots, "state_slots", torch.int32, (ctx.num_seqs,)).data_ptr()
         out = torch.empty((t, channels), dtype=out_dtype, device=y.device)
         a.out_code = _CODE[out_dtype]
+        if activation not in ("silu", None):
+            raise OpsError(f"delta_conv: unknown activation {activation!r}")
+        a.no_activation = int(activation is None)
         a.out, a.num_tokens, a.channels, a.num_taps, a.nseg, a.unit_eps = out.data_ptr(), t, channels, k, len(segments), unit_eps
         at = 0
         for i, (heads, width, mode) in enumerate(segments):
@@ -798,7 +880,7 @@ class HipOps:
 
     # ---- routed experts --------------------------------------------------------------
     def route_top(self, x, router, router_bias, top, scoring="softmax_top", groups=1, keep=None, group_score="top2",
-                  correction=None, renormalise=False, weight_scale=1.0):
+                  correction=None, renormalise=False, weight_scale=1.0, gate_row=False):
         """Router logits ``x W^T + b`` in float32, the ``top`` largest per token and the softmax
         over those alone: (int32 [T, top], float32 [T, top]). ``scoring="sigmoid"``: the choice goes
         by ``sigmoid`` of the logits, which are also the weights, as they are; ``"softmax_all"``: by the
@@ -806,11 +888,14 @@ class HipOps:
         best of ``groups`` equal groups of neighbours can be chosen, a group's score being the sum of
         its two largest entries (``group_score="top2"``) or its largest (``"max"``). With scores over all
         experts: ``correction`` [E] is added to them for the choice alone, ``renormalise`` divides the
-        chosen scores by their sum (+ 1e-20), ``weight_scale`` multiplies the weights at the end."""
+        chosen scores by their sum (+ 1e-20), ``weight_scale`` multiplies the weights at the end.
+        ``gate_row``: the router's last row is no expert; the sigmoid of its product is returned as well,
+        float32 [T]."""
         t, h = x.shape
         _need(x, "x")
-        n = router.shape[0]
-        _need(router, "router", torch.float32, (n, h))
+        n = router.shape[0] - int(bool(gate_row))
+        _need(router, "router", torch.float32, (n + int(bool(gate_row)), h))
+        gate = torch.empty((t,), dtype=torch.float32, device=x.device) if gate_row else None
         if correction is not None:
             _need(correction, "correction of the choice", torch.float32, (n,))
         if router_bias is not None:
@@ -822,8 +907,8 @@ class HipOps:
                                                      c_int(top), c_int({"softmax_top": 0, "sigmoid": 1, "softmax_all": 2}[scoring]),
                                                      c_int(groups), c_int(groups if keep is None else keep),
                                                      c_int(group_score == "max"), _ptr(correction),
-                                                     c_int(bool(renormalise)), c_float(weight_scale), _stream()))
-        return index, weight
+                                                     c_int(bool(renormalise)), c_float(weight_scale), _ptr(gate), _stream()))
+        return (index, weight, gate) if gate_row else (index, weight)
 
     def moe_swiglu(self, x, gate_up, down, index, weight, activation="swiglu", limit=0.0, out=None, weight_on_input=False):
         """``sum_j weight[t, j] * down[e] (silu(gate[e] x) * (up[e] x))`` with ``e = index[t, j]``;
@@ -955,14 +1040,7 @@ class HipOps:
         return out
 
     def swiglu(self, gate_up, scale=None, order=None):
-        _need(gate_up, "gate_up")
-        t, two_i = gate_up.shape
-        if two_i % 2:
-            raise OpsError(f"gate_up has odd width {two_i}")
-        out = torch.empty((t, two_i // 2), dtype=gate_up.dtype, device=gate_up.device)
-        self._check(self.lib, self.lib.qrt_swiglu(_ptr(gate_up), _ptr(out), _CODE[gate_up.dtype],
-                                                  c_int(t), c_int(two_i // 2), _ptr(scale), _ptr(order), _stream()))
-        return out
+        return self.gated_act(gate_up, scale=scale, order=order)
 
     # ---- matrix products -------------------------------------------------------
     def linear(self, x, w, out_f32=False):
@@ -1111,27 +1189,27 @@ class HipOps:
         return max(1, min(8, 256 // blocks, (k // 32) // 12))
 
 
-    def gated_linear(self, x, w_gate_up, activation="swiglu", limit=0.0):
-        """``swiglu(linear(x, w_gate_up))`` with ``w_gate_up`` [2I, K], gate rows first. With few
+    def gated_linear(self, x, w_gate_up, activation="swiglu", limit=0.0, row_scale=None):
+        """``gated_act(linear(x, w_gate_up), ...)`` with ``w_gate_up`` [2I, K], gate rows first. With few
         rows in bfloat16 one kernel forms both halves and applies the activation in its epilogue,
         so the [T, 2I] intermediate never reaches memory."""
         m, k = x.shape
         two_i, kw = w_gate_up.shape
         if k != kw or two_i % 2:
             raise OpsError(f"gated_linear: x is {tuple(x.shape)}, weight is {tuple(w_gate_up.shape)}")
-        if activation != "swiglu":  # the products' fused epilogue is SwiGLU's
-            return self.gated_act(self.linear(x, w_gate_up), activation, limit)
         if x.dtype == torch.bfloat16 and w_gate_up.dtype == torch.bfloat16 and k % 32 == 0:
             _need(x, "x")
             _need(w_gate_up, "weight")
             kernel = self._own_kernel(m, two_i // 2, k, "gated")
             if kernel is not None:
                 out = torch.empty((m, two_i // 2), dtype=torch.bfloat16, device=x.device)
-                self._check(self.lib, self.lib.qrt_gemm_bf16(
-                    _ptr(x), _ptr(w_gate_up), _ptr(out), BF16, c_int(m),
-                    c_int(two_i // 2), c_int(k), c_int(1), c_int(kernel), c_int(1), _stream()))
+                if row_scale is not None:
+                    _need(row_scale, "row factors", torch.float32, (m,))
+                self._check(self.lib, self.lib.qrt_gated_gemm_bf16(
+                    _ptr(x), _ptr(w_gate_up), _ptr(out), BF16, c_int(m), c_int(two_i // 2), c_int(k), c_int(kernel),
+                    c_int(ACTIVATIONS[activation]), c_float(limit), _ptr(row_scale), _stream()))
                 return out
-        return self.swiglu(self.linear(x, w_gate_up))
+        return self.gated_act(self.linear(x, w_gate_up), activation, limit, row_scale=row_scale)
 
     # ---- q/k norm, rotation, cache write ----------------------------------------
     def _qk(self, args: _QkArgs, dtype, num_pages=0):

@@ -1,6 +1,6 @@
 """Layer parts. Importing this package registers the shipped kinds."""
 
-from . import attention, block, delta, embedding, entry, latent, mlp, moe, norm, parallel, retention, rope, statespace  # noqa: F401
+from . import attention, block, delta, embedding, entry, latent, memory, mlp, moe, norm, parallel, retention, rope, statespace  # noqa: F401
 from .base import (  # noqa: F401
     Block,
     CacheView,

@@ -31,7 +31,16 @@ query temperature (``q_temp`` = (coef, every): the normed queries at position ``
 ``1 + coef * ln(floor((p + 1) / every) + 1)``, float32); turned values (``value_turn``, a base: the value
 of position ``j`` is rotated by ``j`` over all its elements, first half against second half with
 frequencies ``base^(-2m/value_dim)``, and cached so; each head's output at position ``i`` is rotated back
-by ``i``, so that what a query takes from a key depends on their distance alone).
+by ``i``, so that what a query takes from a key depends on their distance alone); short convolutions over
+time (``conv``, a number of taps: every channel of the q, k and v projections becomes
+``sum_j taps[:, j] u_(t - conv + 1 + j)``, zeros before the sequence's start, straight after the product and
+before norm and rotation; tensors ``q_conv``, ``k_conv``, ``v_conv``; the last ``conv - 1`` projected values
+are the request's state, kept in its slot); rotation in pairs of neighbours (``neighbour_pairs``: element
+``2i`` of a head's first ``dims`` turns against ``2i + 1``, where the encoding turns ``i`` against
+``i + dims / 2``: the rows of the query and key projections, with their taps, biases and norm weights, are
+brought into the encoding's order when the weights are placed; queries and keys share the order, and
+neither a score nor a head's norm depends on it). A norm without weights after a rotation is the norm
+before it: a rotation leaves a head's root mean square as it is.
 """
 
 from __future__ import annotations
@@ -70,6 +79,8 @@ class GroupedQueryAttention(Mixer):
         values_are_keys: bool = False,
         q_temp: tuple[float, int] | None = None,
         value_turn: float | None = None,
+        conv: int | None = None,
+        neighbour_pairs: bool = False,
         tensors=None,
     ):
         super().__init__(tensors)
@@ -124,14 +135,45 @@ class GroupedQueryAttention(Mixer):
         if position is not None:
             self.position = part_class("position", position.kind)(**position.args, tensors=position.tensors)
         self.qkv = self.o = self.q_norm = self.k_norm = None
+        self.conv = None if conv is None else int(conv)
+        self.taps = None
+        if self.conv is not None:
+            if not 1 <= self.conv <= 16:
+                raise ValueError(f"the convolutions have 1 to 16 taps, not {conv}")
+            if self.joint_norm or output_gate or bias:
+                raise NotImplementedError("convolutions behind the projections, with biases, an output gate or a q/k norm "
+                                          "over the whole projection")
+        self.row_order = None
+        if neighbour_pairs and position is not None:
+            if self.position.fused_form != "half" or self.value_turn is not None:
+                raise ValueError("pairs of neighbours are brought into the order of a half rotation of plain queries and keys")
+            n = self.position.dims
+            self.row_order = torch.tensor([*range(0, n, 2), *range(1, n, 2), *range(n, self.head_dim)], dtype=torch.long)
 
     def children(self):
         return (self.position,) if self.position is not None else ()
+
+    @property
+    def channels(self) -> int:
+        """Columns of q | k | v."""
+        v = 0 if self.values_are_keys else self.num_kv_heads * self.value_dim
+        return (self.num_heads + self.num_kv_heads) * self.head_dim + v
 
     def cache_spec(self):
         return CacheSpec("paged_kv", heads=self.num_kv_heads, head_dim=self.head_dim, window=self.window,
                          chunk=self.chunk, value_dim=None if self.value_dim == self.head_dim else self.value_dim,
                          keep_first=self.keep_first)
+
+    def cache_specs(self):
+        specs = super().cache_specs()
+        if self.conv is not None:
+            specs += (CacheSpec("state", shape=(self.channels, max(self.conv - 1, 1)), dtype="float32"),)
+        return specs
+
+    def _in_order(self, rows: torch.Tensor, heads: int) -> torch.Tensor:
+        """The rows of ``heads`` heads with every head's elements in the encoding's order."""
+        order = self.row_order.to(rows.device)
+        return rows.view(heads, self.head_dim, -1)[:, order].reshape(rows.shape)
 
     def tensor_decls(self):
         h, d, dv = self.hidden_size, self.head_dim, self.value_dim
@@ -144,6 +186,10 @@ class GroupedQueryAttention(Mixer):
         decls.append(TensorDecl(self._name("o"), (h, self.num_heads * dv)))
         if self.output_gate:
             decls.append(TensorDecl(self._name("g"), (self.num_heads * dv, h)))
+        if self.conv is not None:
+            for n, rows in (("q", self.num_heads * d), ("k", self.num_kv_heads * d), ("v", self.num_kv_heads * dv)):
+                if n != "v" or not self.values_are_keys:
+                    decls.append(TensorDecl(self._name(n + "_conv"), (rows, self.conv), init="taps"))
         if self.has_bias:
             decls += [TensorDecl(self._name("q_bias"), (self.num_heads * d,)),
                       TensorDecl(self._name("k_bias"), (self.num_kv_heads * d,))]
@@ -162,6 +208,17 @@ class GroupedQueryAttention(Mixer):
         names = [self._name("q"), self._name("k")] + ([] if self.values_are_keys else [self._name("v")]) \
             + ([self._name("g")] if self.output_gate else [])
         self.qkv = fetch.fused(names, dim=0)
+        nq, nkv, d = self.num_heads, self.num_kv_heads, self.head_dim
+        if self.conv is not None:
+            parts = ("q", "k") if self.values_are_keys else ("q", "k", "v")
+            self.taps = torch.cat([fetch.vector_f32(self._name(n + "_conv")) for n in parts], dim=0)
+        if self.row_order is not None:
+            rows = (nq + nkv) * d
+            self.qkv = fetch.constant(torch.cat([self._in_order(self.qkv[:rows], nq + nkv), self.qkv[rows:]], dim=0))
+            if self.taps is not None:
+                self.taps = torch.cat([self._in_order(self.taps[:rows], nq + nkv), self.taps[rows:]], dim=0)
+        if self.taps is not None:
+            self.taps = fetch.constant(self.taps)
         self.o = fetch.matrix(self._name("o"))
         if self.turn_freq_cpu is not None:
             self.turn_freq = fetch.constant(self.turn_freq_cpu)
@@ -169,10 +226,14 @@ class GroupedQueryAttention(Mixer):
             pieces = [fetch.vector_f32(self._name(n)) for n in ("q_bias", "k_bias", "v_bias")[: 2 if self.values_are_keys else 3]]
             if self.output_gate:
                 pieces.append(torch.zeros(self.num_heads * self.value_dim, dtype=torch.float32, device=pieces[0].device))
+            if self.row_order is not None:
+                pieces[:2] = [self._in_order(pieces[0], nq), self._in_order(pieces[1], nkv)]
             self.bias = fetch.constant(torch.cat(pieces))
         if self.qk_norm_eps is not None and self.qk_norm_weight:
             self.q_norm = fetch.vector_f32(self._name("q_norm"))
             self.k_norm = fetch.vector_f32(self._name("k_norm"))
+            if self.row_order is not None:
+                self.q_norm, self.k_norm = (fetch.constant(self._in_order(w, 1)) for w in (self.q_norm, self.k_norm))
         elif self.qk_norm_eps is not None:  # a norm without weights: weights of one
             self.q_norm = self.k_norm = fetch.constant(torch.ones(self.head_dim, dtype=torch.float32))
 
@@ -193,6 +254,12 @@ class GroupedQueryAttention(Mixer):
         ops = ctx.ops
         nq, nkv, d, dv = self.num_heads, self.num_kv_heads, self.head_dim, self.value_dim
         qkv = ops.linear(x, self.qkv)
+        if self.conv is not None:
+            cache, tail = cache
+            whole, rest = divmod(self.channels, 128)  # what a wave of the convolution takes at a time
+            segments = tuple(s for s in ((whole, 128, 0), (1, rest, 0)) if s[0] * s[1])
+            qkv = ops.delta_conv(ctx, qkv, self.channels, self.taps, tail.state, segments, 0.0, out_dtype=ctx.dtype,
+                                 activation=None)
         eps = self.qk_norm_eps if self.qk_norm_eps is not None else 0.0
         if self.joint_norm:
             # biases, the norm over each whole projection, the queries' temperature and the cache

@@ -7,7 +7,8 @@ configuration the numbers came from.
 
 Roles and the call each must answer (``T`` tokens of this step, ``H`` width):
 
-* embedding      ``forward(ctx, ids[T] int32) -> residual[T, H] float32``
+* embedding      ``forward(ctx, ids[T] int32) -> residual[T, H] float32``; one that keeps something per
+                 request (``cache_specs()`` not empty) also gets ``cache``, a tuple of views
 * norm           ``forward(ctx, residual[T, H] float32, delta[T, H] | None, rows=None, read=None) -> [T|R, H]``
                  adds ``delta`` into ``residual`` in place, then normalises; over several
                  residual streams ``[T, S, H]`` ``delta`` is a ``StreamUpdate`` and ``read``
@@ -91,6 +92,10 @@ class Part:
         return None
 
     def children(self) -> Sequence["Part"]:
+        return ()
+
+    def cache_specs(self) -> tuple[CacheSpec, ...]:
+        """What the part keeps between steps, per request: mixers do, an embedding may."""
         return ()
 
     def step_cost(self, spans: Sequence[tuple[int, int]], rows: int, elem_bytes: int) -> StepCost:
@@ -192,10 +197,11 @@ class NormedUpdate:
 @dataclass
 class ScaledUpdate:
     """Several sub-layer outputs that join the residual stream in one sum, each times a vector of
-    its own, element by element: ``x <- x + sum_i scale_i * y_i``. Like a plain ``delta`` it is
+    its own, element by element: ``x <- x + sum_i scale_i * y_i (+ vector)``. Like a plain ``delta`` it is
     applied by the norm that comes next."""
 
     parts: list  # of (y, scale): y [T, H] or float32 planes [P, T, H] whose sum it is; scale float32 [H]
+    vector: torch.Tensor | None = None  # float32 [H], the same for every token
 
 
 @dataclass

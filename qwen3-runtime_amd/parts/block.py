@@ -179,14 +179,18 @@ class HyperConnectionBlock(Block):
 class ParallelScaledBlock(Block):
     """Mixer and feed-forward side by side: one norm, ``n = norm_in(x)``, both read it, and
     ``x <- x + s1 * mixer(n) + s2 * feed_forward(n)`` with a vector per sub-layer (tensors ``scale1``,
-    ``scale2``; ``layer_scale=False``: no vectors, the plain sum). The two outputs go on as one
+    ``scale2``; ``layer_scale=False``: no vectors, the sum times the constant ``mult``). The two outputs go on as one
     ``ScaledUpdate``, which the next layer's norm adds in the pass in which it normalises. A block
     without feed-forward has the first term only."""
 
     norm_names = ("input",)
 
-    def __init__(self, mixer, feed_forward, norms, hidden_size: int, layer_scale: bool = True, tensors=None):
+    def __init__(self, mixer, feed_forward, norms, hidden_size: int, layer_scale: bool = True, mult: float = 1.0,
+                 tensors=None):
         super().__init__(tensors)
+        self.mult = float(mult)
+        if layer_scale and self.mult != 1.0:
+            raise ValueError("vectors on the sub-layers' outputs, or a constant, not both")
         self.mixer = mixer
         self.feed_forward = feed_forward
         self.norm_in = norms["input"]
@@ -210,7 +214,7 @@ class ParallelScaledBlock(Block):
         else:
             import torch
 
-            self.scale1 = self.scale2 = fetch.constant(torch.ones(self.hidden_size, dtype=torch.float32))
+            self.scale1 = self.scale2 = fetch.constant(torch.full((self.hidden_size,), self.mult, dtype=torch.float32))
 
     def step_cost(self, spans, rows, elem_bytes):
         cost = super().step_cost(spans, rows, elem_bytes)

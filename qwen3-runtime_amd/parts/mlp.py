@@ -3,7 +3,8 @@
 ``down( silu(gate(x)) * up(x) )`` with gate and up as one fused matrix whose
 rows are gate's followed by up's (reference: qwen3_runtime/models/qwen3.py:130-138,
 qwen3_runtime/utils/loader.py:51-53); ``silu(g) = g * sigmoid(g)``
-(reference: qwen3_runtime/layers/ops.py:23-25), evaluated in float32 here.
+(reference: qwen3_runtime/layers/ops.py:23-25), evaluated in float32 here. ``activation="clamped"`` with
+``limit``: ``g = min(gate x, limit)``, ``u = clamp(up x, -limit, limit)``, ``g sigmoid(1.702 g) (u + 1)`` in its place.
 
 ``act_mlp``: ``down( act(up(x)) )`` without a gate; ``act`` is ``relu2`` (the square of relu), in float32.
 """
@@ -17,8 +18,12 @@ from .plan import TensorDecl
 
 @register_part("feed_forward", "swiglu")
 class SwiGLU(FeedForward):
-    def __init__(self, hidden_size: int, intermediate_size: int, tensors=None):
+    def __init__(self, hidden_size: int, intermediate_size: int, activation: str = "swiglu", limit: float = 0.0,
+                 tensors=None):
         super().__init__(tensors)
+        if activation not in ("swiglu", "clamped"):
+            raise ValueError(f"unknown activation {activation!r} (swiglu, clamped)")
+        self.how = {} if activation == "swiglu" else {"activation": activation, "limit": float(limit)}
         self.hidden_size = int(hidden_size)
         self.intermediate_size = int(intermediate_size)
         self.gate_up = None
@@ -37,7 +42,7 @@ class SwiGLU(FeedForward):
         self.down = fetch.matrix(self._name("down"))
 
     def forward(self, ctx, x):
-        act = ctx.ops.gated_linear(x, self.gate_up)
+        act = ctx.ops.gated_linear(x, self.gate_up, **self.how)
         return ctx.ops.linear_for_residual(act, self.down)
 
 

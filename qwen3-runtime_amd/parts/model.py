@@ -45,6 +45,10 @@ class DecoderModel:
         self._check_caches()
 
     def _check_caches(self) -> None:
+        specs = self.embedding.cache_specs()
+        if [s.group_key() for s in specs] != [self.plan.caches[c].group_key() for c in self.plan.embedding_cache]:
+            raise ValueError(f"the embedding needs the caches {list(specs)}, the plan gives "
+                             f"{[self.plan.caches[c] for c in self.plan.embedding_cache]}")
         for i, step in enumerate(self.plan.order):
             specs = self.blocks[step.layer].mixer.cache_specs()
             ids = step.cache_ids()
@@ -111,16 +115,17 @@ class DecoderModel:
         for part in self.parts():
             part.load(fetch)
 
-    def forward(self, ctx: StepContext, ids, caches: Sequence[CacheView | None], rows=None):
+    def forward(self, ctx: StepContext, ids, caches: Sequence[CacheView | None], rows=None,
+                embedding_cache: Sequence[CacheView] = ()):
         """``ids`` int32 [T]; ``caches[i]`` is the view for ``plan.order[i]`` (a tuple of views for
-        a step that names several caches).
+        a step that names several caches); ``embedding_cache`` the embedding's own views, if it has any.
 
         Returns logits ``[R, V]`` float32 for the packed row indices ``rows``
         (int32 tensor), or None when ``rows`` is None: the pass then only fills
         the caches.
         """
         ctx.per_pass.clear()
-        residual = self.embedding.forward(ctx, ids)
+        residual = self.embedding.forward(ctx, ids, tuple(embedding_cache)) if embedding_cache else self.embedding.forward(ctx, ids)
         delta = None
         # entries read the embedding's output; the stream itself is updated in place, so they get a copy
         origin = residual.clone() if self.entries else None

@@ -16,7 +16,8 @@ experts of the ``keep`` best groups can be chosen. ``activation="clamped"`` with
 ``limit``: ``g = min(gate x, limit)``, ``u = clamp(up x, -limit, limit)``, ``y = g sigmoid(1.702 g) (u + 1)``
 in place of ``silu(g) u``. ``shared_size``: one more expert of that inner width (tensors
 ``shared_gate``, ``shared_up``, ``shared_down``; ``shared_limit`` its clamp) that every token passes
-and whose output is added unweighted. ``correction`` (with ``softmax_all`` or ``sigmoid`` scores): a
+and whose output is added unweighted, or (``shared_gate``: a tensor ``shared_sg`` [1, width]) times the
+token's own ``sigmoid(W_sg x)``, one number, float32. ``correction`` (with ``softmax_all`` or ``sigmoid`` scores): a
 tensor ``correction`` [experts] is added to the scores for the choice alone; the weights are the
 chosen experts' scores without it. ``renormalise``: the chosen scores are divided by their sum
 (plus 1e-20). ``weight_scale``: the weights are multiplied by it at the end.
@@ -27,6 +28,8 @@ so the weight multiplies them in float32 in front of the activation.
 """
 
 from __future__ import annotations
+
+import torch
 
 from ..registry import register_part
 from .base import FeedForward, StepCost
@@ -43,7 +46,8 @@ class RoutedSwiGLU(FeedForward):
                  router_bias: bool = True, scoring: str = "softmax_top", groups: int = 1, keep: int | None = None,
                  activation: str = "swiglu", limit: float = 0.0, shared_size: int | None = None,
                  shared_limit: float | None = None, group_score: str = "top2", correction: bool = False,
-                 renormalise: bool = False, weight_scale: float = 1.0, weight_on: str = "output", tensors=None):
+                 renormalise: bool = False, weight_scale: float = 1.0, weight_on: str = "output", shared_gate: bool = False,
+                 tensors=None):
         super().__init__(tensors)
         self.hidden_size = int(hidden_size)
         self.intermediate_size = int(intermediate_size)
@@ -75,6 +79,9 @@ class RoutedSwiGLU(FeedForward):
             raise ValueError(f"{self.keep} groups of {self.num_experts // self.groups} experts hold fewer than the {self.top} chosen")
         self.shared_size = None if shared_size is None else int(shared_size)
         self.shared_limit = self.limit if shared_limit is None else float(shared_limit)
+        self.shared_gate = bool(shared_gate)
+        if self.shared_gate and not self.shared_size:
+            raise ValueError("a gate on the shared expert comes with one")
         self.router = self.router_bias = self.gate_up = self.down = None
         self.shared_gate_up = self.shared_down = self.correction = None
 
@@ -95,6 +102,8 @@ class RoutedSwiGLU(FeedForward):
             s = self.shared_size
             decls += [TensorDecl(self._name("shared_gate"), (s, h)), TensorDecl(self._name("shared_up"), (s, h)),
                       TensorDecl(self._name("shared_down"), (h, s))]
+        if self.shared_gate:
+            decls.append(TensorDecl(self._name("shared_sg"), (1, h)))
         return decls
 
     def load(self, fetch):
@@ -112,6 +121,8 @@ class RoutedSwiGLU(FeedForward):
         if self.shared_size:
             self.shared_gate_up = fetch.fused([self._name("shared_gate"), self._name("shared_up")], dim=0)
             self.shared_down = fetch.matrix(self._name("shared_down"))
+        if self.shared_gate:  # one more row that the router multiplies with every token
+            self.router = fetch.constant(torch.cat([self.router, fetch.vector_f32(self._name("shared_sg"))], dim=0))
 
     def step_cost(self, spans, rows, elem_bytes):
         # only the experts that some token chose are read, and each token multiplies `top` of them
@@ -128,6 +139,9 @@ class RoutedSwiGLU(FeedForward):
             for part in ("shared_gate", "shared_up", "shared_down"):
                 cost.weight_bytes[self._name(part)] = self.shared_size * h * elem_bytes
             cost.flop += 2.0 * tokens * 3 * h * self.shared_size
+        if self.shared_gate:
+            cost.weight_bytes[self._name("shared_sg")] = h * 4
+            cost.flop += 2.0 * tokens * h
         return cost
 
     def forward(self, ctx, x):
@@ -140,14 +154,20 @@ class RoutedSwiGLU(FeedForward):
         how = {"group_score": self.group_score} if self.group_score != "top2" else {}
         if self.has_correction or self.renormalise or self.weight_scale != 1.0:
             how.update(correction=self.correction, renormalise=self.renormalise, weight_scale=self.weight_scale)
-        index, weight = ops.route_top(x, self.router, self.router_bias, self.top, scoring=self.scoring,
-                                      groups=self.groups, keep=self.keep, **how)
+        opened = {}
+        if self.shared_gate:
+            index, weight, gate = ops.route_top(x, self.router, self.router_bias, self.top, scoring=self.scoring,
+                                                groups=self.groups, keep=self.keep, gate_row=True, **how)
+            opened["row_scale"] = gate
+        else:
+            index, weight = ops.route_top(x, self.router, self.router_bias, self.top, scoring=self.scoring,
+                                          groups=self.groups, keep=self.keep, **how)
         more = {"activation": self.activation, "limit": self.limit}
         if self.weight_on == "input":
             more["weight_on_input"] = True
         if not self.shared_size:
             return ops.moe_swiglu(x, self.gate_up, self.down, index, weight, **more)
-        act = ops.gated_linear(x, self.shared_gate_up, activation=self.activation, limit=self.shared_limit)
+        act = ops.gated_linear(x, self.shared_gate_up, activation=self.activation, limit=self.shared_limit, **opened)
         # few tokens: the shared expert's product leaves float32 planes with one to spare, the routed
         # experts write theirs into it, and the norm that comes next adds them all up
         planes = ops.linear_planes_with_spare(act, self.shared_down)

@@ -17,6 +17,9 @@ streams weighted by ``read``; a ``ScaledUpdate`` (the outputs of sub-layers that
 each times a vector) joins one stream as ``x + sum_i s_i * y_i``; a norm built with ``streams=S`` and called without ``read`` takes
 the plain sum (the model's last norm).
 
+``weight_offset``: the weight is stored less this constant and multiplies as ``weight_offset + w`` (1: a
+weight stored around zero).
+
 ``groups``: the RMS norm in parts: the vector is divided into that many equal parts of neighbours, each
 over its own root mean square, and the whole multiplied by the weight; also the norm on a pending
 output (``NormedUpdate.groups``) that this norm adds first.
@@ -35,8 +38,10 @@ from .plan import TensorDecl
 class RMSNorm(Norm):
     has_bias = False
 
-    def __init__(self, size: int, eps: float, streams: int = 1, delta_scale: float = 1.0, groups: int = 1, tensors=None):
+    def __init__(self, size: int, eps: float, streams: int = 1, delta_scale: float = 1.0, groups: int = 1,
+                 weight_offset: float = 0.0, tensors=None):
         super().__init__(tensors)
+        self.weight_offset = float(weight_offset)
         self.groups = int(groups)
         if self.groups < 1 or int(size) % self.groups:
             raise ValueError(f"a norm of {size} elements in {groups} equal parts")
@@ -52,13 +57,15 @@ class RMSNorm(Norm):
             raise ValueError("a scaled residual sum goes with the RMS norm over one stream")
 
     def tensor_decls(self):
-        decls = [TensorDecl(self._name("weight"), (self.size,), init="norm")]
+        decls = [TensorDecl(self._name("weight"), (self.size,), init="norm_zero" if self.weight_offset else "norm")]
         if self.has_bias:
             decls.append(TensorDecl(self._name("bias"), (self.size,), init="matrix"))
         return decls
 
     def load(self, fetch):
         self.weight = fetch.vector_f32(self._name("weight"))
+        if self.weight_offset:
+            self.weight = fetch.constant(self.weight + self.weight_offset)
         if self.has_bias:
             self.bias = fetch.vector_f32(self._name("bias"))
         if self.streams > 1:
@@ -90,7 +97,8 @@ class RMSNorm(Norm):
             # outputs of sub-layers that ran side by side, each times its vector
             if self.has_bias or self.delta_scale != 1.0:
                 raise NotImplementedError("a sum of scaled updates meets the plain RMS norm only")
-            return ctx.ops.scaled_add_rmsnorm(residual, delta.parts, self.weight, self.eps, ctx.dtype, rows)
+            more = {} if delta.vector is None else {"vector": delta.vector}
+            return ctx.ops.scaled_add_rmsnorm(residual, delta.parts, self.weight, self.eps, ctx.dtype, rows, **more)
         if self.has_bias:
             return ctx.ops.mix_norm(residual, delta, None, self.weight, self.bias, self.eps, ctx.dtype, rows)
         if self.delta_scale != 1.0:

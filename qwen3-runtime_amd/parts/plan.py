@@ -35,7 +35,8 @@ class TensorDecl:
     ``init`` tells the random-weights mode how to draw it: ``"matrix"`` and
     ``"embedding"`` are zero-mean normal, ``"norm"`` is a scale around one, ``"mixing"``
     a square matrix around the identity, ``"log_rate"`` the logarithm of a decay rate (around -2:
-    a recurrent state that forgets over tens of tokens).
+    a recurrent state that forgets over tens of tokens), ``"norm_zero"`` a norm's weight stored around
+    zero, ``"taps"`` those of a short convolution, ``"open_gate"`` the bias of a forget gate (around 3: it stays nearly open).
     ``storage`` is ``"float"`` (stored as bfloat16, float32 or float16) or ``"int"``
     (an integer table, held as int32; drawn as zeros in the random-weights mode unless
     ``init`` is ``"index:<n>"``, uniform in ``[0, n)``).
@@ -180,9 +181,14 @@ class ModelPlan:
     eos_token_id: int | None = None
     # parts of role "entry" that steps of the order may name (``RunStep.entry``)
     entries: Sequence[PartSpec] = ()
+    # the caches of an embedding that keeps something per request (the last token it saw, say), in the
+    # order of its ``cache_specs()``; no step of the order names them
+    embedding_cache: Sequence[int] = ()
 
     def __post_init__(self) -> None:
-        writers: set[int] = set()
+        writers: set[int] = set(self.embedding_cache)
+        if any(not 0 <= cache < len(self.caches) for cache in writers) or len(writers) != len(self.embedding_cache):
+            raise ValueError(f"the embedding names caches {list(self.embedding_cache)}; the plan has {len(self.caches)}")
         for i, step in enumerate(self.order):
             if not 0 <= step.layer < len(self.layers):
                 raise ValueError(f"order[{i}] names layer {step.layer}; the plan has {len(self.layers)}")

@@ -139,3 +139,4 @@ def _load_builtin() -> None:
     from .models import roserax  # noqa: F401  (registers Roserax)
     from .models import zuvasun  # noqa: F401  (registers Zuvasun)
     from .models import sarudra  # noqa: F401  (registers Sarudra)
+    from .models import dekinex  # noqa: F401  (registers Dekinex)

@@ -75,7 +75,8 @@ class RandomSource:
     values do not depend on which other tensors exist or on the order they are
     asked for. ``"matrix"`` and ``"embedding"`` tensors are N(0, std);
     ``"norm"`` tensors are ``1 + N(0, norm_jitter)`` (all ones when the jitter
-    is zero), ``"mixing"`` matrices the identity plus ``N(0, norm_jitter)``. Values are rounded to ``store_dtype``. Integer tables
+    is zero), ``"norm_zero"`` ones ``N(0, norm_jitter)``, ``"mixing"`` matrices the identity plus
+    ``N(0, norm_jitter)``, ``"log_rate"`` and ``"open_gate"`` vectors N(-2, 1) and N(3, 1), ``"taps"`` of a short convolution N(0, 0.5). Values are rounded to ``store_dtype``. Integer tables
     (``storage="int"``) are int32: zeros, or uniform in ``[0, n)`` for ``init="index:<n>"``.
     """
 
@@ -118,8 +119,14 @@ class RandomSource:
         x = torch.randn(decl.shape, generator=gen, dtype=torch.float32, device=device)
         if decl.init == "norm":
             x = 1.0 + self.norm_jitter * x
+        elif decl.init == "norm_zero":
+            x = self.norm_jitter * x
+        elif decl.init == "taps":
+            x = 0.5 * x
         elif decl.init == "log_rate":
             x = -2.0 + x
+        elif decl.init == "open_gate":
+            x = 3.0 + x
         elif decl.init == "mixing":
             x = torch.eye(decl.shape[0], decl.shape[1], dtype=torch.float32, device=device) + self.norm_jitter * x
         else:

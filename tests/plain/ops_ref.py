@@ -221,12 +221,16 @@ def mix_norm(streams, update, read, weight, bias, eps, out_dtype, rows=None, com
 
 
 def route_top(x, router, router_bias, top, scoring="softmax_top", groups=1, keep=None, group_score="top2",
-              correction=None, renormalise=False, weight_scale=1.0):
-    """float32 logits x W^T + b; the ``top`` largest per token (ties: the lower index first) and
+              correction=None, renormalise=False, weight_scale=1.0, gate_row=False):
+    """``gate_row``: the router's last row is no expert; sigmoid of its product is returned as well, [T]. float32 logits x W^T + b; the ``top`` largest per token (ties: the lower index first) and
     the softmax over those alone. Returns (int32 [T, top], float32 [T, top]). With sigmoid scoring
     the scores are the weights; with groups only the best ``keep`` groups' experts can be chosen.
     ``correction`` [E] is added to the scores for the choice alone; ``renormalise`` divides the chosen
     scores by their sum (+ 1e-20); ``weight_scale`` multiplies the weights at the end."""
+    if gate_row:
+        gate = torch.sigmoid(x.to(torch.float32) @ router[-1].to(torch.float32))
+        return (*route_top(x, router[:-1], router_bias, top, scoring, groups, keep, group_score, correction, renormalise,
+                           weight_scale), gate)
     logits = x.to(torch.float32) @ router.to(torch.float32).T
     if router_bias is not None:
         logits = logits + router_bias.to(torch.float32)
@@ -319,8 +323,74 @@ def bias_rotate_pairs(x, bias, positions, freq, rot_heads, head_dim):
     return x
 
 
-def delta_conv(y, channels, taps, tail, cu_q, slots, segments, unit_eps, first=0, bias=None, out_dtype=torch.float32):
-    """Causal convolution (+ ``bias``) + silu + unit vectors per head, span by span, over the columns
+def embed_pairs(ids, positions, cu_q, slots, table, pairs, mul_prev, mul_cur, last):
+    """Rows of ``table`` plus rows of ``pairs`` picked by (previous token, token); a sequence's first token
+    has the last row. ``last`` int32 [slots, 1]: each request's last token, brought up to date."""
+    buckets = pairs.shape[0] - 1
+    out = torch.empty((ids.numel(), table.shape[1]), dtype=torch.float32, device=table.device)
+    for s in range(len(cu_q) - 1):
+        a, b, slot = int(cu_q[s]), int(cu_q[s + 1]), int(slots[s])
+        prev = int(last[slot, 0])
+        for t in range(a, b):
+            cur = int(ids[t])
+            row = buckets if int(positions[t]) == 0 else (prev * mul_prev + cur * mul_cur) % buckets
+            out[t] = table[cur].float() + pairs[row].float()
+            prev = cur
+        if b > a:
+            last[slot, 0] = prev
+    return out
+
+
+def memory_gates(logits, bias, cap, top, cu_q, slots, heads):
+    """From the logits [T, heads input | heads forget] (+ ``bias``, softly held to ``cap``): float32 [T, 3, heads],
+    the logarithms of what a token keeps of the memory and of what its write weighs, and the running
+    maximum, which starts from ``top`` [slots, heads] and is left there."""
+    z = cap * torch.tanh((logits.to(torch.float32) + bias) / cap)
+    log_in, log_forget = z[:, :heads], torch.nn.functional.logsigmoid(z[:, heads:])
+    out = torch.empty((z.shape[0], 3, heads), dtype=torch.float32, device=z.device)
+    for s in range(len(cu_q) - 1):
+        slot = int(slots[s])
+        m = top[slot].clone()
+        for t in range(int(cu_q[s]), int(cu_q[s + 1])):
+            new = torch.maximum(log_forget[t] + m, log_in[t])
+            out[t, 0], out[t, 1], out[t, 2] = log_forget[t] + m - new, log_in[t] - new, new
+            m = new
+        top[slot] = m
+    return out
+
+
+def matrix_memory(y, gates, state, cu_q, slots, heads, dim, vdim):
+    """S <- keep S + write k [v | 1]^T, o = S^T q per sequence and head from the slot's state [slots, heads,
+    vdim + 1, dim]; ``y``'s first columns are q | k | v. Returns (o [T, heads, vdim], the last column's [T, heads])."""
+    t = y.shape[0]
+    y = y.to(torch.float32)
+    q, k = y[:, : heads * dim].view(t, heads, dim), y[:, heads * dim: 2 * heads * dim].reshape(t, heads, dim)
+    v = y[:, 2 * heads * dim: 2 * heads * dim + heads * vdim].reshape(t, heads, vdim)
+    v = torch.cat([v, torch.ones_like(v[..., :1])], dim=-1)
+    keep, write = torch.exp(gates[:, 0]), torch.exp(gates[:, 1])
+    out = torch.empty((t, heads, vdim + 1), dtype=torch.float32, device=y.device)
+    for s in range(len(cu_q) - 1):
+        slot = int(slots[s])
+        st = state[slot].clone()
+        for i in range(int(cu_q[s]), int(cu_q[s + 1])):
+            st = st * keep[i][:, None, None] + (write[i][:, None] * v[i])[:, :, None] * k[i][:, None, :]
+            out[i] = torch.einsum("hvd,hd->hv", st, q[i])
+        state[slot] = st
+    return out[..., :vdim].contiguous(), out[..., vdim].contiguous()
+
+
+def memory_out(read, norm_read, gates, weight, out_gate, eps, q_scale, out_dtype):
+    """Per head ``o = s read / (max(|s norm_read|, exp(-m)) + 1e-6)`` (s = ``q_scale``), over its root mean square,
+    times the weight of all heads and sigmoid(out_gate); [T, heads * vdim]."""
+    floor = torch.maximum((norm_read * q_scale).abs(), torch.exp(-gates[:, 2])) + 1e-6
+    o = read * q_scale / floor[..., None]
+    o = (o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + eps)).reshape(o.shape[0], -1)
+    return (o * weight * torch.sigmoid(out_gate.to(torch.float32))).to(out_dtype)
+
+
+def delta_conv(y, channels, taps, tail, cu_q, slots, segments, unit_eps, first=0, bias=None, out_dtype=torch.float32,
+               activation="silu"):
+    """Causal convolution (+ ``bias``) + silu (``activation`` None: without) + unit vectors per head, span by span, over the columns
     ``first .. first + channels``; ``tail`` updated in place."""
     y = y[:, first:]
     k = taps.shape[1]
@@ -333,7 +403,7 @@ def delta_conv(y, channels, taps, tail, cu_q, slots, segments, unit_eps, first=0
         acc = torch.zeros_like(x) if bias is None else bias[None, :].expand_as(x).clone()
         for j in range(k):
             acc = acc + full[j: j + (b - a)] * taps[:, j]
-        out[a:b] = acc * torch.sigmoid(acc)
+        out[a:b] = acc if activation is None else acc * torch.sigmoid(acc)
         if k > 1:
             tail[slot, :, : k - 1] = full[full.shape[0] - (k - 1):].T
     first = 0
@@ -521,13 +591,15 @@ def unary_act(x, kind):
     return torch.relu(x.to(torch.float32)).pow(2).to(x.dtype)
 
 
-def scaled_add_rmsnorm(residual, parts, weight, eps, out_dtype, rows=None, compute=torch.float32):
-    """``residual += sum_i scale_i * y_i`` in place (each ``y_i`` a matrix or planes), then the rows' RMS
+def scaled_add_rmsnorm(residual, parts, weight, eps, out_dtype, rows=None, compute=torch.float32, vector=None):
+    """``residual += sum_i scale_i * y_i (+ vector)`` in place (each ``y_i`` a matrix or planes), then the rows' RMS
     norm; with ``rows`` only those, and ``residual`` is left alone."""
     total = None
     for y, scale in parts:
         term = planes_sum(y) * scale.to(torch.float32)
         total = term if total is None else total + term
+    if vector is not None:
+        total = vector.expand_as(residual) if total is None else total + vector
     return add_rmsnorm(residual, total, weight, eps, out_dtype, rows, compute)
 
 
@@ -593,8 +665,20 @@ class TorchOps:
             latent_store(y, first, rank, rot_dim, weight, eps, positions, freq, cache.k, cache.v, cache.group.slots,
                          cache.group.page_size, neighbours, magnitude)
 
-    def scaled_add_rmsnorm(self, residual, parts, weight, eps, out_dtype, rows=None):
-        return scaled_add_rmsnorm(residual, parts, weight, eps, out_dtype, rows, self.compute)
+    def scaled_add_rmsnorm(self, residual, parts, weight, eps, out_dtype, rows=None, vector=None):
+        return scaled_add_rmsnorm(residual, parts, weight, eps, out_dtype, rows, self.compute, vector)
+
+    def embed_pairs(self, ctx, ids, table, pairs, mul_prev, mul_cur, last):
+        return embed_pairs(ids, ctx.positions, ctx.cu_q, ctx.state_slots, table, pairs, mul_prev, mul_cur, last)
+
+    def memory_gates(self, ctx, logits, bias, cap, top, heads):
+        return memory_gates(logits, bias, cap, top, ctx.cu_q, ctx.state_slots, heads)
+
+    def matrix_memory(self, ctx, y, gates, state, heads, dim, vdim):
+        return matrix_memory(y, gates, state, ctx.cu_q, ctx.state_slots, heads, dim, vdim)
+
+    def memory_out(self, read, norm_read, gates, weight, out_gate, eps, q_scale, out_dtype):
+        return memory_out(read, norm_read, gates, weight, out_gate, eps, q_scale, out_dtype)
 
     def qk_joint_norm_store(self, qk, nq, nkv, d, bias, q_w, k_w, eps, positions, q_temp, values_are_keys, cache):
         if cache is None:
@@ -637,15 +721,18 @@ class TorchOps:
         acc += planes_sum(y)
         return acc
 
-    def gated_act(self, gate_up, activation="swiglu", limit=0.0):
+    def gated_act(self, gate_up, activation="swiglu", limit=0.0, row_scale=None):
         i = gate_up.shape[-1] // 2
-        return gated(gate_up[..., :i].to(self.compute), gate_up[..., i:].to(self.compute), activation, limit).to(gate_up.dtype)
+        act = gated(gate_up[..., :i].to(self.compute), gate_up[..., i:].to(self.compute), activation, limit)
+        return (act if row_scale is None else act * row_scale[:, None]).to(gate_up.dtype)
 
     def bias_rotate_pairs(self, x, bias, positions, freq, rot_heads, head_dim):
         return bias_rotate_pairs(x, bias, positions, freq, rot_heads, head_dim)
 
-    def delta_conv(self, ctx, y, channels, taps, tail, segments, unit_eps, first=0, bias=None, out_dtype=torch.float32):
-        return delta_conv(y, channels, taps, tail, ctx.cu_q, ctx.state_slots, segments, unit_eps, first, bias, out_dtype)
+    def delta_conv(self, ctx, y, channels, taps, tail, segments, unit_eps, first=0, bias=None, out_dtype=torch.float32,
+                   activation="silu"):
+        return delta_conv(y, channels, taps, tail, ctx.cu_q, ctx.state_slots, segments, unit_eps, first, bias, out_dtype,
+                          activation)
 
     def delta_rule(self, ctx, qkv, beta, a_logits, a_log, dt_bias, state, heads, kv_heads, dim, vdim, per_channel):
         return delta_rule(qkv, beta, a_logits, a_log, dt_bias, state, ctx.cu_q, ctx.state_slots, heads, kv_heads,
@@ -673,9 +760,9 @@ class TorchOps:
         return mix_norm(streams, update, read, weight, bias, eps, out_dtype, rows, self.compute)
 
     def route_top(self, x, router, router_bias, top, scoring="softmax_top", groups=1, keep=None, group_score="top2",
-                  correction=None, renormalise=False, weight_scale=1.0):
+                  correction=None, renormalise=False, weight_scale=1.0, gate_row=False):
         return route_top(x, router, router_bias, top, scoring, groups, keep, group_score, correction, renormalise,
-                         weight_scale)
+                         weight_scale, gate_row)
 
     def moe_swiglu(self, x, gate_up, down, index, weight, activation="swiglu", limit=0.0, weight_on_input=False):
         return moe_swiglu(x, gate_up, down, index, weight, self.compute, activation, limit, weight_on_input)
@@ -703,8 +790,8 @@ class TorchOps:
     def swiglu(self, gate_up):
         return swiglu(gate_up, self.compute)
 
-    def gated_linear(self, x, w_gate_up, activation="swiglu", limit=0.0):
-        return self.gated_act(linear(x, w_gate_up, False, self.compute), activation, limit)
+    def gated_linear(self, x, w_gate_up, activation="swiglu", limit=0.0, row_scale=None):
+        return self.gated_act(linear(x, w_gate_up, False, self.compute), activation, limit, row_scale)
 
     def argmax(self, logits):
         return argmax(logits)
