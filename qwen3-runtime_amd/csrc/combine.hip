@@ -218,9 +218,10 @@ extern "C" int qrt_norm_add_rmsnorm(float* residual, const void* y, int y_code, 
 
 // ------------------------------------------------ a sum of scaled sub-layer outputs, then the norm
 // x = residual[r] + sum_i s_i * y_i[r] (+ vector)  (element by element; written back without `rows`);
-// out[b] = x / rms(x) * w.  Everything float32. One block of 1,024 threads per row; a thread keeps
-// its elements in registers (rows up to 4,096 wide; the rest of a wider row is computed again),
-// all terms, vectors and weights asked for before the first is used. The terms are added in order.
+// out[b] = x / rms(x) * w.  Everything float32. One block per row; a thread keeps KEEP pieces of VEC
+// neighbouring elements in registers (the rest of a wider row is computed again), all terms, vectors and
+// weights asked for before the first is used. The terms are added in order. Few rows: 1,024 threads and a
+// piece each; many rows: 256 threads with several pieces.
 #define SA_TERMS 4
 struct ScaledTerms {
   Planes y[SA_TERMS];
@@ -229,72 +230,149 @@ struct ScaledTerms {
   const float* vector;  // [H] or null: one more addend, the same for every row
 };
 
-template <int N>
-__device__ __forceinline__ float scaled_sum_at(const ScaledTerms& s, float x, size_t at, int i) {
-  float part[N > 0 ? N : 1], sc[N > 0 ? N : 1];
-  const float v = s.vector ? s.vector[i] : 0.f;
+// VEC neighbouring elements of a sub-layer output, float32
+template <int VEC>
+__device__ __forceinline__ void planes_piece(const Planes& y, size_t i, float* v) {
+  typedef float fvec_t __attribute__((ext_vector_type(VEC)));
+  typedef bf16_t bvec_t __attribute__((ext_vector_type(VEC)));
+  if (y.code == QRT_BF16) {
+    const bvec_t x = *(const bvec_t*)((const bf16_t*)y.p + i);
 #pragma unroll
-  for (int k = 0; k < N; ++k) {
-    part[k] = planes_at(s.y[k], at);
-    sc[k] = s.scale[k][i];
+    for (int e = 0; e < VEC; ++e) v[e] = (float)x[e];
+    return;
   }
+  const float* p = (const float*)y.p;
+  if (y.planes == 1) {
+    const fvec_t x = *(const fvec_t*)(p + i);
 #pragma unroll
-  for (int k = 0; k < N; ++k) x = fmaf(sc[k], part[k], x);
-  return x + v;
+    for (int e = 0; e < VEC; ++e) v[e] = x[e];
+    return;
+  }
+  fvec_t part[8];
+#pragma unroll
+  for (int k = 0; k < 8; ++k) part[k] = *(const fvec_t*)(p + (size_t)(k < y.planes ? k : 0) * y.plane_stride + i);
+#pragma unroll
+  for (int e = 0; e < VEC; ++e) {
+    v[e] = 0.f;
+#pragma unroll
+    for (int k = 0; k < 8; ++k) v[e] += k < y.planes ? part[k][e] : 0.f;
+  }
+  for (int k = 8; k < y.planes; ++k) {
+    const fvec_t x = *(const fvec_t*)(p + (size_t)k * y.plane_stride + i);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) v[e] += x[e];
+  }
 }
 
-template <typename TO, int N>
-__global__ __launch_bounds__(1024) void scaled_add_rmsnorm_kernel(float* __restrict__ residual, ScaledTerms s,
-                                                                  const float* __restrict__ weight, float eps,
-                                                                  const int* __restrict__ rows, TO* __restrict__ out,
-                                                                  int hidden) {
+template <int N, int VEC>
+__device__ __forceinline__ void scaled_sum_piece(const ScaledTerms& s, const float* __restrict__ residual, size_t row, int i, float* x) {
+  typedef float fvec_t __attribute__((ext_vector_type(VEC)));
+  float part[N > 0 ? N : 1][VEC];
+  fvec_t sc[N > 0 ? N : 1], add;
+  const fvec_t r = *(const fvec_t*)(residual + row + i);
+#pragma unroll
+  for (int k = 0; k < N; ++k) {
+    planes_piece<VEC>(s.y[k], row + i, part[k]);
+    sc[k] = *(const fvec_t*)(s.scale[k] + i);
+  }
+  if (s.vector) add = *(const fvec_t*)(s.vector + i);  // the same for the launch
+#pragma unroll
+  for (int e = 0; e < VEC; ++e) {
+    x[e] = r[e];
+#pragma unroll
+    for (int k = 0; k < N; ++k) x[e] = fmaf(sc[k][e], part[k][e], x[e]);
+    if (s.vector) x[e] += add[e];
+  }
+}
+
+template <typename TO, int N, int VEC, int THREADS, int KEEP>
+__global__ __launch_bounds__(THREADS) void scaled_add_rmsnorm_kernel(float* __restrict__ residual, ScaledTerms s,
+                                                                     const float* __restrict__ weight, float eps,
+                                                                     const int* __restrict__ rows, TO* __restrict__ out,
+                                                                     int hidden) {
+  typedef float fvec_t __attribute__((ext_vector_type(VEC)));
+  typedef TO ovec_t __attribute__((ext_vector_type(VEC)));
+  constexpr int STRIDE = THREADS * VEC;
   __shared__ float red[32];
   const int b = blockIdx.x;
   const int r = rows ? rows[b] : b;
   const size_t row = (size_t)r * hidden;
-  float vx[NM_KEEP], wn[NM_KEEP];
+  const int i0 = threadIdx.x * VEC;
+  float x[KEEP][VEC];
+  fvec_t w[KEEP];
 #pragma unroll
-  for (int j = 0; j < NM_KEEP; ++j) {
-    const int i = min((int)threadIdx.x + 1024 * j, hidden - 1);
-    vx[j] = scaled_sum_at<N>(s, residual[row + i], row + i, i);
-    wn[j] = weight[i];
+  for (int j = 0; j < KEEP; ++j) {
+    const int i = min(i0 + j * STRIDE, hidden - VEC);  // beyond the row: its last piece, dropped below
+    scaled_sum_piece<N, VEC>(s, residual, row, i, x[j]);
+    w[j] = *(const fvec_t*)(weight + i);
   }
+  auto keep = [&](int i, const float* v) {
+    fvec_t u;
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) u[e] = v[e];
+    *(fvec_t*)(residual + row + i) = u;
+  };
   float sx = 0.f;
 #pragma unroll
-  for (int j = 0; j < NM_KEEP; ++j) {
-    const int i = threadIdx.x + 1024 * j;
+  for (int j = 0; j < KEEP; ++j) {
+    const int i = i0 + j * STRIDE;
     if (i < hidden) {
-      sx += vx[j] * vx[j];
-      if (!rows) residual[row + i] = vx[j];
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) sx += x[j][e] * x[j][e];
     }
   }
-  for (int i = threadIdx.x + 1024 * NM_KEEP; i < hidden; i += 1024) {
-    const float x = scaled_sum_at<N>(s, residual[row + i], row + i, i);
-    sx += x * x;
-    if (!rows) residual[row + i] = x;
-  }
-  sx = block_sum(sx, red);
-  const float ix = 1.0f / sqrtf(sx / (float)hidden + eps);
 #pragma unroll
-  for (int j = 0; j < NM_KEEP; ++j) {
-    const int i = threadIdx.x + 1024 * j;
-    if (i < hidden) out[(size_t)b * hidden + i] = from_f32<TO>(vx[j] * ix * wn[j]);
+  for (int j = 0; j < KEEP; ++j)
+    if (!rows && i0 + j * STRIDE < hidden) keep(i0 + j * STRIDE, x[j]);
+  for (int i = i0 + KEEP * STRIDE; i < hidden; i += STRIDE) {
+    float v[VEC];
+    scaled_sum_piece<N, VEC>(s, residual, row, i, v);
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) sx += v[e] * v[e];
+    if (!rows) keep(i, v);
   }
-  for (int i = threadIdx.x + 1024 * NM_KEEP; i < hidden; i += 1024) {
-    const float x = rows ? scaled_sum_at<N>(s, residual[row + i], row + i, i) : residual[row + i];
-    out[(size_t)b * hidden + i] = from_f32<TO>(x * ix * weight[i]);
+  const float ix = 1.0f / sqrtf(block_sum(sx, red) / (float)hidden + eps);
+  auto finish = [&](int i, const float* v, const fvec_t& ww) {
+    ovec_t y;
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) y[e] = from_f32<TO>(v[e] * ix * ww[e]);
+    *(ovec_t*)(out + (size_t)b * hidden + i) = y;
+  };
+#pragma unroll
+  for (int j = 0; j < KEEP; ++j)
+    if (i0 + j * STRIDE < hidden) finish(i0 + j * STRIDE, x[j], w[j]);
+  for (int i = i0 + KEEP * STRIDE; i < hidden; i += STRIDE) {
+    float v[VEC];
+    if (rows) {
+      scaled_sum_piece<N, VEC>(s, residual, row, i, v);
+    } else {
+      const fvec_t u = *(const fvec_t*)(residual + row + i);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) v[e] = u[e];
+    }
+    finish(i, v, *(const fvec_t*)(weight + i));
   }
+}
+
+template <typename TO, int N>
+static void scaled_add_rmsnorm_launch(float* residual, const ScaledTerms& s, const float* weight, float eps, const int* rows, TO* out,
+                                      int num_out, int hidden, bool vec4, hipStream_t stream) {
+  if (!vec4) scaled_add_rmsnorm_kernel<TO, N, 1, 1024, 4><<<num_out, 1024, 0, stream>>>(residual, s, weight, eps, rows, out, hidden);
+  else if (num_out <= 512) scaled_add_rmsnorm_kernel<TO, N, 4, 1024, 1><<<num_out, 1024, 0, stream>>>(residual, s, weight, eps, rows, out, hidden);
+  else scaled_add_rmsnorm_kernel<TO, N, 4, 256, 3><<<num_out, 256, 0, stream>>>(residual, s, weight, eps, rows, out, hidden);
 }
 
 // y, y_code, y_planes, scale: `count` entries each; all planes [P, T, H] lie `plane_stride` elements apart
 extern "C" int qrt_scaled_add_rmsnorm(float* residual, const void* const* y, const int* y_code, const int* y_planes,
                                       const float* const* scale, int count, const float* vector, long plane_stride,
-                                      const float* weight, float eps, const int* rows, void* out, int out_dtype, int num_out, int hidden,
-                                      hipStream_t stream) {
+                                      const float* weight, float eps, const int* rows, void* out, int out_dtype, int num_out,
+                                      int hidden, hipStream_t stream) {
   QRT_CHECK(num_out >= 0 && hidden > 0 && count >= (vector ? 0 : 1) && count <= SA_TERMS, "scaled_add_rmsnorm: %d terms (1..%d)", count, SA_TERMS);
   ScaledTerms s;
   s.count = count;
   s.vector = vector;
+  bool vec4 = hidden % 4 == 0 && plane_stride % 4 == 0 && (uintptr_t)residual % 16 == 0 && (uintptr_t)weight % 16 == 0 &&
+              (uintptr_t)out % 16 == 0 && (uintptr_t)vector % 16 == 0;
   for (int k = 0; k < SA_TERMS; ++k) {
     if (count == 0) {
       s.y[k] = Planes{nullptr, QRT_F32, 1, 0};
@@ -306,14 +384,15 @@ extern "C" int qrt_scaled_add_rmsnorm(float* residual, const void* const* y, con
     QRT_CHECK(y_code[kk] == QRT_F32 || (y_code[kk] == QRT_BF16 && y_planes[kk] == 1), "scaled_add_rmsnorm: planes are float32");
     s.y[k] = Planes{y[kk], y_code[kk], y_planes[kk], plane_stride};
     s.scale[k] = scale[kk];
+    vec4 = vec4 && (uintptr_t)y[kk] % 16 == 0 && (uintptr_t)scale[kk] % 16 == 0;
   }
   if (num_out == 0) return 0;
   QRT_CHECK(out_dtype == QRT_F32 || out_dtype == QRT_BF16, "scaled_add_rmsnorm: unknown dtype %d", out_dtype);
-#define SA_LAUNCH(N)                                                                                                          \
-  if (out_dtype == QRT_F32)                                                                                                   \
-    scaled_add_rmsnorm_kernel<float, N><<<num_out, 1024, 0, stream>>>(residual, s, weight, eps, rows, (float*)out, hidden);   \
-  else                                                                                                                        \
-    scaled_add_rmsnorm_kernel<bf16_t, N><<<num_out, 1024, 0, stream>>>(residual, s, weight, eps, rows, (bf16_t*)out, hidden)
+#define SA_LAUNCH(N)                                                                                                               \
+  if (out_dtype == QRT_F32)                                                                                                        \
+    scaled_add_rmsnorm_launch<float, N>(residual, s, weight, eps, rows, (float*)out, num_out, hidden, vec4, stream);               \
+  else                                                                                                                             \
+    scaled_add_rmsnorm_launch<bf16_t, N>(residual, s, weight, eps, rows, (bf16_t*)out, num_out, hidden, vec4, stream)
   if (count == 0) { SA_LAUNCH(0); }
   else if (count == 1) { SA_LAUNCH(1); }
   else if (count == 2) { SA_LAUNCH(2); }

@@ -24,39 +24,58 @@ struct GatesArgs {
   int heads;
 };
 
-__device__ __forceinline__ double shift_up(double x, int by) { return __shfl_up(x, by, 64); }
-
-__global__ __launch_bounds__(256) void memory_gates_kernel(GatesArgs a) {
-  const int lane = threadIdx.x & 63, head = blockIdx.x * 4 + uniform_wave_number(), seq = blockIdx.y;
-  if (head >= a.heads) return;  // the whole wave
+// A block of W waves: a head each (W = 4, spans of up to 64 tokens), or one head whose tiles of 64 tokens
+// the waves take side by side (W = 16): what a tile does to the maximum before it is one pair of numbers,
+// m -> F + max(m, u) with the tile's sum and its largest i_s - F_s, so every wave finds the maximum before its
+// own tile from the pairs of the tiles before, in their order. Spans of one token need no scan.
+template <int W>
+__global__ __launch_bounds__(64 * W) void memory_gates_kernel(GatesArgs a) {
+  __shared__ double tile_sum[16], tile_max[16];
+  constexpr bool SPREAD = W == 16;
+  const int lane = threadIdx.x & 63, wave = uniform_wave_number(), seq = blockIdx.y;
+  const int head = SPREAD ? blockIdx.x : blockIdx.x * W + wave;
+  if (head >= a.heads) return;  // the whole wave; with one head a block, never
   const int t0 = a.cu_q[seq], t1 = a.cu_q[seq + 1];
+  if (t0 >= t1) return;
   float* top = a.top + (size_t)a.state_slots[seq] * a.heads + head;
   const float bi = a.bias[head], bf = a.bias[a.heads + head];
   float m = *top;
-  float zi = 0.f, zf = 0.f;
-  auto fetch = [&](int base) {
-    const float* row = a.logits + (size_t)min(base + lane, t1 - 1) * 2 * a.heads;
-    zi = row[head];
-    zf = row[a.heads + head];
-  };
-  if (t0 < t1) fetch(t0);
-  for (int base = t0; base < t1; base += 64) {
-    const int t = base + lane;
+  // the lane that has a tile's sum and maximum: lanes behind the last token carry them on
+  const int last = t1 - t0 > 1 ? 63 : 0;
+  for (int base = t0; base < t1; base += SPREAD ? 1024 : 64) {
+    const int t = base + lane + (SPREAD ? 64 * wave : 0);
     const bool ok = t < t1;
-    const float li = a.cap * tanhf((zi + bi) / a.cap), c = a.cap * tanhf((zf + bf) / a.cap);
+    const float* row = a.logits + (size_t)min(t, t1 - 1) * 2 * a.heads;
+    const float li = a.cap * tanhf((row[head] + bi) / a.cap), c = a.cap * tanhf((row[a.heads + head] + bf) / a.cap);
     const float lf = fminf(c, 0.f) - log1pf(expf(-fabsf(c)));
-    if (base + 64 < t1) fetch(base + 64);
     double F = ok ? (double)lf : 0.0;
-#pragma unroll
-    for (int o = 1; o < 64; o <<= 1) {
-      const double before = shift_up(F, o);
-      if (lane >= o) F += before;
-    }
     double u = ok ? (double)li - F : -INFINITY;
+    if (t1 - t0 > 1) {
 #pragma unroll
-    for (int o = 1; o < 64; o <<= 1) {
-      const double before = shift_up(u, o);
-      if (lane >= o) u = fmax(u, before);
+      for (int o = 1; o < 64; o <<= 1) {
+        const double before = __shfl_up(F, o, 64);
+        if (lane >= o) F += before;
+      }
+      u = ok ? (double)li - F : -INFINITY;
+#pragma unroll
+      for (int o = 1; o < 64; o <<= 1) {
+        const double before = __shfl_up(u, o, 64);
+        if (lane >= o) u = fmax(u, before);
+      }
+    }
+    float next = 0.f;  // the maximum behind this round's tokens
+    if (SPREAD) {
+      if (lane == last) {
+        tile_sum[wave] = F;
+        tile_max[wave] = u;
+      }
+      __syncthreads();
+      float run = m;
+      for (int j = 0; j < 16; ++j) {
+        if (j == wave) m = run;
+        run = (float)(tile_sum[j] + fmax((double)run, tile_max[j]));
+      }
+      next = run;
     }
     const float mt = (float)(F + fmax((double)m, u));
     float mp = __shfl_up(mt, 1, 64);
@@ -67,17 +86,20 @@ __global__ __launch_bounds__(256) void memory_gates_kernel(GatesArgs a) {
       o[a.heads] = li - mt;
       o[2 * a.heads] = mt;
     }
-    m = __shfl(mt, min(63, t1 - 1 - base), 64);
+    m = SPREAD ? next : __shfl(mt, last, 64);
+    if (SPREAD) __syncthreads();             // the pairs have been read
   }
-  if (lane == 0 && t0 < t1) *top = m;
+  if (lane == 0 && (!SPREAD || wave == 0)) *top = m;
 }
 
+// max_span: the most tokens a sequence has in this step
 extern "C" int qrt_memory_gates(const float* logits, const float* bias, float cap, float* top, float* out, const int* cu_q,
-                                const int* state_slots, int heads, int num_tokens, int num_seqs, hipStream_t stream) {
+                                const int* state_slots, int heads, int num_tokens, int num_seqs, int max_span, hipStream_t stream) {
   QRT_CHECK(heads > 0 && cap > 0.f && num_tokens >= 0 && num_seqs >= 0 && num_seqs <= 65535, "memory_gates: bad sizes");
   if (num_tokens == 0 || num_seqs == 0) return 0;
   const GatesArgs a{logits, bias, cap, top, out, cu_q, state_slots, heads};
-  memory_gates_kernel<<<dim3((heads + 3) / 4, num_seqs), 256, 0, stream>>>(a);
+  if (max_span > 64) memory_gates_kernel<16><<<dim3(heads, num_seqs), 1024, 0, stream>>>(a);
+  else memory_gates_kernel<4><<<dim3((heads + 3) / 4, num_seqs), 256, 0, stream>>>(a);
   QRT_LAUNCH_CHECK("memory_gates");
   return 0;
 }

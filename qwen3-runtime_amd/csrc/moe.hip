@@ -65,11 +65,28 @@ __global__ __launch_bounds__(1024) void route_top_kernel(const T* __restrict__ x
                                                          float weight_scale, float* __restrict__ gate) {
   __shared__ float logit[MAX_EXPERTS];
   __shared__ float score[MAX_EXPERTS];
+  __shared__ float gate_part[16];
   const int t = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const T* xr = x + (size_t)t * hidden;
   const bool wide = hidden % 4 == 0;
-  // with `gate` the router has one more row, no expert: the sigmoid of its product is the token's gate
-  for (int e = wave; e < experts + (gate ? 1 : 0); e += 16) {
+  // with `gate` the router has one more row, no expert: the sigmoid of its product is the token's gate. The
+  // block's threads share that row, on their way beside the waves' own rows
+  float gate_acc = 0.f;
+  if (gate) {
+    const float* wr = router + (size_t)experts * hidden;
+    if (wide) {
+      typedef T xvec_t __attribute__((ext_vector_type(4)));
+      for (int c = threadIdx.x * 4; c < hidden; c += 4096) {
+        const f32x4_t wv = *(const f32x4_t*)(wr + c);
+        const xvec_t xv = *(const xvec_t*)(xr + c);
+#pragma unroll
+        for (int k = 0; k < 4; ++k) gate_acc = fmaf(to_f32<T>(xv[k]), wv[k], gate_acc);
+      }
+    } else {
+      for (int c = threadIdx.x; c < hidden; c += 1024) gate_acc = fmaf(to_f32<T>(xr[c]), wr[c], gate_acc);
+    }
+  }
+  for (int e = wave; e < experts; e += 16) {
     const float* wr = router + (size_t)e * hidden;
     float acc = 0.f;
     if (wide) {
@@ -85,12 +102,18 @@ __global__ __launch_bounds__(1024) void route_top_kernel(const T* __restrict__ x
       for (int c = lane; c < hidden; c += 64) acc = fmaf(to_f32<T>(xr[c]), wr[c], acc);
     }
     const float z = wave_sum(acc);
-    if (lane == 0) {
-      if (e < experts) logit[e] = z + (bias ? bias[e] : 0.f);
-      else gate[t] = 1.0f / (1.0f + expf(-z));
-    }
+    if (lane == 0) logit[e] = z + (bias ? bias[e] : 0.f);
+  }
+  if (gate) {
+    gate_acc = wave_sum(gate_acc);
+    if (lane == 0) gate_part[wave] = gate_acc;
   }
   __syncthreads();
+  if (gate && threadIdx.x == 64) {
+    float z = 0.f;
+    for (int i = 0; i < 16; ++i) z += gate_part[i];
+    gate[t] = 1.0f / (1.0f + expf(-z));
+  }
   if (wave != 0) return;
   if (sigmoid_scores == 1) {
     // scores sigmoid(z) take the logits' place: the choice goes by them, and they are the weights

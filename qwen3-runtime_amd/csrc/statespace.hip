@@ -1,4 +1,4 @@
-// The state-space recurrence over spans of many tokens, chunk by chunk on MFMA, for bfloat16 inputs.
+// The state-space and matrix-memory recurrences over spans of many tokens, chunk by chunk on MFMA, for bfloat16 inputs.
 //
 //   D_t = softplus(step_t + bias), a_t = exp(-exp(a_log) D_t)
 //   S <- a_t S + D_t x_t B_t^T;   y_t = S C_t + skip x_t            (S [P, N] per sequence and head)
@@ -16,6 +16,12 @@
 // overflows however fast a head forgets. The recurrence written out token by token is in retention.hip;
 // the two differ by the rounding of float32 sums.
 //
+// Matrix memory (GATES) is the same recurrence with other names: values x, keys B, queries C (a head's
+// own), no skip, and per token and head the logarithms of what it keeps of the state (in place of a's) and
+// of what its write weighs (in place of D's). Its state has one more row, the sum of the weighted keys n; its
+// read-out n . q is the brackets' sum over s plus what is left of n_0 . q, both of which the block has at
+// hand, so the blocks of a head's first channels keep n in float32 beside their tiles, a thread an element.
+//
 // A block of four waves owns one head of one sequence and 64 of its P channels, and walks the span's
 // chunks in order with the state in registers: wave w holds channels 16 w .. 16 w + 15, S transposed as
 // the accumulator tiles of the update (tile i: rows n = 16 i + 4 quad + r, column p = lane & 15), which
@@ -30,15 +36,18 @@
 #include <math.h>
 
 struct SpaceArgs {
-  const bf16_t* xbc;         // [T, channels]: x heads | B groups | C groups
+  const bf16_t* xbc;         // [T, channels]: x heads, B groups and C groups from the columns below on
   int channels;
+  int x_first, b_first, c_first;
   const void* step; long step_stride; int step_code;   // [T, heads] step logits
   const float* step_bias; const float* a_log; const float* skip;  // [heads]
-  float* state;              // [slots, heads, P, N]
+  float* state;              // [slots, heads, P, N]; GATES: [slots, heads, P + 1, N]
   float* out;                // [T, heads, P]
   const int* cu_q; const int* state_slots;
   const int* seq_ids;        // the sequences of this launch; null: all of the step's
   int heads, groups, n, p;
+  const float* gates;        // [T, 3, heads]: log keep, log write (a third row is not read); null: step sizes
+  float* last_out;           // [T, heads]: n . q (GATES)
 };
 
 constexpr int CHUNK = 64;
@@ -81,7 +90,7 @@ __device__ __forceinline__ float wave_running_sum(float x) {
 }
 
 // KS steps of 32 state elements (N padded with zeros)
-template <int KS>
+template <int KS, bool GATES>
 __global__ __launch_bounds__(256, 1) void state_space_chunk_kernel(SpaceArgs a) {
   constexpr int NP = 32 * KS, BROW = NP + 16;
   constexpr int B_TASKS = 32 * KS, TASKS = B_TASKS + 64;     // 8 x 8 pieces of B and of x
@@ -96,6 +105,7 @@ __global__ __launch_bounds__(256, 1) void state_space_chunk_kernel(SpaceArgs a) 
   float* acs = dts + CHUNK;                // [64] base-2 logarithms of the decay since the chunk's start, the token's own included
   float* since = acs + CHUNK;              // [64] 2^acs: what is left of the state before the chunk
   float* left = since + CHUNK;             // [64] step size times what is left of the token's write at the chunk's end
+  float* nvec = left + CHUNK;              // [NP] the sum of the weighted keys before the chunk (GATES)
 
   const int tid = threadIdx.x, lane = tid & 63, wave = uniform_wave_number();
   const int r16 = lane & 15, quad = lane >> 4;
@@ -104,13 +114,22 @@ __global__ __launch_bounds__(256, 1) void state_space_chunk_kernel(SpaceArgs a) 
   const int t0 = a.cu_q[seq], t1 = a.cu_q[seq + 1];
   if (t1 <= t0) return;
   const int N = a.n, P = a.p, group = head / (a.heads / a.groups);
-  const int x_col = head * P + p0, b_col = a.heads * P + group * N, c_col = b_col + a.groups * N;
-  const float rate = expf(a.a_log[head]) * 1.4426950408889634f, bias = a.step_bias[head], skip = a.skip[head];
+  const int x_col = a.x_first + head * P + p0, b_col = a.b_first + group * N, c_col = a.c_first + group * N;
+  const float rate = GATES ? 0.f : expf(a.a_log[head]) * 1.4426950408889634f, bias = GATES ? 0.f : a.step_bias[head];
+  const float skip = GATES ? 0.f : a.skip[head];
+  const int state_rows = GATES ? P + 1 : P;
+  const bool has_n = GATES && blockIdx.y == 0;  // the same for the block
   const bool has_tile = p0 + 16 * wave < P;   // the same for the whole wave
   const int my_p = p0 + 16 * wave + r16;
   const bool p_ok = my_p < P;
 
-  float* st = a.state + (((size_t)a.state_slots[seq] * a.heads + head) * P + (p_ok ? my_p : 0)) * N;
+  float* st = a.state + (((size_t)a.state_slots[seq] * a.heads + head) * state_rows + (p_ok ? my_p : 0)) * N;
+  float* st_n = a.state + (((size_t)a.state_slots[seq] * a.heads + head) * state_rows + P) * N;  // GATES
+  float own_n = 0.f;
+  if (has_n) {
+    if (tid < N) own_n = st_n[tid];
+    if (tid < NP) nvec[tid] = own_n;
+  }
   f32x4_t S[2 * KS];
 #pragma unroll
   for (int i = 0; i < 2 * KS; ++i) {
@@ -119,7 +138,7 @@ __global__ __launch_bounds__(256, 1) void state_space_chunk_kernel(SpaceArgs a) 
   }
 
   bf16x8_t pre[R][8], pre_b[KS], pre_c[KS];
-  float pre_step = 0.f;
+  float pre_step = 0.f, pre_write = 0.f;
   const bool padded = N < NP || p0 + 64 > P;   // some pieces lie outside the state: zeros (the same for the block)
   // piece `task`: of B (tokens 8 sg .., channels 8 cg ..) or of x
   auto where = [&](int task, int& sg, int& cg, bool& is_b, bool& ok) {
@@ -174,7 +193,12 @@ __global__ __launch_bounds__(256, 1) void state_space_chunk_kernel(SpaceArgs a) 
         pre_c[k] = *(const bf16x8_t*)(base + at_row[k] + back + c_col);
       }
     }
-    if (tid < CHUNK) {
+    if (GATES && tid < CHUNK) {
+      const float* row = a.gates + (size_t)min(c0 + tid, t1 - 1) * 3 * a.heads + head;
+      pre_step = row[0];
+      pre_write = row[a.heads];
+    }
+    if (!GATES && tid < CHUNK) {
       const size_t at = (size_t)min(c0 + tid, t1 - 1) * a.step_stride + head;
       pre_step = a.step_code == QRT_F32 ? ((const float*)a.step)[at] : (float)((const bf16_t*)a.step)[at];
     }
@@ -212,9 +236,16 @@ __global__ __launch_bounds__(256, 1) void state_space_chunk_kernel(SpaceArgs a) 
       *(bf16x8_t*)(crow + row * BROW + 8 * cg) = pre_c[k];
     }
     if (wave == 0) {
-      const float z = pre_step + bias;
-      const float d = c0 + lane < t1 ? (z > 20.f ? z : log1pf(expf(z))) : 0.f;
-      const float v = wave_running_sum(-rate * d);
+      float d, log_keep;  // what the token's write weighs; the base-2 logarithm of what it keeps of the state
+      if (GATES) {
+        d = c0 + lane < t1 ? expf(pre_write) : 0.f;
+        log_keep = c0 + lane < t1 ? pre_step * 1.4426950408889634f : 0.f;
+      } else {
+        const float z = pre_step + bias;
+        d = c0 + lane < t1 ? (z > 20.f ? z : log1pf(expf(z))) : 0.f;
+        log_keep = -rate * d;
+      }
+      const float v = wave_running_sum(log_keep);
       dts[lane] = d;
       acs[lane] = v;
       since[lane] = __builtin_amdgcn_exp2f(v);
@@ -231,6 +262,7 @@ __global__ __launch_bounds__(256, 1) void state_space_chunk_kernel(SpaceArgs a) 
       // the bracket: rows t = 16 wave + r16, keys 32 kb + 8 quad + e
       const int t = 16 * wave + r16;
       const float lt = acs[t];
+      float n_read = 0.f, row_sum = 0.f;  // this lane's share of n_0 . q_t and of the row's bracket
       for (int kb = 0; kb <= (wave >> 1); ++kb) {
         // everything the rows need from LDS is asked for before the first product
         bf16x8_t kk[2][KS], cc[KS];
@@ -247,6 +279,17 @@ __global__ __launch_bounds__(256, 1) void state_space_chunk_kernel(SpaceArgs a) 
           ls[s2] = *(const f32x4_t*)(acs + 32 * kb + 8 * quad + 4 * s2);
           dd[s2] = *(const f32x4_t*)(dts + 32 * kb + 8 * quad + 4 * s2);
         }
+        if (has_n && kb == 0) {
+#pragma unroll
+          for (int j = 0; j < KS; ++j) {
+            const f32x4_t n0 = *(const f32x4_t*)(nvec + 32 * j + 8 * quad), n1 = *(const f32x4_t*)(nvec + 32 * j + 8 * quad + 4);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+              n_read = fmaf(n0[e], (float)cc[j][e], n_read);
+              n_read = fmaf(n1[e], (float)cc[j][e + 4], n_read);
+            }
+          }
+        }
         f32x4_t sc[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
 #pragma unroll
         for (int j = 0; j < KS; ++j)
@@ -258,7 +301,8 @@ __global__ __launch_bounds__(256, 1) void state_space_chunk_kernel(SpaceArgs a) 
           const int s = 32 * kb + 8 * quad + e;
           // keys after the row's token: the exponent is held at 0 (so that nothing overflows) and the weight is 0
           const float w = __builtin_amdgcn_exp2f(fminf(lt - ls[e >> 2][e & 3], 0.f)) * dd[e >> 2][e & 3];
-          m[e] = sc[e >> 2][e & 3] * (s <= t ? w : 0.f) + (s == t ? skip : 0.f);
+          m[e] = sc[e >> 2][e & 3] * (s <= t ? w : 0.f) + (!GATES && s == t ? skip : 0.f);
+          if (GATES) row_sum += m[e];
         }
         bf16x8_t terms[READ_TERMS];
         split_terms<READ_TERMS>(m, terms);
@@ -266,8 +310,29 @@ __global__ __launch_bounds__(256, 1) void state_space_chunk_kernel(SpaceArgs a) 
 #pragma unroll
         for (int k = 0; k < READ_TERMS; ++k) *(bf16x8_t*)(pm + ((combo * READ_TERMS + k) * 64 + lane) * 8) = terms[k];
       }
+      if (has_n) {
+        float q_n = fmaf(since[t], n_read, row_sum);
+        q_n += __shfl_xor(q_n, 16, 64);
+        q_n += __shfl_xor(q_n, 32, 64);
+        if (quad == 0 && c0 + t < t1) a.last_out[(size_t)(c0 + t) * a.heads + head] = q_n;
+      }
     }
     __syncthreads();
+    if (has_n && tid < NP) {  // the sum of the weighted keys moves on: nobody reads nvec before the next barrier
+      float acc = 0.f;
+#pragma unroll
+      for (int sg = 0; sg < CHUNK / 8; ++sg) {
+        const bf16x8_t kv = *(const bf16x8_t*)(bt + tid * TROW + 8 * sg);
+        const f32x4_t l0 = *(const f32x4_t*)(left + 8 * sg), l1 = *(const f32x4_t*)(left + 8 * sg + 4);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          acc = fmaf(l0[e], (float)kv[e], acc);
+          acc = fmaf(l1[e], (float)kv[e + 4], acc);
+        }
+      }
+      own_n = fmaf(since[CHUNK - 1], own_n, acc);
+      nvec[tid] = own_n;
+    }
     if (has_tile) {
       bf16x8_t sterm[KS][READ_TERMS], xa[2];
 #pragma unroll
@@ -349,6 +414,7 @@ __global__ __launch_bounds__(256, 1) void state_space_chunk_kernel(SpaceArgs a) 
     }
     __syncthreads();  // the next chunk takes the same LDS
   }
+  if (has_n && tid < N) st_n[tid] = own_n;
   if (p_ok) {
 #pragma unroll
     for (int i = 0; i < 2 * KS; ++i) {
@@ -358,18 +424,18 @@ __global__ __launch_bounds__(256, 1) void state_space_chunk_kernel(SpaceArgs a) 
   }
 }
 
-template <int KS>
+template <int KS, bool GATES>
 static int space_launch(const SpaceArgs& a, int num_seqs, hipStream_t stream) {
   constexpr int NP = 32 * KS, BROW = NP + 16;
-  constexpr size_t smem = (size_t)(2 * CHUNK * BROW + NP * TROW + CHUNK * TROW + 6 * READ_TERMS * 512) * sizeof(bf16_t) + 4 * CHUNK * sizeof(float);
+  constexpr size_t smem = (size_t)(2 * CHUNK * BROW + NP * TROW + CHUNK * TROW + 6 * READ_TERMS * 512) * sizeof(bf16_t) + (4 * CHUNK + (GATES ? NP : 0)) * sizeof(float);
   static_assert(smem <= 160 * 1024, "the chunk does not fit a compute unit's LDS");
   static bool allowed = smem <= 64 * 1024;  // once: not again inside every stream capture
   if (!allowed) {
-    if (hipFuncSetAttribute((const void*)state_space_chunk_kernel<KS>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem) != hipSuccess)
+    if (hipFuncSetAttribute((const void*)state_space_chunk_kernel<KS, GATES>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem) != hipSuccess)
       return qrt_fail("state_space_chunks: cannot get %zu bytes of LDS", smem);
     allowed = true;
   }
-  state_space_chunk_kernel<KS><<<dim3(a.heads, (a.p + 63) / 64, num_seqs), 256, smem, stream>>>(a);
+  state_space_chunk_kernel<KS, GATES><<<dim3(a.heads, (a.p + 63) / 64, num_seqs), 256, smem, stream>>>(a);
   return 0;
 }
 
@@ -379,16 +445,21 @@ extern "C" int qrt_state_space_chunks(const SpaceArgs* args, int num_seqs, hipSt
   QRT_CHECK(a.heads > 0 && a.groups > 0 && a.heads % a.groups == 0, "state_space_chunks: %d heads in %d groups", a.heads, a.groups);
   QRT_CHECK(a.n >= 8 && a.n <= 256 && a.n % 8 == 0 && a.p >= 8 && a.p % 8 == 0,
             "state_space_chunks: a state of %d x %d (multiples of 8, the first up to 256)", a.n, a.p);
-  QRT_CHECK(a.channels == a.heads * a.p + 2 * a.groups * a.n, "state_space_chunks: %d channels", a.channels);
+  QRT_CHECK(a.channels % 8 == 0 && a.x_first % 8 == 0 && a.b_first % 8 == 0 && a.c_first % 8 == 0 && a.x_first >= 0 &&
+                a.b_first >= 0 && a.c_first >= 0 && a.x_first + a.heads * a.p <= a.channels &&
+                a.b_first + a.groups * a.n <= a.channels && a.c_first + a.groups * a.n <= a.channels,
+            "state_space_chunks: rows of %d channels, the three parts from %d, %d and %d on", a.channels, a.x_first, a.b_first, a.c_first);
   QRT_CHECK((uintptr_t)a.xbc % 16 == 0 && (uintptr_t)a.state % 16 == 0 && (uintptr_t)a.out % 16 == 0, "state_space_chunks: not aligned to 16 bytes");
-  QRT_CHECK(a.step && a.step_bias && a.a_log && a.skip && a.step_stride >= a.heads, "state_space_chunks: no step logits, bias, rate or skip");
+  QRT_CHECK(a.gates ? a.last_out != nullptr : a.step && a.step_bias && a.a_log && a.skip && a.step_stride >= a.heads, "state_space_chunks: no step logits, bias, rate or skip");
   QRT_CHECK(num_seqs >= 0 && num_seqs <= 65535, "state_space_chunks: %d sequences", num_seqs);
   if (num_seqs == 0) return 0;
   int rc;
-  if (a.n <= 32) rc = space_launch<1>(a, num_seqs, stream);
-  else if (a.n <= 64) rc = space_launch<2>(a, num_seqs, stream);
-  else if (a.n <= 128) rc = space_launch<4>(a, num_seqs, stream);
-  else rc = space_launch<8>(a, num_seqs, stream);
+#define GO(KS) rc = a.gates ? space_launch<KS, true>(a, num_seqs, stream) : space_launch<KS, false>(a, num_seqs, stream)
+  if (a.n <= 32) GO(1);
+  else if (a.n <= 64) GO(2);
+  else if (a.n <= 128) GO(4);
+  else GO(8);
+#undef GO
   if (rc != 0) return rc;
   QRT_LAUNCH_CHECK("state_space_chunks");
   return 0;

@@ -129,10 +129,10 @@ class _RetentionArgs(Structure):
 
 class _SpaceArgs(Structure):
     _fields_ = [
-        ("xbc", c_void_p), ("channels", c_int), ("step", c_void_p), ("step_stride", c_long), ("step_code", c_int),
+        ("xbc", c_void_p), ("channels", c_int), ("x_first", c_int), ("b_first", c_int), ("c_first", c_int), ("step", c_void_p), ("step_stride", c_long), ("step_code", c_int),
         ("step_bias", c_void_p), ("a_log", c_void_p), ("skip", c_void_p), ("state", c_void_p), ("out", c_void_p),
         ("cu_q", c_void_p), ("state_slots", c_void_p), ("seq_ids", c_void_p),
-        ("heads", c_int), ("groups", c_int), ("n", c_int), ("p", c_int),
+        ("heads", c_int), ("groups", c_int), ("n", c_int), ("p", c_int), ("gates", c_void_p), ("last_out", c_void_p),
     ]
 
 
@@ -596,6 +596,7 @@ class HipOps:
             b.xbc, b.channels, b.step, b.step_stride, b.step_code = xbc.data_ptr(), c, step.data_ptr(), step.stride(0), _CODE[step.dtype]
             b.state, b.out, b.cu_q, b.state_slots, b.seq_ids = state.data_ptr(), out.data_ptr(), cu_q, slots, _addr(chunked)
             b.heads, b.groups, b.n, b.p = heads, groups, n, vdim
+            b.x_first, b.b_first, b.c_first = 0, heads * vdim, heads * vdim + groups * n
             for name, ptr in consts.items():
                 setattr(b, name, ptr)
             self._check(self.lib, self.lib.qrt_state_space_chunks(byref(b), c_int(num_chunked), _stream()))
@@ -625,13 +626,16 @@ class HipOps:
         _need(ctx.state_slots, "state_slots", torch.int32, (ctx.num_seqs,))
         out = torch.empty((t, 3, heads), dtype=torch.float32, device=logits.device)
         self._check(self.lib, self.lib.qrt_memory_gates(_ptr(logits), _ptr(bias), c_float(cap), _ptr(top), _ptr(out), _ptr(ctx.cu_q),
-                                                        _ptr(ctx.state_slots), c_int(heads), c_int(t), c_int(ctx.num_seqs), _stream()))
+                                                        _ptr(ctx.state_slots), c_int(heads), c_int(t), c_int(ctx.num_seqs),
+                                                        c_int(ctx.max_q_len), _stream()))
         return out
 
     def matrix_memory(self, ctx, y, gates, state, heads, dim, vdim):
         """``S <- keep S + write k [v | 1]^T; o = S^T q`` over each sequence's tokens from its slot's state (float32
         [slots, heads, vdim + 1, dim], updated in place). ``y`` [T, W]: its first columns are q | k | v; ``gates``
-        as ``memory_gates`` leaves them. Returns (o float32 [T, heads, vdim], the last column's [T, heads])."""
+        as ``memory_gates`` leaves them. Returns (o float32 [T, heads, vdim], the last column's [T, heads]). Float32
+        inputs, short spans and odd sizes go token by token; long spans of bfloat16 inputs chunk by chunk, in
+        a launch of their own beside the short ones of the same step."""
         t, w = y.shape
         c = 2 * heads * dim + heads * vdim
         _need(y, "q | k | v", shape=(ctx.num_tokens, w))
@@ -641,13 +645,24 @@ class HipOps:
         _need(gates, "gates", torch.float32, (t, 3, heads))
         out = torch.empty((t, heads, vdim), dtype=torch.float32, device=y.device)
         last = torch.empty((t, heads), dtype=torch.float32, device=y.device)
-        a = _RetentionArgs()
-        a.qkv, a.qkv_code, a.channels, a.q_first, a.k_first, a.v_first = y.data_ptr(), _CODE[y.dtype], w, 0, heads * dim, 2 * heads * dim
-        a.gates, a.last_out, a.state, a.out = gates.data_ptr(), last.data_ptr(), state.data_ptr(), out.data_ptr()
-        a.cu_q = _need(ctx.cu_q, "cu_q", torch.int32, (ctx.num_seqs + 1,)).data_ptr()
-        a.state_slots = _need(ctx.state_slots, "state_slots", torch.int32, (ctx.num_seqs,)).data_ptr()
-        a.heads, a.dim, a.vdim = heads, dim, vdim
-        self._check(self.lib, self.lib.qrt_retention(byref(a), c_int(t), c_int(ctx.num_seqs), c_int(state.shape[0]), _stream()))
+        cu_q = _need(ctx.cu_q, "cu_q", torch.int32, (ctx.num_seqs + 1,)).data_ptr()
+        slots = _need(ctx.state_slots, "state_slots", torch.int32, (ctx.num_seqs,)).data_ptr()
+        chunked, short, num_chunked, short_tokens = self._space_split(ctx, y, dim, vdim)
+        if num_chunked:
+            b = _SpaceArgs()
+            b.xbc, b.channels, b.x_first, b.b_first, b.c_first = y.data_ptr(), w, 2 * heads * dim, heads * dim, 0
+            b.gates, b.last_out, b.state, b.out = gates.data_ptr(), last.data_ptr(), state.data_ptr(), out.data_ptr()
+            b.cu_q, b.state_slots, b.seq_ids = cu_q, slots, _addr(chunked)
+            b.heads, b.groups, b.n, b.p = heads, heads, dim, vdim
+            self._check(self.lib, self.lib.qrt_state_space_chunks(byref(b), c_int(num_chunked), _stream()))
+        if num_chunked < ctx.num_seqs:
+            a = _RetentionArgs()
+            a.qkv, a.qkv_code, a.channels, a.q_first, a.k_first, a.v_first = y.data_ptr(), _CODE[y.dtype], w, 0, heads * dim, 2 * heads * dim
+            a.gates, a.last_out, a.state, a.out = gates.data_ptr(), last.data_ptr(), state.data_ptr(), out.data_ptr()
+            a.cu_q, a.state_slots, a.seq_ids = cu_q, slots, _addr(short)
+            a.heads, a.dim, a.vdim = heads, dim, vdim
+            self._check(self.lib, self.lib.qrt_retention(byref(a), c_int(short_tokens), c_int(ctx.num_seqs - num_chunked),
+                                                         c_int(state.shape[0]), _stream()))
         return out, last
 
     def memory_out(self, read, norm_read, gates, weight, out_gate, eps, q_scale, out_dtype):
