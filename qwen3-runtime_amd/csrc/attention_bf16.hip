@@ -1,5 +1,5 @@
 // Paged attention on MFMA for bfloat16, one head size per build (QRT_HEAD_DIM,
-// a multiple of 16). Serves prompt portions, single decoded tokens and batches
+// a multiple of 16; values of another size: QRT_VALUE_DIM, likewise). Serves prompt portions, single decoded tokens and batches
 // that mix both, with optional splitting of the keys across blocks.
 //
 // Rows. For one sequence and one key/value head the work is a matrix of
@@ -17,7 +17,7 @@
 // up with the scores of 8 consecutive keys for its row: exactly the B operand
 // (P^T) of the second product O^T = V^T P^T, whose A operand is then 8
 // consecutive keys of one head element: one 16-byte read from the value page,
-// which stores values transposed ([page, head, D, offset]). No data crosses
+// which stores values transposed ([page, head, DV, offset]). No data crosses
 // lanes except the row maximum and sum.
 //
 // Softmax is online, float32, in base 2 (scale * log2 e is folded into the
@@ -36,6 +36,12 @@
 #if QRT_HEAD_DIM % 16 != 0 || QRT_HEAD_DIM < 16 || QRT_HEAD_DIM > 512
 #error "QRT_HEAD_DIM must be a multiple of 16 between 16 and 512"
 #endif
+#ifndef QRT_VALUE_DIM
+#define QRT_VALUE_DIM QRT_HEAD_DIM
+#endif
+#if QRT_VALUE_DIM % 16 != 0 || QRT_VALUE_DIM < 16 || QRT_VALUE_DIM > 512
+#error "QRT_VALUE_DIM must be a multiple of 16 between 16 and 512"
+#endif
 
 
 // 8 head elements from ``p`` for the quads that hold real data, zeros for the others: a head
@@ -52,15 +58,15 @@ __device__ __forceinline__ bf16x8_t load_tail(const bf16_t* p, int quad) {
 
 struct AttnTileArgs {
   const bf16_t* q;        // [T, nq * D]
-  bf16_t* out;            // [T, nq * D]
+  bf16_t* out;            // [T, nq * DV]
   const bf16_t* k_cache;  // [pages, nkv, page_size, D]
-  const bf16_t* v_cache;  // [pages, nkv, D, page_size]
+  const bf16_t* v_cache;  // [pages, nkv, DV, page_size]
   const int* cu_q;        // [S + 1]
   const int* kv_lens;     // [S]
   const int* block_table; // [S, table_width]
   const int* tile_seq;    // [num_tiles]
   const int* tile_row0;   // [num_tiles]
-  float* part_o;          // [T, nq, num_splits, D]   (num_splits > 1)
+  float* part_o;          // [T, nq, num_splits, DV]   (num_splits > 1)
   float* part_lse;        // [T, nq, num_splits]      base-2 log of the split's sum, -inf if empty
   int table_width, num_tiles, nq, nkv, page_size, window, num_splits, waves;
   float scale_log2;
@@ -76,7 +82,7 @@ struct AttnTileArgs {
   // key heads itself, attends over the cache up to the token before, adds the token's own key
   // and value from registers, and stores them into the cache for the steps to come. `q` is
   // then unused.
-  const bf16_t* qkv;       // [T, qkv_stride]: nq query heads, nkv key heads, nkv value heads of D
+  const bf16_t* qkv;       // [T, qkv_stride]: nq query heads, nkv key heads, nkv value heads of DV
   long qkv_stride;
   const float* q_weight;   // [D] or null: no norm
   const float* k_weight;
@@ -94,7 +100,7 @@ struct AttnTileArgs {
   int chunk;               // > 0: a query sees the keys of its own chunk of this many positions (no window then)
   float cap_in, cap_out;   // score cap c > 0: cap_in = scale / c, cap_out = c / scale; 0: no cap
   // An output gate: the result at (token, head, element) is multiplied by the sigmoid of
-  // gate[token * gate_stride + head * D + element] (the gate's columns of the product that made
+  // gate[token * gate_stride + head * DV + element] (the gate's columns of the product that made
   // q, k and v, say). Applied where the output is written: here, or in the merge of key splits.
   const bf16_t* gate;
   long gate_stride;
@@ -108,8 +114,8 @@ struct AttnTileArgs {
   // p_j = exp(s_j) / (1 + sum exp(s_j)): added where the sums are final (here, or in the merge).
   int sink;
   int rope_pairs;          // with `rope`: pairs (j, j + rope_pairs) that turn, a multiple of 32 up to D / 2
-  // Turned values: [T, D], the cosines of a token's D / 2 angles, then their sines; null: values as they
-  // are. The cached values are turned by their own positions, element j against j + D / 2, and a row's
+  // Turned values: [T, DV], the cosines of a token's DV / 2 angles, then their sines; null: values as they
+  // are. The cached values are turned by their own positions, element j against j + DV / 2, and a row's
   // output is turned back by its token's angles where it is written (here, or in the merge).
   const float* turn;
 };
@@ -133,16 +139,18 @@ __device__ __forceinline__ void cap_scores(f32x4_t sc[2], float cap_in, float ca
   }
 }
 
-constexpr int D = QRT_HEAD_DIM;
+constexpr int D = QRT_HEAD_DIM;      // of queries and keys
+constexpr int DV = QRT_VALUE_DIM;    // of values and outputs
+constexpr int DMAX = D > DV ? D : DV;
 constexpr int KFULL = D / 32;        // 32-wide steps of the first product
 constexpr bool KTAIL = (D % 32) != 0;  // one 16-wide step more
-constexpr int DB = D / 16;           // 16-wide blocks of the head dimension
+constexpr int DB = DV / 16;          // 16-wide blocks of a value
 
 // sigmoid of the gate's element for output row `row` (= token * nq + head) and head element d; 1 without a gate
 __device__ __forceinline__ float gate_factor(const bf16_t* __restrict__ gate, long gate_stride, int nq, size_t row, int d) {
   if (!gate) return 1.0f;
   const size_t token = row / nq;
-  const float x = (float)gate[token * gate_stride + (row - token * nq) * D + d];
+  const float x = (float)gate[token * gate_stride + (row - token * nq) * DV + d];
   return 1.0f / (1.0f + __expf(-x));
 }
 
@@ -154,7 +162,7 @@ __device__ __forceinline__ void turn_back(f32x4_t* o, const float* __restrict__ 
   if constexpr (DB % 2 == 0) {
 #pragma unroll
     for (int i = 0; i < DB / 2; ++i) {
-      const f32x4_t c = *(const f32x4_t*)(angles + 16 * i + 4 * quad), s = *(const f32x4_t*)(angles + D / 2 + 16 * i + 4 * quad);
+      const f32x4_t c = *(const f32x4_t*)(angles + 16 * i + 4 * quad), s = *(const f32x4_t*)(angles + DV / 2 + 16 * i + 4 * quad);
       const f32x4_t u = o[i], v = o[i + DB / 2];
       o[i] = u * c + v * s;
       o[i + DB / 2] = v * c - u * s;
@@ -174,8 +182,8 @@ __device__ __forceinline__ void turn_back(f32x4_t* o, const float* __restrict__ 
       else if (i == H) p = upper ? across[0] : across[DB - 1];
       else p = upper ? across[i - H] : across[i - H - 1];
       const bool low = i < H || (i == H && !upper);
-      const int j = 16 * i + 4 * quad - (low ? 0 : D / 2);
-      const f32x4_t c = *(const f32x4_t*)(angles + j), s = *(const f32x4_t*)(angles + D / 2 + j);
+      const int j = 16 * i + 4 * quad - (low ? 0 : DV / 2);
+      const f32x4_t c = *(const f32x4_t*)(angles + j), s = *(const f32x4_t*)(angles + DV / 2 + j);
       o[i] = low ? o[i] * c + p * s : o[i] * c - p * s;
     }
   }
@@ -376,7 +384,7 @@ __device__ __forceinline__ void block_load(const AttnTileArgs& a, int kvh, int b
     if (KTAIL) blk.kt[kb] = load_tail(kp + 32 * KFULL, quad);
   }
   const int kv0 = min(max(base + 8 * quad, lo & ~7), pos_max & ~7);
-  const bf16_t* vp = live ? a.v_cache + (((size_t)pg[2] * a.nkv + kvh) * D + r16) * ps + page_mod<P2>(kv0, ps) : a.v_cache;
+  const bf16_t* vp = live ? a.v_cache + (((size_t)pg[2] * a.nkv + kvh) * DV + r16) * ps + page_mod<P2>(kv0, ps) : a.v_cache;
 #pragma unroll
   for (int i = 0; i < DB; ++i)
     blk.v[i] = ONCE ? load_once8(vp + (size_t)16 * i * ps) : *(const bf16x8_t*)(vp + (size_t)16 * i * ps);
@@ -439,7 +447,7 @@ __device__ __forceinline__ void add_sink(float& m, float& l_total, f32x4_t* o) {
 template <int RT, bool P2>
 // (Heads wider than 256: a wave's accumulator, queries and one block of keys and values fill most of
 // the 512 registers a lane can have, so one block of waves a compute unit and one tile a wave.)
-__global__ __launch_bounds__(256, (RT <= 2 && D <= 256) ? 2 : 1) void attention_bf16_kernel(AttnTileArgs a) {
+__global__ __launch_bounds__(256, (RT <= 2 && DMAX <= 256) ? 2 : 1) void attention_bf16_kernel(AttnTileArgs a) {
   const int lane = threadIdx.x & 63, wave = uniform_wave_number();
   const int r16 = lane & 15, quad = lane >> 4;
   // blocks of one tile are neighbours in the launch order, one per key head: with as many key
@@ -553,10 +561,10 @@ __global__ __launch_bounds__(256, (RT <= 2 && D <= 256) ? 2 : 1) void attention_
     lt += __shfl_xor(lt, 32, 64);
     if (!row_valid[t]) continue;
     if (a.sink && a.num_splits == 1) add_sink(m[t], lt, o[t]);
-    if (a.turn && a.num_splits == 1) turn_back(o[t], a.turn + row_index[t] / a.nq * D, quad);
+    if (a.turn && a.num_splits == 1) turn_back(o[t], a.turn + row_index[t] / a.nq * DV, quad);
     const float inv = lt > 0.f ? 1.0f / lt : 0.f;
     if (a.num_splits == 1) {
-      bf16_t* op = a.out + row_index[t] * D;
+      bf16_t* op = a.out + row_index[t] * DV;
 #pragma unroll
       for (int i = 0; i < DB; ++i) {
         bf16x4_t w;
@@ -566,7 +574,7 @@ __global__ __launch_bounds__(256, (RT <= 2 && D <= 256) ? 2 : 1) void attention_
         *(bf16x4_t*)(op + 16 * i + 4 * quad) = w;
       }
     } else {
-      float* op = a.part_o + (row_index[t] * a.num_splits + split) * D;
+      float* op = a.part_o + (row_index[t] * a.num_splits + split) * DV;
 #pragma unroll
       for (int i = 0; i < DB; ++i) {
         f32x4_t w = o[t][i] * inv;
@@ -645,7 +653,7 @@ __device__ __forceinline__ void tile_probabilities(const f32x4_t sc[2], float sc
 }
 
 constexpr int VROW = 48;                        // elements per value row (one head element, 32 keys) in LDS
-constexpr int STAGE_ELEMS = 32 * KROW + D * VROW;
+constexpr int STAGE_ELEMS = 32 * KROW + DV * VROW;
 
 //
 // G = 2: eight waves, two groups of four that both own the block's rows and take the blocks of
@@ -745,27 +753,24 @@ __global__ __launch_bounds__(256 * G, G == 1 ? 2 : 1) void attention_bf16_prefil
   // outside is masked with the scores or zeroed by a select): with loads under branches the
   // compiler can no longer count which are in flight and waits for all of them in the middle of
   // the products.
-  const size_t page_stride = (size_t)a.nkv * ps * D;  // elements per page, keys and values alike
+  const size_t k_stride = (size_t)a.nkv * ps * D, v_stride = (size_t)a.nkv * ps * DV;  // elements per page
   const bf16_t* k_head = a.k_cache + (size_t)kvh * ps * D;
-  const bf16_t* v_head = a.v_cache + (size_t)kvh * D * ps;
+  const bf16_t* v_head = a.v_cache + (size_t)kvh * DV * ps;
   const int w8 = 8 * wave;  // this wave's group within a block
-  constexpr int LANE_PIECES = (D + 63) / 64;   // 16-byte pieces per lane, of keys and of values
-  constexpr bool ALL_LANES = D % 64 == 0;
-  struct Pieces { bf16x8_t k[LANE_PIECES], v[LANE_PIECES]; };
+  constexpr int K_PIECES = (D + 63) / 64, V_PIECES = (DV + 63) / 64;   // 16-byte pieces per lane
+  struct Pieces { bf16x8_t k[K_PIECES], v[V_PIECES]; };
   Pieces set_a, set_b;  // two blocks of keys on their way: one asked for a round ago, one just now
   auto group_start = [&](int b) { return min(max((b << 5) + w8, lo & ~7), blk_pos_max & ~7); };
   auto lookup = [&](int b) { return table[page_div<P2>(group_start(b), ps, psh)]; };
   auto fetch = [&](int b, int page, Pieces& in) {  // global -> registers
     const int off = page_mod<P2>(group_start(b), ps);
-    const bf16_t* kp = k_head + (size_t)page * page_stride + (size_t)off * D;  // 8 keys: 8 D elements in a row
-    const bf16_t* vp = v_head + (size_t)page * page_stride + off;
+    const bf16_t* kp = k_head + (size_t)page * k_stride + (size_t)off * D;  // 8 keys: 8 D elements in a row
+    const bf16_t* vp = v_head + (size_t)page * v_stride + off;
 #pragma unroll
-    for (int i = 0; i < LANE_PIECES; ++i) {
+    for (int i = 0; i < (K_PIECES > V_PIECES ? K_PIECES : V_PIECES); ++i) {
       const int c = lane + 64 * i;
-      if (ALL_LANES || c < D) {
-        in.k[i] = *(const bf16x8_t*)(kp + 8 * c);
-        in.v[i] = *(const bf16x8_t*)(vp + (size_t)c * ps);
-      }
+      if (i < K_PIECES && (D % 64 == 0 || c < D)) in.k[i] = *(const bf16x8_t*)(kp + 8 * c);
+      if (i < V_PIECES && (DV % 64 == 0 || c < DV)) in.v[i] = *(const bf16x8_t*)(vp + (size_t)c * ps);
     }
   };
   auto stash = [&](int b, int stage, const Pieces& in) {  // registers -> LDS: block b into its stage
@@ -777,9 +782,9 @@ __global__ __launch_bounds__(256 * G, G == 1 ? 2 : 1) void attention_bf16_prefil
     const int g0 = (b << 5) + w8;
     const int keep = g0 + 7 >= lo ? blk_pos_max - g0 + 1 : 0;
 #pragma unroll
-    for (int i = 0; i < LANE_PIECES; ++i) {
+    for (int i = 0; i < (K_PIECES > V_PIECES ? K_PIECES : V_PIECES); ++i) {
       const int c = lane + 64 * i;
-      if (ALL_LANES || c < D) {
+      if (i < K_PIECES && (D % 64 == 0 || c < D)) {
         // keys: piece c of the group is key c / (D / 8) of it, elements 8 (c % (D / 8)) onward; row
         // 16 s2 + r16 of the stage holds the key that lane r16 of sub-block s2 multiplies (key
         // 8 q + 4 s2 + r of the block sits in row 16 s2 + 4 q + r), so that the 16 lanes of an
@@ -787,8 +792,8 @@ __global__ __launch_bounds__(256 * G, G == 1 ? 2 : 1) void attention_bf16_prefil
         const int kl = c / (D / 8), part = c - kl * (D / 8);
         const int row = 16 * (kl >> 2) + (w8 >> 1) + (kl & 3);
         *(bf16x8_t*)(kb + row * KROW + 8 * part) = in.k[i];
-        *(bf16x8_t*)(vb + c * VROW + w8) = keep_first(in.v[i], keep);
       }
+      if (i < V_PIECES && (DV % 64 == 0 || c < DV)) *(bf16x8_t*)(vb + c * VROW + w8) = keep_first(in.v[i], keep);
     }
   };
 
@@ -944,10 +949,10 @@ __global__ __launch_bounds__(256 * G, G == 1 ? 2 : 1) void attention_bf16_prefil
     lt += __shfl_xor(lt, 32, 64);
     if (!row_valid[t] || !wave_has_rows || grp != 0) continue;
     if (a.sink && a.num_splits == 1) add_sink(m[t], lt, o[t]);
-    if (a.turn && a.num_splits == 1) turn_back(o[t], a.turn + row_index[t] / a.nq * D, quad);
+    if (a.turn && a.num_splits == 1) turn_back(o[t], a.turn + row_index[t] / a.nq * DV, quad);
     const float inv = lt > 0.f ? 1.0f / lt : 0.f;
     if (a.num_splits == 1) {
-      bf16_t* op = a.out + row_index[t] * D;
+      bf16_t* op = a.out + row_index[t] * DV;
 #pragma unroll
       for (int i = 0; i < DB; ++i) {
         bf16x4_t w;
@@ -957,7 +962,7 @@ __global__ __launch_bounds__(256 * G, G == 1 ? 2 : 1) void attention_bf16_prefil
         *(bf16x4_t*)(op + 16 * i + 4 * quad) = w;
       }
     } else {
-      float* op = a.part_o + (row_index[t] * a.num_splits + split) * D;
+      float* op = a.part_o + (row_index[t] * a.num_splits + split) * DV;
 #pragma unroll
       for (int i = 0; i < DB; ++i) {
         f32x4_t w = o[t][i] * inv;
@@ -978,15 +983,15 @@ __device__ __forceinline__ void merge_few(const float* __restrict__ part_o, cons
                                           const bf16_t* __restrict__ gate, long gate_stride, int nq, int sink,
                                           const float* __restrict__ turn) {
   float ls[MAX], pv[2][MAX];
-  const int second = turn ? D / 2 : (int)blockDim.x;
-  const int d0 = min((int)threadIdx.x, D - 1), d1 = min((int)threadIdx.x + second, D - 1);
+  const int second = turn ? DV / 2 : (int)blockDim.x;
+  const int d0 = min((int)threadIdx.x, DV - 1), d1 = min((int)threadIdx.x + second, DV - 1);
   const float g0 = gate_factor(gate, gate_stride, nq, row, d0), g1 = gate_factor(gate, gate_stride, nq, row, d1);
 #pragma unroll
   for (int s = 0; s < MAX; ++s) {
     const int sc = min(s, num_splits - 1);
     ls[s] = lse[sc];
-    pv[0][s] = part_o[(row * num_splits + sc) * D + d0];
-    pv[1][s] = part_o[(row * num_splits + sc) * D + d1];
+    pv[0][s] = part_o[(row * num_splits + sc) * DV + d0];
+    pv[1][s] = part_o[(row * num_splits + sc) * DV + d1];
   }
   float mx = -INFINITY;
 #pragma unroll
@@ -1007,18 +1012,18 @@ __device__ __forceinline__ void merge_few(const float* __restrict__ part_o, cons
     }
   }
   if (turn) {
-    if ((int)threadIdx.x < D / 2) {
-      const float* angles = turn + row / nq * D + threadIdx.x;
-      const float c = angles[0], s = angles[D / 2], inv = wsum > 0.f ? 1.0f / wsum : 0.f;
+    if ((int)threadIdx.x < DV / 2) {
+      const float* angles = turn + row / nq * DV + threadIdx.x;
+      const float c = angles[0], s = angles[DV / 2], inv = wsum > 0.f ? 1.0f / wsum : 0.f;
       const float u = acc[0] * inv, v = acc[1] * inv;
-      out[row * D + threadIdx.x] = (bf16_t)((u * c + v * s) * g0);
-      out[row * D + threadIdx.x + D / 2] = (bf16_t)((v * c - u * s) * g1);
+      out[row * DV + threadIdx.x] = (bf16_t)((u * c + v * s) * g0);
+      out[row * DV + threadIdx.x + DV / 2] = (bf16_t)((v * c - u * s) * g1);
     }
     return;
   }
-  if ((int)threadIdx.x < D) out[row * D + threadIdx.x] = (bf16_t)(wsum > 0.f ? acc[0] / wsum * g0 : 0.f);
-  if ((int)(threadIdx.x + blockDim.x) < D)
-    out[row * D + threadIdx.x + blockDim.x] = (bf16_t)(wsum > 0.f ? acc[1] / wsum * g1 : 0.f);
+  if ((int)threadIdx.x < DV) out[row * DV + threadIdx.x] = (bf16_t)(wsum > 0.f ? acc[0] / wsum * g0 : 0.f);
+  if ((int)(threadIdx.x + blockDim.x) < DV)
+    out[row * DV + threadIdx.x + blockDim.x] = (bf16_t)(wsum > 0.f ? acc[1] / wsum * g1 : 0.f);
 }
 
 // out[row] = sum_s 2^(lse_s - M) O_s / sum_s 2^(lse_s - M); empty splits weigh 0
@@ -1030,7 +1035,7 @@ __global__ void attention_merge_kernel(const float* __restrict__ part_o, const f
   // rows are (token, query head); with a token list the grid walks the listed tokens' rows only
   const size_t row = tokens ? (size_t)tokens[blockIdx.x / nq] * nq + blockIdx.x % nq : blockIdx.x;
   const float* lse = part_lse + row * num_splits;
-  if (num_splits <= 64 && D <= 2 * (int)blockDim.x) {
+  if (num_splits <= 64 && DV <= 2 * (int)blockDim.x) {
     if (num_splits <= 8) merge_few<8>(part_o, lse, out, num_splits, row, gate, gate_stride, nq, sink, turn);
     else if (num_splits <= 16) merge_few<16>(part_o, lse, out, num_splits, row, gate, gate_stride, nq, sink, turn);
     else if (num_splits <= 32) merge_few<32>(part_o, lse, out, num_splits, row, gate, gate_stride, nq, sink, turn);
@@ -1043,27 +1048,27 @@ __global__ void attention_merge_kernel(const float* __restrict__ part_o, const f
   auto element = [&](int d) -> float {
     float acc = 0.f, wsum = sink ? exp2f(-mx) : 0.f;
     if (mx != -INFINITY) {
-      const float* po = part_o + row * num_splits * D + d;
+      const float* po = part_o + row * num_splits * DV + d;
 #pragma unroll 8
       for (int s = 0; s < num_splits; ++s) {
         const float w = exp2f(lse[s] - mx);
         wsum += w;
-        if (w > 0.f) acc += w * po[(size_t)s * D];
+        if (w > 0.f) acc += w * po[(size_t)s * DV];
       }
     }
     return wsum > 0.f ? acc / wsum : 0.f;
   };
   if (turn) {
-    for (int d = threadIdx.x; d < D / 2; d += blockDim.x) {
-      const float* angles = turn + row / nq * D + d;
-      const float c = angles[0], s = angles[D / 2], u = element(d), v = element(d + D / 2);
-      out[row * D + d] = (bf16_t)((u * c + v * s) * gate_factor(gate, gate_stride, nq, row, d));
-      out[row * D + d + D / 2] = (bf16_t)((v * c - u * s) * gate_factor(gate, gate_stride, nq, row, d + D / 2));
+    for (int d = threadIdx.x; d < DV / 2; d += blockDim.x) {
+      const float* angles = turn + row / nq * DV + d;
+      const float c = angles[0], s = angles[DV / 2], u = element(d), v = element(d + DV / 2);
+      out[row * DV + d] = (bf16_t)((u * c + v * s) * gate_factor(gate, gate_stride, nq, row, d));
+      out[row * DV + d + DV / 2] = (bf16_t)((v * c - u * s) * gate_factor(gate, gate_stride, nq, row, d + DV / 2));
     }
     return;
   }
-  for (int d = threadIdx.x; d < D; d += blockDim.x)
-    out[row * D + d] = (bf16_t)(element(d) * gate_factor(gate, gate_stride, nq, row, d));
+  for (int d = threadIdx.x; d < DV; d += blockDim.x)
+    out[row * DV + d] = (bf16_t)(element(d) * gate_factor(gate, gate_stride, nq, row, d));
 }
 
 // ------------------------------------------------------------------ decoding
@@ -1212,12 +1217,12 @@ __device__ __forceinline__ void head_as_operand(const bf16_t* __restrict__ x, co
 constexpr bool DECODE_ONCE = true;  // measured: 2 % off a decode step at batch 1 and at batch 64, level at batch 8
 
 template <bool P2, bool FUSED = false>
-__global__ __launch_bounds__(64 * DW, D <= 128 ? 2 : 1) void attention_bf16_decode_kernel(AttnTileArgs a) {
-  // per wave: maximum and sum per row, unnormalised accumulator [16][D]
+__global__ __launch_bounds__(64 * DW, DMAX <= 128 ? 2 : 1) void attention_bf16_decode_kernel(AttnTileArgs a) {
+  // per wave: maximum and sum per row, unnormalised accumulator [16][DV]
   extern __shared__ float lds[];
   float* lds_m = lds;                 // [DW][16]
   float* lds_l = lds + DW * 16;       // [DW][16]
-  float* lds_o = lds + 2 * DW * 16;   // [DW][16][D]
+  float* lds_o = lds + 2 * DW * 16;   // [DW][16][DV]
 
   const int lane = threadIdx.x & 63, wave = uniform_wave_number();
   const int r16 = lane & 15, quad = lane >> 4;
@@ -1279,33 +1284,33 @@ __global__ __launch_bounds__(64 * DW, D <= 128 ? 2 : 1) void attention_bf16_deco
   auto own_token = [&]() {
     const bf16_t* raw = a.qkv + (size_t)q_begin * a.qkv_stride;
     const float* rope = a.rope ? a.rope + (size_t)q_begin * 2 * a.rope_pairs : nullptr;
-    const float* turn = a.turn ? a.turn + (size_t)q_begin * D : nullptr;
+    const float* turn = a.turn ? a.turn + (size_t)q_begin * DV : nullptr;
     head_as_operand(raw + (size_t)head * D, a.q_weight, rope, a.rope_pairs, a.eps, quad, qreg);
     const bool at_end = split == last_split;
     const bool adds_own = at_end && wave == DW - 1, stores_own = at_end && wave == (2 * DW - 2) % DW;
     if (adds_own || stores_own) {  // uniform over the wave
       const bf16_t* kraw = raw + ((size_t)a.nq + kvh) * D;
-      const bf16_t* vraw = raw + ((size_t)a.nq + a.nkv + kvh) * D;
+      const bf16_t* vraw = raw + ((size_t)a.nq + a.nkv) * D + (size_t)kvh * DV;
       bf16x8_t kreg[KFULL > 0 ? KFULL : 1];
       head_as_operand(kraw, a.k_weight, rope, a.rope_pairs, a.eps, quad, kreg);
       // the token's own value, turned by its position where values are
       auto own_value = [&](int d) -> bf16_t {
         if (!turn) return vraw[d];
-        const bool low = d < D / 2;
-        const int j = low ? d : d - D / 2;
-        const float x = (float)vraw[d], y = (float)vraw[low ? d + D / 2 : j], c = turn[j], sn = turn[D / 2 + j];
+        const bool low = d < DV / 2;
+        const int j = low ? d : d - DV / 2;
+        const float x = (float)vraw[d], y = (float)vraw[low ? d + DV / 2 : j], c = turn[j], sn = turn[DV / 2 + j];
         return (bf16_t)(low ? x * c - y * sn : x * c + y * sn);
       };
       if (stores_own) {
         const int slot = a.slots[q_begin];
         const int page = slot / a.page_size, off = slot - page * a.page_size;
         bf16_t* kdst = (bf16_t*)a.k_cache + (((size_t)page * a.nkv + kvh) * a.page_size + off) * D;
-        bf16_t* vdst = (bf16_t*)a.v_cache + ((size_t)page * a.nkv + kvh) * D * a.page_size + off;
+        bf16_t* vdst = (bf16_t*)a.v_cache + ((size_t)page * a.nkv + kvh) * DV * a.page_size + off;
         if (r16 == 0) {
 #pragma unroll
           for (int i = 0; i < KFULL; ++i) *(bf16x8_t*)(kdst + 32 * i + 8 * quad) = kreg[i];
         }
-        for (int d = lane; d < D; d += 64) vdst[(size_t)d * a.page_size] = own_value(d);
+        for (int d = lane; d < DV; d += 64) vdst[(size_t)d * a.page_size] = own_value(d);
       }
       if (adds_own) {
         // a block of keys that holds this one key, in the place of key first_pos: operand row 0
@@ -1389,7 +1394,7 @@ __global__ __launch_bounds__(64 * DW, D <= 128 ? 2 : 1) void attention_bf16_deco
 #pragma unroll
   for (int i = 0; i < DB; ++i)
 #pragma unroll
-    for (int r = 0; r < 4; ++r) lds_o[(wave * 16 + r16) * D + 16 * i + 4 * quad + r] = o[i][r];
+    for (int r = 0; r < 4; ++r) lds_o[(wave * 16 + r16) * DV + 16 * i + 4 * quad + r] = o[i][r];
   __syncthreads();
 
   const size_t tile_row0 = (size_t)q_begin * a.nq;  // rows of this sequence start here, in units of heads
@@ -1406,37 +1411,37 @@ __global__ __launch_bounds__(64 * DW, D <= 128 ? 2 : 1) void attention_bf16_deco
 #pragma unroll
       for (int w = 0; w < DW; ++w) {
         const float f = exp2f(lds_m[w * 16 + row] - mm);
-        num += f * lds_o[(w * 16 + row) * D + d];
+        num += f * lds_o[(w * 16 + row) * DV + d];
         den += f * lds_l[w * 16 + row];
       }
     }
     return den > 0.f ? num / den : 0.f;
   };
   if (a.turn && a.num_splits == 1) {  // the two elements of a pair at a time, turned back
-    for (int idx = threadIdx.x; idx < n_rows * (D / 2); idx += 64 * DW) {
-      const int row = idx / (D / 2), d = idx - row * (D / 2);
+    for (int idx = threadIdx.x; idx < n_rows * (DV / 2); idx += 64 * DW) {
+      const int row = idx / (DV / 2), d = idx - row * (DV / 2);
       float mm, den;
-      const float u = joined(row, d, mm, den), v = joined(row, d + D / 2, mm, den);
+      const float u = joined(row, d, mm, den), v = joined(row, d + DV / 2, mm, den);
       const int rt = row / g, rh = row - rt * g;
       const size_t row_index = tile_row0 + (size_t)rt * a.nq + kvh * g + rh;
-      const float* angles = a.turn + (size_t)(q_begin + rt) * D + d;
-      const float c = angles[0], sn = angles[D / 2];
-      a.out[row_index * D + d] = (bf16_t)((u * c + v * sn) * gate_factor(a.gate, a.gate_stride, a.nq, row_index, d));
-      a.out[row_index * D + d + D / 2] = (bf16_t)((v * c - u * sn) * gate_factor(a.gate, a.gate_stride, a.nq, row_index, d + D / 2));
+      const float* angles = a.turn + (size_t)(q_begin + rt) * DV + d;
+      const float c = angles[0], sn = angles[DV / 2];
+      a.out[row_index * DV + d] = (bf16_t)((u * c + v * sn) * gate_factor(a.gate, a.gate_stride, a.nq, row_index, d));
+      a.out[row_index * DV + d + DV / 2] = (bf16_t)((v * c - u * sn) * gate_factor(a.gate, a.gate_stride, a.nq, row_index, d + DV / 2));
     }
     return;  // one split: there are no parts to mark empty
   }
-  for (int idx = threadIdx.x; idx < 16 * D; idx += 64 * DW) {
-    const int row = idx / D, d = idx - row * D;
+  for (int idx = threadIdx.x; idx < 16 * DV; idx += 64 * DW) {
+    const int row = idx / DV, d = idx - row * DV;
     if (row >= n_rows) continue;
     float mm, den;
     const float val = joined(row, d, mm, den);
     const int rt = row / g, rh = row - rt * g;
     const size_t row_index = tile_row0 + (size_t)rt * a.nq + kvh * g + rh;
     if (a.num_splits == 1) {
-      a.out[row_index * D + d] = (bf16_t)(val * gate_factor(a.gate, a.gate_stride, a.nq, row_index, d));
+      a.out[row_index * DV + d] = (bf16_t)(val * gate_factor(a.gate, a.gate_stride, a.nq, row_index, d));
     } else {
-      a.part_o[(row_index * a.num_splits + split) * D + d] = val;
+      a.part_o[(row_index * a.num_splits + split) * DV + d] = val;
       if (d == 0) a.part_lse[row_index * a.num_splits + split] = den > 0.f ? mm + log2f(den) : -INFINITY;
     }
   }
@@ -1472,7 +1477,7 @@ extern "C" int qrt_attention_bf16_decode(const AttnTileArgs* args, int num_rows_
   AttnTileArgs a = *args;
   QRT_CHECK(a.nq > 0 && a.nkv > 0 && a.nq % a.nkv == 0, "attention: %d query heads do not divide into %d key heads",
             a.nq, a.nkv);
-  QRT_CHECK(D <= 256, "attention (decode): head size %d is above 256", D);
+  QRT_CHECK(DMAX <= 256, "attention (decode): head size %d is above 256", DMAX);
   QRT_CHECK(a.page_size > 0 && a.page_size % 8 == 0,
             "attention (bfloat16): page size %d must be a multiple of 8", a.page_size);
   QRT_CHECK(a.num_splits >= 1 && a.num_splits <= 65535 && a.nkv <= 65535, "attention: bad split or head count");
@@ -1481,8 +1486,8 @@ extern "C" int qrt_attention_bf16_decode(const AttnTileArgs* args, int num_rows_
   QRT_CHECK(a.chunk >= 0 && !(a.chunk > 0 && a.window > 0), "attention: a window or a mask of chunks, not both");
   QRT_CHECK(a.keep_first >= 0 && (a.keep_first == 0 || a.window > 0), "attention: first keys are kept beside a window");
   QRT_CHECK((a.cap_in > 0.f) == (a.cap_out > 0.f), "attention: a score cap needs both of its factors");
-  QRT_CHECK(!a.gate || a.gate_stride >= (long)a.nq * D, "attention: the gate's rows are %ld elements apart, %d heads of %d need more",
-            a.gate_stride, a.nq, D);
+  QRT_CHECK(!a.gate || a.gate_stride >= (long)a.nq * DV, "attention: the gate's rows are %ld elements apart, %d heads of %d need more",
+            a.gate_stride, a.nq, DV);
   QRT_CHECK(a.items ? a.split_blocks > 0 && a.max_items >= a.num_tiles && a.max_items <= 65535
                     : a.split_blocks == 0,
             "attention (decode): pieces of %d blocks with a list of %d items for %d sequences", a.split_blocks,
@@ -1491,7 +1496,7 @@ extern "C" int qrt_attention_bf16_decode(const AttnTileArgs* args, int num_rows_
   const bool p2 = (a.page_size & (a.page_size - 1)) == 0;  // shifts instead of divisions
   dim3 grid(a.num_tiles, a.nkv, a.num_splits), block(64 * DW);
   if (a.items) grid = dim3(a.nkv, a.max_items, 1);
-  constexpr size_t smem = (size_t)(2 * DW * 16 + DW * 16 * D) * sizeof(float);
+  constexpr size_t smem = (size_t)(2 * DW * 16 + DW * 16 * DV) * sizeof(float);
   if (smem > 64 * 1024) {  // head size 256: a little more LDS than a block gets without asking
     static bool allowed = false;  // once: not again inside every stream capture
     if (!allowed) {
@@ -1506,7 +1511,7 @@ extern "C" int qrt_attention_bf16_decode(const AttnTileArgs* args, int num_rows_
   if (a.qkv) {
     // one token per sequence, its query, key and value taken from the product that made them
     if constexpr (D % 64 == 0) {
-      QRT_CHECK(a.nq / a.nkv <= 16 && a.slots && a.qkv_stride >= (long)(a.nq + 2 * a.nkv) * D && a.qkv_stride % 8 == 0 &&
+      QRT_CHECK(a.nq / a.nkv <= 16 && a.slots && a.qkv_stride >= (long)(a.nq + a.nkv) * D + (long)a.nkv * DV && a.qkv_stride % 8 == 0 &&
                     (uintptr_t)a.qkv % 16 == 0,
                 "attention (decode, own token from the product): %d query heads per key head, stride %ld",
                 a.nq / a.nkv, a.qkv_stride);
@@ -1534,7 +1539,7 @@ extern "C" int qrt_attention_bf16_decode(const AttnTileArgs* args, int num_rows_
   if (a.num_splits > 1) {
     const int merge_rows = a.merge_tokens ? a.num_merge_tokens * a.nq : num_rows_total;
     if (merge_rows > 0)
-      attention_merge_kernel<<<dim3(merge_rows), dim3(D > 128 ? 256 : (D >= 64 ? 64 : 32)), 0, stream>>>(
+      attention_merge_kernel<<<dim3(merge_rows), dim3(DV > 128 ? 256 : (DV >= 64 ? 64 : 32)), 0, stream>>>(
           a.part_o, a.part_lse, a.out, a.num_splits, a.merge_tokens, a.nq, a.gate, a.gate_stride, a.sink, a.turn);
     QRT_LAUNCH_CHECK("attention_merge");
   }
@@ -1554,8 +1559,8 @@ extern "C" int qrt_attention_bf16(const AttnTileArgs* args, int num_rows_total, 
   QRT_CHECK(a.chunk >= 0 && !(a.chunk > 0 && a.window > 0), "attention: a window or a mask of chunks, not both");
   QRT_CHECK(a.keep_first >= 0 && (a.keep_first == 0 || a.window > 0), "attention: first keys are kept beside a window");
   QRT_CHECK((a.cap_in > 0.f) == (a.cap_out > 0.f), "attention: a score cap needs both of its factors");
-  QRT_CHECK(!a.gate || a.gate_stride >= (long)a.nq * D, "attention: the gate's rows are %ld elements apart, %d heads of %d need more",
-            a.gate_stride, a.nq, D);
+  QRT_CHECK(!a.gate || a.gate_stride >= (long)a.nq * DV, "attention: the gate's rows are %ld elements apart, %d heads of %d need more",
+            a.gate_stride, a.nq, DV);
   if (a.num_tiles == 0) return 0;
   const bool p2 = (a.page_size & (a.page_size - 1)) == 0;  // shifts instead of divisions
   QRT_CHECK((long long)a.num_tiles * a.nkv < (1ll << 31), "attention: %d tiles x %d key heads is too many blocks", a.num_tiles, a.nkv);
@@ -1594,7 +1599,7 @@ extern "C" int qrt_attention_bf16(const AttnTileArgs* args, int num_rows_total, 
   if (a.num_splits > 1) {
     const int merge_rows = a.merge_tokens ? a.num_merge_tokens * a.nq : num_rows_total;
     if (merge_rows > 0)
-      attention_merge_kernel<<<dim3(merge_rows), dim3(D > 128 ? 256 : (D >= 64 ? 64 : 32)), 0, stream>>>(
+      attention_merge_kernel<<<dim3(merge_rows), dim3(DV > 128 ? 256 : (DV >= 64 ? 64 : 32)), 0, stream>>>(
           a.part_o, a.part_lse, a.out, a.num_splits, a.merge_tokens, a.nq, a.gate, a.gate_stride, a.sink, a.turn);
     QRT_LAUNCH_CHECK("attention_merge");
   }

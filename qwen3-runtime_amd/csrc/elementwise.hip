@@ -597,35 +597,36 @@ __global__ __launch_bounds__(256) void qk_norm_rope_store_wide_kernel(QkArgs a, 
   }
 
   // values: 8 tokens of one head
+  const int Dv = a.value_dim, half_v = Dv >> 1;
   const long item = (long)(blockIdx.x - rope_blocks) * 4 + wave;
   const int token_groups = (a.num_tokens + 7) >> 3;
   if (item >= (long)token_groups * a.nv) return;
   const int tg = (int)(item / a.nv), hv = (int)(item - (long)tg * a.nv);
   const int t0 = 8 * tg, nvalid = min(8, a.num_tokens - t0);
-  const int row = D + 8;  // padded: the 8 tokens of an element lie in different banks
+  const int row = Dv + 8;  // padded: the 8 tokens of an element lie in different banks
   T* tile = (T*)smem_raw + (size_t)wave * 8 * row;
-  const int chunks = D >> 3;
+  const int chunks = Dv >> 3;
   if (a.v_rope) {  // 8 neighbouring pairs at a time, turned on their way into LDS
-    const int hc = D >> 4;
+    const int hc = Dv >> 4;
     for (int idx = lane; idx < 8 * hc; idx += 64) {
       const int j = idx / hc, c = idx - j * hc;
       if (j < nvalid) {
-        const T* src = (const T*)a.v_in + (size_t)(t0 + j) * a.v_stride + (size_t)hv * D + 8 * c;
-        const float* angles = a.v_rope + (size_t)(t0 + j) * D + 8 * c;
-        const Vec8<T> u = *(const Vec8<T>*)src, v = *(const Vec8<T>*)(src + half);
+        const T* src = (const T*)a.v_in + (size_t)(t0 + j) * a.v_stride + (size_t)hv * Dv + 8 * c;
+        const float* angles = a.v_rope + (size_t)(t0 + j) * Dv + 8 * c;
+        const Vec8<T> u = *(const Vec8<T>*)src, v = *(const Vec8<T>*)(src + half_v);
         Vec8<T> y1, y2;
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
-          const float x1 = to_f32<T>(u.v[e]), x2 = to_f32<T>(v.v[e]), cs = angles[e], sn = angles[half + e];
+          const float x1 = to_f32<T>(u.v[e]), x2 = to_f32<T>(v.v[e]), cs = angles[e], sn = angles[half_v + e];
           y1.v[e] = from_f32<T>(x1 * cs - x2 * sn);
           y2.v[e] = from_f32<T>(x2 * cs + x1 * sn);
         }
         *(Vec8<T>*)(tile + j * row + 8 * c) = y1;
-        *(Vec8<T>*)(tile + j * row + half + 8 * c) = y2;
+        *(Vec8<T>*)(tile + j * row + half_v + 8 * c) = y2;
         if (a.v_out) {
-          T* dense = (T*)a.v_out + ((size_t)(t0 + j) * a.nv + hv) * D + 8 * c;
+          T* dense = (T*)a.v_out + ((size_t)(t0 + j) * a.nv + hv) * Dv + 8 * c;
           *(Vec8<T>*)dense = y1;
-          *(Vec8<T>*)(dense + half) = y2;
+          *(Vec8<T>*)(dense + half_v) = y2;
         }
       }
     }
@@ -633,9 +634,9 @@ __global__ __launch_bounds__(256) void qk_norm_rope_store_wide_kernel(QkArgs a, 
   for (int idx = lane; idx < 8 * chunks; idx += 64) {
     const int j = idx / chunks, c = idx - j * chunks;
     if (j < nvalid) {
-      const Vec8<T> r = *(const Vec8<T>*)((const T*)a.v_in + (size_t)(t0 + j) * a.v_stride + (size_t)hv * D + 8 * c);
+      const Vec8<T> r = *(const Vec8<T>*)((const T*)a.v_in + (size_t)(t0 + j) * a.v_stride + (size_t)hv * Dv + 8 * c);
       *(Vec8<T>*)(tile + j * row + 8 * c) = r;
-      if (a.v_out) *(Vec8<T>*)((T*)a.v_out + ((size_t)(t0 + j) * a.nv + hv) * D + 8 * c) = r;
+      if (a.v_out) *(Vec8<T>*)((T*)a.v_out + ((size_t)(t0 + j) * a.nv + hv) * Dv + 8 * c) = r;
     }
   }
   if (!a.slots) return;
@@ -646,8 +647,8 @@ __global__ __launch_bounds__(256) void qk_norm_rope_store_wide_kernel(QkArgs a, 
   const bool wide = nvalid == 8 && (s0 & 7) == 0 && (a.page_size & 7) == 0 && __all(in_line);
   if (wide) {
     const int page = s0 / a.page_size, off = s0 - page * a.page_size;
-    T* base = (T*)a.v_cache + ((size_t)page * a.nv + hv) * D * a.page_size + off;
-    for (int d = lane; d < D; d += 64) {
+    T* base = (T*)a.v_cache + ((size_t)page * a.nv + hv) * Dv * a.page_size + off;
+    for (int d = lane; d < Dv; d += 64) {
       Vec8<T> o;
 #pragma unroll
       for (int j = 0; j < 8; ++j) o.v[j] = tile[j * row + d];
@@ -657,8 +658,8 @@ __global__ __launch_bounds__(256) void qk_norm_rope_store_wide_kernel(QkArgs a, 
     for (int j = 0; j < nvalid; ++j) {
       const int sj = __shfl(my_slot, j, 64);
       const int page = sj / a.page_size, off = sj - page * a.page_size;
-      T* base = (T*)a.v_cache + ((size_t)page * a.nv + hv) * D * a.page_size + off;
-      for (int d = lane; d < D; d += 64) base[(size_t)d * a.page_size] = tile[j * row + d];
+      T* base = (T*)a.v_cache + ((size_t)page * a.nv + hv) * Dv * a.page_size + off;
+      for (int d = lane; d < Dv; d += 64) base[(size_t)d * a.page_size] = tile[j * row + d];
     }
   }
 }
@@ -690,7 +691,8 @@ extern "C" int qrt_qk_norm_rope_store(const QkArgs* args, int dtype, long num_ca
   const int D = a.head_dim;
   // few tokens (decoding): the time is the launch and one round of memory latency, and the
   // one-head-per-wave kernel has the shorter chain
-  const bool wide = a.num_tokens >= 32 && D >= 16 && a.value_dim == D && (D & (D - 1)) == 0 && a.rot_pairs % 8 == 0 && a.q_stride % 8 == 0 && a.k_stride % 8 == 0 &&
+  const size_t smem = (size_t)waves * 8 * (a.value_dim + 8) * esize;
+  const bool wide = a.num_tokens >= 32 && D >= 16 && a.value_dim % 16 == 0 && smem <= 64 * 1024 && (D & (D - 1)) == 0 && a.rot_pairs % 8 == 0 && a.q_stride % 8 == 0 && a.k_stride % 8 == 0 &&
                     a.v_stride % 8 == 0 && lined_up(a.q_in) && lined_up(a.k_in) && lined_up(a.v_in) &&
                     lined_up(a.q_out) && lined_up(a.k_out) && lined_up(a.v_out) && lined_up(a.k_cache) &&
                     lined_up(a.v_cache);
@@ -705,7 +707,6 @@ extern "C" int qrt_qk_norm_rope_store(const QkArgs* args, int dtype, long num_ca
     const long rope_blocks = (rope_items + waves - 1) / waves, v_blocks = (v_items + waves - 1) / waves;
     QRT_CHECK(rope_blocks + v_blocks < (1l << 31), "qk_norm_rope_store: too many tokens");
     dim3 grid((unsigned)(rope_blocks + v_blocks)), block(64 * waves);
-    const size_t smem = (size_t)waves * 8 * (D + 8) * esize;
     if (dtype == QRT_F32)
       qk_norm_rope_store_wide_kernel<float><<<grid, block, smem, stream>>>(a, lph, (int)rope_blocks, ppw);
     else if (dtype == QRT_BF16)

@@ -2,7 +2,7 @@
 
 Two kinds of library of the engine's own: ``core`` (everything whose sizes are
 run-time arguments) and ``attn_bf16_d<D>`` (the MFMA attention kernel, one build
-per head size). A part defined elsewhere brings its kernels with
+per head size, ``attn_bf16_d<D>v<DV>`` where values have another size than keys). A part defined elsewhere brings its kernels with
 ``register_library(name, sources)`` and loads them with ``ops.hip.load_library``:
 same flags, same cache, same error reporting, no edit here. A library is rebuilt when the hash of its sources and flags changes. The build
 is plain ``hipcc`` for gfx950: seconds per file, no Python headers involved, so
@@ -108,10 +108,11 @@ def library_spec(name: str) -> tuple[list, list[str]]:
     if name in _REGISTERED:
         return list(_REGISTERED[name][0]), list(_REGISTERED[name][1])
     if name.startswith("attn_bf16_d"):
-        d = int(name[len("attn_bf16_d"):])
-        if d % 16 or not 16 <= d <= 512:
-            raise BuildError(f"the bfloat16 attention kernel takes head sizes 16..512 in steps of 16, not {d}")
-        return ["runtime.hip", "attention_bf16.hip"], [f"-DQRT_HEAD_DIM={d}"]
+        # attn_bf16_d<D>, or attn_bf16_d<D>v<DV> where values have another size than keys
+        sizes = [int(x) for x in name[len("attn_bf16_d"):].split("v")]
+        if not 1 <= len(sizes) <= 2 or any(x % 16 or not 16 <= x <= 512 for x in sizes):
+            raise BuildError(f"the bfloat16 attention kernel takes head sizes 16..512 in steps of 16, not {sizes}")
+        return ["runtime.hip", "attention_bf16.hip"], [f"-DQRT_HEAD_DIM={sizes[0]}"] + [f"-DQRT_VALUE_DIM={x}" for x in sizes[1:]]
     raise BuildError(f"unknown library {name!r}; registered from outside: {registered_libraries()}")
 
 
@@ -179,10 +180,14 @@ def build_library(name: str, force: bool = False) -> Path:
     return so
 
 
-def build_all(head_dims=(16, 32, 48, 64, 80, 96, 112, 128, 160, 176, 256, 320, 448, 512), force: bool = True) -> list[Path]:
+def build_all(head_dims=(16, 32, 48, 64, 80, 96, 112, 128, 160, 176, 256, 320, 448, 512),
+              value_dims=((16, 48), (32, 16), (32, 80), (64, 16), (64, 32), (64, 128), (80, 48), (128, 64), (256, 16)),
+              force: bool = True) -> list[Path]:
     """Every library the tests, the smoke run and the measurements load (head sizes above 256 are
-    those of latent rows: latent plus turned key part). Three libraries at a time."""
-    names = ["core", "peaks"] + [f"attn_bf16_d{d}" for d in head_dims] + registered_libraries()
+    those of latent rows: latent plus turned key part; ``value_dims``: sizes of keys and values where they
+    differ). Three libraries at a time."""
+    names = ["core", "peaks"] + [f"attn_bf16_d{d}" for d in head_dims] + \
+        [f"attn_bf16_d{d}v{dv}" for d, dv in value_dims] + registered_libraries()
     first = build_library(names[0], force=force)  # the one with many sources compiles them side by side itself
     with ThreadPoolExecutor(3) as pool:
         return [first] + list(pool.map(lambda n: build_library(n, force=force), names[1:]))

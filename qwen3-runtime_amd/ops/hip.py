@@ -180,7 +180,7 @@ def _load(name: str) -> ctypes.CDLL:
 
 
 _core: ctypes.CDLL | None = None
-_attn: dict[int, ctypes.CDLL] = {}
+_attn: dict[tuple[int, int], ctypes.CDLL] = {}
 
 
 def core_library() -> ctypes.CDLL:
@@ -190,10 +190,12 @@ def core_library() -> ctypes.CDLL:
     return _core
 
 
-def attention_library(head_dim: int) -> ctypes.CDLL:
-    if head_dim not in _attn:
-        _attn[head_dim] = _load(f"attn_bf16_d{head_dim}")
-    return _attn[head_dim]
+def attention_library(head_dim: int, value_dim: int | None = None) -> ctypes.CDLL:
+    """The MFMA attention kernels of one size of keys and (None: the same) of values."""
+    key = (head_dim, value_dim or head_dim)
+    if key not in _attn:
+        _attn[key] = _load(f"attn_bf16_d{head_dim}" + ("" if key[1] == head_dim else f"v{key[1]}"))
+    return _attn[key]
 
 
 _extra: dict[str, ctypes.CDLL] = {}
@@ -1397,9 +1399,10 @@ class HipOps:
                                gate=None, keep_first=0, sink=False, rot_pairs=None, value_turn=None) -> bool:
         """Whether ``decode_attention`` serves this step: one token per sequence, bfloat16, a head
         size that keeps a rotation pair in one lane (a multiple of 64, up to 256; ``rot_pairs``, the pairs
-        of a head that turn, a multiple of 32), at most 16
+        of a head that turn, a multiple of 32; values of a multiple of 16, up to 256), at most 16
         query heads per key head, and a layer that writes its own cache."""
-        if value_dim not in (None, d) or (rot_pairs is not None and rot_pairs % 32):
+        dv = d if value_dim is None else value_dim
+        if dv % 16 or dv > 256 or (rot_pairs is not None and rot_pairs % 32) or qkv.shape[1] % 8:
             return False
         return (self.fuse_decode and qkv.dtype == torch.bfloat16 and ctx.max_q_len == 1
                 and ctx.num_tokens == ctx.num_seqs and d % 64 == 0 and d <= 256 and nq // nkv <= 16
@@ -1415,9 +1418,10 @@ class HipOps:
         key and value from registers and stores them into the cache for later steps. Saves the
         kernel between the product and the attention, and the round trip of the queries."""
         t, width = qkv.shape
+        dv = d if value_dim is None else int(value_dim)
         extra = 0 if gate is None else gate.shape[1]  # the gate's columns, behind q | k | v
-        _need(qkv, "qkv", torch.bfloat16, (t, (nq + 2 * nkv) * d + extra))
-        self._check_cache(cache, nkv, d, qkv.dtype)
+        _need(qkv, "qkv", torch.bfloat16, (t, (nq + nkv) * d + nkv * dv + extra))
+        self._check_cache(cache, nkv, d, qkv.dtype, dv)
         for name, w in (("q_norm", q_w), ("k_norm", k_w)):
             if w is not None:
                 _need(w, name, torch.float32, (d,))
@@ -1433,10 +1437,10 @@ class HipOps:
         own = {"qkv": qkv, "q_weight": q_w, "k_weight": k_w, "eps": eps,
                "rope": None if inv_freq is None else self.rope_table(ctx, inv_freq, angles_key),
                "rope_pairs": 0 if inv_freq is None else inv_freq.numel()}
-        out = torch.empty((t, nq * d), dtype=qkv.dtype, device=qkv.device)
+        out = torch.empty((t, nq * dv), dtype=qkv.dtype, device=qkv.device)
         self._launch_attention(None, out, cache, ctx, nq, nkv, d, scale, window or 0, None, True, own,
                                chunk=chunk or 0, softcap=softcap or 0.0, gate=gate, keep_first=keep_first, sink=sink,
-                               turn=self._turn_table(ctx, value_turn, d))
+                               turn=self._turn_table(ctx, value_turn, dv), dv=dv)
         return out
 
     def _turn_table(self, ctx, value_turn, dv):
@@ -1471,9 +1475,9 @@ class HipOps:
         out = torch.empty((t, nq * dv), dtype=q.dtype, device=q.device)
         if keep_first and not window:
             raise OpsError("first keys are kept in sight beside a window")
-        if dv == d and q.dtype == torch.bfloat16 and d % 16 == 0 and d <= 512 and ps % 8 == 0:
+        if q.dtype == torch.bfloat16 and d % 16 == 0 and d <= 512 and dv % 16 == 0 and dv <= 512 and ps % 8 == 0:
             self._attention_mfma(q, out, cache, ctx, nq, nkv, d, scale, window or 0, chunk or 0, softcap or 0.0, gate,
-                                 keep_first=int(keep_first), sink=bool(sink), turn=self._turn_table(ctx, value_turn, dv))
+                                 keep_first=int(keep_first), sink=bool(sink), turn=self._turn_table(ctx, value_turn, dv), dv=dv)
         else:
             a = _AttnArgs()
             a.q, a.out, a.k_cache, a.v_cache = q.data_ptr(), out.data_ptr(), cache.k.data_ptr(), cache.v.data_ptr()
@@ -1616,7 +1620,7 @@ class HipOps:
     split_launch_min_kv = 1024
 
     def _attention_mfma(self, q, out, cache, ctx, nq, nkv, d, scale, window, chunk=0, softcap=0.0, gate=None,
-                        keep_first=0, sink=False, turn=None):
+                        keep_first=0, sink=False, turn=None, dv=None):
         """Which kernel for which sequences. Steps of decoded tokens only: the decode kernel.
         Other steps: the prompt kernels; but sequences of at most 16 rows with a long context
         (decoded tokens beside a prompt portion) would each walk all their keys in one block
@@ -1626,11 +1630,13 @@ class HipOps:
             raise OpsError(f"the bfloat16 attention kernels take a positive score scale, not {scale}")
         g = nq // nkv
         seqs = range(ctx.num_seqs)
-        more = {"keep_first": keep_first, "sink": sink, "turn": turn}
-        if ctx.max_q_len * g <= 16 and d <= 256:
+        dv = dv or d
+        widest = max(d, dv)
+        more = {"keep_first": keep_first, "sink": sink, "turn": turn, "dv": dv}
+        if ctx.max_q_len * g <= 16 and widest <= 256:
             return self._launch_attention(q, out, cache, ctx, nq, nkv, d, scale, window, None, True, chunk=chunk, softcap=softcap, gate=gate, **more)
         small = [s for s in seqs if ctx.q_lens_host[s] * g <= 16]
-        if (d <= 256 and small and len(small) < ctx.num_seqs
+        if (widest <= 256 and small and len(small) < ctx.num_seqs
                 and max(ctx.kv_lens_host[s] for s in small) >= self.split_launch_min_kv):
             small_set = set(small)
             big = [s for s in seqs if s not in small_set]
@@ -1640,13 +1646,16 @@ class HipOps:
         self._launch_attention(q, out, cache, ctx, nq, nkv, d, scale, window, None, False, chunk=chunk, softcap=softcap, gate=gate, **more)
 
     def _launch_attention(self, q, out, cache, ctx, nq, nkv, d, scale, window, subset, decode, own=None,
-                          chunk=0, softcap=0.0, gate=None, keep_first=0, sink=False, turn=None):
+                          chunk=0, softcap=0.0, gate=None, keep_first=0, sink=False, turn=None, dv=None):
         """One launch over the sequences in ``subset`` (None: all of the step's). ``own``: the
         decode kernel takes the tokens' queries, own keys and own values from the q/k/v product
         (``decode_attention``); ``q`` is then None. ``chunk``: a mask of chunks in place of a
-        window; ``softcap``: the cap on the scaled scores; ``gate`` [T, nq * d] (columns of a wider
-        matrix will do): its sigmoid multiplies the output where the kernels write it."""
-        lib = attention_library(d)
+        window; ``softcap``: the cap on the scaled scores; ``gate`` [T, nq * dv] (columns of a wider
+        matrix will do): its sigmoid multiplies the output where the kernels write it. ``dv``: the size
+        of a value (None: ``d``)."""
+        dv = dv or d
+        widest = max(d, dv)
+        lib = attention_library(d, dv)
         # how far back a query can see at most: what the choices below (key splits, pieces) go by
         reach = window or chunk
         g = nq // nkv
@@ -1661,10 +1670,10 @@ class HipOps:
         waves = 1 if max_rows <= 16 else (2 if max_rows <= 32 else 4)
         # long portions: several row tiles per wave, so that loaded keys and values serve more rows
         # (heads wider than 256 fill a lane's registers with one tile)
-        row_tiles = 1 if max_rows <= 64 or d > 256 else (self.prefill_row_tiles if d <= 128 else min(2, self.prefill_row_tiles))
+        row_tiles = 1 if max_rows <= 64 or widest > 256 else (self.prefill_row_tiles if widest <= 128 else min(2, self.prefill_row_tiles))
         # the list depends on the rows a tile holds (head geometry and kernel choice): layers of
         # another geometry in the same step get a list of their own
-        key = ("attn_plan", g, nkv, d, waves, row_tiles, decode, None if subset is None else tuple(subset), reach)
+        key = ("attn_plan", g, nkv, widest, waves, row_tiles, decode, None if subset is None else tuple(subset), reach)
         plan = ctx.scratch.get(key)
         if plan is None:  # the same for every layer of the step
             dev = out.device
@@ -1688,17 +1697,17 @@ class HipOps:
             ctx.scratch[key] = plan
         tiles, n_tiles, tokens, groups = plan
         splits = ctx.scratch.get("attn_splits") or (
-            self.choose_decode_splits(n_tiles, nkv, seen_kv) if decode else self.choose_splits(n_tiles, nkv, seen_kv, d))
+            self.choose_decode_splits(n_tiles, nkv, seen_kv) if decode else self.choose_splits(n_tiles, nkv, seen_kv, widest))
         a = _AttnTileArgs()
         a.chunk = chunk
         # beside a window the sequence's first keys stay in sight; a sink: one more term in the softmax's sum
         a.keep_first, a.sink = int(keep_first), int(bool(sink))
-        a.turn = _addr(turn)  # float32 [T, d]: angles by which the outputs are turned back
+        a.turn = _addr(turn)  # float32 [T, dv]: angles by which the outputs are turned back
         if softcap:
             a.cap_in, a.cap_out = scale / softcap, softcap / scale
         if gate is not None:
-            if gate.dtype != torch.bfloat16 or tuple(gate.shape) != (ctx.num_tokens, nq * d) or gate.stride(1) != 1:
-                raise OpsError(f"gate {tuple(gate.shape)} {gate.dtype} does not fit {ctx.num_tokens} tokens of {nq} heads of {d}")
+            if gate.dtype != torch.bfloat16 or tuple(gate.shape) != (ctx.num_tokens, nq * dv) or gate.stride(1) != 1:
+                raise OpsError(f"gate {tuple(gate.shape)} {gate.dtype} does not fit {ctx.num_tokens} tokens of {nq} heads of {dv}")
             a.gate, a.gate_stride = gate.data_ptr(), gate.stride(0)
         piece = None
         if decode and n_tiles <= 1024:
@@ -1738,7 +1747,7 @@ class HipOps:
         a.use_lds = groups
         a.scale_log2 = scale * math.log2(math.e)
         if splits > 1:
-            part_o = torch.empty((ctx.num_tokens * nq * splits, d), dtype=torch.float32, device=out.device)
+            part_o = torch.empty((ctx.num_tokens * nq * splits, dv), dtype=torch.float32, device=out.device)
             part_lse = torch.empty((ctx.num_tokens * nq * splits,), dtype=torch.float32, device=out.device)
             a.part_o, a.part_lse = part_o.data_ptr(), part_lse.data_ptr()
         if piece:
