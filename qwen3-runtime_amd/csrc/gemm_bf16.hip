@@ -27,13 +27,16 @@ __device__ __forceinline__ bf16x8_t load_k8(const bf16_t* __restrict__ row, int 
   return v;
 }
 
-// What the gated products do with a gate and an up value: an activation of common.h, times a factor per
-// row of the activations (null: 1).
+// What the gated products do with a gate and an up value (their template's GATED: 0 no gate, 1 SwiGLU and
+// nothing else, 2 what is given here): an activation of common.h, times a factor per row of the
+// activations (null: 1).
 struct GatedEpilogue {
   int kind;
   float limit;
   const float* row_scale;
+  template <int GATED>
   __device__ __forceinline__ float apply(float g, float u, int m) const {
+    if (GATED == 1) return gated_act(g, u, QRT_ACT_SWIGLU, 0.f);
     const float v = gated_act(g, u, kind, limit);
     return row_scale ? v * row_scale[m] : v;
   }
@@ -117,7 +120,7 @@ __global__ __launch_bounds__(256) void gemm_bf16_kernel(const bf16_t* __restrict
 // GATED: W holds 2N rows, gate rows then up rows; the block owns matching
 // tiles of both and writes silu(gate) * up, so the gated feed-forward's
 // intermediate [M, 2N] never reaches memory.
-template <int MB, int NW, int NT, int U, bool GATED, typename TO>
+template <int MB, int NW, int NT, int U, int GATED, typename TO>
 __global__ __launch_bounds__(64 * NW) void gemm_bf16_skinny_kernel(const bf16_t* __restrict__ A,
                                                                     const bf16_t* __restrict__ W,
                                                                     TO* __restrict__ C, int M, int N, int K, GatedEpilogue ep) {
@@ -204,7 +207,7 @@ __global__ __launch_bounds__(64 * NW) void gemm_bf16_skinny_kernel(const bf16_t*
         if (nn + r < N) {
           // the gate and the up value are rounded to bfloat16 first, as the unfused kernels see them
           const float g = (float)(bf16_t)sum[r];
-          const float out = GATED ? ep.apply(g, (float)(bf16_t)sum2[r], m) : sum[r];
+          const float out = GATED ? ep.template apply<GATED>(g, (float)(bf16_t)sum2[r], m) : sum[r];
           C[(size_t)m * N + nn + r] = from_f32<TO>(out);
         }
       }
@@ -212,7 +215,7 @@ __global__ __launch_bounds__(64 * NW) void gemm_bf16_skinny_kernel(const bf16_t*
   }
 }
 
-template <int MB, int NW, int NT, int U, bool GATED>
+template <int MB, int NW, int NT, int U, int GATED>
 static int launch_skinny(const bf16_t* a, const bf16_t* w, void* c, int out_dtype, int M, int N, int K, const GatedEpilogue& ep,
                          hipStream_t stream) {
   dim3 grid((N + 16 * NT - 1) / (16 * NT)), block(64 * NW);
@@ -227,7 +230,7 @@ static int launch_skinny(const bf16_t* a, const bf16_t* w, void* c, int out_dtyp
   return 0;
 }
 
-template <bool GATED>
+template <int GATED>
 static int skinny(const bf16_t* a, const bf16_t* w, void* c, int out_dtype, int M, int N, int K, const GatedEpilogue& ep, hipStream_t st) {
   const int tiles = (N + 15) / 16;
   if (tiles >= 2048) return launch_skinny<1, 8, 2, 8, GATED>(a, w, c, out_dtype, M, N, K, ep, st);
@@ -266,7 +269,7 @@ static int skinny(const bf16_t* a, const bf16_t* w, void* c, int out_dtype, int 
 typedef const void __attribute__((address_space(1)))* global_ptr_t;
 typedef void __attribute__((address_space(3)))* lds_ptr_t;
 
-template <int NW, int NT, int U, bool GATED, typename TO>
+template <int NW, int NT, int U, int GATED, typename TO>
 __global__ __launch_bounds__(64 * NW) void gemm_bf16_rows_kernel(const bf16_t* __restrict__ A,
                                                                   const bf16_t* __restrict__ W,
                                                                   TO* __restrict__ C, int M, int N, int K, GatedEpilogue ep) {
@@ -367,7 +370,7 @@ __global__ __launch_bounds__(64 * NW) void gemm_bf16_rows_kernel(const bf16_t* _
       for (int r = 0; r < 4; ++r) {
         if (nn + r < N) {
           const float g = (float)(bf16_t)sum[r];  // rounded to bfloat16 first, as the unfused kernels see them
-          const float out = GATED ? ep.apply(g, (float)(bf16_t)sum2[r], m) : sum[r];
+          const float out = GATED ? ep.template apply<GATED>(g, (float)(bf16_t)sum2[r], m) : sum[r];
           C[(size_t)m * N + nn + r] = from_f32<TO>(out);
         }
       }
@@ -375,7 +378,7 @@ __global__ __launch_bounds__(64 * NW) void gemm_bf16_rows_kernel(const bf16_t* _
   }
 }
 
-template <int NW, int NT, int U, bool GATED>
+template <int NW, int NT, int U, int GATED>
 static int launch_rows(const bf16_t* a, const bf16_t* w, void* c, int out_dtype, int M, int N, int K, const GatedEpilogue& ep,
                        hipStream_t stream, int k_parts) {
   constexpr int WT = GATED ? 2 * NT : NT;
@@ -408,7 +411,7 @@ static int launch_rows(const bf16_t* a, const bf16_t* w, void* c, int out_dtype,
 // (19.1 us at the 4B size, 5.2 TB/s; 81.4 at the 32B size, 6.4 TB/s). The whole result: two tiles a block, except where K is a multiple of 2,048 (the rows of
 // two tiles then start in the same memory channels: 14.0 us against 11.2 for the 8B q/k/v product)
 // and for a few hundred tiles of long rows. K cut into planes: two tiles a block from K = 9,728 on.
-template <bool GATED>
+template <int GATED>
 static int few_rows(const bf16_t* a, const bf16_t* w, void* c, int out_dtype, int M, int N, int K, const GatedEpilogue& ep, hipStream_t st,
                     int k_parts) {
   const int tiles = (N + 15) / 16;
@@ -466,7 +469,7 @@ __device__ bf16x8_t qrt_zero_tile[64];
 //     batch (the others, read one pair ahead of their products).
 // Within a chunk, loads past the end of K are issued all the same, at clamped addresses, and count
 // as zero; behind the last chunk nothing is fetched, and its waits count accordingly.
-template <int MB, int KW, int NWV, int NT, int KC, bool GATED, typename TO>
+template <int MB, int KW, int NWV, int NT, int KC, int GATED, typename TO>
 __global__ __launch_bounds__(64 * KW * NWV) void gemm_bf16_mid_rows_kernel(const bf16_t* __restrict__ A,
                                                                             const bf16_t* __restrict__ W,
                                                                             TO* __restrict__ C, int M, int N, int K, GatedEpilogue ep) {
@@ -649,7 +652,7 @@ __global__ __launch_bounds__(64 * KW * NWV) void gemm_bf16_mid_rows_kernel(const
       for (int r = 0; r < 4; ++r) {
         if (GATED) {  // gate and up value rounded to bfloat16 first, as the unfused kernels see them
           const float g = (float)(bf16_t)acc[t][b][r];
-          o[r] = ep.apply(g, (float)(bf16_t)acc[NT + t][b][r], m);
+          o[r] = ep.template apply<GATED>(g, (float)(bf16_t)acc[NT + t][b][r], m);
         } else {
           o[r] = acc[t][b][r];
         }
@@ -659,7 +662,7 @@ __global__ __launch_bounds__(64 * KW * NWV) void gemm_bf16_mid_rows_kernel(const
   }
 }
 
-template <int MB, int KW, int NWV, int NT, int KC, bool GATED>
+template <int MB, int KW, int NWV, int NT, int KC, int GATED>
 static int launch_mid_rows(const bf16_t* a, const bf16_t* w, void* c, int out_dtype, int M, int N, int K, const GatedEpilogue& ep,
                            hipStream_t stream, int k_parts) {
   constexpr int WT = GATED ? 2 * NT : NT;
@@ -708,19 +711,20 @@ static int launch_mid_rows(const bf16_t* a, const bf16_t* w, void* c, int out_dt
 template <int MB>
 static int mid_rows(const bf16_t* a, const bf16_t* w, void* c, int out_dtype, int M, int N, int K, const GatedEpilogue& ep, int gated,
                     hipStream_t st, int k_parts) {
-  if (gated) return launch_mid_rows<MB, 1, 3, 1, 6, true>(a, w, c, out_dtype, M, N, K, ep, st, 1);
+  if (gated == 1) return launch_mid_rows<MB, 1, 3, 1, 6, 1>(a, w, c, out_dtype, M, N, K, ep, st, 1);
+  if (gated) return launch_mid_rows<MB, 1, 3, 1, 6, 2>(a, w, c, out_dtype, M, N, K, ep, st, 1);
   if (k_parts > 1) {
     if constexpr (MB % 2 == 0) {
-      if (MB > 4 || K % 2048 == 0) return launch_mid_rows<MB, 1, 8, 1, 4, false>(a, w, c, out_dtype, M, N, K, ep, st, k_parts);
+      if (MB > 4 || K % 2048 == 0) return launch_mid_rows<MB, 1, 8, 1, 4, 0>(a, w, c, out_dtype, M, N, K, ep, st, k_parts);
     } else {
-      if (K % 2048 == 0) return launch_mid_rows<MB, 1, 4, 1, 4, false>(a, w, c, out_dtype, M, N, K, ep, st, k_parts);
+      if (K % 2048 == 0) return launch_mid_rows<MB, 1, 4, 1, 4, 0>(a, w, c, out_dtype, M, N, K, ep, st, k_parts);
     }
-    if constexpr (MB <= 4) return launch_mid_rows<MB, 1, 4, 2, 8, false>(a, w, c, out_dtype, M, N, K, ep, st, k_parts);
+    if constexpr (MB <= 4) return launch_mid_rows<MB, 1, 4, 2, 8, 0>(a, w, c, out_dtype, M, N, K, ep, st, k_parts);
   }
   if constexpr (MB <= 4) {
-    if (N >= 32768) return launch_mid_rows<MB, 1, 4, 2, 8, false>(a, w, c, out_dtype, M, N, K, ep, st, 1);
-    if (K % 2048 == 0) return launch_mid_rows<MB, 3, 2, 1, 4, false>(a, w, c, out_dtype, M, N, K, ep, st, 1);
-    return launch_mid_rows<MB, 2, 2, 1, 8, false>(a, w, c, out_dtype, M, N, K, ep, st, 1);
+    if (N >= 32768) return launch_mid_rows<MB, 1, 4, 2, 8, 0>(a, w, c, out_dtype, M, N, K, ep, st, 1);
+    if (K % 2048 == 0) return launch_mid_rows<MB, 3, 2, 1, 4, 0>(a, w, c, out_dtype, M, N, K, ep, st, 1);
+    return launch_mid_rows<MB, 2, 2, 1, 8, 0>(a, w, c, out_dtype, M, N, K, ep, st, 1);
   }
   return qrt_fail("gemm_bf16: above 64 rows only the gated form and products cut along K have a kernel of their own (M=%d)", M);
 }
@@ -750,7 +754,7 @@ static int launch(const bf16_t* a, const bf16_t* w, void* c, int out_dtype, int 
 static int gemm(const void* a, const void* w, void* c, int out_dtype, int M, int N, int K, int gated, int shared, int k_parts,
                 const GatedEpilogue& ep, hipStream_t stream) {
   QRT_CHECK(M >= 0 && N > 0 && K > 0, "gemm_bf16: bad sizes M=%d N=%d K=%d", M, N, K);
-  QRT_CHECK(gated == 0 || gated == 1, "gemm_bf16: unknown mode %d", gated);
+  QRT_CHECK(gated >= 0 && gated <= 2, "gemm_bf16: unknown mode %d", gated);
   QRT_CHECK(shared == 0 || shared == 1, "gemm_bf16: unknown kernel choice %d", shared);
   QRT_CHECK(k_parts >= 1 && k_parts <= 64, "gemm_bf16: bad number of K parts %d", k_parts);
   QRT_CHECK(k_parts == 1 || (!gated && out_dtype == QRT_F32), "gemm_bf16: K parts need no gate and float32 output");
@@ -770,11 +774,13 @@ static int gemm(const void* a, const void* w, void* c, int out_dtype, int M, int
     return mid_rows<8>(A, W, c, out_dtype, M, N, K, ep, gated, stream, k_parts);
   }
   if (M <= 16 && aligned && K % 64 == 0)  // through LDS by direct loads: whole cache lines
-    return gated ? few_rows<true>(A, W, c, out_dtype, M, N, K, ep, stream, 1)
-                 : few_rows<false>(A, W, c, out_dtype, M, N, K, ep, stream, k_parts);
+    return gated == 1 ? few_rows<1>(A, W, c, out_dtype, M, N, K, ep, stream, 1)
+           : gated    ? few_rows<2>(A, W, c, out_dtype, M, N, K, ep, stream, 1)
+                      : few_rows<0>(A, W, c, out_dtype, M, N, K, ep, stream, k_parts);
   QRT_CHECK(k_parts == 1, "gemm_bf16: K parts need M <= 16 or the LDS-sharing kernel, and K %% 64 == 0 (M=%d K=%d)", M, K);
-  if (M <= 16 && aligned) return gated ? skinny<true>(A, W, c, out_dtype, M, N, K, ep, stream)
-                                       : skinny<false>(A, W, c, out_dtype, M, N, K, ep, stream);
+  if (M <= 16 && aligned) return gated == 1 ? skinny<1>(A, W, c, out_dtype, M, N, K, ep, stream)
+                                : gated    ? skinny<2>(A, W, c, out_dtype, M, N, K, ep, stream)
+                                           : skinny<0>(A, W, c, out_dtype, M, N, K, ep, stream);
   QRT_CHECK(gated == 0, "gemm_bf16: the gated form needs K a multiple of 32 and M <= 16, or the LDS-sharing kernel "
             "(M=%d K=%d)", M, K);
   if (M <= 16) return launch<1, 2>(A, W, c, out_dtype, M, N, K, stream);
@@ -784,6 +790,7 @@ static int gemm(const void* a, const void* w, void* c, int out_dtype, int M, int
 
 extern "C" int qrt_gemm_bf16(const void* a, const void* w, void* c, int out_dtype, int M, int N, int K, int gated,
                              int shared, int k_parts, hipStream_t stream) {
+  QRT_CHECK(gated == 0 || gated == 1, "gemm_bf16: unknown mode %d", gated);
   return gemm(a, w, c, out_dtype, M, N, K, gated, shared, k_parts, GatedEpilogue{QRT_ACT_SWIGLU, 0.f, nullptr}, stream);
 }
 
@@ -791,5 +798,6 @@ extern "C" int qrt_gemm_bf16(const void* a, const void* w, void* c, int out_dtyp
 extern "C" int qrt_gated_gemm_bf16(const void* a, const void* w, void* c, int out_dtype, int M, int N, int K, int shared,
                                    int act_kind, float limit, const float* row_scale, hipStream_t stream) {
   QRT_CHECK(act_kind == QRT_ACT_SWIGLU || act_kind == QRT_ACT_CLAMPED, "gated_gemm_bf16: unknown activation %d", act_kind);
-  return gemm(a, w, c, out_dtype, M, N, K, 1, shared, 1, GatedEpilogue{act_kind, limit, row_scale}, stream);
+  const int mode = act_kind == QRT_ACT_SWIGLU && !row_scale ? 1 : 2;
+  return gemm(a, w, c, out_dtype, M, N, K, mode, shared, 1, GatedEpilogue{act_kind, limit, row_scale}, stream);
 }
