@@ -29,7 +29,7 @@ feed-forward a mixture of 16 experts, 2 a token) have the widths, heads, layers 
 ``qwen3_4b``; ``--preset zisedra_4b`` (delta rule beside windowed attention) and ``--preset roserax_4b``
 (latent attention, retention, windowed attention with kept first tokens and a sink) have those sizes
 too, ``*_2b`` and ``*_8b`` smaller and larger ones, as have ``--preset zuvasun_4b`` (latent attention with shared
-latents, attention whose values are its keys) ``--preset sarudra_4b`` (state-space mixers, windowed
+latents, attention whose values are its keys), ``--preset sarudra_4b`` (state-space mixers, windowed
 attention with turned values) and ``--preset dekinex_4b`` (matrix memories, windowed attention behind short
 convolutions).
 

@@ -63,7 +63,7 @@ __global__ __launch_bounds__(64 * W) void memory_gates_kernel(GatesArgs a) {
         if (lane >= o) u = fmax(u, before);
       }
     }
-    float next = 0.f;  // the maximum behind this round's tokens
+    float next = 0.f;  // the maximum behind these 1,024 tokens
     if (SPREAD) {
       if (lane == last) {
         tile_sum[wave] = F;

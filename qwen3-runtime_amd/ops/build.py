@@ -180,7 +180,7 @@ def build_library(name: str, force: bool = False) -> Path:
     return so
 
 
-def build_all(head_dims=(16, 32, 48, 64, 80, 96, 112, 128, 160, 176, 256, 320, 448, 512),
+def build_all(head_dims=(16, 32, 48, 64, 80, 96, 112, 128, 160, 176, 192, 208, 256, 320, 448, 512),
               value_dims=((16, 48), (32, 16), (32, 80), (64, 16), (64, 32), (64, 128), (80, 48), (128, 64), (256, 16)),
               force: bool = True) -> list[Path]:
     """Every library the tests, the smoke run and the measurements load (head sizes above 256 are
